@@ -150,6 +150,9 @@ typedef struct mesh_tensor_info {
 /* Header-only scan of a GGUF file: hyper-parameters and container facts, no tensor data touched.
  * The bounded parse of mesh-client/src/models/gguf.rs:318-420 (scan_gguf_compact_meta). */
 int mesh_gguf_probe(const char *gguf_path, mesh_model_info *out);
+/* The same summary for a GGUF file or a model folder (config.json; sizes that differ between layers: the largest; the
+ * container fields are 0 for a folder). */
+int mesh_model_probe(const char *path, mesh_model_info *out);
 /* Directory entry of one tensor by name -- the lookup rpc_server::set_tensor_gguf does (patches/0001:203-209).
  * MESH_ERR_INVALID if the tensor is absent, MESH_ERR_FORMAT if its bytes would leave the file. */
 int mesh_gguf_tensor(const char *gguf_path, const char *name, mesh_tensor_info *out);
@@ -166,6 +169,9 @@ typedef struct mesh_session mesh_session;
  * device buffer and has no such limit. */
 #define MESH_LOGITS_TOKENS_MAX 128
 
+#define MESH_PRECISION_DEFAULT 0
+#define MESH_PRECISION_F32 1
+
 typedef struct mesh_stage_opts {
     const char *device;     /* "ROCm0" / "HIP0" / "0"; NULL = current device               (-d, launch.rs:920-952) */
     int32_t n_ctx;          /* KV positions per sequence; 0 = 4096                          (-c, launch.rs:474-504) */
@@ -176,16 +182,22 @@ typedef struct mesh_stage_opts {
                                KvCacheQuant::for_model_size (launch.rs:568-591) are supported: f16/f16, q8_0/q4_0, q4_0/q4_0 */
     const char *tuning;     /* kernel-selection switches as "name=value,name=value"; NULL = the defaults.  See
                                mesh_session_set_option for the names.  No counterpart in the reference. */
+    int32_t precision;      /* MESH_PRECISION_DEFAULT, or MESH_PRECISION_F32: every product, activation and cache row in 32
+                               bits (models in a folder only; MESH_ERR_UNSUPPORTED for GGUF models) */
 } mesh_stage_opts;
 
 typedef struct mesh_batch {
     int32_t n_tokens;
     const int32_t *pos;     /* [n_tokens] cache position of each token */
     const int32_t *seq_id;  /* [n_tokens] sequence of each token; NULL = all 0 */
+    const int32_t *token_id;/* [n_tokens] token ids, for models whose layers read them (a folder model; not needed when
+                               the input itself is MESH_TOKENS through the host-pointer call); NULL otherwise */
+    const uint8_t *want;    /* [n_tokens], MESH_LOGITS output only: nonzero = return this token's logits, rows in batch
+                               order; NULL = every token's.  All zero is allowed and returns no bytes. */
 } mesh_batch;
 
-/* Load layers [layer_begin, layer_end) of the GGUF model at gguf_path into HBM (layer_end < 0 = to the last
- * layer).  What `rpc-server --gguf PATH` plus the SET_TENSOR_GGUF traffic of start-up amount to
+/* Load layers [layer_begin, layer_end) of the model at gguf_path into HBM (layer_end < 0 = to the last layer): a
+ * GGUF file, or a folder with config.json and model.safetensors (architectures described layer by layer).  What `rpc-server --gguf PATH` plus the SET_TENSOR_GGUF traffic of start-up amount to
  * (mesh-llm/src/inference/launch.rs:887-1030; patches/0001:179-266). */
 int mesh_stage_open(const char *gguf_path, int layer_begin, int layer_end, const mesh_stage_opts *opts, mesh_stage **out);
 void mesh_stage_close(mesh_stage *stage);
@@ -200,13 +212,18 @@ void mesh_stage_session_free(mesh_session *session);
 /* Run the stage over a batch: `in` holds n_tokens rows of n_embd in in_fmt (MESH_F32 / MESH_F16 / MESH_Q8_0, the
  * boundary tensor of the previous stage) or int32 token ids (MESH_TOKENS); each token's K/V is stored at
  * (seq_id, pos) and it attends to positions [0, pos] of its sequence.  `out` receives the boundary hidden state
- * packed in out_fmt, or logits (MESH_LOGITS).  *out_len = bytes written (set even when out_cap is too small).
+ * packed in out_fmt, or logits (MESH_LOGITS).  A model with recurrent layers carries a state per sequence: a call's tokens
+ * of a sequence are then neighbours, ascend by one, and go on where the sequence stands, or start at position 0, which
+ * gives the sequence a fresh state; anything else is MESH_ERR_INVALID.  *out_len = bytes written (set even when out_cap is too small).
  * Host pointers; blocks until done.  The GRAPH_COMPUTE + tensor push of one step (patches/0002:443-451,544-622). */
 int mesh_stage_decode(mesh_session *session, const mesh_batch *batch, const void *in, int in_fmt,
                       void *out, int out_fmt, size_t out_cap, size_t *out_len);
 /* Same with device pointers for in/out; queued on the session's stream, returns without waiting. */
 int mesh_stage_decode_dev(mesh_session *session, const mesh_batch *batch, const void *d_in, int in_fmt,
                           void *d_out, int out_fmt, size_t out_cap, size_t *out_len);
+/* Forget what sequence seq_id holds: its slot is free for another request, which starts at position 0.  No counterpart in the
+ * reference (llama_memory_seq_rm inside llama.cpp). */
+int mesh_session_seq_reset(mesh_session *session, int seq_id);
 /* The session's hipStream_t (for events), and a wait for everything queued on it. */
 void *mesh_session_stream(mesh_session *session);
 int mesh_session_synchronize(mesh_session *session);
@@ -281,6 +298,8 @@ int mesh_session_f16_saturations(mesh_session *session, uint64_t *count);
  *     moe_fuse_quant=1     the expert combine step quantises for the next layer
  *     moe_gemm=1, moe_gemm_min_pairs=4   prefill-sized expert products on the large-tile GEMM
  *     grouped_oversub=8    grouped expert mat-vec: workgroups per compute unit and item
+ *     linear_tile_min_tokens=128  bf16 products of at least this many tokens on the large matrix-core tile
+ *     step_fused=1         bf16 models, one token: norms, activations and residual updates ride in the products
  *     graphs=0             decode steps of up to 32 tokens replayed from captured HIP graphs
  *
  * MESH_ERR_INVALID: unknown name, value out of range, or a stage-level switch passed to set_option.  No counterpart in

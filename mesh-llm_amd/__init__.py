@@ -66,13 +66,14 @@ class StageOpts(ctypes.Structure):
     """mesh_stage_opts"""
     _fields_ = [("device", ctypes.c_char_p), ("n_ctx", ctypes.c_int32), ("n_seq_max", ctypes.c_int32),
                 ("n_batch_max", ctypes.c_int32), ("kv_type", ctypes.c_int32), ("kv_type_v", ctypes.c_int32),
-                ("tuning", ctypes.c_char_p)]
+                ("tuning", ctypes.c_char_p), ("precision", ctypes.c_int32)]
 
 
 class Batch(ctypes.Structure):
     """mesh_batch"""
     _fields_ = [("n_tokens", ctypes.c_int32), ("pos", ctypes.POINTER(ctypes.c_int32)),
-                ("seq_id", ctypes.POINTER(ctypes.c_int32))]
+                ("seq_id", ctypes.POINTER(ctypes.c_int32)), ("token_id", ctypes.POINTER(ctypes.c_int32)),
+                ("want", ctypes.POINTER(ctypes.c_uint8))]
 
 
 class Profile(ctypes.Structure):
@@ -82,6 +83,8 @@ class Profile(ctypes.Structure):
 
 PROF_GEMV, PROF_ROPE, PROF_ATTN, PROF_CODEC, PROF_PREP = 0, 1, 2, 3, 4
 TOKENS, LOGITS = 100, 101
+PRECISION_DEFAULT, PRECISION_F32 = 0, 1
+LOGITS_TOKENS_MAX = 128     # MESH_LOGITS_TOKENS_MAX
 _pp = ctypes.POINTER(ctypes.c_void_p)
 _psz = ctypes.POINTER(ctypes.c_size_t)
 
@@ -92,6 +95,7 @@ SIGNATURES.update({
     "mesh_mul_mat_dev": (_i32, [_vp, _vp, _i64, _vp, _vp]),
     "mesh_weight_download": (_i32, [_vp, _vp]),
     "mesh_gguf_probe": (_i32, [_cp, ctypes.POINTER(ModelInfo)]),
+    "mesh_model_probe": (_i32, [_cp, ctypes.POINTER(ModelInfo)]),
     "mesh_gguf_tensor": (_i32, [_cp, _cp, ctypes.POINTER(TensorInfo)]),
     "mesh_stage_open": (_i32, [_cp, _i32, _i32, ctypes.POINTER(StageOpts), _pp]),
     "mesh_stage_close": (None, [_vp]),
@@ -101,6 +105,7 @@ SIGNATURES.update({
     "mesh_stage_session_free": (None, [_vp]),
     "mesh_stage_decode": (_i32, [_vp, ctypes.POINTER(Batch), _vp, _i32, _vp, _i32, _sz, _psz]),
     "mesh_stage_decode_dev": (_i32, [_vp, ctypes.POINTER(Batch), _vp, _i32, _vp, _i32, _sz, _psz]),
+    "mesh_session_seq_reset": (_i32, [_vp, _i32]),
     "mesh_session_stream": (_vp, [_vp]),
     "mesh_session_synchronize": (_i32, [_vp]),
     "mesh_session_graph_replays": (_i64, [_vp]),
@@ -288,6 +293,13 @@ def gguf_probe(path):
     return info
 
 
+def model_probe(path):
+    """Summary of a GGUF file or a model folder."""
+    info = ModelInfo()
+    check(lib().mesh_model_probe(os.fsencode(path), ctypes.byref(info)))
+    return info
+
+
 def gguf_tensor(path, name):
     info = TensorInfo()
     check(lib().mesh_gguf_tensor(os.fsencode(path), name.encode(), ctypes.byref(info)))
@@ -296,15 +308,18 @@ def gguf_tensor(path, name):
 
 # ---------------------------------------------------------------------------------------------- stage
 class Stage:
-    """Layers [layer_begin, layer_end) of a GGUF model resident on the GPU (mesh_stage)."""
+    """Layers [layer_begin, layer_end) of a model resident on the GPU (mesh_stage): a GGUF file, or a folder with config.json
+    and model.safetensors."""
 
-    def __init__(self, gguf_path, layer_begin, layer_end=-1, n_ctx=0, n_seq_max=0, n_batch_max=0, device=None, kv_types=None, tuning=None):
+    def __init__(self, gguf_path, layer_begin, layer_end=-1, n_ctx=0, n_seq_max=0, n_batch_max=0, device=None, kv_types=None, tuning=None,
+                 precision=PRECISION_DEFAULT):
         """kv_types: (K, V) cache row types, one of (F16, F16), (Q8_0, Q4_0), (Q4_0, Q4_0); None = f16 / f16.
-        tuning: kernel-selection switches, {"name": value} or "name=value,..." (mesh_stage_opts.tuning)."""
+        tuning: kernel-selection switches, {"name": value} or "name=value,..." (mesh_stage_opts.tuning).
+        precision: PRECISION_F32 runs a folder model in 32 bits throughout."""
         kt, vt = kv_types if kv_types else (0, 0)
         if isinstance(tuning, dict):
             tuning = ",".join("%s=%d" % (k, int(v)) for k, v in tuning.items())
-        opts = StageOpts(device.encode() if device else None, n_ctx, n_seq_max, n_batch_max, kt, vt, tuning.encode() if tuning else None)
+        opts = StageOpts(device.encode() if device else None, n_ctx, n_seq_max, n_batch_max, kt, vt, tuning.encode() if tuning else None, precision)
         self._h = ctypes.c_void_p()
         check(lib().mesh_stage_open(os.fsencode(gguf_path), layer_begin, layer_end, ctypes.byref(opts), ctypes.byref(self._h)))
         self.info = ModelInfo()
@@ -336,17 +351,28 @@ class Session:
         check(lib().mesh_stage_session_new(stage._h, ctypes.byref(self._h)))
 
     @staticmethod
-    def _batch(pos, seq):
+    def _batch(pos, seq, token_ids=None, want=None):
         import numpy as np
         pos = np.ascontiguousarray(pos, dtype=np.int32)
         seq = np.zeros_like(pos) if seq is None else np.ascontiguousarray(seq, dtype=np.int32)
         b = Batch(pos.size, pos.ctypes.data_as(ctypes.POINTER(ctypes.c_int32)), seq.ctypes.data_as(ctypes.POINTER(ctypes.c_int32)))
-        return b, (pos, seq)
+        if token_ids is not None:
+            token_ids = np.ascontiguousarray(token_ids, dtype=np.int32)
+            b.token_id = token_ids.ctypes.data_as(ctypes.POINTER(ctypes.c_int32))
+        if want is not None:
+            want = np.ascontiguousarray(want, dtype=np.uint8)
+            b.want = want.ctypes.data_as(ctypes.POINTER(ctypes.c_uint8))
+        for extra in (token_ids, want):
+            if extra is not None and extra.size != pos.size:
+                raise ValueError("token_ids and want take one entry per token")
+        return b, (pos, seq, token_ids, want)
 
-    def decode(self, inp, pos, seq=None, in_fmt=F32, out_fmt=F32):
-        """Host form.  inp: numpy array holding the packed input (f32 rows, f16 bits, q8_0 bytes or int32 ids)."""
+    def decode(self, inp, pos, seq=None, in_fmt=F32, out_fmt=F32, token_ids=None, want=None):
+        """Host form.  inp: numpy array holding the packed input (f32 rows, f16 bits, q8_0 bytes or int32 ids).
+        token_ids: ids of the tokens, for layers that read them when the input is not the ids themselves.
+        want: one flag per token, for LOGITS output: the tokens whose rows are returned (default all)."""
         import numpy as np
-        b, keep = self._batch(pos, seq)
+        b, keep = self._batch(pos, seq, token_ids, want)
         inp = np.ascontiguousarray(inp)
         T = b.n_tokens
         if out_fmt == LOGITS:
@@ -364,8 +390,8 @@ class Session:
         check(rc)
         return out[:n.value]
 
-    def decode_dev(self, d_in, pos, d_out, out_cap, seq=None, in_fmt=F32, out_fmt=F32):
-        b, keep = self._batch(pos, seq)
+    def decode_dev(self, d_in, pos, d_out, out_cap, seq=None, in_fmt=F32, out_fmt=F32, token_ids=None, want=None):
+        b, keep = self._batch(pos, seq, token_ids, want)
         n = ctypes.c_size_t(0)
         check(lib().mesh_stage_decode_dev(self._h, ctypes.byref(b), d_in, in_fmt, d_out, out_fmt, out_cap, ctypes.byref(n)))
         return n.value
@@ -376,6 +402,10 @@ class Session:
 
     def synchronize(self):
         check(lib().mesh_session_synchronize(self._h))
+
+    def seq_reset(self, seq_id):
+        """Give back what sequence seq_id holds (mesh_session_seq_reset)."""
+        check(lib().mesh_session_seq_reset(self._h, seq_id))
 
     def attn_dev(self, layer, d_q, pos, d_out, seq=None, matrix_cores=True):
         """Decode attention of one layer over this session's KV cache (mesh_session_attn_dev); device pointers."""

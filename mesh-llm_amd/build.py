@@ -41,10 +41,11 @@ def build(verbose=False):
         for obj, warn in results:
             if warn:
                 print(warn, file=sys.stderr)
-    cmd = [HIPCC, "--offload-arch=gfx950", "-shared", "-fPIC", "-o", LIB, *[o for o, _ in results]]
+    cmd = [HIPCC, "--offload-arch=gfx950", "-shared", "-fPIC", "-o", LIB + ".part", *[o for o, _ in results]]
     r = subprocess.run(cmd, capture_output=True, text=True)
     if r.returncode != 0:
         raise RuntimeError("link failed:\n%s\n%s" % (" ".join(cmd), r.stderr))
+    os.replace(LIB + ".part", LIB)          # never a half-written library under the name others load
     return LIB
 
 

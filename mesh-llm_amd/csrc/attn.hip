@@ -77,7 +77,7 @@ int rope_kv(const RopeKvArgs &a, int T, hipStream_t stream) {
     if (T <= 0) return MESH_OK;
     if (a.head_dim % 2 || a.n_rot % 2 || a.n_rot > a.head_dim || a.head_dim > ROPE_HD_MAX)
         return fail(MESH_ERR_INVALID, "rope: bad head_dim/n_rot %d/%d", a.head_dim, a.n_rot);
-    if (!kv_type_supported(a.k_type) || !kv_type_supported(a.v_type) || ((a.k_type != MESH_F16 || a.v_type != MESH_F16) && a.head_dim % 32))
+    if (!kv_type_supported(a.k_type) || !kv_type_supported(a.v_type) || ((kv_quantised(a.k_type) || kv_quantised(a.v_type)) && a.head_dim % 32))
         return fail(MESH_ERR_UNSUPPORTED, "rope: KV cache types %d/%d with head_dim %d", a.k_type, a.v_type, a.head_dim);
     MESH_LAUNCH(rope_kv_kernel, dim3((unsigned)(a.n_head + 2 * a.n_kv), (unsigned)T), dim3(64), 0, stream, a.pos, a.seq, a.q, a.k, a.v, a.n_head, a.n_kv, a.head_dim, a);
     MESH_LAUNCH_CHECK();
@@ -93,14 +93,15 @@ constexpr int KPT = 4;                      // keys per thread per pass: 8 x 16-
 // for a normal float may flush to zero, which a softmax weight of that size is anyway.
 __device__ __forceinline__ float exp2_fast(float x) { return __builtin_amdgcn_exp2f(x); }
 
-// Sum over the LPK (8 or 16) consecutive lanes that share a key, result in every one of them: data-parallel-primitive
+// Sum over the LPK (8, 16 or 32) consecutive lanes that share a key, result in every one of them: data-parallel-primitive
 // moves inside a row of 16 lanes (swap neighbours, swap pairs, mirror the 8, mirror the 16) instead of LDS permutes.
 template <int LPK>
 __device__ __forceinline__ float slot_sum(float v) {
     v += __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), 0xB1, 0xF, 0xF, false));    // quad_perm [1,0,3,2]
     v += __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), 0x4E, 0xF, 0xF, false));    // quad_perm [2,3,0,1]
     v += __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), 0x141, 0xF, 0xF, false));   // row_half_mirror
-    if (LPK == 16) v += __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), 0x140, 0xF, 0xF, false));   // row_mirror
+    if (LPK >= 16) v += __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), 0x140, 0xF, 0xF, false));   // row_mirror
+    if (LPK == 32) v += __shfl_xor(v, 16);
     return v;
 }
 
@@ -125,8 +126,9 @@ __global__ __launch_bounds__(ATTN_THREADS) void attn_kernel(AttnArgs a) {
     const int tid = threadIdx.x, slot = tid / LPK, ds = (tid % LPK) * 8, wave = tid >> 6;
     const int seq = a.seq[t];
     const int n_keys = a.pos[t] + 1;
-    const int per = (n_keys + a.n_splits - 1) / a.n_splits;
-    const int j0 = split * per;
+    const int first = a.window > 0 && n_keys > a.window ? n_keys - a.window : 0;
+    const int per = (n_keys - first + a.n_splits - 1) / a.n_splits;
+    const int j0 = first + split * per;
     const int j1 = j0 + per < n_keys ? j0 + per : n_keys;
 
     constexpr int KRB = kv_row_bytes(KT, HD), VRB = kv_row_bytes(VT, HD);
@@ -144,7 +146,7 @@ __global__ __launch_bounds__(ATTN_THREADS) void attn_kernel(AttnArgs a) {
         l[h] = 0.f;
         voff[h] = 0.f;
         qoff[h] = 0.f;
-        if (KT != MESH_F16) {
+        if (kv_quantised(KT)) {
 #pragma unroll
             for (int i = 0; i < 8; ++i) qoff[h] += q[h][i];
             qoff[h] *= -KvAffine<KT>::off;
@@ -175,7 +177,7 @@ __global__ __launch_bounds__(ATTN_THREADS) void attn_kernel(AttnArgs a) {
                 float s = qoff[h];
 #pragma unroll
                 for (int e = 0; e < 8; ++e) s = fmaf(q[h][e], kf[e], s);
-                if (KT != MESH_F16) s *= kd;
+                if (kv_quantised(KT)) s *= kd;
                 s = slot_sum<LPK>(s);
                 sc[i][h] = ok ? s : -INFINITY;
             }
@@ -194,7 +196,7 @@ __global__ __launch_bounds__(ATTN_THREADS) void attn_kernel(AttnArgs a) {
 #pragma unroll
             for (int i = 0; i < KPT; ++i) { p[i] = exp2_fast(sc[i][h] - mn); ps += p[i]; }
             l[h] = l[h] * corr + ps;
-            if (VT != MESH_F16) {       // from here on p carries the row scale; the offset term is summed apart
+            if (kv_quantised(VT)) {       // from here on p carries the row scale; the offset term is summed apart
                 float po = 0.f;
 #pragma unroll
                 for (int i = 0; i < KPT; ++i) { p[i] *= vd[i]; po += p[i]; }
@@ -210,7 +212,7 @@ __global__ __launch_bounds__(ATTN_THREADS) void attn_kernel(AttnArgs a) {
             m[h] = mn;
         }
     }
-    if (VT != MESH_F16) {
+    if (kv_quantised(VT)) {
 #pragma unroll
         for (int h = 0; h < G; ++h)
 #pragma unroll
@@ -250,7 +252,8 @@ __global__ __launch_bounds__(ATTN_THREADS) void attn_kernel(AttnArgs a) {
         for (int w2 = 0; w2 < ATTN_WAVES; ++w2) { sum += s_acc[w2][h][dd]; ll += s_l[w2][h]; }
         const size_t row = (size_t)t * a.n_head + h0 + h;
         if (single) {
-            a.out[row * HD + dd] = sum / ll;
+            if (a.out_bf16) a.out_bf16[row * HD + dd] = f32_to_bf16_bits(sum / ll);
+            else a.out[row * HD + dd] = sum / ll;
         } else {
             a.part[(row * a.n_splits + split) * HD + dd] = sum;
             if (dd == 0) {
@@ -264,8 +267,8 @@ __global__ __launch_bounds__(ATTN_THREADS) void attn_kernel(AttnArgs a) {
 // Merge of the KV splits: grid (n_head, T), head_dim threads.  Split statistics go through LDS so every thread
 // sees them with broadcast reads and the partial rows are fetched with independent loads.
 // (leading scalar arguments: preloaded into SGPRs, see gemv.hip)
-__global__ __launch_bounds__(128) void attn_combine_kernel(const float *p_part, const float *p_ml, float *p_out, _Float16 *p_out16_k8,
-                                                           uint8_t *p_out_q16, int p_n_splits, int p_n_head, int p_head_dim) {
+__global__ __launch_bounds__(256) void attn_combine_kernel(const float *p_part, const float *p_ml, float *p_out, _Float16 *p_out16_k8,
+                                                           uint8_t *p_out_q16, uint16_t *p_out_bf16, int p_n_splits, int p_n_head, int p_head_dim) {
     __shared__ float s_m[ATTN_SPLITS_CAP], s_l[ATTN_SPLITS_CAP];
     const int h = blockIdx.x, t = blockIdx.y, dd = threadIdx.x;
     const size_t row = (size_t)t * p_n_head + h;
@@ -296,6 +299,8 @@ __global__ __launch_bounds__(128) void attn_combine_kernel(const float *p_part, 
     } else if (p_out16_k8) {
         const size_t kk = (size_t)h * p_head_dim + dd, KK = (size_t)p_n_head * p_head_dim;
         p_out16_k8[(size_t)(t / 16) * 16 * KK + ((kk >> 3) * 16 + (t % 16)) * 8 + (kk & 7)] = (_Float16)(num / den);
+    } else if (p_out_bf16) {
+        p_out_bf16[row * p_head_dim + dd] = f32_to_bf16_bits(num / den);
     } else {
         p_out[row * p_head_dim + dd] = num / den;
     }
@@ -311,10 +316,9 @@ static int launch_attn(const AttnArgs &a, int T, hipStream_t stream) {
         return MESH_OK;                                                                             \
     }
     MESH_ATTN_CASE(1)
-    MESH_ATTN_CASE(2)
-    MESH_ATTN_CASE(4)
-    if (HD == 128) { MESH_ATTN_CASE(5) MESH_ATTN_CASE(8) }
-    if (HD == 64) { MESH_ATTN_CASE(7) }
+    if constexpr (HD <= 128) { MESH_ATTN_CASE(2) MESH_ATTN_CASE(4) }
+    if constexpr (HD == 128) { MESH_ATTN_CASE(5) MESH_ATTN_CASE(8) }
+    if constexpr (HD == 64) { MESH_ATTN_CASE(7) }
 #undef MESH_ATTN_CASE
     // any other group size: one query head per workgroup (K/V re-read per head)
     MESH_LAUNCH((attn_kernel<HD, 1, KT, VT>), dim3((unsigned)a.n_splits, (unsigned)(a.n_kv * a.group), (unsigned)T), block, 0, stream, a);
@@ -325,9 +329,12 @@ static int launch_attn(const AttnArgs &a, int T, hipStream_t stream) {
 template <int HD>
 static int launch_attn_typed(const AttnArgs &a, int T, hipStream_t stream) {
     if (a.k_type == MESH_F16 && a.v_type == MESH_F16) return launch_attn<HD, MESH_F16, MESH_F16>(a, T, stream);
-    if (a.k_type == MESH_Q8_0 && a.v_type == MESH_Q4_0) return launch_attn<HD, MESH_Q8_0, MESH_Q4_0>(a, T, stream);
-    if (a.k_type == MESH_Q4_0 && a.v_type == MESH_Q4_0) return launch_attn<HD, MESH_Q4_0, MESH_Q4_0>(a, T, stream);
-    return fail(MESH_ERR_UNSUPPORTED, "attention: KV cache types %d/%d (f16/f16, q8_0/q4_0 and q4_0/q4_0 have kernels)", a.k_type, a.v_type);
+    if (a.k_type == MESH_F32 && a.v_type == MESH_F32) return launch_attn<HD, MESH_F32, MESH_F32>(a, T, stream);
+    if constexpr (HD <= 128) {
+        if (a.k_type == MESH_Q8_0 && a.v_type == MESH_Q4_0) return launch_attn<HD, MESH_Q8_0, MESH_Q4_0>(a, T, stream);
+        if (a.k_type == MESH_Q4_0 && a.v_type == MESH_Q4_0) return launch_attn<HD, MESH_Q4_0, MESH_Q4_0>(a, T, stream);
+    }
+    return fail(MESH_ERR_UNSUPPORTED, "attention: KV cache types %d/%d at this head_dim (f16/f16, f32/f32, q8_0/q4_0 and q4_0/q4_0 have kernels)", a.k_type, a.v_type);
 }
 
 bool kv_pair_supported(int k_type, int v_type) {
@@ -342,13 +349,14 @@ int attention(const AttnArgs &a, int T, hipStream_t stream) {
     int rc;
     if (a.head_dim == 128) rc = launch_attn_typed<128>(a, T, stream);
     else if (a.head_dim == 64) rc = launch_attn_typed<64>(a, T, stream);
-    else return fail(MESH_ERR_UNSUPPORTED, "attention: head_dim %d has no kernel (64 and 128 do)", a.head_dim);
+    else if (a.head_dim == 256) rc = launch_attn_typed<256>(a, T, stream);
+    else return fail(MESH_ERR_UNSUPPORTED, "attention: head_dim %d has no kernel (64, 128 and 256 do)", a.head_dim);
     if (rc != MESH_OK || a.n_splits == 1) return rc;
     return attention_combine(a, T, stream);
 }
 
 int attention_combine(const AttnArgs &a, int T, hipStream_t stream) {
-    MESH_LAUNCH(attn_combine_kernel, dim3((unsigned)a.n_head, (unsigned)T), dim3((unsigned)a.head_dim), 0, stream, a.part, a.ml, a.out, a.out16_k8, a.out_q16, a.n_splits, a.n_head, a.head_dim);
+    MESH_LAUNCH(attn_combine_kernel, dim3((unsigned)a.n_head, (unsigned)T), dim3((unsigned)a.head_dim), 0, stream, a.part, a.ml, a.out, a.out16_k8, a.out_q16, a.out_bf16, a.n_splits, a.n_head, a.head_dim);
     MESH_LAUNCH_CHECK();
     return MESH_OK;
 }
@@ -371,7 +379,7 @@ __global__ __launch_bounds__(64) void kv_export_kernel(int type, const uint8_t *
 }
 
 int kv_import(int type, uint8_t *cache, const uint16_t *half, int n_kv, int n_ctx, int head_dim, int seq, int pos0, int n_pos, hipStream_t stream) {
-    if (!kv_type_supported(type) || head_dim > ROPE_HD_MAX || (type != MESH_F16 && head_dim % 32)) return fail(MESH_ERR_UNSUPPORTED, "kv_import: type %d, head_dim %d", type, head_dim);
+    if (!kv_type_supported(type) || head_dim > ROPE_HD_MAX || (kv_quantised(type) && head_dim % 32)) return fail(MESH_ERR_UNSUPPORTED, "kv_import: type %d, head_dim %d", type, head_dim);
     MESH_LAUNCH(kv_import_kernel, dim3((unsigned)n_kv, (unsigned)n_pos), dim3(64), 0, stream, type, cache, half, n_kv, n_ctx, head_dim, seq, pos0);
     MESH_LAUNCH_CHECK();
     return MESH_OK;

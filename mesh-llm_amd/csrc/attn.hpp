@@ -29,7 +29,7 @@ int rope_kv(const RopeKvArgs &a, int T, hipStream_t stream);
 struct AttnArgs {
     const float *q = nullptr;      // [T][n_head][head_dim]
     const uint8_t *kcache = nullptr, *vcache = nullptr;    // rows of k_type / v_type
-    int k_type = MESH_F16, v_type = MESH_F16;              // (f16, f16), (q8_0, q4_0) or (q4_0, q4_0)
+    int k_type = MESH_F16, v_type = MESH_F16;              // (f16, f16), (q8_0, q4_0) or (q4_0, q4_0); attention() also (f32, f32)
     const int32_t *pos = nullptr, *seq = nullptr;
     float *part = nullptr;         // [T][n_head][n_splits][head_dim]
     float *ml = nullptr;           // [T][n_head][n_splits][2]
@@ -43,10 +43,13 @@ struct AttnArgs {
     // attention_chunk only, optional: scratch of 2 * n_kv * n_ctx * head_dim f16 values; with it a long chunk over a
     // quantised cache decodes the rows it needs once, into the scratch, instead of once per query tile
     _Float16 *chunk_kv16 = nullptr;
+    // or, when set, as bf16 rows [T][n_head * head_dim] (every kernel here), also instead of `out`
+    uint16_t *out_bf16 = nullptr;
+    int window = 0;                // token t sees the positions (pos[t] - window, pos[t]]; 0: all of [0, pos[t]]
     float scale = 1.f;
     int n_head = 0, n_kv = 0, group = 1, head_dim = 0, n_ctx = 0, n_splits = 1;
 };
-// token t attends to cache positions [0, pos[t]] of sequence seq[t]
+// token t attends to cache positions [0, pos[t]] of sequence seq[t], or to the last `window` of them
 int attention(const AttnArgs &a, int T, hipStream_t stream);
 // merge of the split partials (a.part, a.ml) into a.out; a no-op contract for n_splits == 1 is the caller's business
 int attention_combine(const AttnArgs &a, int T, hipStream_t stream);
@@ -55,7 +58,7 @@ int attention_combine(const AttnArgs &a, int T, hipStream_t stream);
 bool attention_mma_supported(const AttnArgs &a);
 int attention_mma(const AttnArgs &a, int T, hipStream_t stream);
 // The same for a chunk of T consecutive positions pos0 .. pos0 + T - 1 of one sequence, on the matrix cores
-// (attn_prefill.hip; head_dim 128).  a.pos / a.seq / a.part / a.ml are not used.
+// (attn_prefill.hip; head_dim 64 or 128).  a.pos / a.seq / a.part / a.ml are not used.
 int attention_chunk(const AttnArgs &a, int T, int pos0, int seq, hipStream_t stream);
 bool kv_pair_supported(int k_type, int v_type);
 

@@ -1,6 +1,6 @@
 // GQA decode attention on the matrix cores, for batches of decode tokens over long KV ranges.
 //
-// Same contract as attn_kernel of attn.hip (token t attends to cache positions [0, pos[t]] of sequence seq[t]; split-KV
+// Same contract as attn_kernel of attn.hip (token t attends to cache positions [0, pos[t]] of sequence seq[t], or the last `window` of them; split-KV
 // partials merged by attn_combine_kernel), same place in the worker's graph (flash_attn_ext under -fa on,
 // mesh-llm/src/inference/launch.rs:1350-1353).  The per-key work of that kernel is vector ALU work that grows with the
 // number of query heads per KV head; here the query heads of a KV head are the 16 columns of an MFMA tile, so the
@@ -87,7 +87,7 @@ __device__ __forceinline__ void mm_wave_lds_sync() {
 template <int HD, int KT, int VT>
 __global__ __launch_bounds__(MMA_THREADS) void attn_mma_kernel(const float *p_q, const int32_t *p_pos, const int32_t *p_seq,
                                                                const uint8_t *p_kcache, const uint8_t *p_vcache, int p_n_splits,
-                                                               int p_n_ctx, int p_n_kv, int p_group, int p_n_head, float p_scale,
+                                                               int p_n_ctx, int p_n_kv, int p_group, int p_n_head, float p_scale, int p_window,
                                                                const AttnArgs a) {
     constexpr int NC = HD / 32;             // 32-dim chunks of the score product
     constexpr int NDB = HD / 16;            // 16-dim blocks of the output
@@ -105,8 +105,9 @@ __global__ __launch_bounds__(MMA_THREADS) void attn_mma_kernel(const float *p_q,
     const int G = p_group;
     const int seq = p_seq[t];
     const int n_keys = p_pos[t] + 1;
-    const int per = (n_keys + p_n_splits - 1) / p_n_splits;
-    const int j0 = split * per;
+    const int first = p_window > 0 && n_keys > p_window ? n_keys - p_window : 0;
+    const int per = (n_keys - first + p_n_splits - 1) / p_n_splits;
+    const int j0 = first + split * per;
     const int j1 = j0 + per < n_keys ? j0 + per : n_keys;
 
     // Q^T operand: head column c, dims 32*cc + 8*g + j, in log2 units
@@ -248,6 +249,8 @@ __global__ __launch_bounds__(MMA_THREADS) void attn_mma_kernel(const float *p_q,
             } else if (a.out16_k8) {
                 const size_t kk = ((size_t)kvh * G + h) * HD + dd, KK = (size_t)p_n_head * HD;
                 a.out16_k8[(size_t)(t / 16) * 16 * KK + ((kk >> 3) * 16 + (t % 16)) * 8 + (kk & 7)] = (_Float16)(sum / ll);
+            } else if (a.out_bf16) {
+                a.out_bf16[row * HD + dd] = f32_to_bf16_bits(sum / ll);
             } else {
                 a.out[row * HD + dd] = sum / ll;
             }
@@ -264,9 +267,9 @@ __global__ __launch_bounds__(MMA_THREADS) void attn_mma_kernel(const float *p_q,
 template <int HD>
 static int launch_mma(const AttnArgs &a, int T, hipStream_t stream) {
     const dim3 grid((unsigned)a.n_splits, (unsigned)a.n_kv, (unsigned)T), block(MMA_THREADS);
-    if (a.k_type == MESH_F16 && a.v_type == MESH_F16) MESH_LAUNCH((attn_mma_kernel<HD, MESH_F16, MESH_F16>), grid, block, 0, stream, a.q, a.pos, a.seq, a.kcache, a.vcache, a.n_splits, a.n_ctx, a.n_kv, a.group, a.n_head, a.scale, a);
-    else if (a.k_type == MESH_Q8_0 && a.v_type == MESH_Q4_0) MESH_LAUNCH((attn_mma_kernel<HD, MESH_Q8_0, MESH_Q4_0>), grid, block, 0, stream, a.q, a.pos, a.seq, a.kcache, a.vcache, a.n_splits, a.n_ctx, a.n_kv, a.group, a.n_head, a.scale, a);
-    else if (a.k_type == MESH_Q4_0 && a.v_type == MESH_Q4_0) MESH_LAUNCH((attn_mma_kernel<HD, MESH_Q4_0, MESH_Q4_0>), grid, block, 0, stream, a.q, a.pos, a.seq, a.kcache, a.vcache, a.n_splits, a.n_ctx, a.n_kv, a.group, a.n_head, a.scale, a);
+    if (a.k_type == MESH_F16 && a.v_type == MESH_F16) MESH_LAUNCH((attn_mma_kernel<HD, MESH_F16, MESH_F16>), grid, block, 0, stream, a.q, a.pos, a.seq, a.kcache, a.vcache, a.n_splits, a.n_ctx, a.n_kv, a.group, a.n_head, a.scale, a.window, a);
+    else if (a.k_type == MESH_Q8_0 && a.v_type == MESH_Q4_0) MESH_LAUNCH((attn_mma_kernel<HD, MESH_Q8_0, MESH_Q4_0>), grid, block, 0, stream, a.q, a.pos, a.seq, a.kcache, a.vcache, a.n_splits, a.n_ctx, a.n_kv, a.group, a.n_head, a.scale, a.window, a);
+    else if (a.k_type == MESH_Q4_0 && a.v_type == MESH_Q4_0) MESH_LAUNCH((attn_mma_kernel<HD, MESH_Q4_0, MESH_Q4_0>), grid, block, 0, stream, a.q, a.pos, a.seq, a.kcache, a.vcache, a.n_splits, a.n_ctx, a.n_kv, a.group, a.n_head, a.scale, a.window, a);
     else return fail(MESH_ERR_UNSUPPORTED, "attention_mma: KV cache types %d/%d", a.k_type, a.v_type);
     MESH_LAUNCH_CHECK();
     return MESH_OK;

@@ -1,8 +1,9 @@
-// Causal GQA attention for a prefill chunk on the matrix cores (head_dim 128; f16 or quantised KV cache rows, which
+// Causal GQA attention for a prefill chunk on the matrix cores (head_dim 64 or 128, written below for 128; f16 or quantised KV cache rows, which
 // are dequantised to f16 on their way into LDS).
 //
 // The chunk is T consecutive positions pos0 .. pos0 + T - 1 of one sequence whose keys and values are already in
-// the cache (rope_kv appended them); token t attends to cache positions [0, pos0 + t].  A workgroup takes 32
+// the cache (rope_kv appended them); token t attends to cache positions [0, pos0 + t], or to the last `window` of them
+// (a workgroup then starts its walk at the first key its first query sees).  A workgroup takes 32
 // queries of every head of one KV-head group (one wave per head), walks the keys in tiles of 32 and keeps the
 // running softmax in registers:
 //   S^T = K . Q^T        (32 keys x 32 queries, v_mfma_f32_32x32x16_f16 over the 128 dims)
@@ -25,14 +26,13 @@
 
 namespace mesh {
 
-constexpr int PF_HD = 128;
 constexpr int PF_TILE = 32;                 // queries per workgroup
-constexpr int PF_KPITCH = PF_HD + 8;        // halfs per key row of the K tile in LDS (bank-conflict padding)
 
 // Column (dword) of key pair kp in dim row `dim` of the transposed V tile.  Rows 32 apart start on the same LDS bank
 // (32 rows of 18 or 34 dwords are a multiple of the 64 banks), and the staging writes of a wave touch four such rows at once; the
 // XOR moves them onto different banks.  It keeps dwords 2j, 2j + 1 neighbours, which the 8-byte fragment reads need.
 __device__ __forceinline__ int pf_vcol(int dim, int kp) { return kp ^ ((dim >> 5) << 2); }
+constexpr int PF_EXPAND_HD = 128;            // kv_expand_kernel's head_dim
 constexpr int PF_EXPAND_MIN_T = 128;         // chunks from this many tokens decode a quantised cache to f16 once, ahead of the walk
 constexpr float PF_RESCALE_STEP = 8.f;      // the softmax reference moves only when the running maximum exceeds it by this (log2)
 
@@ -47,9 +47,9 @@ __device__ __forceinline__ uint32_t pf_pack(float a, float b) {
 }
 
 // the 8 values a (key, piece) pair contributes to a tile, as packed f16
-template <int TYPE>
+template <int TYPE, int HD>
 __device__ __forceinline__ uint4 pf_row_piece(const uint8_t *row, int piece) {
-    const KvRaw<TYPE> r = kv_load<TYPE, PF_HD>(row, piece * 8);
+    const KvRaw<TYPE> r = kv_load<TYPE, HD>(row, piece * 8);
     if constexpr (TYPE == MESH_F16) {
         return r.v;
     } else {
@@ -62,15 +62,18 @@ __device__ __forceinline__ uint4 pf_row_piece(const uint8_t *row, int piece) {
 }
 
 // NT: tiles of 32 keys per step (1 or 2; two give the wave two independent score chains and half the barriers per key, at
-// ~50 more registers).  NP: (key, 8-dim piece) pairs of a step one thread carries in registers, at least 512 NT /
+// ~50 more registers).  NP: (key, 8-dim piece) pairs of a step one thread carries in registers, at least 4 HD NT /
 // (threads of the workgroup); 0 for small workgroups, which load each step's rows where they write them.
-template <int KT, int VT, int NP, int NT>
+template <int HD, int KT, int VT, int NP, int NT>
 __global__ __launch_bounds__(512) void attn_chunk_kernel(const AttnArgs a, int T, int pos0, int seq, int hpw, int fwd_from, int qtiles, int n_ksplit) {
-    constexpr int KRB = kv_row_bytes(KT, PF_HD), VRB = kv_row_bytes(VT, PF_HD);
+    constexpr int KRB = kv_row_bytes(KT, HD), VRB = kv_row_bytes(VT, HD);
+    constexpr int PIECES = HD / 8;                  // 8-dim pieces of a row
+    constexpr int NKC = HD / 16, NDB = HD / 32;     // steps of the score product along the dims, 32-dim blocks of the output
+    constexpr int PF_KPITCH = HD + 8;               // halfs per key row of the K tile in LDS (bank-conflict padding)
     constexpr int PF_KEYS = 32 * NT;                // keys per step
     constexpr int PF_VPITCH = PF_KEYS / 2 + 2;      // dwords (key pairs) per dim row of the transposed V tile
     __shared__ __align__(16) _Float16 sK[PF_KEYS * PF_KPITCH];
-    __shared__ __align__(16) uint32_t sVt[PF_HD * PF_VPITCH];
+    __shared__ __align__(16) uint32_t sVt[HD * PF_VPITCH];
     const int tid = threadIdx.x, lane = tid & 63, nthreads = blockDim.x;
     // wave -> (head of the workgroup, one of its `qtiles` consecutive query tiles): groups of fewer than four heads fill the
     // workgroup with several query tiles of the same heads, which share the K / V tiles like heads do
@@ -89,23 +92,24 @@ __global__ __launch_bounds__(512) void attn_chunk_kernel(const AttnArgs a, int T
     const int tq = qt * PF_TILE + qcol;
     const bool q_live = tq < T;
     const int pos_q = pos0 + tq;
+    const int win_lo = a.window > 0 ? pos_q - a.window : -1;      // keys up to this one are out of the query's sight
 
     // Q^T fragments of this lane's query, scaled so that the scores are in log2 units
     const float qs = a.scale * 1.44269504088896341f;
-    pf_h8 qf[8];
+    pf_h8 qf[NKC];
     {
-        const float *qp = a.q + ((size_t)(q_live ? tq : 0) * a.n_head + h) * PF_HD + 8 * half;
+        const float *qp = a.q + ((size_t)(q_live ? tq : 0) * a.n_head + h) * HD + 8 * half;
 #pragma unroll
-        for (int kc = 0; kc < 8; ++kc) {
+        for (int kc = 0; kc < NKC; ++kc) {
             const float4 v0 = *reinterpret_cast<const float4 *>(qp + kc * 16), v1 = *reinterpret_cast<const float4 *>(qp + kc * 16 + 4);
             const float z = q_live ? qs : 0.f;
             const pf_u4 p = {pf_pack(v0.x * z, v0.y * z), pf_pack(v0.z * z, v0.w * z), pf_pack(v1.x * z, v1.y * z), pf_pack(v1.z * z, v1.w * z)};
             qf[kc] = __builtin_bit_cast(pf_h8, p);
         }
     }
-    pf_f16v o[4];
+    pf_f16v o[NDB];
 #pragma unroll
-    for (int db = 0; db < 4; ++db)
+    for (int db = 0; db < NDB; ++db)
 #pragma unroll
         for (int i = 0; i < 16; ++i) o[db][i] = 0.f;
     float m = -INFINITY, l = 0.f;
@@ -115,26 +119,30 @@ __global__ __launch_bounds__(512) void attn_chunk_kernel(const AttnArgs a, int T
     const int n_keys_own = qt * PF_TILE < T ? pos0 + q_end : 0;                     // keys any of them may see
     const int wg_end = (qg + 1) * qtiles * PF_TILE < T ? (qg + 1) * qtiles * PF_TILE : T;
     const int n_keys_wg = pos0 + wg_end;                                            // keys the workgroup's last tile walks
-    const int per_split = (((n_keys_wg + n_ksplit - 1) / n_ksplit) + 63) & ~63;
-    const int k_lo = ks * per_split;
+    // keys before the window of the workgroup's (and of this wave's) first query are not walked
+    const int wg_first = a.window > 0 ? (pos0 + qg * qtiles * PF_TILE - a.window + 1 > 0 ? (pos0 + qg * qtiles * PF_TILE - a.window + 1) & ~(PF_KEYS - 1) : 0) : 0;
+    const int own_first = a.window > 0 ? pos0 + qt * PF_TILE - a.window + 1 : 0;
+    const int full_from = a.window > 0 ? pos0 + qt * PF_TILE + PF_TILE - a.window : 0;     // from this key on, inside every query's window
+    const int per_split = (((n_keys_wg - wg_first + n_ksplit - 1) / n_ksplit) + 63) & ~63;
+    const int k_lo = wg_first + ks * per_split;
     const int n_keys = k_lo + per_split < n_keys_wg ? k_lo + per_split : n_keys_wg;   // end of this workgroup's walk
     const int n_keys_mine = n_keys_own < n_keys ? n_keys_own : n_keys;              // and of this wave's
     // K is staged as it is: (key, 8-dim piece) pairs, 16 bytes each.  V is staged transposed: an item is the same 8 dims
     // of two neighbouring keys, written as 8 dwords, one per dim, each holding the pair of keys.  Rows past the context
     // end are clamped (masked below).
     auto k_row = [&](int k0, int p) {
-        int kr = k0 + (p >> 4);
+        int kr = k0 + p / PIECES;
         kr = kr < a.n_ctx ? kr : a.n_ctx - 1;
-        return pf_row_piece<KT>(a.kcache + (base + kr) * KRB, p & 15);
+        return pf_row_piece<KT, HD>(a.kcache + (base + kr) * KRB, p % PIECES);
     };
     auto v_row = [&](int k0, int p, int second) {
-        int kr = k0 + 2 * (p >> 4) + second;
+        int kr = k0 + 2 * (p / PIECES) + second;
         kr = kr < a.n_ctx ? kr : a.n_ctx - 1;
-        return pf_row_piece<VT>(a.vcache + (base + kr) * VRB, p & 15);
+        return pf_row_piece<VT, HD>(a.vcache + (base + kr) * VRB, p % PIECES);
     };
-    auto k_put = [&](int p, const uint4 &r) { *reinterpret_cast<uint4 *>(sK + (p >> 4) * PF_KPITCH + (p & 15) * 8) = r; };
+    auto k_put = [&](int p, const uint4 &r) { *reinterpret_cast<uint4 *>(sK + (p / PIECES) * PF_KPITCH + (p % PIECES) * 8) = r; };
     auto v_put = [&](int p, const uint4 &r0, const uint4 &r1) {
-        const int kp = p >> 4, piece = p & 15;
+        const int kp = p / PIECES, piece = p % PIECES;
         const uint32_t w0[4] = {r0.x, r0.y, r0.z, r0.w}, w1[4] = {r1.x, r1.y, r1.z, r1.w};
         uint32_t *dst = sVt + piece * 8 * PF_VPITCH + pf_vcol(piece * 8, kp);
 #pragma unroll
@@ -151,12 +159,12 @@ __global__ __launch_bounds__(512) void attn_chunk_kernel(const AttnArgs a, int T
 #pragma unroll
         for (int i = 0; i < NPK; ++i) {
             const int p = tid + i * nthreads;
-            if (p < PF_KEYS * 16) rk[i] = k_row(k0, p);
+            if (p < PF_KEYS * PIECES) rk[i] = k_row(k0, p);
         }
 #pragma unroll
         for (int i = 0; i < NPV; ++i) {
             const int p = tid + i * nthreads;
-            if (p < PF_KEYS * 8) { rv[i][0] = v_row(k0, p, 0); rv[i][1] = v_row(k0, p, 1); }
+            if (p < PF_KEYS * PIECES / 2) { rv[i][0] = v_row(k0, p, 0); rv[i][1] = v_row(k0, p, 1); }
         }
     };
     if constexpr (NP > 0) fetch_step(k_lo);
@@ -165,22 +173,23 @@ __global__ __launch_bounds__(512) void attn_chunk_kernel(const AttnArgs a, int T
 #pragma unroll
             for (int i = 0; i < NPK; ++i) {
                 const int p = tid + i * nthreads;
-                if (p < PF_KEYS * 16) k_put(p, rk[i]);
+                if (p < PF_KEYS * PIECES) k_put(p, rk[i]);
             }
 #pragma unroll
             for (int i = 0; i < NPV; ++i) {
                 const int p = tid + i * nthreads;
-                if (p < PF_KEYS * 8) v_put(p, rv[i][0], rv[i][1]);
+                if (p < PF_KEYS * PIECES / 2) v_put(p, rv[i][0], rv[i][1]);
             }
         } else {
-            for (int p = tid; p < PF_KEYS * 16; p += nthreads) k_put(p, k_row(k0, p));
-            for (int p = tid; p < PF_KEYS * 8; p += nthreads) v_put(p, v_row(k0, p, 0), v_row(k0, p, 1));
+            for (int p = tid; p < PF_KEYS * PIECES; p += nthreads) k_put(p, k_row(k0, p));
+            for (int p = tid; p < PF_KEYS * PIECES / 2; p += nthreads) v_put(p, v_row(k0, p, 0), v_row(k0, p, 1));
         }
         __syncthreads();
         if constexpr (NP > 0) {
             if (k0 + PF_KEYS < n_keys) fetch_step(k0 + PF_KEYS);
         }
-        if (k0 < n_keys_mine) {     // (an earlier query tile of the workgroup is done before the last one)
+        // (an earlier query tile of the workgroup is done before the last one, and with a window starts before it)
+        if (k0 < n_keys_mine && k0 + PF_KEYS > own_first) {
         // the second 32 keys of the step lie past every query of the tile at the end of the walk
         const bool two = NT == 2 && k0 + 32 < n_keys_mine;
 
@@ -193,7 +202,7 @@ __global__ __launch_bounds__(512) void attn_chunk_kernel(const AttnArgs a, int T
             for (int i = 0; i < 16; ++i) s[t][i] = t == 0 ? 0.f : (two ? 0.f : -INFINITY);
         if (two) {
 #pragma unroll
-            for (int kc = 0; kc < 8; ++kc)
+            for (int kc = 0; kc < NKC; ++kc)
 #pragma unroll
                 for (int t = 0; t < NT; ++t) {
                     const pf_h8 kf = *reinterpret_cast<const pf_h8 *>(sK + (32 * t + qcol) * PF_KPITCH + kc * 16 + 8 * half);
@@ -201,20 +210,20 @@ __global__ __launch_bounds__(512) void attn_chunk_kernel(const AttnArgs a, int T
                 }
         } else {
 #pragma unroll
-            for (int kc = 0; kc < 8; ++kc) {
+            for (int kc = 0; kc < NKC; ++kc) {
                 const pf_h8 kf = *reinterpret_cast<const pf_h8 *>(sK + qcol * PF_KPITCH + kc * 16 + 8 * half);
                 s[0] = __builtin_amdgcn_mfma_f32_32x32x16_f16(kf, qf[kc], s[0], 0, 0, 0);
             }
         }
         // register i of tile t is key k0 + 32 * t + 8 * (i / 4) + 4 * half + i % 4 for query qcol.  Only a step that
-        // reaches past the first query's position has anything to mask (a dead query column has q = 0 and is never stored).
-        if (k0 + PF_KEYS - 1 > pos0 + qt * PF_TILE) {
+        // reaches past the first query's position, or starts before the last query's window, has anything to mask (a dead query column has q = 0 and is never stored).
+        if (k0 + PF_KEYS - 1 > pos0 + qt * PF_TILE || k0 < full_from) {
 #pragma unroll
             for (int t = 0; t < NT; ++t)
 #pragma unroll
                 for (int i = 0; i < 16; ++i) {
                     const int key = k0 + 32 * t + 8 * (i >> 2) + 4 * half + (i & 3);
-                    s[t][i] = key <= pos_q ? s[t][i] : -INFINITY;
+                    s[t][i] = key <= pos_q && key > win_lo ? s[t][i] : -INFINITY;
                 }
         }
         float mxt[NT];
@@ -228,8 +237,8 @@ __global__ __launch_bounds__(512) void attn_chunk_kernel(const AttnArgs a, int T
         mx = fmaxf(mx, __shfl_xor(mx, 32));
         // m is the reference the exponentials are taken against.  It follows the running maximum only when that has
         // moved by more than PF_RESCALE_STEP (log2 units), so that most steps skip the rescale of the 64 accumulator
-        // registers; in between p <= 2^PF_RESCALE_STEP, which f16 holds comfortably.  (Key 0 is visible to every
-        // query, so after the first step m is finite for every live column.)
+        // registers; in between p <= 2^PF_RESCALE_STEP, which f16 holds comfortably.  (Without a window key 0
+        // is visible to every query, so after the first step m is finite for every live column.)
         if (__builtin_amdgcn_ballot_w64(mx > m + PF_RESCALE_STEP) != 0ull) {
             const float m_new = mx > m + PF_RESCALE_STEP ? mx : m;
             // 1 for lanes that stay, exp2(-inf) = 0 while nothing is accumulated.  A query that has seen no key yet and
@@ -239,12 +248,11 @@ __global__ __launch_bounds__(512) void attn_chunk_kernel(const AttnArgs a, int T
             l *= corr;
             m = m_new;
 #pragma unroll
-            for (int db = 0; db < 4; ++db)
+            for (int db = 0; db < NDB; ++db)
 #pragma unroll
                 for (int i = 0; i < 16; ++i) o[db][i] *= corr;
         }
-        // (Without key splits key 0 is visible to every query, so m is finite from the first step on.  In a later split a
-        // query may see no key at all: all its scores are -inf and so is m; the reference 0 then gives p = 0, not NaN.)
+        // (In a later split, or in the first steps of a windowed walk, a query may see no key at all: all its scores are -inf and so is m; the reference 0 then gives p = 0, not NaN.)
         const float mref = m == -INFINITY ? 0.f : m;
         // P^T as the B operand: the lane's own registers, 8 per MFMA
         pf_h8 pf[NT][2];
@@ -265,7 +273,7 @@ __global__ __launch_bounds__(512) void attn_chunk_kernel(const AttnArgs a, int T
         ps += __shfl_xor(ps, 32);
         l += ps;
 #pragma unroll
-        for (int db = 0; db < 4; ++db) {
+        for (int db = 0; db < NDB; ++db) {
             // dim row db * 32 + qcol, this half's keys of tile t: key pairs 16 * t + 2 * half + 4 * j (+ 1), j = 0 .. 3
             const uint32_t *vrow = sVt + (db * 32 + qcol) * PF_VPITCH + 2 * half;
 #pragma unroll
@@ -285,9 +293,9 @@ __global__ __launch_bounds__(512) void attn_chunk_kernel(const AttnArgs a, int T
         // un-normalised partial and (maximum, sum) of this key split, in the layout of the split-KV decode kernels
         if (q_live) {
             const size_t prow = ((size_t)tq * a.n_head + h) * n_ksplit + ks;
-            float *pp = a.part + prow * PF_HD;
+            float *pp = a.part + prow * HD;
 #pragma unroll
-            for (int db = 0; db < 4; ++db)
+            for (int db = 0; db < NDB; ++db)
 #pragma unroll
                 for (int i4 = 0; i4 < 4; ++i4)
                     *reinterpret_cast<float4 *>(pp + db * 32 + 8 * i4 + 4 * half) =
@@ -302,22 +310,34 @@ __global__ __launch_bounds__(512) void attn_chunk_kernel(const AttnArgs a, int T
         const int t_pad = (T + 15) & ~15;
         if (tq < t_pad) {
             const float inv = q_live ? 1.0f / l : 0.f;
-            const size_t KK = (size_t)a.n_head * PF_HD;
+            const size_t KK = (size_t)a.n_head * HD;
             _Float16 *ob = a.out16_k8 + (size_t)(tq >> 4) * 16 * KK + (size_t)(tq & 15) * 8;
 #pragma unroll
-            for (int db = 0; db < 4; ++db)
+            for (int db = 0; db < NDB; ++db)
 #pragma unroll
                 for (int i4 = 0; i4 < 4; ++i4) {
-                    const size_t kk = (size_t)h * PF_HD + db * 32 + 8 * i4 + 4 * half;
+                    const size_t kk = (size_t)h * HD + db * 32 + 8 * i4 + 4 * half;
                     *reinterpret_cast<uint2 *>(ob + (kk >> 3) * 128 + (kk & 7)) =
                         make_uint2(pf_pack(o[db][4 * i4] * inv, o[db][4 * i4 + 1] * inv), pf_pack(o[db][4 * i4 + 2] * inv, o[db][4 * i4 + 3] * inv));
                 }
         }
+    } else if (a.out_bf16) {
+        if (q_live) {
+            const float inv = 1.0f / l;
+            uint16_t *op = a.out_bf16 + ((size_t)tq * a.n_head + h) * HD;
+            auto two16 = [&](float lo, float hi) { return (uint32_t)f32_to_bf16_bits(lo * inv) | ((uint32_t)f32_to_bf16_bits(hi * inv) << 16); };
+#pragma unroll
+            for (int db = 0; db < NDB; ++db)
+#pragma unroll
+                for (int i4 = 0; i4 < 4; ++i4)
+                    *reinterpret_cast<uint2 *>(op + db * 32 + 8 * i4 + 4 * half) =
+                        make_uint2(two16(o[db][4 * i4], o[db][4 * i4 + 1]), two16(o[db][4 * i4 + 2], o[db][4 * i4 + 3]));
+        }
     } else if (q_live) {
         const float inv = 1.0f / l;
-        float *op = a.out + ((size_t)tq * a.n_head + h) * PF_HD;
+        float *op = a.out + ((size_t)tq * a.n_head + h) * HD;
 #pragma unroll
-        for (int db = 0; db < 4; ++db)
+        for (int db = 0; db < NDB; ++db)
 #pragma unroll
             for (int i4 = 0; i4 < 4; ++i4)
                 *reinterpret_cast<float4 *>(op + db * 32 + 8 * i4 + 4 * half) =
@@ -330,15 +350,15 @@ __global__ __launch_bounds__(512) void attn_chunk_kernel(const AttnArgs a, int T
 template <int KT, int VT>
 __global__ __launch_bounds__(256) void kv_expand_kernel(const uint8_t *kcache, const uint8_t *vcache, uint4 *k16, uint4 *v16, int n_keys, int n_ctx,
                                                         int n_kv, int seq) {
-    constexpr int KRB = kv_row_bytes(KT, PF_HD), VRB = kv_row_bytes(VT, PF_HD);
+    constexpr int KRB = kv_row_bytes(KT, PF_EXPAND_HD), VRB = kv_row_bytes(VT, PF_EXPAND_HD);
     const size_t idx = (size_t)blockIdx.x * 256 + threadIdx.x;
     const int piece = (int)(idx & 15);
     const size_t row = idx >> 4;
     if (row >= (size_t)n_kv * n_keys) return;
     const int kvh = (int)(row / n_keys), key = (int)(row % n_keys);
     const size_t src = ((size_t)seq * n_kv + kvh) * n_ctx + key, dst = (size_t)kvh * n_ctx + key;
-    k16[dst * 16 + piece] = pf_row_piece<KT>(kcache + src * KRB, piece);
-    v16[dst * 16 + piece] = pf_row_piece<VT>(vcache + src * VRB, piece);
+    k16[dst * 16 + piece] = pf_row_piece<KT, PF_EXPAND_HD>(kcache + src * KRB, piece);
+    v16[dst * 16 + piece] = pf_row_piece<VT, PF_EXPAND_HD>(vcache + src * VRB, piece);
 }
 
 static int pf_n_cu() {
@@ -355,7 +375,8 @@ static int pf_n_cu() {
 int attention_chunk(const AttnArgs &a_in, int T, int pos0, int seq, hipStream_t stream) {
     if (T <= 0) return MESH_OK;
     AttnArgs a = a_in;
-    if (a.head_dim != PF_HD) return fail(MESH_ERR_UNSUPPORTED, "attention_chunk: head_dim %d (128 only)", a.head_dim);
+    if (a.head_dim != 128 && (a.head_dim != 64 || a.k_type != MESH_F16))
+        return fail(MESH_ERR_UNSUPPORTED, "attention_chunk: head_dim %d, cache type %d (128, and 64 with f16 rows)", a.head_dim, a.k_type);
     if (a.group < 1 || a.n_head != a.group * a.n_kv || pos0 < 0 || pos0 + T > a.n_ctx || seq < 0)
         return fail(MESH_ERR_INVALID, "attention_chunk: bad head layout or chunk [%d, %d) outside the context of %d", pos0, pos0 + T, a.n_ctx);
     if (a.k_type != MESH_F16 && a.chunk_kv16 && T >= PF_EXPAND_MIN_T) {
@@ -389,7 +410,7 @@ int attention_chunk(const AttnArgs &a_in, int T, int pos0, int seq, hipStream_t 
     // workgroup per CU, at most 8 ways, at least 256 keys each, within the buffers' rows of (token, split).
     int n_ksplit = 1;
     {
-        const int wgs = (int)(grid.x * grid.y * grid.z), n_keys = pos0 + T;
+        const int wgs = (int)(grid.x * grid.y * grid.z), n_keys = a.window > 0 ? std::min(pos0 + T, a.window + PF_TILE) : pos0 + T;
         if (a.part && a.ml && a.part_rows > 0 && wgs < pf_n_cu())
             n_ksplit = std::max(1, std::min(std::min(pf_n_cu() / wgs, 8), std::min(n_keys / 256, (int)(a.part_rows / (size_t)T))));
         if (n_ksplit > ATTN_SPLITS_CAP) n_ksplit = ATTN_SPLITS_CAP;
@@ -404,15 +425,16 @@ int attention_chunk(const AttnArgs &a_in, int T, int pos0, int seq, hipStream_t 
     // (Two tiles per step everywhere.  With 5 heads per KV head one tile per step keeps the kernel under 170 registers, so
     // that two 5-wave workgroups share a CU instead of one: measured slower, 16.5 against 14.8 ms over 32 layers of 4096 tokens.)
     // NP by the threads of the workgroup: 1024 / threads pairs each, rounded up
-#define MESH_CHUNK_LAUNCH(KT, VT)                                                                                         \
+#define MESH_CHUNK_LAUNCH(HD, KT, VT)                                                                                     \
     do {                                                                                                                  \
-        if (waves == 8) MESH_LAUNCH((attn_chunk_kernel<KT, VT, 2, 2>), grid, block, 0, stream, a, T, pos0, seq, hpw, fwd_from, qtiles, n_ksplit);      \
-        else if (waves == 6) MESH_LAUNCH((attn_chunk_kernel<KT, VT, 3, 2>), grid, block, 0, stream, a, T, pos0, seq, hpw, fwd_from, qtiles, n_ksplit); \
-        else MESH_LAUNCH((attn_chunk_kernel<KT, VT, 4, 2>), grid, block, 0, stream, a, T, pos0, seq, hpw, fwd_from, qtiles, n_ksplit);                  \
+        if (waves == 8) MESH_LAUNCH((attn_chunk_kernel<HD, KT, VT, 2, 2>), grid, block, 0, stream, a, T, pos0, seq, hpw, fwd_from, qtiles, n_ksplit);      \
+        else if (waves == 6) MESH_LAUNCH((attn_chunk_kernel<HD, KT, VT, 3, 2>), grid, block, 0, stream, a, T, pos0, seq, hpw, fwd_from, qtiles, n_ksplit); \
+        else MESH_LAUNCH((attn_chunk_kernel<HD, KT, VT, 4, 2>), grid, block, 0, stream, a, T, pos0, seq, hpw, fwd_from, qtiles, n_ksplit);                  \
     } while (0)
-    if (a.k_type == MESH_F16 && a.v_type == MESH_F16) MESH_CHUNK_LAUNCH(MESH_F16, MESH_F16);
-    else if (a.k_type == MESH_Q8_0 && a.v_type == MESH_Q4_0) MESH_CHUNK_LAUNCH(MESH_Q8_0, MESH_Q4_0);
-    else if (a.k_type == MESH_Q4_0 && a.v_type == MESH_Q4_0) MESH_CHUNK_LAUNCH(MESH_Q4_0, MESH_Q4_0);
+    if (a.head_dim == 64) MESH_CHUNK_LAUNCH(64, MESH_F16, MESH_F16);
+    else if (a.k_type == MESH_F16 && a.v_type == MESH_F16) MESH_CHUNK_LAUNCH(128, MESH_F16, MESH_F16);
+    else if (a.k_type == MESH_Q8_0 && a.v_type == MESH_Q4_0) MESH_CHUNK_LAUNCH(128, MESH_Q8_0, MESH_Q4_0);
+    else if (a.k_type == MESH_Q4_0 && a.v_type == MESH_Q4_0) MESH_CHUNK_LAUNCH(128, MESH_Q4_0, MESH_Q4_0);
     else return fail(MESH_ERR_UNSUPPORTED, "attention_chunk: KV cache types %d/%d", a.k_type, a.v_type);
 #undef MESH_CHUNK_LAUNCH
     MESH_LAUNCH_CHECK();

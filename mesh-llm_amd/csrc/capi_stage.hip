@@ -109,6 +109,18 @@ int mesh_gguf_probe(const char *gguf_path, mesh_model_info *out) {
     return MESH_OK;
 }
 
+int mesh_model_probe(const char *path, mesh_model_info *out) {
+    if (!path || !out) return fail(MESH_ERR_INVALID, "mesh_model_probe: null argument");
+    if (!is_model_folder(path)) return mesh_gguf_probe(path, out);
+    ModelSpec spec;
+    const int rc = model_spec_from_folder(path, spec);
+    if (rc != MESH_OK) return rc;
+    HParams hp;
+    hparams_from_spec(spec, hp);
+    fill_info(hp, out);
+    return MESH_OK;
+}
+
 int mesh_gguf_tensor(const char *gguf_path, const char *name, mesh_tensor_info *out) {
     if (!name || !out) return fail(MESH_ERR_INVALID, "mesh_gguf_tensor: null argument");
     GgufFile g;
@@ -160,6 +172,12 @@ void *mesh_session_stream(mesh_session *session) { return session ? static_cast<
 int mesh_session_synchronize(mesh_session *session) {
     if (!session) return fail(MESH_ERR_INVALID, "mesh_session_synchronize: null session");
     MESH_HIP_TRY(hipStreamSynchronize(session->stream));
+    return MESH_OK;
+}
+
+int mesh_session_seq_reset(mesh_session *session, int seq_id) {
+    if (!session || seq_id < 0 || seq_id >= session->stage->n_seq_max) return fail(MESH_ERR_INVALID, "mesh_session_seq_reset: bad session or sequence id");
+    if (session->hybrid) session->hybrid->seq_len[(size_t)seq_id] = 0;       // (cache rows and states are replaced as the next request is fed)
     return MESH_OK;
 }
 
@@ -249,6 +267,7 @@ static int kv_xfer(mesh_session *s, int layer, int seq_id, int pos0, int n_pos, 
     if (!s || !k || !v) return fail(MESH_ERR_INVALID, "mesh_session_kv: null argument");
     const mesh_stage *st = s->stage;
     const HParams &hp = st->hp;
+    if (st->hybrid) return fail(MESH_ERR_UNSUPPORTED, "mesh_session_kv: architecture '%s' carries more than key / value rows from token to token", hp.arch.c_str());
     if (layer < st->layer_begin || layer >= st->layer_end) return fail(MESH_ERR_INVALID, "mesh_session_kv: layer %d not in this stage [%d,%d)", layer, st->layer_begin, st->layer_end);
     if (seq_id < 0 || seq_id >= st->n_seq_max || pos0 < 0 || n_pos <= 0 || pos0 + n_pos > st->n_ctx)
         return fail(MESH_ERR_INVALID, "mesh_session_kv: sequence %d positions [%d,%d) outside the cache", seq_id, pos0, pos0 + n_pos);

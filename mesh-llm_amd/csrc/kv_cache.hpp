@@ -2,7 +2,8 @@
 //
 // A row is the head_dim values of one (sequence, kv head, position).  Three row types, the KV tiers of
 // KvCacheQuant::for_model_size (mesh-llm/src/inference/launch.rs:568-591: f16/f16 below 5 GB of model, q8_0 K with
-// q4_0 V up to 50 GB, q4_0/q4_0 above):
+// q4_0 V up to 50 GB, q4_0/q4_0 above), and 32-bit rows for stages that compute everything in 32 bits:
+//   MESH_F32   head_dim floats
 //   MESH_F16   head_dim halfs
 //   MESH_Q8_0  head_dim int8 quants, then head_dim/32 f16 scales          (ggml block_q8_0 values, regrouped)
 //   MESH_Q4_0  head_dim/2 bytes of nibbles, then head_dim/32 f16 scales   (ggml block_q4_0 values, regrouped)
@@ -17,28 +18,35 @@
 
 namespace mesh {
 
-__host__ __device__ constexpr int kv_quant_bytes(int type, int hd) { return type == MESH_F16 ? hd * 2 : type == MESH_Q8_0 ? hd : hd / 2; }
+__host__ __device__ constexpr int kv_quant_bytes(int type, int hd) { return type == MESH_F32 ? hd * 4 : type == MESH_F16 ? hd * 2 : type == MESH_Q8_0 ? hd : hd / 2; }
+// rows of quants with scales of their own
+__host__ __device__ constexpr bool kv_quantised(int type) { return type == MESH_Q8_0 || type == MESH_Q4_0; }
 __host__ __device__ constexpr int kv_row_bytes(int type, int hd) {
-    return (kv_quant_bytes(type, hd) + (type == MESH_F16 ? 0 : hd / 32 * 2) + 7) & ~7;
+    return (kv_quant_bytes(type, hd) + (kv_quantised(type) ? hd / 32 * 2 : 0) + 7) & ~7;
 }
-inline bool kv_type_supported(int type) { return type == MESH_F16 || type == MESH_Q8_0 || type == MESH_Q4_0; }
+inline bool kv_type_supported(int type) { return type == MESH_F32 || type == MESH_F16 || type == MESH_Q8_0 || type == MESH_Q4_0; }
 
 #if defined(__HIPCC__)
 // ---------------------------------------------------------------------------------------------- lane access
 // What a lane holding dimensions [ds, ds + 8) of a row fetches, and its decoding to value = scale * (u - off).
 template <int TYPE> struct KvRaw;
+template <> struct KvRaw<MESH_F32> { float4 a, b; };
 template <> struct KvRaw<MESH_F16> { uint4 v; };
 template <> struct KvRaw<MESH_Q8_0> { uint2 v; uint16_t d; };
 template <> struct KvRaw<MESH_Q4_0> { uint32_t v; uint16_t d; };
 
 template <int TYPE> __device__ __forceinline__ void kv_zero(KvRaw<TYPE> &r);
+template <> __device__ __forceinline__ void kv_zero<MESH_F32>(KvRaw<MESH_F32> &r) { r.a = r.b = make_float4(0.f, 0.f, 0.f, 0.f); }
 template <> __device__ __forceinline__ void kv_zero<MESH_F16>(KvRaw<MESH_F16> &r) { r.v = make_uint4(0, 0, 0, 0); }
 template <> __device__ __forceinline__ void kv_zero<MESH_Q8_0>(KvRaw<MESH_Q8_0> &r) { r.v = make_uint2(0x80808080u, 0x80808080u); r.d = 0; }
 template <> __device__ __forceinline__ void kv_zero<MESH_Q4_0>(KvRaw<MESH_Q4_0> &r) { r.v = 0x88888888u; r.d = 0; }
 
 template <int TYPE, int HD> __device__ __forceinline__ KvRaw<TYPE> kv_load(const uint8_t *row, int ds) {
     KvRaw<TYPE> r;
-    if constexpr (TYPE == MESH_F16) {
+    if constexpr (TYPE == MESH_F32) {
+        r.a = *reinterpret_cast<const float4 *>(row + ds * 4);
+        r.b = *reinterpret_cast<const float4 *>(row + ds * 4 + 16);
+    } else if constexpr (TYPE == MESH_F16) {
         r.v = *reinterpret_cast<const uint4 *>(row + ds * 2);
     } else if constexpr (TYPE == MESH_Q8_0) {
         r.v = *reinterpret_cast<const uint2 *>(row + ds);
@@ -52,9 +60,13 @@ template <int TYPE, int HD> __device__ __forceinline__ KvRaw<TYPE> kv_load(const
 
 template <int TYPE> struct KvAffine { static constexpr float off = TYPE == MESH_Q8_0 ? 128.f : TYPE == MESH_Q4_0 ? 8.f : 0.f; };
 
-// u[8] are small non-negative integers (quantised types; the stored quant plus `off`) or the values themselves (f16)
+// u[8] are small non-negative integers (quantised types; the stored quant plus `off`) or the values themselves (f16, f32)
 template <int TYPE> __device__ __forceinline__ float kv_decode(const KvRaw<TYPE> &r, float (&u)[8]) {
-    if constexpr (TYPE == MESH_F16) {
+    if constexpr (TYPE == MESH_F32) {
+        u[0] = r.a.x; u[1] = r.a.y; u[2] = r.a.z; u[3] = r.a.w;
+        u[4] = r.b.x; u[5] = r.b.y; u[6] = r.b.z; u[7] = r.b.w;
+        return 1.f;
+    } else if constexpr (TYPE == MESH_F16) {
         u[0] = f16_bits_to_f32((uint16_t)(r.v.x & 0xFFFF)); u[1] = f16_bits_to_f32((uint16_t)(r.v.x >> 16));
         u[2] = f16_bits_to_f32((uint16_t)(r.v.y & 0xFFFF)); u[3] = f16_bits_to_f32((uint16_t)(r.v.y >> 16));
         u[4] = f16_bits_to_f32((uint16_t)(r.v.z & 0xFFFF)); u[5] = f16_bits_to_f32((uint16_t)(r.v.z >> 16));
@@ -78,6 +90,10 @@ template <int TYPE> __device__ __forceinline__ float kv_decode(const KvRaw<TYPE>
 // is a reduction over the 32 lanes of a block; q4_0 takes the FIRST element of largest magnitude, as the serial
 // reference loop does.
 __device__ __forceinline__ void kv_store_row(int type, uint8_t *row, const float *vec, int hd, int lane) {
+    if (type == MESH_F32) {
+        for (int i = lane; i < hd; i += 64) reinterpret_cast<float *>(row)[i] = vec[i];
+        return;
+    }
     if (type == MESH_F16) {
         for (int i = lane; i < hd; i += 64) reinterpret_cast<uint16_t *>(row)[i] = f32_to_f16_bits(vec[i]);
         return;
@@ -116,6 +132,7 @@ __device__ __forceinline__ void kv_store_row(int type, uint8_t *row, const float
 
 // element i of a row as f32 (the value the attention kernels see)
 __device__ __forceinline__ float kv_fetch(int type, const uint8_t *row, int hd, int i) {
+    if (type == MESH_F32) return reinterpret_cast<const float *>(row)[i];
     if (type == MESH_F16) return f16_bits_to_f32(reinterpret_cast<const uint16_t *>(row)[i]);
     const float d = f16_bits_to_f32(reinterpret_cast<const uint16_t *>(row + kv_quant_bytes(type, hd))[i >> 5]);
     if (type == MESH_Q8_0) return (float)(int8_t)row[i] * d;

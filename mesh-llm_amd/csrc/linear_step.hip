@@ -1,0 +1,231 @@
+// The single-token product: y = W x for a bf16 matrix and one f32 vector, bound by the weight stream.
+//
+// A wave takes R rows at a time; its 64 lanes cover 512 consecutive k per 16-byte load and R * U loads are in flight while
+// the R * U before them are multiplied.  The input vector sits in LDS as f32.  Every workgroup derives it itself from what
+// the launch before left (residual update with its output norm, polynomial activation: linear.hpp), which saves a launch
+// between two products; the first weight loads go out before that work and travel behind it.  Sums of squares a later norm
+// needs are left per workgroup and added in workgroup order by the consumer, so the result does not depend on timing.
+#include "linear.hpp"
+
+#include <algorithm>
+
+namespace mesh {
+
+constexpr int STEP_THREADS = 512, STEP_WAVES = STEP_THREADS / 64;
+constexpr size_t STEP_LDS_MAX = 160 * 1024 - 1024;
+
+__device__ __forceinline__ float step_wave_sum(float v) {
+#pragma unroll
+    for (int o = 32; o > 0; o >>= 1) v += __shfl_xor(v, o);
+    return v;
+}
+// sum over the workgroup in a fixed order, the same in every thread
+__device__ __forceinline__ float step_block_sum(float v, float *scratch, int lane, int wave) {
+    v = step_wave_sum(v);
+    __syncthreads();
+    if (lane == 0) scratch[wave] = v;
+    __syncthreads();
+    float s = 0.f;
+#pragma unroll
+    for (int w = 0; w < STEP_WAVES; ++w) s += scratch[w];
+    return s;
+}
+
+template <int R, int U, StepIn IN, StepOut OUT>
+__global__ __launch_bounds__(STEP_THREADS) void linear_step_kernel(const uint16_t *p_w, int p_Kp, int p_groups, int p_width, int p_K, const StepArgs a) {
+    extern __shared__ __align__(16) uint8_t smem[];
+    __shared__ float scratch[STEP_WAVES][4];
+    float *xs = reinterpret_cast<float *>(smem);
+    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+    const int K = p_K, Kp = p_Kp;
+    const int batches = (Kp + 512 * U - 1) / (512 * U);
+    const int g_step = gridDim.x * STEP_WAVES;
+    int grp = blockIdx.x * STEP_WAVES + wave, batch = 0;
+    auto row_of = [&](int gr, int r) { return OUT == STEP_OUT_MIN_GRU ? r * p_width + gr : gr * R + r; };
+    auto fetch = [&](uint4 (&b)[R][U], int gr, int bt) {
+#pragma unroll
+        for (int r = 0; r < R; ++r) {
+            const uint16_t *wr = p_w + (size_t)row_of(gr, r) * Kp;
+#pragma unroll
+            for (int u = 0; u < U; ++u) {
+                const int k = (bt * U + u) * 512 + lane * 8;
+                b[r][u] = make_uint4(0, 0, 0, 0);
+                if (k < Kp) b[r][u] = *reinterpret_cast<const uint4 *>(wr + k);
+            }
+        }
+    };
+    uint4 b0[R][U], b1[R][U];
+    if (grp < p_groups) fetch(b0, grp, 0);
+
+    // ---- the input vector
+    if constexpr (IN == STEP_IN_VEC) {
+        for (int k = tid; k < Kp; k += STEP_THREADS) xs[k] = k < K ? a.in[k] : 0.f;
+    } else if constexpr (IN == STEP_IN_POLY) {
+        float p2 = 0.f, p4 = 0.f, p6 = 0.f;
+        for (int i = tid; i < a.n_part; i += STEP_THREADS) { p2 += a.part[i]; p4 += a.part[a.n_part + i]; p6 += a.part[2 * a.n_part + i]; }
+        p2 = step_block_sum(p2, &scratch[0][0], lane, wave);
+        p4 = step_block_sum(p4, &scratch[0][0], lane, wave);
+        p6 = step_block_sum(p6, &scratch[0][0], lane, wave);
+        const float c1 = a.coef[0] / sqrtf(p2 / (float)K + a.eps), c2 = a.coef[1] / sqrtf(p4 / (float)K + a.eps), c3 = a.coef[2] / sqrtf(p6 / (float)K + a.eps);
+        const float c0 = a.coef[3];
+        for (int k = tid; k < Kp; k += STEP_THREADS) {
+            const float u = k < K ? a.in[k] : 0.f;
+            xs[k] = k < K ? ((c3 * u + c2) * u + c1) * u + c0 : 0.f;
+        }
+    } else {
+        float ss = 0.f;
+        for (int i = tid; i < a.n_part; i += STEP_THREADS) ss += a.part[i];
+        ss = step_block_sum(ss, &scratch[0][0], lane, wave);
+        const float rinv = 1.0f / sqrtf(ss / (float)K + a.eps);
+        float sx = 0.f;
+        for (int k = tid; k < Kp; k += STEP_THREADS) {
+            float v = 0.f;
+            if (k < K) {
+                v = a.in[k] + a.y[k] * rinv * a.gain[k];
+                if (blockIdx.x == 0) a.x_out[k] = v;
+            }
+            xs[k] = v;
+            sx = fmaf(v, v, sx);
+        }
+        if constexpr (IN == STEP_IN_RESIDUAL_NORM) {
+            sx = step_block_sum(sx, &scratch[0][0], lane, wave);
+            const float z = a.norm_gain[0] / sqrtf(sx / (float)K + a.eps);
+            for (int k = tid; k < Kp; k += STEP_THREADS) xs[k] *= z;
+        }
+    }
+    __syncthreads();
+
+    // ---- rows
+    float acc[R], s2 = 0.f, s4 = 0.f, s6 = 0.f;
+#pragma unroll
+    for (int r = 0; r < R; ++r) acc[r] = 0.f;
+    auto finish = [&](int gr) {
+        float v[R];
+#pragma unroll
+        for (int r = 0; r < R; ++r) { v[r] = step_wave_sum(acc[r]); acc[r] = 0.f; }
+        if constexpr (OUT == STEP_OUT_MIN_GRU) {
+            if (lane == 0) {
+                const float pz = v[0] + a.bias_z[gr], u = v[1] + a.bias_x[gr];
+                const float z = 1.0f / (1.0f + expf(-pz)), keep = 1.0f / (1.0f + expf(pz));
+                const float cand = u >= 0.f ? u + 0.5f : 1.0f / (1.0f + expf(-u));
+                float *st = a.state + (size_t)a.seq[0] * p_width + gr;
+                const float s = (a.pos[0] == 0 ? 0.f : keep * *st) + z * cand;
+                *st = s;
+                a.out[gr] = s * (v[2] / (1.0f + expf(-v[2])));
+            }
+        } else {
+#pragma unroll
+            for (int r = 0; r < R; ++r) {
+                const int m = gr * R + r;
+                if (m >= a.W.M) continue;
+                float o = v[r];
+                if constexpr (OUT == STEP_OUT_SIDE) {
+                    const float e = bf16_bits_to_f32(a.side[(size_t)a.tok[0] * a.side_stride + a.side_offset + m]);
+                    o = 0.5f * o * (1.0f + tanhf(0.7978845608028654f * (o + 0.044715f * o * o * o))) * e;
+                }
+                if (lane == 0) a.out[m] = o;
+                const float q = o * o;
+                if constexpr (OUT == STEP_OUT_SUMSQ || OUT == STEP_OUT_POWERS) s2 += q;
+                if constexpr (OUT == STEP_OUT_POWERS) { s4 += q * q; s6 += q * q * q; }
+            }
+        }
+    };
+    auto use = [&](const uint4 (&b)[R][U], int bt) {
+#pragma unroll
+        for (int u = 0; u < U; ++u) {
+            const int k = (bt * U + u) * 512 + lane * 8;
+            if (k < Kp) {
+                const float4 xa = *reinterpret_cast<const float4 *>(xs + k), xb = *reinterpret_cast<const float4 *>(xs + k + 4);
+                const float xf[8] = {xa.x, xa.y, xa.z, xa.w, xb.x, xb.y, xb.z, xb.w};
+#pragma unroll
+                for (int r = 0; r < R; ++r) {
+                    const uint32_t w[4] = {b[r][u].x, b[r][u].y, b[r][u].z, b[r][u].w};
+#pragma unroll
+                    for (int j = 0; j < 8; ++j) acc[r] = fmaf(__uint_as_float((j & 1) ? (w[j >> 1] & 0xFFFF0000u) : (w[j >> 1] << 16)), xf[j], acc[r]);
+                }
+            }
+        }
+    };
+    // (group, batch) pairs in order; each is fetched while the one before it is used
+    auto step = [&](uint4 (&cur)[R][U], uint4 (&next)[R][U]) {
+        const int gr = grp, bt = batch;
+        if (++batch == batches) { batch = 0; grp += g_step; }
+        if (grp < p_groups) fetch(next, grp, batch);
+        use(cur, bt);
+        if (bt == batches - 1) finish(gr);
+    };
+    while (grp < p_groups) {
+        step(b0, b1);
+        if (grp >= p_groups) break;
+        step(b1, b0);
+    }
+    if constexpr (OUT == STEP_OUT_SUMSQ || OUT == STEP_OUT_POWERS) {
+        // (every lane of a wave holds the wave's sums)
+        __syncthreads();
+        if (lane == 0) { scratch[wave][0] = s2; scratch[wave][1] = s4; scratch[wave][2] = s6; }
+        __syncthreads();
+        if (tid < (OUT == STEP_OUT_POWERS ? 3 : 1)) {
+            float s = 0.f;
+            for (int w = 0; w < STEP_WAVES; ++w) s += scratch[w][tid];
+            a.out_part[(size_t)tid * gridDim.x + blockIdx.x] = s;
+        }
+    }
+}
+
+bool linear_step_supported(const LinearWeight &W) { return (size_t)W.Kp * sizeof(float) <= STEP_LDS_MAX; }
+
+static int rows_per_group(const StepArgs &a) { return a.out_kind == STEP_OUT_MIN_GRU ? 3 : a.W.M < 4096 ? 1 : 2; }
+static int step_groups(const StepArgs &a) { return a.out_kind == STEP_OUT_MIN_GRU ? a.width : (a.W.M + rows_per_group(a) - 1) / rows_per_group(a); }
+
+int linear_step_grid(const StepArgs &a) {
+    // as many workgroups as the chip holds at once, two per CU; more rows mean more turns per wave, equally many for all
+    const int wgs = (step_groups(a) + STEP_WAVES - 1) / STEP_WAVES;
+    const int turns = (wgs + STEP_PARTS_MAX - 1) / STEP_PARTS_MAX;
+    return (wgs + turns - 1) / turns;
+}
+
+template <int R, int U, StepIn IN, StepOut OUT>
+static int launch_step(const StepArgs &a, hipStream_t stream) {
+    const size_t lds = (size_t)a.W.Kp * sizeof(float);
+    static bool ready = false;        // (hosts are single-threaded per session; a second thread sets the same attribute)
+    if (!ready) {
+        MESH_HIP_TRY(hipFuncSetAttribute(reinterpret_cast<const void *>(linear_step_kernel<R, U, IN, OUT>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)STEP_LDS_MAX));
+        ready = true;
+    }
+    MESH_LAUNCH((linear_step_kernel<R, U, IN, OUT>), dim3((unsigned)linear_step_grid(a)), dim3(STEP_THREADS), lds, stream, a.W.w, a.W.Kp, step_groups(a), a.width, a.W.K, a);
+    MESH_LAUNCH_CHECK();
+    return MESH_OK;
+}
+template <StepIn IN, StepOut OUT>
+static int launch_step_rows(const StepArgs &a, hipStream_t stream) {
+    return rows_per_group(a) == 1 ? launch_step<1, 4, IN, OUT>(a, stream) : launch_step<2, 4, IN, OUT>(a, stream);
+}
+
+int linear_step(const StepArgs &a, hipStream_t stream) {
+    const LinearWeight &W = a.W;
+    if (!W.w || !a.in || !a.out || W.M < 1 || W.Kp % LINEAR_K_PAD || W.Kp < W.K || W.Mp < W.M || !linear_step_supported(W))
+        return fail(MESH_ERR_INVALID, "linear_step: bad operands (%d x %d)", W.M, W.K);
+    const bool resid = a.in_kind == STEP_IN_RESIDUAL || a.in_kind == STEP_IN_RESIDUAL_NORM;
+    if ((resid && (!a.y || !a.gain || !a.part || !a.x_out || a.x_out == a.in || a.n_part < 1 || a.n_part > STEP_PARTS_MAX)) ||
+        (a.in_kind == STEP_IN_RESIDUAL_NORM && !a.norm_gain) || (a.in_kind == STEP_IN_POLY && (!a.part || !a.coef || a.n_part < 1 || a.n_part > STEP_PARTS_MAX)))
+        return fail(MESH_ERR_INVALID, "linear_step: input description incomplete");
+    if (((a.out_kind == STEP_OUT_SUMSQ || a.out_kind == STEP_OUT_POWERS) && !a.out_part) ||
+        (a.out_kind == STEP_OUT_MIN_GRU && (!a.state || !a.pos || !a.seq || !a.bias_z || !a.bias_x || a.width < 1 || W.M != 3 * a.width)) ||
+        (a.out_kind == STEP_OUT_SIDE && (!a.side || !a.tok)))
+        return fail(MESH_ERR_INVALID, "linear_step: output description incomplete");
+#define MESH_STEP_CASE(IN, OUT) \
+    if (a.in_kind == IN && a.out_kind == OUT) return launch_step_rows<IN, OUT>(a, stream);
+    MESH_STEP_CASE(STEP_IN_VEC, STEP_OUT_PLAIN)
+    MESH_STEP_CASE(STEP_IN_RESIDUAL, STEP_OUT_PLAIN)
+    MESH_STEP_CASE(STEP_IN_RESIDUAL_NORM, STEP_OUT_PLAIN)
+    MESH_STEP_CASE(STEP_IN_VEC, STEP_OUT_SUMSQ)
+    MESH_STEP_CASE(STEP_IN_POLY, STEP_OUT_SUMSQ)
+    MESH_STEP_CASE(STEP_IN_RESIDUAL, STEP_OUT_POWERS)
+    MESH_STEP_CASE(STEP_IN_RESIDUAL, STEP_OUT_SIDE)
+#undef MESH_STEP_CASE
+    if (a.in_kind == STEP_IN_VEC && a.out_kind == STEP_OUT_MIN_GRU) return launch_step<3, 2, STEP_IN_VEC, STEP_OUT_MIN_GRU>(a, stream);
+    if (a.in_kind == STEP_IN_RESIDUAL && a.out_kind == STEP_OUT_MIN_GRU) return launch_step<3, 2, STEP_IN_RESIDUAL, STEP_OUT_MIN_GRU>(a, stream);
+    return fail(MESH_ERR_UNSUPPORTED, "linear_step: no kernel for input %d with output %d", (int)a.in_kind, (int)a.out_kind);
+}
+
+}  // namespace mesh

@@ -114,6 +114,14 @@ __device__ __forceinline__ uint16_t f32_to_f16_bits(float f) {
 }
 __device__ __forceinline__ float f16_bits_to_f32(uint16_t h) { return __half2float(__ushort_as_half(h)); }
 
+// bfloat16 bits <-> f32: round to nearest even, NaN kept a NaN
+__device__ __forceinline__ uint16_t f32_to_bf16_bits(float f) {
+    const uint32_t w = __float_as_uint(f);
+    if ((w & 0x7FFFFFFFu) > 0x7F800000u) return (uint16_t)((w >> 16) | 0x40u);
+    return (uint16_t)((w + 0x7FFFu + ((w >> 16) & 1u)) >> 16);
+}
+__device__ __forceinline__ float bf16_bits_to_f32(uint16_t h) { return __uint_as_float((uint32_t)h << 16); }
+
 // The f16 producers of the batched paths clamp what f16 cannot hold to +-65504.  A caller can ask how often that happened
 // (mesh_session_f16_saturations): every producer that can meet such a value is handed the session's counter and notes each
 // group of values it clamps.  `sat` may be null (no counting).

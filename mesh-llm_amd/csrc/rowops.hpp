@@ -1,0 +1,60 @@
+// Element-wise and per-row work between the products of a hybrid model's layers (rowops.hip), many tokens at a time, and
+// the gated recurrence (recurrent.hip).  "act" outputs are rows of ld elements of `act` type whose columns from n on are
+// written as zeros (linear.hpp: the activations of a product).
+#pragma once
+
+#include "linear.hpp"
+
+namespace mesh {
+
+// x[t] = table[tok[t]] * scale + position vector of pos[t]: entries 2i and 2i + 1 are sin and cos of pos * freq[i]
+int embed_rows(const uint16_t *table, const int32_t *tok, const int32_t *pos, const float *freq, float scale, int T, int n, float *x, hipStream_t stream);
+
+// x[t] += y[t] / rms(y[t]) * gain (y null: x as it is), and act[t] = x[t]
+int residual_norm_rows(float *x, const float *y, const float *gain, float eps, int T, int n, void *out, ActType act, int ld, hipStream_t stream);
+
+// act[i] = x[row[i]] / rms * gain[0] for i < n_rows (row null: i)
+int scalar_norm_rows(const float *x, const int32_t *row, const float *gain, float eps, int n_rows, int n, void *out, ActType act, int ld, hipStream_t stream);
+
+// act[t] = c0 N(u) + c1 N(u^2) + c2 N(u^3) + c3 with u = u[t][0..n), powers element by element, N(v) = v / rms(v)
+int poly_norm_rows(const float *u, const float *coef, float eps, int T, int n, void *out, ActType act, int ld, hipStream_t stream);
+
+// act[t][i] = gelu_tanh(g[t][i]) * side[tok[t]][offset + i]
+int side_gate_rows(const float *g, const uint16_t *side, const int32_t *tok, int stride, int offset, int T, int n, void *out, ActType act, int ld, hipStream_t stream);
+
+// Norm over a whole q / k projection and KV append for attention whose values are the un-normalised keys.  qk: [T][(n_head +
+// n_kv) * hd], q first; each head's entries from dim on are zero.  q[t] = q / rms(q over all heads) * q_norm; the cache
+// gets k / rms(k) * k_norm as the key and k as the value, rows of hd of kv_type (f16 or f32).
+struct QkAppendArgs {
+    const float *qk = nullptr;
+    float *q = nullptr;                // [T][n_head * hd]
+    uint8_t *kcache = nullptr, *vcache = nullptr;       // this layer's, [n_seq][n_kv][n_ctx] rows
+    int kv_type = MESH_F16;
+    const float *q_norm = nullptr, *k_norm = nullptr;   // [n_head * hd], [n_kv * hd], zero where the head is padded
+    const int32_t *pos = nullptr, *seq = nullptr;
+    unsigned *sat = nullptr;           // counts values clamped to the f16 range
+    float eps = 0.f;
+    int n_head = 0, n_kv = 0, dim = 0, hd = 0, n_ctx = 0;
+};
+int qk_norm_append(const QkAppendArgs &a, int T, hipStream_t stream);
+
+// Gated recurrence over the tokens of a call, in order within each sequence:
+//   z = sigmoid(pz + bias_z), u = px + bias_x, c = u + 1/2 where u >= 0 and sigmoid(u) elsewhere,
+//   S = (1 - z) S + z c,  act[t] = S * silu(pg)
+// with (pz, px, pg) = zxg[t] (three rows of width).  A sequence's tokens are neighbours in the call and ascend; its state is
+// read from `state` [n_seq][width] unless its first token is at position 0, and the last one is left there.  ws:
+// min_gru_workspace(T, width) floats.
+struct MinGruArgs {
+    const float *zxg = nullptr;
+    const float *bias_z = nullptr, *bias_x = nullptr;
+    float *state = nullptr;
+    const int32_t *pos = nullptr, *seq = nullptr;
+    float *ws = nullptr;
+    void *out = nullptr;
+    ActType act = ACT_BF16;
+    int ld = 0, width = 0;
+};
+size_t min_gru_workspace(int T, int width);
+int min_gru(const MinGruArgs &a, int T, hipStream_t stream);
+
+}  // namespace mesh

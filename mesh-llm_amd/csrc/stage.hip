@@ -20,6 +20,7 @@
 #include "gemm.hpp"
 #include "gemv.hpp"
 #include "moe.hpp"
+#include "registry.hpp"
 
 namespace mesh {
 
@@ -31,8 +32,8 @@ int dequantize_dev(int type, const void *src, float *dst, int64_t n, hipStream_t
 int hparams_from_gguf(const GgufFile &g, HParams &hp) {
     if (!g.get_str("general.architecture", hp.arch)) return fail(MESH_ERR_FORMAT, "gguf: general.architecture missing");
     const std::string &a = hp.arch;
-    if (a != "llama" && a != "qwen2" && a != "qwen3" && a != "qwen3moe")
-        return fail(MESH_ERR_UNSUPPORTED, "architecture '%s' is not supported (llama, qwen2, qwen3, qwen3moe are)", a.c_str());
+    if (!find_arch(a, CONTAINER_GGUF))
+        return fail(MESH_ERR_UNSUPPORTED, "architecture '%s' is not supported (%s are)", a.c_str(), arch_names(CONTAINER_GGUF).c_str());
     auto need = [&](const char *suffix, uint32_t &out) -> int {
         if (!g.get_u32(a + suffix, out)) return fail(MESH_ERR_FORMAT, "gguf: key %s%s missing or not an unsigned integer", a.c_str(), suffix);
         return MESH_OK;
@@ -71,6 +72,21 @@ int hparams_from_gguf(const GgufFile &g, HParams &hp) {
     return MESH_OK;
 }
 
+
+void hparams_from_spec(const ModelSpec &s, HParams &hp) {
+    hp.arch = s.arch;
+    hp.n_layer = (uint32_t)s.layers.size();
+    hp.n_embd = (uint32_t)s.width;
+    hp.n_vocab = (uint32_t)s.vocab;
+    hp.rms_eps = s.eps;
+    hp.rope_freq_base = 0.f;
+    for (const LayerSpec &l : s.layers) {
+        hp.n_head = std::max(hp.n_head, (uint32_t)l.mixer.heads);
+        hp.n_head_kv = std::max(hp.n_head_kv, (uint32_t)l.mixer.kv_heads);
+        hp.head_dim = std::max(hp.head_dim, (uint32_t)l.mixer.dim);
+        hp.n_ff = std::max(hp.n_ff, (uint32_t)l.ff);
+    }
+}
 
 // ------------------------------------------------------------------------------------------------ loading
 namespace {
@@ -214,13 +230,39 @@ struct Loader {
 
 }  // namespace
 
+int stage_select_device(const mesh_stage_opts *opts, mesh_stage *st) {
+    int rc;
+    if (opts && opts->device && opts->device[0] && (rc = mesh_device_select(opts->device)) != MESH_OK) return rc;
+    if (mesh_device_count() < 1) return fail(MESH_ERR_DEVICE, "mesh_stage_open: no GPU available");
+    MESH_HIP_TRY(hipGetDevice(&st->device));
+    return MESH_OK;
+}
+
+// what every kind of model takes from the options
+static int stage_common_opts(const mesh_stage_opts *opts, mesh_stage *st) {
+    int rc;
+    if ((rc = tuning_process_default(st->tune)) != MESH_OK) return rc;
+    if (opts && opts->tuning && (rc = tuning_parse(st->tune, opts->tuning, "mesh_stage_opts.tuning")) != MESH_OK) return rc;
+    st->n_ctx = opts && opts->n_ctx > 0 ? opts->n_ctx : 4096;
+    st->n_seq_max = opts && opts->n_seq_max > 0 ? opts->n_seq_max : 1;
+    st->n_batch_max = opts && opts->n_batch_max > 0 ? opts->n_batch_max : 512;
+    if (opts && opts->precision != MESH_PRECISION_DEFAULT && opts->precision != MESH_PRECISION_F32)
+        return fail(MESH_ERR_INVALID, "mesh_stage_open: precision %d unknown", opts->precision);
+    return MESH_OK;
+}
+
 int stage_open(const char *path, int layer_begin, int layer_end, const mesh_stage_opts *opts, mesh_stage **out) {
     if (!path || !out) return fail(MESH_ERR_INVALID, "mesh_stage_open: null argument");
     *out = nullptr;
-    GgufFile g;
-    int rc = g.open(path);
-    if (rc != MESH_OK) return rc;
+    int rc;
     std::unique_ptr<mesh_stage> st(new mesh_stage());
+    if (is_model_folder(path)) {
+        if ((rc = stage_common_opts(opts, st.get())) != MESH_OK || (rc = hybrid_open(path, layer_begin, layer_end, opts, st.get())) != MESH_OK) return rc;
+        *out = st.release();
+        return MESH_OK;
+    }
+    GgufFile g;
+    if ((rc = g.open(path)) != MESH_OK) return rc;
     if ((rc = hparams_from_gguf(g, st->hp)) != MESH_OK) return rc;
     const HParams &hp = st->hp;
     if (layer_end < 0) layer_end = (int)hp.n_layer;
@@ -228,20 +270,14 @@ int stage_open(const char *path, int layer_begin, int layer_end, const mesh_stag
         return fail(MESH_ERR_INVALID, "mesh_stage_open: layer range [%d,%d) does not fit a %u-layer model", layer_begin, layer_end, hp.n_layer);
     st->layer_begin = layer_begin;
     st->layer_end = layer_end;
-    if ((rc = tuning_process_default(st->tune)) != MESH_OK) return rc;
-    if (opts && opts->tuning && (rc = tuning_parse(st->tune, opts->tuning, "mesh_stage_opts.tuning")) != MESH_OK) return rc;
-    st->n_ctx = opts && opts->n_ctx > 0 ? opts->n_ctx : 4096;
-    st->n_seq_max = opts && opts->n_seq_max > 0 ? opts->n_seq_max : 1;
-    st->n_batch_max = opts && opts->n_batch_max > 0 ? opts->n_batch_max : 512;
+    if ((rc = stage_common_opts(opts, st.get())) != MESH_OK) return rc;
+    if (opts && opts->precision == MESH_PRECISION_F32)
+        return fail(MESH_ERR_UNSUPPORTED, "mesh_stage_open: architecture '%s' has no 32-bit path", hp.arch.c_str());
     st->k_type = opts && opts->kv_type ? opts->kv_type : MESH_F16;
     st->v_type = opts && opts->kv_type_v ? opts->kv_type_v : (st->k_type == MESH_F16 ? MESH_F16 : MESH_Q4_0);
     if (!kv_pair_supported(st->k_type, st->v_type))
         return fail(MESH_ERR_UNSUPPORTED, "mesh_stage_open: KV cache types %d/%d not supported (f16/f16, q8_0/q4_0 and q4_0/q4_0 are)", st->k_type, st->v_type);
-    if (opts && opts->device && opts->device[0]) {
-        if ((rc = mesh_device_select(opts->device)) != MESH_OK) return rc;
-    }
-    if (mesh_device_count() < 1) return fail(MESH_ERR_DEVICE, "mesh_stage_open: no GPU available");
-    MESH_HIP_TRY(hipGetDevice(&st->device));
+    if ((rc = stage_select_device(opts, st.get())) != MESH_OK) return rc;
     if (hp.head_dim != 64 && hp.head_dim != 128)
         return fail(MESH_ERR_UNSUPPORTED, "mesh_stage_open: head_dim %u has no attention kernel (64 and 128 do)", hp.head_dim);
 
@@ -324,11 +360,10 @@ int stage_open(const char *path, int layer_begin, int layer_end, const mesh_stag
     return MESH_OK;
 }
 
-static int sess_alloc(mesh_session *s, void **p, size_t bytes);
 static bool layer_is_kquant_dense(const LayerWeights &L);
 
 // ------------------------------------------------------------------------------------------------ session
-static int sess_alloc(mesh_session *s, void **p, size_t bytes) {
+int sess_alloc(mesh_session *s, void **p, size_t bytes) {
     hipError_t e = hipMalloc(p, bytes ? bytes : 16);
     if (e != hipSuccess) return fail(e == hipErrorOutOfMemory ? MESH_ERR_NOMEM : MESH_ERR_DEVICE, "hipMalloc(%zu) failed: %s", bytes, hipGetErrorString(e));
     s->allocations.push_back(*p);
@@ -346,24 +381,19 @@ constexpr int LOGITS_TOKENS_MAX = MESH_LOGITS_TOKENS_MAX;        // logits rows 
 #define PREFILL_MIN_TOKENS (s->tune.gemm_min_tokens)
 #define MOE_GEMM_MIN_PAIRS_PER_EXPERT ((size_t)s->tune.moe_gemm_min_pairs)
 
-int session_new(mesh_stage *st, mesh_session **out) {
-    if (!st || !out) return fail(MESH_ERR_INVALID, "mesh_stage_session_new: null argument");
-    *out = nullptr;
-    MESH_HIP_TRY(hipSetDevice(st->device));
-    std::unique_ptr<mesh_session> s(new mesh_session());
-    s->stage = st;
+// KV cache and activation buffers of a K-quant model
+static int kquant_session_alloc(mesh_session *s) {
+    mesh_stage *st = s->stage;
     const HParams &hp = st->hp;
     const size_t nl = st->layers.size(), B = (size_t)st->n_batch_max;
-    MESH_HIP_TRY(hipStreamCreateWithFlags(&s->stream, hipStreamNonBlocking));
-    s->tune = st->tune;
     const size_t kv_rows = (size_t)st->n_seq_max * hp.n_head_kv * (size_t)st->n_ctx;
     s->k_layer_bytes = kv_rows * (size_t)kv_row_bytes(st->k_type, (int)hp.head_dim);
     s->v_layer_bytes = kv_rows * (size_t)kv_row_bytes(st->v_type, (int)hp.head_dim);
     int rc;
     void *p = nullptr;
-    if ((rc = sess_alloc(s.get(), &p, nl * s->k_layer_bytes)) != MESH_OK) return rc;
+    if ((rc = sess_alloc(s, &p, nl * s->k_layer_bytes)) != MESH_OK) return rc;
     s->kcache = static_cast<uint8_t *>(p);
-    if ((rc = sess_alloc(s.get(), &p, nl * s->v_layer_bytes)) != MESH_OK) return rc;
+    if ((rc = sess_alloc(s, &p, nl * s->v_layer_bytes)) != MESH_OK) return rc;
     s->vcache = static_cast<uint8_t *>(p);
     MESH_HIP_TRY(hipMemsetAsync(s->kcache, 0, nl * s->k_layer_bytes, s->stream));
     MESH_HIP_TRY(hipMemsetAsync(s->vcache, 0, nl * s->v_layer_bytes, s->stream));
@@ -371,7 +401,7 @@ int session_new(mesh_stage *st, mesh_session **out) {
     const size_t ff = std::max<size_t>(hp.n_ff, (size_t)hp.n_ff_exp * std::max<uint32_t>(hp.n_expert_used, 1));
     auto fbuf = [&](float **dst, size_t n) -> int {
         void *q = nullptr;
-        int r = sess_alloc(s.get(), &q, n * sizeof(float));
+        int r = sess_alloc(s, &q, n * sizeof(float));
         *dst = static_cast<float *>(q);
         return r;
     };
@@ -381,18 +411,18 @@ int session_new(mesh_stage *st, mesh_session **out) {
         (rc = fbuf(&s->v, B * KD)) || (rc = fbuf(&s->attn, B * QD)) || (rc = fbuf(&s->ffn, B * ff)) ||
         (rc = fbuf(&s->attn_part, part_rows * QD)) || (rc = fbuf(&s->attn_ml, part_rows * hp.n_head * 2)))
         return rc;
-    if ((rc = sess_alloc(s.get(), &p, 256)) != MESH_OK) return rc;
+    if ((rc = sess_alloc(s, &p, 256)) != MESH_OK) return rc;
     s->f16_sat = static_cast<unsigned *>(p);
     MESH_HIP_TRY(hipMemsetAsync(p, 0, 256, s->stream));
     if (hp.n_ff && hp.n_ff % QK_K == 0) {
-        if ((rc = sess_alloc(s.get(), &p, xq_bytes((int)hp.n_ff))) != MESH_OK) return rc;
+        if ((rc = sess_alloc(s, &p, xq_bytes((int)hp.n_ff))) != MESH_OK) return rc;
         s->ffn_xq = static_cast<uint8_t *>(p);
     }
     // (either skinny kernel may be picked per call, so the buffers are there from the smaller of their thresholds on)
     const int skinny_alloc_from = s->tune.skinny_min_tokens > 0 ? s->tune.skinny_min_tokens : 4;
     if (B >= (size_t)std::min(PREFILL_MIN_TOKENS, skinny_alloc_from)) {
         const size_t B16 = (B + 15) / 16 * 16;       // the skinny GEMM reads whole blocks of 16 tokens
-        if ((rc = sess_alloc(s.get(), &p, B16 * std::max<size_t>(hp.n_embd, QD) * 2)) != MESH_OK) return rc;
+        if ((rc = sess_alloc(s, &p, B16 * std::max<size_t>(hp.n_embd, QD) * 2)) != MESH_OK) return rc;
         s->xn16 = static_cast<uint16_t *>(p);
         MESH_HIP_TRY(hipMemsetAsync(p, 0, B16 * std::max<size_t>(hp.n_embd, QD) * 2, s->stream));     // unused token columns stay finite
         {
@@ -404,31 +434,31 @@ int session_new(mesh_stage *st, mesh_session **out) {
             size_t bytes = (tok + 15) / 16 * q16_block_bytes((int)((kmax + 255) / 256 * 256));
             // mixture of experts: the down projections read one row of n_ff_exp per (token, slot) pair
             if (hp.n_expert) bytes = std::max(bytes, (tok * hp.n_expert_used + 15) / 16 * q16_block_bytes((int)((hp.n_ff_exp + 255) / 256 * 256)));
-            if ((rc = sess_alloc(s.get(), &p, bytes)) != MESH_OK) return rc;
+            if ((rc = sess_alloc(s, &p, bytes)) != MESH_OK) return rc;
             s->xq = static_cast<uint8_t *>(p);
         }
         if (st->k_type != MESH_F16 && hp.head_dim == 128 && B >= 128) {
             // f16 copy of one sequence's K and V rows of one layer: a long prefill chunk decodes the quantised cache once
             // per layer into it (attn.hpp: chunk_kv16).  Zeroed, so that rows past a chunk's last key are finite.
             const size_t bytes = 2 * (size_t)hp.n_head_kv * st->n_ctx * hp.head_dim * 2;
-            if ((rc = sess_alloc(s.get(), &p, bytes)) != MESH_OK) return rc;
+            if ((rc = sess_alloc(s, &p, bytes)) != MESH_OK) return rc;
             s->chunk_kv16 = static_cast<uint16_t *>(p);
             MESH_HIP_TRY(hipMemsetAsync(p, 0, bytes, s->stream));
         }
         if (hp.n_ff > 0) {
             // (two blocks of 16 tokens: the hand-over is for calls the skinny GEMM takes in one launch)
-            if ((rc = sess_alloc(s.get(), &p, SKINNY_F16_NORM_TOKENS_MAX * (size_t)hp.n_embd * 2)) != MESH_OK) return rc;
+            if ((rc = sess_alloc(s, &p, SKINNY_F16_NORM_TOKENS_MAX * (size_t)hp.n_embd * 2)) != MESH_OK) return rc;
             s->norm16 = static_cast<uint16_t *>(p);
             MESH_HIP_TRY(hipMemsetAsync(p, 0, SKINNY_F16_NORM_TOKENS_MAX * (size_t)hp.n_embd * 2, s->stream));
             if ((rc = fbuf(&s->norm_part, (size_t)SKINNY_F16_NORM_PARTS_MAX * SKINNY_F16_NORM_TOKENS_MAX)) != MESH_OK) return rc;
-            if ((rc = sess_alloc(s.get(), &p, B16 * (size_t)hp.n_ff * 2)) != MESH_OK) return rc;
+            if ((rc = sess_alloc(s, &p, B16 * (size_t)hp.n_ff * 2)) != MESH_OK) return rc;
             s->ffn16 = static_cast<uint16_t *>(p);
             if ((rc = fbuf(&s->ffn_up, B * (size_t)hp.n_ff)) != MESH_OK) return rc;
         }
         if (B >= (size_t)PREFILL_MIN_TOKENS) {
             // a split launch holds at most one 128 x 128 f32 tile per CU: 16.8 MB on 256 CUs
             s->gemm_part_bytes = (size_t)32 << 20;
-            if ((rc = sess_alloc(s.get(), &p, s->gemm_part_bytes)) != MESH_OK) return rc;
+            if ((rc = sess_alloc(s, &p, s->gemm_part_bytes)) != MESH_OK) return rc;
             s->gemm_part = static_cast<float *>(p);
         }
     }
@@ -437,13 +467,13 @@ int session_new(mesh_stage *st, mesh_session **out) {
         if ((rc = fbuf(&s->moe_logits, B * ne)) || (rc = fbuf(&s->moe_w, B * k)) || (rc = fbuf(&s->moe_out, B * k * hp.n_embd)) ||
             (rc = fbuf(&s->expert_mask, ne)))
             return rc;
-        if ((rc = sess_alloc(s.get(), &p, B * k * sizeof(int32_t))) != MESH_OK) return rc;
+        if ((rc = sess_alloc(s, &p, B * k * sizeof(int32_t))) != MESH_OK) return rc;
         s->moe_ids = static_cast<int32_t *>(p);
         // work items: 4 pairs each for the mat-vec kernel, 16 for the matrix-core one; the buffer fits either
         const size_t items = (size_t)std::max(moe_max_items((int)(B * k), (int)ne) * MOE_ITEM_INTS,
                                               moe_max_items((int)(B * k), (int)ne, SKINNY_ITEM_PAIRS) * moe_item_ints(SKINNY_ITEM_PAIRS)) / MOE_ITEM_INTS + 1;
         // (+ the item count, + the arrival counter of the router launch whose last workgroup routes and groups)
-        if ((rc = sess_alloc(s.get(), &p, (items * MOE_ITEM_INTS + 2) * sizeof(int32_t))) != MESH_OK) return rc;
+        if ((rc = sess_alloc(s, &p, (items * MOE_ITEM_INTS + 2) * sizeof(int32_t))) != MESH_OK) return rc;
         s->moe_items = static_cast<int32_t *>(p);
         s->moe_n_items = s->moe_items + items * MOE_ITEM_INTS;
         s->moe_arrive = reinterpret_cast<int *>(s->moe_n_items + 1);
@@ -454,26 +484,45 @@ int session_new(mesh_stage *st, mesh_session **out) {
             // down-projection rows, all indexed by slot (moe.hpp: moe_sort)
             const size_t slots = (size_t)moe_sort_slots((int)(B * k), (int)ne), tiles = (size_t)moe_sort_max_tiles((int)(B * k), (int)ne);
             const size_t pairs4 = (B * k + 3) / 4 * 4;
-            if ((rc = sess_alloc(s.get(), &p, (pairs4 + slots + 4 * tiles + 4) * sizeof(int32_t))) != MESH_OK) return rc;
+            if ((rc = sess_alloc(s, &p, (pairs4 + slots + 4 * tiles + 4) * sizeof(int32_t))) != MESH_OK) return rc;
             s->moe_sorted.slot_of_pair = static_cast<int32_t *>(p);
             s->moe_sorted.pair_of_slot = s->moe_sorted.slot_of_pair + pairs4;
             s->moe_sorted.tiles = s->moe_sorted.pair_of_slot + slots;           // (a multiple of 16 ints in: 16-byte aligned)
             s->moe_sorted.counts = s->moe_sorted.tiles + 4 * tiles;
-            if ((rc = sess_alloc(s.get(), &p, slots * hp.n_embd * 2)) != MESH_OK) return rc;
+            if ((rc = sess_alloc(s, &p, slots * hp.n_embd * 2)) != MESH_OK) return rc;
             s->moe_x16 = static_cast<uint16_t *>(p);
-            if ((rc = sess_alloc(s.get(), &p, slots * (size_t)hp.n_ff_exp * 2)) != MESH_OK) return rc;
+            if ((rc = sess_alloc(s, &p, slots * (size_t)hp.n_ff_exp * 2)) != MESH_OK) return rc;
             s->moe_ffn16 = static_cast<uint16_t *>(p);
             if ((rc = fbuf(&s->moe_out_slots, slots * hp.n_embd)) != MESH_OK) return rc;
             MESH_HIP_TRY(hipMemsetAsync(s->moe_x16, 0, slots * hp.n_embd * 2, s->stream));          // unused slots stay finite
             MESH_HIP_TRY(hipMemsetAsync(s->moe_ffn16, 0, slots * (size_t)hp.n_ff_exp * 2, s->stream));
         }
     }
-    if ((rc = sess_alloc(s.get(), &p, 3 * B * sizeof(int32_t))) != MESH_OK) return rc;
+    if (st->output.present() && (rc = fbuf(&s->logit_rows, B * hp.n_embd)) != MESH_OK) return rc;
+    return MESH_OK;
+}
+
+int session_new(mesh_stage *st, mesh_session **out) {
+    if (!st || !out) return fail(MESH_ERR_INVALID, "mesh_stage_session_new: null argument");
+    *out = nullptr;
+    MESH_HIP_TRY(hipSetDevice(st->device));
+    std::unique_ptr<mesh_session> s(new mesh_session());
+    s->stage = st;
+    const HParams &hp = st->hp;
+    const size_t B = (size_t)st->n_batch_max;
+    MESH_HIP_TRY(hipStreamCreateWithFlags(&s->stream, hipStreamNonBlocking));
+    s->tune = st->tune;
+    int rc = st->hybrid ? hybrid_session_alloc(s.get()) : kquant_session_alloc(s.get());
+    if (rc != MESH_OK) return rc;
+    void *p = nullptr;
+    if ((rc = sess_alloc(s.get(), &p, 4 * B * sizeof(int32_t))) != MESH_OK) return rc;
     s->d_pos = static_cast<int32_t *>(p);
     s->d_seq = s->d_pos + B;
     s->d_tok = s->d_seq + B;
-    MESH_HIP_TRY(hipHostMalloc(reinterpret_cast<void **>(&s->h_meta), META_SLOTS * 3 * B * sizeof(int32_t), hipHostMallocDefault));
-    memset(s->h_meta, 0, META_SLOTS * 3 * B * sizeof(int32_t));
+    s->d_rows = s->d_tok + B;
+    MESH_HIP_TRY(hipMemsetAsync(p, 0, 4 * B * sizeof(int32_t), s->stream));
+    MESH_HIP_TRY(hipHostMalloc(reinterpret_cast<void **>(&s->h_meta), META_SLOTS * 4 * B * sizeof(int32_t), hipHostMallocDefault));
+    memset(s->h_meta, 0, META_SLOTS * 4 * B * sizeof(int32_t));
     // staging for packed in/out of the host-pointer entry point: f32 rows of n_embd in; the same or logits rows out
     // (logits of at most LOGITS_TOKENS_MAX tokens per call: a row of a 152k vocabulary is 0.6 MB)
     s->io_stage_bytes = B * (size_t)hp.n_embd * sizeof(float);
@@ -497,7 +546,7 @@ static GemvMat mat_of(const DevTensor &w, float *y, int ldy, const DevTensor *bi
 // to f16; faster at every batch size, so the default is 1).  Callers that want the all-f32 vector-ALU kernel at small
 // batches raise it.
 // quantised: the cache rows are q8_0 / q4_0
-static int attn_splits_for(const Tuning &tune, int T, int n_kv, int max_keys, bool quantised) {
+int attn_splits_for(const Tuning &tune, int T, int n_kv, int max_keys, bool quantised) {
     // One workgroup per compute unit (256 on gfx950) measured best from batch 1 to 16 with f16 rows, which that many
     // workgroups stream at the memory's rate.  Quantised rows are bound by the instructions that decode them, and two
     // workgroups per CU hide each other's waits: 3-7% of the step at batch 8-32 (Qwen2.5-32B shape, q8_0 / q4_0 cache:
@@ -537,14 +586,10 @@ LaunchTimer launch_timer() {
     return t;
 }
 
-struct ProfScope {
-    mesh_session *prev_s;
-    int prev_kind;
-    ProfScope(mesh_session *ses, int kind) : prev_s(t_prof_session), prev_kind(t_prof_kind) {
-        if (ses->profile) { t_prof_session = ses; t_prof_kind = kind; }
-    }
-    ~ProfScope() { t_prof_session = prev_s; t_prof_kind = prev_kind; }
-};
+ProfScope::ProfScope(mesh_session *ses, int kind) : prev_s(t_prof_session), prev_kind(t_prof_kind) {
+    if (ses->profile) { t_prof_session = ses; t_prof_kind = kind; }
+}
+ProfScope::~ProfScope() { t_prof_session = prev_s; t_prof_kind = prev_kind; }
 
 int profile_collect(mesh_session *s) {
     MESH_HIP_TRY(hipStreamSynchronize(s->stream));
@@ -869,6 +914,7 @@ static int run_layer_prefill(mesh_session *s, const LayerWeights &L, size_t il, 
 // Runs the layers over the T token rows already in s->x.  pos/seq are on the device in s->d_pos / s->d_seq.
 static int run_layers(mesh_session *s, int T, int max_keys) {
     mesh_stage *st = s->stage;
+    if (st->hybrid) return hybrid_run_layers(s, T, max_keys);
     const HParams &hp = st->hp;
     hipStream_t stream = s->stream;
     const int E = (int)hp.n_embd, QD = (int)(hp.n_head * hp.head_dim), KD = (int)(hp.n_head_kv * hp.head_dim);
@@ -1168,8 +1214,8 @@ static int run_layers_graphed(mesh_session *s, int T, int max_keys) {
     // chunk's.  Such calls are always launched eagerly.
     if (s->chunk_pos0 >= 0 && T >= PREFILL_MIN_TOKENS) return run_layers(s, T, max_keys);
     const mesh_stage *st = s->stage;
-    const int n_splits = attn_splits_for(s->tune, T, (int)st->hp.n_head_kv, max_keys, st->k_type != MESH_F16);
-    const uint64_t key = (uint64_t)T | ((uint64_t)n_splits << 8) | ((uint64_t)(s->expert_mask_on ? 1 : 0) << 20);
+    const int n_splits = st->hybrid ? 0 : attn_splits_for(s->tune, T, (int)st->hp.n_head_kv, max_keys, st->k_type != MESH_F16);
+    const uint64_t key = st->hybrid ? hybrid_graph_key(s, T, max_keys) : (uint64_t)T | ((uint64_t)n_splits << 8) | ((uint64_t)(s->expert_mask_on ? 1 : 0) << 20);
     auto it = s->graphs.find(key);
     if (it == s->graphs.end()) {
         if (s->graphs.size() >= GRAPH_MAX_ENTRIES) return run_layers(s, T, max_keys);
@@ -1200,8 +1246,15 @@ static int run_layers_graphed(mesh_session *s, int T, int max_keys) {
     return MESH_OK;
 }
 
-int stage_decode_dev(mesh_session *s, const mesh_batch *b, const void *d_in, int in_fmt, void *d_out, int out_fmt,
-                     size_t out_cap, size_t *out_len) {
+// rows of x picked by `row`, packed: grid (rows), 256 threads
+__global__ __launch_bounds__(256) void gather_rows_kernel(const float *x, const int32_t *row, int n, float *out) {
+    const float *src = x + (size_t)row[blockIdx.x] * n;
+    for (int i = threadIdx.x; i < n; i += 256) out[(size_t)blockIdx.x * n + i] = src[i];
+}
+
+// ids: the call's token ids in host memory, or null
+static int decode_core(mesh_session *s, const mesh_batch *b, const int32_t *ids, const void *d_in, int in_fmt, void *d_out, int out_fmt,
+                       size_t out_cap, size_t *out_len) {
     if (!s || !d_in || !d_out) return fail(MESH_ERR_INVALID, "mesh_stage_decode: null argument");
     mesh_stage *st = s->stage;
     const HParams &hp = st->hp;
@@ -1217,8 +1270,21 @@ int stage_decode_dev(mesh_session *s, const mesh_batch *b, const void *d_in, int
         return fail(MESH_ERR_INVALID, "mesh_stage_decode: logits output needs a stage that ends at the last layer of a file with output weights");
     if (!logits_out && out_fmt != MESH_F32 && out_fmt != MESH_F16 && out_fmt != MESH_Q8_0)
         return fail(MESH_ERR_INVALID, "mesh_stage_decode: output format %d unknown", out_fmt);
-    const size_t need = logits_out ? (size_t)T * (size_t)st->output.M * 4 : mesh_act_packed_size(out_fmt, T, hp.n_embd);
-    if (need == 0) return fail(MESH_ERR_INVALID, "mesh_stage_decode: n_embd %u is not a whole number of blocks of format %d", hp.n_embd, out_fmt);
+    // tokens whose logits are wanted (batch->want; none given: all)
+    int n_rows = T;
+    const bool picked = logits_out && b->want;
+    if (picked) {
+        n_rows = 0;
+        for (int i = 0; i < T; ++i) n_rows += b->want[i] != 0;
+    }
+    if (st->hybrid) {
+        if (!ids) return fail(MESH_ERR_INVALID, "mesh_stage_decode: the layers of architecture '%s' read the token ids (batch.token_id)", hp.arch.c_str());
+        for (int i = 0; i < T; ++i)
+            if (ids[i] < 0 || ids[i] >= (int)hp.n_vocab) return fail(MESH_ERR_INVALID, "mesh_stage_decode: token id %d outside the vocabulary of %u", ids[i], hp.n_vocab);
+        if ((rc = hybrid_check_batch(s, b)) != MESH_OK) return rc;
+    }
+    const size_t need = logits_out ? (size_t)n_rows * (size_t)st->output.M * 4 : mesh_act_packed_size(out_fmt, T, hp.n_embd);
+    if (need == 0 && !picked) return fail(MESH_ERR_INVALID, "mesh_stage_decode: n_embd %u is not a whole number of blocks of format %d", hp.n_embd, out_fmt);
     if (out_len) *out_len = need;
     if (out_cap < need) return fail(MESH_ERR_INVALID, "mesh_stage_decode: output needs %zu bytes, capacity is %zu", need, out_cap);
     MESH_HIP_TRY(hipSetDevice(st->device));
@@ -1232,12 +1298,39 @@ int stage_decode_dev(mesh_session *s, const mesh_batch *b, const void *d_in, int
     // positions / sequence ids -> device, through a ring of pinned slots so calls may be queued back to back
     const size_t B = (size_t)st->n_batch_max;
     if (s->meta_counter && s->meta_counter % META_SLOTS == 0) MESH_HIP_TRY(hipStreamSynchronize(stream));   // ring wraps: older copies are done
-    int32_t *slot = s->h_meta + (size_t)(s->meta_counter++ % META_SLOTS) * 3 * B;
+    int32_t *slot = s->h_meta + (size_t)(s->meta_counter++ % META_SLOTS) * 4 * B;
     for (int i = 0; i < T; ++i) { slot[i] = b->pos[i]; slot[B + i] = b->seq_id ? b->seq_id[i] : 0; }
-    // (one copy for both: the slot and the device buffer have the same layout, positions at 0 and sequence ids at B; a copy is
-    // a launch of its own on the stream, and the entries between T and B are never read)
-    MESH_HIP_TRY(hipMemcpyAsync(s->d_pos, slot, (B + T) * sizeof(int32_t), hipMemcpyHostToDevice, stream));
+    size_t meta_ints = B + (size_t)T;
+    if (st->hybrid) {
+        for (int i = 0; i < T; ++i) slot[2 * B + i] = ids[i];
+        meta_ints = 2 * B + (size_t)T;
+    }
+    if (picked && n_rows < T && n_rows > 0) {
+        for (int i = 0, r = 0; i < T; ++i)
+            if (b->want[i]) slot[3 * B + (size_t)r++] = i;
+        meta_ints = 3 * B + (size_t)n_rows;
+    }
+    // (one copy for all: the slot and the device buffer have the same layout, positions at 0, sequence ids at B, token ids and
+    // wanted rows behind them; a copy is a launch of its own on the stream, and the entries past each list are never read)
+    MESH_HIP_TRY(hipMemcpyAsync(s->d_pos, slot, meta_ints * sizeof(int32_t), hipMemcpyHostToDevice, stream));
 
+    if (st->hybrid) {
+        // (a call that fails from here on leaves its sequences in a state nothing is known of; they have to start anew)
+        hybrid_note_batch(s, b, false);
+        float *x = nullptr;
+        if (tokens_in) rc = hybrid_embed(s, T);
+        else { ProfScope ps(s, MESH_PROF_CODEC); rc = act_unpack_dev(in_fmt, d_in, s->x, (int64_t)T * hp.n_embd, stream); }
+        if (rc != MESH_OK || (rc = run_layers_graphed(s, T, max_keys)) != MESH_OK) return rc;
+        if (logits_out) {
+            if (n_rows > 0 && (rc = hybrid_logits(s, T, n_rows < T ? s->d_rows : nullptr, n_rows, static_cast<float *>(d_out))) != MESH_OK) return rc;
+        } else {
+            if ((rc = hybrid_finish(s, T, &x)) != MESH_OK) return rc;
+            ProfScope ps(s, MESH_PROF_CODEC);
+            if ((rc = act_pack_dev(out_fmt, x, d_out, (int64_t)T * hp.n_embd, stream)) != MESH_OK) return rc;
+        }
+        hybrid_note_batch(s, b, true);
+        return MESH_OK;
+    }
     if (tokens_in) {
         // embedding rows: one dequantize per token (ids are read on the host side by the caller's contract)
         return fail(MESH_ERR_UNSUPPORTED, "mesh_stage_decode_dev: token input is only available through the host-pointer entry point");
@@ -1246,16 +1339,28 @@ int stage_decode_dev(mesh_session *s, const mesh_batch *b, const void *d_in, int
     if (rc != MESH_OK) return rc;
     if ((rc = run_layers_graphed(s, T, max_keys)) != MESH_OK) return rc;
     if (logits_out) {
+        if (n_rows == 0) return MESH_OK;
+        const float *rows = s->x;
+        if (n_rows < T) {
+            ProfScope ps(s, MESH_PROF_PREP);
+            MESH_LAUNCH(gather_rows_kernel, dim3((unsigned)n_rows), dim3(256), 0, stream, s->x, s->d_rows, (int)hp.n_embd, s->logit_rows);
+            MESH_LAUNCH_CHECK();
+            rows = s->logit_rows;
+        }
         GemvArgs la;
         la.n_mat = 1;
         la.mat[0] = mat_of(st->output, static_cast<float *>(d_out), (int)st->output.M, nullptr);
-        la.x = s->x; la.ldx = (int)hp.n_embd; la.K = (int)hp.n_embd; la.T = T;
+        la.x = rows; la.ldx = (int)hp.n_embd; la.K = (int)hp.n_embd; la.T = n_rows;
         la.norm_w = static_cast<const float *>(st->output_norm.data); la.eps = hp.rms_eps;
         ProfScope ps(s, MESH_PROF_GEMV);
         return gemv(la, stream);
     }
     ProfScope ps(s, MESH_PROF_CODEC);
     return act_pack_dev(out_fmt, s->x, d_out, (int64_t)T * hp.n_embd, stream);
+}
+
+int stage_decode_dev(mesh_session *s, const mesh_batch *b, const void *d_in, int in_fmt, void *d_out, int out_fmt, size_t out_cap, size_t *out_len) {
+    return decode_core(s, b, b ? b->token_id : nullptr, d_in, in_fmt, d_out, out_fmt, out_cap, out_len);
 }
 
 int stage_decode(mesh_session *s, const mesh_batch *b, const void *in, int in_fmt, void *out, int out_fmt, size_t out_cap,
@@ -1266,14 +1371,22 @@ int stage_decode(mesh_session *s, const mesh_batch *b, const void *in, int in_fm
     if (!b || b->n_tokens <= 0) return fail(MESH_ERR_INVALID, "mesh_stage_decode: empty batch");
     if (b->n_tokens > st->n_batch_max) return fail(MESH_ERR_INVALID, "mesh_stage_decode: %d tokens exceed n_batch_max %d", b->n_tokens, st->n_batch_max);
     const int T = b->n_tokens;
-    if (out_fmt == MESH_LOGITS && T > LOGITS_TOKENS_MAX)
-        return fail(MESH_ERR_INVALID, "mesh_stage_decode: logits of %d tokens in one call (at most %d; mesh_stage_decode_dev has no such limit)", T, LOGITS_TOKENS_MAX);
+    int wanted = T;
+    if (b->want) {
+        wanted = 0;
+        for (int i = 0; i < T; ++i) wanted += b->want[i] != 0;
+    }
+    if (out_fmt == MESH_LOGITS && wanted > LOGITS_TOKENS_MAX)
+        return fail(MESH_ERR_INVALID, "mesh_stage_decode: logits of %d tokens in one call (at most %d; mesh_stage_decode_dev has no such limit)", wanted, LOGITS_TOKENS_MAX);
     MESH_HIP_TRY(hipSetDevice(st->device));
     hipStream_t stream = s->stream;
     uint8_t *d_in = static_cast<uint8_t *>(s->io_stage), *d_out = d_in + s->io_stage_bytes;
     int rc;
     int eff_in_fmt = in_fmt;
-    if (in_fmt == MESH_TOKENS) {
+    const int32_t *token_ids = b->token_id;
+    if (in_fmt == MESH_TOKENS && st->hybrid) {
+        token_ids = static_cast<const int32_t *>(in);          // (checked and embedded with the rest of the call)
+    } else if (in_fmt == MESH_TOKENS) {
         if (st->layer_begin != 0 || !st->tok_embd.present())
             return fail(MESH_ERR_INVALID, "mesh_stage_decode: token input needs a stage that starts at layer 0 of a file with token_embd");
         const int32_t *ids = static_cast<const int32_t *>(in);
@@ -1292,13 +1405,13 @@ int stage_decode(mesh_session *s, const mesh_batch *b, const void *in, int in_fm
         MESH_HIP_TRY(hipMemcpyAsync(d_in, s->h_io, in_bytes, hipMemcpyHostToDevice, stream));
     }
     size_t len = 0;
-    if ((rc = stage_decode_dev(s, b, d_in, eff_in_fmt, d_out, out_fmt, std::min(out_cap, s->io_out_bytes), &len)) != MESH_OK) {
+    if ((rc = decode_core(s, b, token_ids, d_in, eff_in_fmt, d_out, out_fmt, std::min(out_cap, s->io_out_bytes), &len)) != MESH_OK) {
         if (out_len) *out_len = len;
         return rc;
     }
     if (out_len) *out_len = len;
     uint8_t *h_out = static_cast<uint8_t *>(s->h_io) + s->io_stage_bytes;
-    MESH_HIP_TRY(hipMemcpyAsync(h_out, d_out, len, hipMemcpyDeviceToHost, stream));
+    if (len) MESH_HIP_TRY(hipMemcpyAsync(h_out, d_out, len, hipMemcpyDeviceToHost, stream));
     MESH_HIP_TRY(hipStreamSynchronize(stream));
     memcpy(out, h_out, len);
     return MESH_OK;
@@ -1310,6 +1423,7 @@ int session_attention(mesh_session *s, int layer, const float *d_q, const mesh_b
     const mesh_stage *st = s->stage;
     const HParams &hp = st->hp;
     const int il = layer - st->layer_begin;
+    if (st->hybrid) return fail(MESH_ERR_UNSUPPORTED, "mesh_session_attn_dev: architecture '%s' runs its attention inside the layer only", hp.arch.c_str());
     if (il < 0 || il >= (int)st->layers.size()) return fail(MESH_ERR_INVALID, "mesh_session_attn_dev: layer %d is not in this stage", layer);
     const int T = b->n_tokens;
     if (T < 1 || T > st->n_batch_max || !b->pos) return fail(MESH_ERR_INVALID, "mesh_session_attn_dev: bad batch");

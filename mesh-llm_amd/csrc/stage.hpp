@@ -7,6 +7,7 @@
 #include <vector>
 
 #include "gguf.hpp"
+#include "hybrid.hpp"
 #include "mesh_common.hpp"
 #include "moe.hpp"
 #include "tuning.hpp"
@@ -25,6 +26,8 @@ struct HParams {
 
 // Fills `hp` from the GGUF key/value table (keys of the form "<arch>.block_count", ...).
 int hparams_from_gguf(const GgufFile &g, HParams &hp);
+// The same summary of a model described layer by layer (sizes that differ between layers: the largest).
+void hparams_from_spec(const ModelSpec &s, HParams &hp);
 
 // A weight matrix resident in HBM.  K-quant matrices are stored in the tiled layout of gemv.hip
 // (same byte count as the GGUF tensor); everything else keeps the GGUF row-major layout.
@@ -63,6 +66,17 @@ int stage_decode(mesh_session *s, const mesh_batch *b, const void *in, int in_fm
 int profile_collect(mesh_session *s);
 int session_attention(mesh_session *s, int layer, const float *d_q, const mesh_batch *b, float *d_out, int matrix_cores);
 int stage_decode_dev(mesh_session *s, const mesh_batch *b, const void *d_in, int in_fmt, void *d_out, int out_fmt, size_t out_cap, size_t *out_len);
+// shared by the runners
+int stage_select_device(const mesh_stage_opts *opts, mesh_stage *st);
+int sess_alloc(mesh_session *s, void **p, size_t bytes);
+int attn_splits_for(const Tuning &tune, int T, int n_kv, int max_keys, bool quantised);
+// names the kernel class of the launches made while it lives (mesh_session_profile)
+struct ProfScope {
+    mesh_session *prev_s;
+    int prev_kind;
+    ProfScope(mesh_session *ses, int kind);
+    ~ProfScope();
+};
 }  // namespace mesh
 
 struct mesh_stage {
@@ -73,6 +87,7 @@ struct mesh_stage {
     int n_ctx = 0, n_seq_max = 1, n_batch_max = 0;
     mesh::Tuning tune;            // process default, then mesh_stage_opts.tuning; fixed from here on
     std::vector<mesh::LayerWeights> layers;
+    std::unique_ptr<mesh::HybridModel> hybrid;         // models described layer by layer; `layers` is empty then
     mesh::DevTensor tok_embd, output_norm, output;
     std::vector<void *> allocations;
     size_t gemm_layout_bytes = 0; // extra HBM held by the GEMM-layout copies
@@ -84,6 +99,7 @@ struct mesh_stage {
 struct mesh_session {
     mesh_stage *stage = nullptr;
     hipStream_t stream = nullptr;
+    std::unique_ptr<mesh::HybridSession> hybrid;       // set with the stage's
     mesh::Tuning tune;            // starts as the stage's copy; mesh_session_set_option changes the session-level switches
     bool graphs_failed = false;   // a failed capture turns graph replay off for the rest of the session
     // KV cache: per local layer, K and V as f16 [n_seq_max][n_head_kv][n_ctx][head_dim]
@@ -121,7 +137,8 @@ struct mesh_session {
     uint16_t *moe_x16 = nullptr, *moe_ffn16 = nullptr;          // k8-major f16: normalised inputs, SwiGLU outputs
     float *moe_out_slots = nullptr;                            // down-projection rows
     int xq_layer = -1;               // layer whose attention-norm activations the previous layer's combine step has left in xq (-1: none)
-    int32_t *d_pos = nullptr, *d_seq = nullptr, *d_tok = nullptr;
+    int32_t *d_pos = nullptr, *d_seq = nullptr, *d_tok = nullptr, *d_rows = nullptr;     // one buffer; d_rows: tokens whose logits are wanted
+    float *logit_rows = nullptr;    // hidden states of those tokens (K-quant models)
     int32_t *h_meta = nullptr;      // pinned staging for pos/seq/token ids (ring of slots)
     unsigned meta_counter = 0;
     void *io_stage = nullptr;       // device staging for packed in/out of the host-pointer entry point
