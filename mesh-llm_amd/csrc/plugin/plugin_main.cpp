@@ -47,10 +47,10 @@ constexpr uint64_t ENDPOINT_KIND_INFERENCE = 1, ENDPOINT_TRANSPORT_HTTP = 1, HEA
 
 struct Config {
     std::string plugin_id = "mesh-stage";
-    std::string gguf;
+    std::string gguf;                // a GGUF file or a model folder
     int layer_begin = 0, layer_end = -1;
     std::string device;
-    int n_ctx = 4096, n_seq_max = 1, n_batch_max = 512;
+    int n_ctx = 4096, n_seq_max = 1, n_batch_max = 512, precision = MESH_PRECISION_DEFAULT;
     bool open_stage = true;          // --no-stage: serve /v1/models from the file's header only (machines without a GPU)
     int http_port = 0;               // 0 = any free port
 };
@@ -225,7 +225,8 @@ static int format_id(const std::string &name, int fallback) {
 
 // POST /v1/stage/decode: headers X-Mesh-Tokens (count), X-Mesh-Pos0 (cache position of the first token; the rest follow),
 // X-Mesh-Seq (sequence id, default 0), X-Mesh-In-Format / X-Mesh-Out-Format (f32 | f16 | q8_0, in also tokens, out also
-// logits; default q8_0); body = the packed input rows.  200 with the packed output rows as application/octet-stream.
+// logits; default q8_0), X-Mesh-Token-Ids (1: the body starts with the tokens' int32 ids, for models whose layers read them),
+// X-Mesh-Want (the tokens whose logits are returned, as places "3,7"; default all); body = the packed input rows.  200 with the packed output rows as application/octet-stream.
 static void handle_decode(int fd, State &st, const std::string &head, const std::string &body) {
     if (!st.session) return http_error(fd, "503 Service Unavailable", "the stage is not open in this process", "stage_unavailable");
     const int T = atoi(header_value(head, "X-Mesh-Tokens").c_str());
@@ -235,21 +236,39 @@ static void handle_decode(int fd, State &st, const std::string &head, const std:
     if (T < 1 || T > st.cfg.n_batch_max || pos0 < 0 || pos0 > (1 << 30) || seq < 0 || in_fmt < 0 || out_fmt < 0 || in_fmt == MESH_LOGITS || out_fmt == MESH_TOKENS)
         return http_error(fd, "400 Bad Request", "X-Mesh-Tokens / X-Mesh-Pos0 / formats out of range", "invalid_request_error");
     // (refused before anything is allocated for it: a row of logits is the whole vocabulary)
-    if (out_fmt == MESH_LOGITS && T > MESH_LOGITS_TOKENS_MAX)
+    std::vector<uint8_t> wanted;
+    const std::string places = header_value(head, "X-Mesh-Want");
+    int rows = T;
+    if (!places.empty()) {
+        wanted.assign((size_t)T, 0);
+        const char *p = places.c_str();
+        while (*p) {
+            char *end = nullptr;
+            const long v = strtol(p, &end, 10);
+            if (end == p || v < 0 || v >= T || (*end && *end != ',')) return http_error(fd, "400 Bad Request", "X-Mesh-Want is not a list of places in the batch", "invalid_request_error");
+            wanted[(size_t)v] = 1;
+            p = *end ? end + 1 : end;
+        }
+        rows = (int)std::count(wanted.begin(), wanted.end(), 1);
+    }
+    if (out_fmt == MESH_LOGITS && rows > MESH_LOGITS_TOKENS_MAX)
         return http_error(fd, "400 Bad Request", "logits of at most " + std::to_string(MESH_LOGITS_TOKENS_MAX) + " tokens per request", "invalid_request_error");
-    const size_t want = in_fmt == MESH_TOKENS ? (size_t)T * 4 : mesh_act_packed_size(in_fmt, T, st.info.n_embd);
+    const size_t id_bytes = atoi(header_value(head, "X-Mesh-Token-Ids").c_str()) == 1 ? (size_t)T * 4 : 0;
+    const size_t want = id_bytes + (in_fmt == MESH_TOKENS ? (size_t)T * 4 : mesh_act_packed_size(in_fmt, T, st.info.n_embd));
     if (body.size() != want) return http_error(fd, "400 Bad Request", "body has " + std::to_string(body.size()) + " bytes, " + std::to_string(want) + " expected", "invalid_request_error");
     std::vector<int32_t> pos((size_t)T), seqs((size_t)T, seq);
     for (int i = 0; i < T; ++i) pos[(size_t)i] = pos0 + i;
-    mesh_batch b{T, pos.data(), seqs.data()};
-    const size_t cap = out_fmt == MESH_LOGITS ? (size_t)T * st.info.n_vocab * 4 : mesh_act_packed_size(out_fmt, T, st.info.n_embd);
+    std::vector<int32_t> ids(id_bytes / 4);
+    if (id_bytes) memcpy(ids.data(), body.data(), id_bytes);
+    mesh_batch b{T, pos.data(), seqs.data(), id_bytes ? ids.data() : nullptr, wanted.empty() ? nullptr : wanted.data()};
+    const size_t cap = out_fmt == MESH_LOGITS ? (size_t)rows * st.info.n_vocab * 4 : mesh_act_packed_size(out_fmt, T, st.info.n_embd);
     std::string out(cap, '\0');
     size_t len = 0;
     int rc;
     {
         std::lock_guard<std::mutex> lk(st.decode_mu);
         if (st.stopping || !st.session) return http_error(fd, "503 Service Unavailable", "the plugin is shutting down", "stage_unavailable");
-        rc = mesh_stage_decode(st.session, &b, body.data(), in_fmt, &out[0], out_fmt, cap, &len);
+        rc = mesh_stage_decode(st.session, &b, body.data() + id_bytes, in_fmt, &out[0], out_fmt, cap, &len);
     }
     if (rc != MESH_OK) return http_error(fd, rc == MESH_ERR_INVALID ? "400 Bad Request" : "500 Internal Server Error", mesh_last_error(), "stage_error");
     out.resize(len);
@@ -327,7 +346,8 @@ static bool http_listen(State &st) {
     return true;
 }
 
-static std::string model_id_of(const std::string &path) {
+static std::string model_id_of(std::string path) {
+    while (path.size() > 1 && path.back() == '/') path.pop_back();        // a model folder
     size_t a = path.find_last_of('/');
     std::string base = a == std::string::npos ? path : path.substr(a + 1);
     if (base.size() > 5 && base.compare(base.size() - 5, 5, ".gguf") == 0) base.resize(base.size() - 5);
@@ -344,7 +364,7 @@ int main(int argc, char **argv) {
         const std::string a = argv[i];
         auto val = [&]() -> const char * { return i + 1 < argc ? argv[++i] : ""; };
         if (a == "--plugin-id") c.plugin_id = val();
-        else if (a == "--gguf" || a == "-m") c.gguf = val();
+        else if (a == "--gguf" || a == "--model" || a == "-m") c.gguf = val();
         else if (a == "--layers") {                                 // BEGIN:END, END exclusive, empty = to the last layer
             const std::string v = val();
             const size_t colon = v.find(':');
@@ -355,21 +375,22 @@ int main(int argc, char **argv) {
         else if (a == "--parallel") c.n_seq_max = atoi(val());
         else if (a == "--batch") c.n_batch_max = atoi(val());
         else if (a == "--http-port") c.http_port = atoi(val());
+        else if (a == "--precision") c.precision = std::string(val()) == "f32" ? MESH_PRECISION_F32 : MESH_PRECISION_DEFAULT;
         else if (a == "--no-stage") c.open_stage = false;
         else {
-            fprintf(stderr, "usage: %s --gguf PATH [--layers B:E] [-d ROCm0] [-c CTX] [--parallel N] [--batch N] [--plugin-id NAME] [--http-port P] [--no-stage]\n", argv[0]);
+            fprintf(stderr, "usage: %s --gguf PATH | --model FOLDER [--precision f32] [--layers B:E] [-d ROCm0] [-c CTX] [--parallel N] [--batch N] [--plugin-id NAME] [--http-port P] [--no-stage]\n", argv[0]);
             return 2;
         }
     }
     if (const char *id = getenv("MESH_LLM_PLUGIN_NAME")) if (*id) c.plugin_id = id;      // the name the host configured (src/plugin/runtime.rs:188) and checks the reply against
     if (c.gguf.empty()) { fprintf(stderr, "[mesh-stage-plugin] --gguf is required\n"); return 2; }
-    if (mesh_gguf_probe(c.gguf.c_str(), &st.info) != MESH_OK) { fprintf(stderr, "[mesh-stage-plugin] %s\n", mesh_last_error()); return 1; }
+    if (mesh_model_probe(c.gguf.c_str(), &st.info) != MESH_OK) { fprintf(stderr, "[mesh-stage-plugin] %s\n", mesh_last_error()); return 1; }
     st.model_id = model_id_of(c.gguf);
     signal(SIGPIPE, SIG_IGN);
     if (c.open_stage) {
         mesh_stage_opts o{};
         o.device = c.device.empty() ? nullptr : c.device.c_str();
-        o.n_ctx = c.n_ctx; o.n_seq_max = c.n_seq_max; o.n_batch_max = c.n_batch_max;
+        o.n_ctx = c.n_ctx; o.n_seq_max = c.n_seq_max; o.n_batch_max = c.n_batch_max; o.precision = c.precision;
         if (mesh_stage_open(c.gguf.c_str(), c.layer_begin, c.layer_end, &o, &st.stage) != MESH_OK ||
             mesh_stage_session_new(st.stage, &st.session) != MESH_OK) {
             fprintf(stderr, "[mesh-stage-plugin] cannot open the stage: %s\n", mesh_last_error());
