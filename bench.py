@@ -1,7 +1,7 @@
 #!/usr/bin/env python3
 """Benchmark of the pipeline-stage hot path on one MI355X.  Prints ONE JSON line.
 
-  python bench.py [--gpus 1] [--steps K] [--warmup W] [--workload stage|codec] [--batches 1,4,16]
+  python bench.py [--gpus 1] [--steps K] [--warmup W] [--workload stage|codec|c4|c5|nadosun] [--batches 1,4,16]
 
 Workloads
   stage   (default) Llama-3-8B-shaped stage, layers 0-15 of 32 (hidden 4096, 32/8 heads, head_dim 128, FFN 14336,
@@ -14,6 +14,9 @@ Workloads
           tier), decode batch 1/8/32 and a 4096-token prefill.  value = batch-1 tokens/s.
   c5      Qwen3-30B-A3B-shaped expert shard: all 48 layers, 64 of the 128 experts per layer (top-8 routing, expert FFN
           768, per-head q/k norms), decode batch 16 at a 4096-token context.  value = tokens/s at batch 16.
+  nadosun Nadosun layers of two sizes (hidden 2048 and 4096: half windowed attention with a feed-forward, half minGRU),
+          bf16 random weights, decode of one token behind 2048 and prefill of 2048; beside it a llama stage of the same
+          width, heads and feed-forward (Q4_K_M), the closest K-quant model.  value = decode tokens/s at hidden 4096.
 
 Timing uses HIP events recorded on the stream the kernels run on (the session's own stream for the stage).
 The cpu_baseline leg times the CPU oracle (a restatement of ggml's reference routines, NOT llama.cpp) on the
@@ -559,12 +562,175 @@ def bench_shape(args):
     return out
 
 
+# ------------------------------------------------------------------------------------------------ Nadosun
+NADOSUN_SIZES = {
+    # width, query / KV heads of 128, feed-forward, window, side input, layers (attention, recurrence, recurrence, attention, ...)
+    "2048": dict(E=2048, H=16, G=4, FF=8192, window=512, side=128, layers=16),
+    "4096": dict(E=4096, H=32, G=8, FF=14336, window=1024, side=256, layers=8),
+}
+NADOSUN_T, NADOSUN_CTX, NADOSUN_VOCAB = 2048, 8192, 4096
+BF16_PEAK_TFLOPS = 2500.0
+
+
+def nadosun_config(sp):
+    att = {"type": "attention", "mlp": {"kind": "dense", "ff": sp["FF"]},
+           "mixer": {"heads": sp["H"], "kv_heads": sp["G"], "dim": 128, "vdim": 128, "scale": 128 ** -0.5, "mask": {"size": sp["window"]}}}
+    gru = {"type": "mingru", "mlp": None, "mixer": {"width": sp["E"]}}
+    return {"architecture": "Nadosun", "vocab": NADOSUN_VOCAB, "width": sp["E"], "embedding": {"scale": 1.0}, "norm": {"eps": 1e-5},
+            "token_side": {"dim": sp["side"]}, "layers": [att if i % 4 in (0, 3) else gru for i in range(sp["layers"])]}
+
+
+def write_nadosun(folder, cfg):
+    """Random bf16 weights of sigma 1 / sqrt(row length), cut from one random block; norms and layer scales near 1."""
+    os.makedirs(folder, exist_ok=True)
+    E, S, n = cfg["width"], cfg["token_side"]["dim"], len(cfg["layers"])
+    shapes = {"embed": (cfg["vocab"], E), "side.embed": (cfg["vocab"], n * S), "final.norm": (), "head": (cfg["vocab"], E)}
+    for i, l in enumerate(cfg["layers"]):
+        p, mx = "l%d." % i, l["mixer"]
+        if l["type"] == "attention":
+            hd, gd = mx["heads"] * mx["dim"], mx["kv_heads"] * mx["dim"]
+            shapes.update({p + "mix.q": (hd, E), p + "mix.k": (gd, E), p + "mix.o": (E, hd), p + "mix.q.norm": (hd,), p + "mix.k.norm": (gd,)})
+        else:
+            W = mx["width"]
+            shapes.update({p + "mix." + t: (W, E) for t in "zxg"})
+            shapes.update({p + "mix.z.b": (W,), p + "mix.x.b": (W,), p + "mix.o": (E, W)})
+        shapes.update({p + "norm1": (), p + "ls1": (E,), p + "side.gate": (S, E), p + "side.proj": (E, S), p + "side.norm": (E,)})
+        if l["mlp"]:
+            shapes.update({p + "mlp.up": (l["mlp"]["ff"], E), p + "mlp.down": (E, l["mlp"]["ff"]), p + "mlp.act": (4,), p + "norm2": (), p + "ls2": (E,)})
+    rng = np.random.Generator(np.random.PCG64(42))
+    base = rng.standard_normal(1 << 24).astype(np.float32)
+
+    def bits(a):
+        u = np.ascontiguousarray(a, np.float32).view(np.uint32)
+        return ((u + 0x7FFF + ((u >> 16) & 1)) >> 16).astype("<u2")
+
+    scaled = {}          # row length -> the block at that scale, as bf16
+
+    head, at = {}, 0
+    for name, sh in shapes.items():
+        nb = int(np.prod(sh, dtype=np.int64)) * 2
+        head[name] = {"dtype": "BF16", "shape": list(sh), "data_offsets": [at, at + nb]}
+        at += nb
+    h = json.dumps(head).encode()
+    with open(os.path.join(folder, "config.json"), "w") as f:
+        json.dump(cfg, f)
+    with open(os.path.join(folder, "model.safetensors"), "wb") as f:
+        f.write(len(h).to_bytes(8, "little") + h)
+        for k, (name, sh) in enumerate(shapes.items()):
+            count = int(np.prod(sh, dtype=np.int64))
+            if len(sh) < 2:
+                f.write(bits(np.full(count, 0.8)).tobytes())
+                continue
+            if sh[1] not in scaled:
+                scaled[sh[1]] = bits(base if "embed" in name else base / np.sqrt(sh[1]))
+            block, start = scaled[sh[1]], (k * 7919 * 64) % (1 << 23)
+            while count:
+                take = min(count, block.size - start)
+                f.write(block[start:start + take].tobytes())
+                count -= take
+                start = 0
+
+
+def nadosun_work(sp):
+    """(bf16 weight bytes of the layers, multiply-adds per token in their products, attention layers, recurrent layers)."""
+    E, A = sp["E"], sum(i % 4 in (0, 3) for i in range(sp["layers"]))
+    R = sp["layers"] - A
+    macs = A * (E * (sp["H"] + sp["G"]) * 128 + E * sp["H"] * 128 + 2 * E * sp["FF"]) + R * 4 * E * E + sp["layers"] * 2 * E * sp["side"]
+    return 2 * macs, macs, A, R
+
+
+def kernel_ms(ses, fn, n):
+    ses.profile(True)
+    for _ in range(n):
+        fn(0)
+    p = ses.profile_read()
+    ses.profile(False)
+    return {k: round(v["ms"] / n, 4) for k, v in p.items()}, {k: v["launches"] // n for k, v in p.items()}
+
+
+def bench_nadosun(args):
+    import shutil
+    import torch
+    import __graft_entry__ as graft
+    import models
+    m = graft.load_package()
+    m.lib()
+    sizes = {}
+    for name, sp in NADOSUN_SIZES.items():
+        T, L = NADOSUN_T, sp["layers"]
+        folder = os.path.join(models.tmp_dir(), "mesh_bench_nadosun")
+        write_nadosun(folder, nadosun_config(sp))
+        st = m.Stage(folder, 0, L, n_ctx=NADOSUN_CTX, n_batch_max=T)
+        shutil.rmtree(folder)
+        path = os.path.join(models.tmp_dir(), "mesh_bench_nadosun_llama.gguf")
+        lc = dict(models.CONFIGS["llama3-8b"], n_layer=L, n_embd=sp["E"], n_head=sp["H"], n_head_kv=sp["G"], n_ff=sp["FF"])
+        models.write_model(path, lc, range(L), seed=42, fast=True)
+        ls = m.Stage(path, 0, L, n_ctx=T + 512, n_batch_max=T)
+        os.unlink(path)
+        print("[bench] nadosun %s: stages open" % name, file=sys.stderr, flush=True)
+        E = sp["E"]
+        wbytes, macs, A, R = nadosun_work(sp)
+        rng = np.random.Generator(np.random.PCG64(1))
+        xs = torch.from_numpy(rng.standard_normal((T, E)).astype(np.float32)).cuda()
+        out = torch.empty(T * E, dtype=torch.float32, device="cuda")
+        ids = rng.integers(0, NADOSUN_VOCAB, T).astype(np.int32)
+        ses, lses = st.session(), ls.session()
+        at = [0]
+
+        def prefill(i):
+            ses.decode_dev(xs.data_ptr(), np.arange(T), out.data_ptr(), T * E * 4, token_ids=ids)
+            at[0] = T
+
+        def step(i):
+            ses.decode_dev(xs.data_ptr(), [at[0]], out.data_ptr(), T * E * 4, token_ids=ids[:1])
+            at[0] += 1
+
+        def lprefill(i):
+            lses.decode_dev(xs.data_ptr(), np.arange(T), out.data_ptr(), T * E * 4)
+
+        def lstep(i):
+            lses.decode_dev(xs.data_ptr(), [sp["window"] - 1], out.data_ptr(), T * E * 4)
+
+        s1, s2 = torch.cuda.ExternalStream(ses.stream), torch.cuda.ExternalStream(lses.stream)
+        for _ in range(args.burn_in):           # untimed; see bench_stage
+            lstep(0)
+        torch.cuda.synchronize()
+        res = {"nadosun": {"prefill_ms": [], "decode_ms": []}, "llama_q4_k_m": {"prefill_ms": [], "decode_ms": []}}
+        steps = min(args.steps, 500)
+        for _ in range(3):                      # both sides in turn
+            res["nadosun"]["prefill_ms"].append(time_on_stream(torch, s1, prefill, 3, 1)[0])
+            res["llama_q4_k_m"]["prefill_ms"].append(time_on_stream(torch, s2, lprefill, 3, 1)[0])
+            res["nadosun"]["decode_ms"].append(time_on_stream(torch, s1, step, steps, args.warmup)[0])
+            res["llama_q4_k_m"]["decode_ms"].append(time_on_stream(torch, s2, lstep, steps, args.warmup)[0])
+        for side, ses_, pf, sf, by, mc in (("nadosun", ses, prefill, step, wbytes, macs),
+                                           ("llama_q4_k_m", lses, lprefill, lstep, ls.weight_bytes, L * (2 * E * sp["H"] * 128 + 2 * E * sp["G"] * 128 + 3 * E * sp["FF"]))):
+            r = res[side]
+            for k in ("prefill_ms", "decode_ms"):
+                r[k] = round(min(r[k]), 4)
+            pms, _ = kernel_ms(ses_, pf, 1)
+            dms, dl = kernel_ms(ses_, sf, 5)
+            r.update({"prefill_tok_s": round(T * 1e3 / r["prefill_ms"], 1), "decode_tok_s": round(1e3 / r["decode_ms"], 1), "weight_GB": round(by / 1e9, 3),
+                      "prefill_kernel_ms": pms, "decode_kernel_ms": dms, "decode_launches": dl,
+                      "products_prefill_TFLOPs": round(2.0 * mc * T / pms["gemv"] / 1e9, 1),
+                      "products_prefill_frac_peak": round(2.0 * mc * T / pms["gemv"] / 1e9 / BF16_PEAK_TFLOPS, 4),
+                      "products_decode_GBps": round(by / dms["gemv"] / 1e6, 1), "products_decode_frac_hbm": round(by / dms["gemv"] / 1e6 / HBM_PEAK_GBS, 4),
+                      "step_frac_hbm": round(by / r["decode_ms"] / 1e6 / HBM_PEAK_GBS, 4)})
+        sizes[name] = dict(shape=dict(sp, attention_layers=A, recurrent_layers=R, tokens=T), **res)
+        ses.close(), lses.close(), st.close(), ls.close()
+    head = sizes["4096"]["nadosun"]
+    return {"metric": "Nadosun decode tok/s, hidden 4096, 8 layers", "value": head["decode_tok_s"], "unit": "tok/s", "n_gpus": 1, "steps": args.steps, "warmup": args.warmup,
+            "ms_per_step": head["decode_ms"], "higher_is_better": True, "scaling": "weak", "vs_baseline": None, "dtype": "bf16", "data": "synthetic",
+            "config": {"workload": "Nadosun layers of two sizes, random bf16 weights, single-token decode behind %d tokens and %d-token prefill, beside llama stages of the "
+                                   "same width, heads and feed-forward in Q4_K_M" % (NADOSUN_T, NADOSUN_T)},
+            "sizes": sizes}
+
+
 def main():
     ap = argparse.ArgumentParser()
     ap.add_argument("--gpus", type=int, default=1)
     ap.add_argument("--steps", type=int, default=100)
     ap.add_argument("--warmup", type=int, default=10)
-    ap.add_argument("--workload", default="stage", choices=["stage", "codec", "c4", "c5"])
+    ap.add_argument("--workload", default="stage", choices=["stage", "codec", "c4", "c5", "nadosun"])
     ap.add_argument("--batches", default=None, help="decode batch sizes; the first is the headline value (default 1,4,16 for the stage workload, the shape's own list for c4 / c5)")
     ap.add_argument("--kv", default="f16", choices=["f16", "q8_0/q4_0", "q4_0/q4_0"],
                     help="KV cache row types K/V (default f16: the tier the reference picks for an 8B Q4_K_M model)")
@@ -577,7 +743,8 @@ def main():
               file=sys.stderr)
         sys.exit(2)
     args.kv_given = any(a == "--kv" or a.startswith("--kv=") for a in sys.argv[1:])
-    out = bench_stage(args) if args.workload == "stage" else bench_codec(args) if args.workload == "codec" else bench_shape(args)
+    out = bench_stage(args) if args.workload == "stage" else bench_codec(args) if args.workload == "codec" else \
+        bench_nadosun(args) if args.workload == "nadosun" else bench_shape(args)
     print(json.dumps(out))
 
 

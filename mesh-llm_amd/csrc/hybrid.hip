@@ -196,7 +196,7 @@ int hybrid_open(const char *folder, int layer_begin, int layer_end, const mesh_s
         HybridLayer &L = hm.layers[(size_t)(i - layer_begin)];
         L.spec = s.layers[(size_t)i];
         if ((rc = ld.layer(L, s, i)) != MESH_OK) return rc;
-        hm.in_max = std::max({hm.in_max, L.in.M, L.up.M, L.side_gate.M});
+        hm.in_max = std::max({hm.in_max, L.in.M, L.up.M, L.side_gate.M * LINEAR_SLICES_MAX});
         hm.act_max = std::max({hm.act_max, L.out.Kp, L.down.Kp, L.side_proj.Kp});
         if (L.spec.mixer.kind == MIXER_ATTENTION) hm.q_max = std::max(hm.q_max, L.spec.mixer.heads * L.head_pad);
         else { hm.has_state = true; hm.state_max = std::max(hm.state_max, L.spec.mixer.width); }
@@ -471,10 +471,15 @@ int hybrid_run_layers(mesh_session *s, int T, int max_keys) {
             }
             if ((rc = product(L.down, h.acta, h.y, E)) != MESH_OK || (rc = add(L.gain2)) != MESH_OK) return rc;
         }
-        if ((rc = product(L.side_gate, h.xa, h.big, hm.spec.side_dim)) != MESH_OK) return rc;
+        int slices;
+        const size_t slice = (size_t)T * hm.spec.side_dim;
+        {
+            ProfScope ps(s, MESH_PROF_GEMV);
+            if ((slices = linear_sliced(L.side_gate, h.xa, act, T, h.big, slice, s->tune.linear_tile_min_tokens, stream)) < 0) return slices;
+        }
         {
             ProfScope ps(s, MESH_PROF_PREP);
-            if ((rc = side_gate_rows(h.big, hm.side, s->d_tok, (int)hm.spec.layers.size() * hm.spec.side_dim, (st->layer_begin + (int)il) * hm.spec.side_dim, T,
+            if ((rc = side_gate_rows(h.big, slices, slice, hm.side, s->d_tok, (int)hm.spec.layers.size() * hm.spec.side_dim, (st->layer_begin + (int)il) * hm.spec.side_dim, T,
                                      hm.spec.side_dim, h.acta, act, L.side_proj.Kp, stream)) != MESH_OK)
                 return rc;
         }

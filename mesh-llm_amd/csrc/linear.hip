@@ -114,7 +114,10 @@ __device__ __forceinline__ void tile_copy16(const uint16_t *src, uint16_t *lds_b
 // 1-D grid of (row blocks x token blocks); the workgroups a die is dealt (every eighth) take a contiguous run of tiles with
 // the token block running fastest, so that the weight rows of a run stay in that die's cache
 __global__ __launch_bounds__(TILE_THREADS) void linear_tile_kernel(const uint16_t *w, const uint16_t *x, float *y, int K, int M, int T, int ldy,
-                                                                   int n_tblocks, int n_tiles) {
+                                                                   int n_tblocks, int n_tiles, int k_slice, size_t y_slice) {
+    // blockIdx.y: slice of K and the partial result it writes
+    const int k_begin = blockIdx.y * k_slice, k_end = k_begin + k_slice < K ? k_begin + k_slice : K;
+    y += blockIdx.y * y_slice;
     __shared__ __align__(16) uint16_t sW0[TILE_M * TILE_K], sW1[TILE_M * TILE_K], sX0[TILE_T * TILE_K], sX1[TILE_T * TILE_K];
     const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
     int tile = blockIdx.x;
@@ -173,14 +176,14 @@ __global__ __launch_bounds__(TILE_THREADS) void linear_tile_kernel(const uint16_
         asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
         __syncthreads();
     };
-    stage(sW0, sX0, 0);
-    for (int k = 0; k < K; k += 2 * TILE_K) {
+    stage(sW0, sX0, k_begin);
+    for (int k = k_begin; k < k_end; k += 2 * TILE_K) {
         arrive();
-        if (k + TILE_K < K) stage(sW1, sX1, k + TILE_K);
+        if (k + TILE_K < k_end) stage(sW1, sX1, k + TILE_K);
         multiply(sW0, sX0);
-        if (k + TILE_K >= K) break;
+        if (k + TILE_K >= k_end) break;
         arrive();
-        if (k + 2 * TILE_K < K) stage(sW0, sX0, k + 2 * TILE_K);
+        if (k + 2 * TILE_K < k_end) stage(sW0, sX0, k + 2 * TILE_K);
         multiply(sW1, sX1);
     }
 #pragma unroll
@@ -208,17 +211,40 @@ static int launch_rows(const LinearWeight &W, const void *x, int T, float *y, in
     return MESH_OK;
 }
 
-int linear(const LinearWeight &W, const void *x, ActType act, int T, float *y, int ldy, int big_from, hipStream_t stream) {
-    if (T <= 0) return MESH_OK;
-    if (!W.w || !x || !y || W.M < 1 || W.Kp % LINEAR_K_PAD || W.Mp % LINEAR_ROW_PAD || W.Mp < W.M || W.Kp < W.K || ldy < W.M || (T + 63) / 64 > 65535)
-        return fail(MESH_ERR_INVALID, "linear: bad operands (%d x %d, %d tokens)", W.M, W.K, T);
-    if (act == ACT_F32) return launch_rows<ACT_F32>(W, x, T, y, ldy, stream);
-    if (T < big_from || W.M < TILE_M) return launch_rows<ACT_BF16>(W, x, T, y, ldy, stream);
+static int launch_tile(const LinearWeight &W, const void *x, int T, float *y, int ldy, int slices, size_t stride, hipStream_t stream) {
     const int mblocks = (W.M + TILE_M - 1) / TILE_M, tblocks = (T + TILE_T - 1) / TILE_T;
-    MESH_LAUNCH(linear_tile_kernel, dim3((unsigned)(mblocks * tblocks)), dim3(TILE_THREADS), 0, stream, W.w, static_cast<const uint16_t *>(x), y, W.Kp, W.M, T, ldy,
-                tblocks, mblocks * tblocks);
+    const int steps = W.Kp / TILE_K, k_slice = (steps + slices - 1) / slices * TILE_K;
+    MESH_LAUNCH(linear_tile_kernel, dim3((unsigned)(mblocks * tblocks), (unsigned)slices), dim3(TILE_THREADS), 0, stream, W.w, static_cast<const uint16_t *>(x), y, W.Kp, W.M,
+                T, ldy, tblocks, mblocks * tblocks, k_slice, stride);
     MESH_LAUNCH_CHECK();
     return MESH_OK;
+}
+
+static bool linear_ok(const LinearWeight &W, const void *x, int T, const float *y, int ldy) {
+    return W.w && x && y && W.M >= 1 && W.Kp % LINEAR_K_PAD == 0 && W.Mp % LINEAR_ROW_PAD == 0 && W.Mp >= W.M && W.Kp >= W.K && ldy >= W.M && (T + 63) / 64 <= 65535;
+}
+
+int linear_sliced(const LinearWeight &W, const void *x, ActType act, int T, float *y, size_t stride, int big_from, hipStream_t stream) {
+    const int tiles = (W.M + TILE_M - 1) / TILE_M * ((T + TILE_T - 1) / TILE_T), steps = W.Kp / TILE_K;
+    int slices = 128 / (tiles > 0 ? tiles : 1);
+    if (slices > LINEAR_SLICES_MAX) slices = LINEAR_SLICES_MAX;
+    if (slices > steps / 4) slices = steps / 4;                  // (a slice of at least four steps)
+    if (slices > 1) slices = (steps + (steps + slices - 1) / slices - 1) / ((steps + slices - 1) / slices);        // every slice has some
+    if (act == ACT_F32 || T < big_from || slices <= 1 || stride < (size_t)T * W.M) {
+        const int rc = linear(W, x, act, T, y, W.M, big_from, stream);
+        return rc == MESH_OK ? 1 : rc;
+    }
+    if (!linear_ok(W, x, T, y, W.M)) return fail(MESH_ERR_INVALID, "linear_sliced: bad operands (%d x %d, %d tokens)", W.M, W.K, T);
+    const int rc = launch_tile(W, x, T, y, W.M, slices, stride, stream);
+    return rc == MESH_OK ? slices : rc;
+}
+
+int linear(const LinearWeight &W, const void *x, ActType act, int T, float *y, int ldy, int big_from, hipStream_t stream) {
+    if (T <= 0) return MESH_OK;
+    if (!linear_ok(W, x, T, y, ldy)) return fail(MESH_ERR_INVALID, "linear: bad operands (%d x %d, %d tokens)", W.M, W.K, T);
+    if (act == ACT_F32) return launch_rows<ACT_F32>(W, x, T, y, ldy, stream);
+    if (T < big_from || W.M < TILE_M) return launch_rows<ACT_BF16>(W, x, T, y, ldy, stream);
+    return launch_tile(W, x, T, y, ldy, 1, 0, stream);
 }
 
 }  // namespace mesh

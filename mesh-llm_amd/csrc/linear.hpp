@@ -25,6 +25,12 @@ inline int linear_k_padded(int K) { return (K + LINEAR_K_PAD - 1) / LINEAR_K_PAD
 // aligned; y: f32 rows of ldy.  big_from: bf16 calls of at least this many tokens take the large-tile kernel.
 int linear(const LinearWeight &W, const void *x, ActType act, int T, float *y, int ldy, int big_from, hipStream_t stream);
 
+// The same for a matrix of few rows (hundreds), which leaves the large tile with few workgroups: K is cut into slices, each of
+// which writes its own partial y, `stride` floats apart; the reader adds them in order.  Returns the slice count (1: y is
+// the product) or a negative status.  y holds at least LINEAR_SLICES_MAX * T * W.M floats.
+constexpr int LINEAR_SLICES_MAX = 8;
+int linear_sliced(const LinearWeight &W, const void *x, ActType act, int T, float *y, size_t stride, int big_from, hipStream_t stream);
+
 // ---- one token ------------------------------------------------------------------------------------------------
 // A mat-vec whose workgroups derive the input vector themselves from what the launch before them left, and whose epilogue
 // does the element-wise work that follows.  Activations are f32 throughout, so the results serve both ActTypes.

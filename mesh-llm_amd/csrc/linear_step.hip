@@ -5,6 +5,7 @@
 // the launch before left (residual update with its output norm, polynomial activation: linear.hpp), which saves a launch
 // between two products; the first weight loads go out before that work and travel behind it.  Sums of squares a later norm
 // needs are left per workgroup and added in workgroup order by the consumer, so the result does not depend on timing.
+#include "act_math.hpp"
 #include "linear.hpp"
 
 #include <algorithm>
@@ -29,6 +30,27 @@ __device__ __forceinline__ float step_block_sum(float v, float *scratch, int lan
 #pragma unroll
     for (int w = 0; w < STEP_WAVES; ++w) s += scratch[w];
     return s;
+}
+
+// four elements of a vector of K, zeros behind its end
+__device__ __forceinline__ float4 ln_load4(const float *p, int k, int K) {
+    if (k + 4 <= K) return *reinterpret_cast<const float4 *>(p + k);
+    return make_float4(k < K ? p[k] : 0.f, k + 1 < K ? p[k + 1] : 0.f, k + 2 < K ? p[k + 2] : 0.f, 0.f);
+}
+// xs[k .. k + 3] = map(k, load(k)) over [0, Kp), four loads of a thread in flight
+template <typename Load, typename Map>
+__device__ __forceinline__ void step_vec(int K, int Kp, int tid, Load load, Map map, float *xs) {
+    constexpr int N = 4;
+    for (int k0 = tid * 4; k0 < Kp; k0 += N * STEP_THREADS * 4) {
+        float4 v[N];
+#pragma unroll
+        for (int i = 0; i < N; ++i) v[i] = load(k0 + i * STEP_THREADS * 4);
+#pragma unroll
+        for (int i = 0; i < N; ++i) {
+            const int k = k0 + i * STEP_THREADS * 4;
+            if (k < Kp) *reinterpret_cast<float4 *>(xs + k) = map(k, v[i]);
+        }
+    }
 }
 
 template <int R, int U, StepIn IN, StepOut OUT>
@@ -59,7 +81,7 @@ __global__ __launch_bounds__(STEP_THREADS) void linear_step_kernel(const uint16_
 
     // ---- the input vector
     if constexpr (IN == STEP_IN_VEC) {
-        for (int k = tid; k < Kp; k += STEP_THREADS) xs[k] = k < K ? a.in[k] : 0.f;
+        step_vec(K, Kp, tid, [&](int k) { return ln_load4(a.in, k, K); }, [&](int k, const float4 &v) { return v; }, xs);
     } else if constexpr (IN == STEP_IN_POLY) {
         float p2 = 0.f, p4 = 0.f, p6 = 0.f;
         for (int i = tid; i < a.n_part; i += STEP_THREADS) { p2 += a.part[i]; p4 += a.part[a.n_part + i]; p6 += a.part[2 * a.n_part + i]; }
@@ -68,25 +90,40 @@ __global__ __launch_bounds__(STEP_THREADS) void linear_step_kernel(const uint16_
         p6 = step_block_sum(p6, &scratch[0][0], lane, wave);
         const float c1 = a.coef[0] / sqrtf(p2 / (float)K + a.eps), c2 = a.coef[1] / sqrtf(p4 / (float)K + a.eps), c3 = a.coef[2] / sqrtf(p6 / (float)K + a.eps);
         const float c0 = a.coef[3];
-        for (int k = tid; k < Kp; k += STEP_THREADS) {
-            const float u = k < K ? a.in[k] : 0.f;
-            xs[k] = k < K ? ((c3 * u + c2) * u + c1) * u + c0 : 0.f;
-        }
+        auto poly = [&](float u) { return ((c3 * u + c2) * u + c1) * u + c0; };
+        step_vec(K, Kp, tid, [&](int k) { return ln_load4(a.in, k, K); },
+                 [&](int k, const float4 &u) {
+                     return make_float4(k < K ? poly(u.x) : 0.f, k + 1 < K ? poly(u.y) : 0.f, k + 2 < K ? poly(u.z) : 0.f, k + 3 < K ? poly(u.w) : 0.f);
+                 }, xs);
     } else {
         float ss = 0.f;
         for (int i = tid; i < a.n_part; i += STEP_THREADS) ss += a.part[i];
+        // the vectors' loads go out before the partial sums are added up
+        constexpr int AHEAD = 2;
+        float4 x4[AHEAD], y4[AHEAD], g4[AHEAD];
+#pragma unroll
+        for (int i = 0; i < AHEAD; ++i) {
+            const int k = (tid + i * STEP_THREADS) * 4;
+            x4[i] = ln_load4(a.in, k, K); y4[i] = ln_load4(a.y, k, K); g4[i] = ln_load4(a.gain, k, K);
+        }
         ss = step_block_sum(ss, &scratch[0][0], lane, wave);
         const float rinv = 1.0f / sqrtf(ss / (float)K + a.eps);
         float sx = 0.f;
-        for (int k = tid; k < Kp; k += STEP_THREADS) {
-            float v = 0.f;
-            if (k < K) {
-                v = a.in[k] + a.y[k] * rinv * a.gain[k];
-                if (blockIdx.x == 0) a.x_out[k] = v;
+        auto update = [&](int k, const float4 &x, const float4 &y, const float4 &g) {
+            if (k >= Kp) return;
+            const float4 v = make_float4(x.x + y.x * rinv * g.x, x.y + y.y * rinv * g.y, x.z + y.z * rinv * g.z, x.w + y.w * rinv * g.w);
+            *reinterpret_cast<float4 *>(xs + k) = v;
+            sx += v.x * v.x + v.y * v.y + v.z * v.z + v.w * v.w;
+            if (blockIdx.x == 0) {
+                const float o[4] = {v.x, v.y, v.z, v.w};
+#pragma unroll
+                for (int j = 0; j < 4; ++j)
+                    if (k + j < K) a.x_out[k + j] = o[j];
             }
-            xs[k] = v;
-            sx = fmaf(v, v, sx);
-        }
+        };
+#pragma unroll
+        for (int i = 0; i < AHEAD; ++i) update((tid + i * STEP_THREADS) * 4, x4[i], y4[i], g4[i]);
+        for (int k = (tid + AHEAD * STEP_THREADS) * 4; k < Kp; k += STEP_THREADS * 4) update(k, ln_load4(a.in, k, K), ln_load4(a.y, k, K), ln_load4(a.gain, k, K));
         if constexpr (IN == STEP_IN_RESIDUAL_NORM) {
             sx = step_block_sum(sx, &scratch[0][0], lane, wave);
             const float z = a.norm_gain[0] / sqrtf(sx / (float)K + a.eps);
@@ -105,13 +142,11 @@ __global__ __launch_bounds__(STEP_THREADS) void linear_step_kernel(const uint16_
         for (int r = 0; r < R; ++r) { v[r] = step_wave_sum(acc[r]); acc[r] = 0.f; }
         if constexpr (OUT == STEP_OUT_MIN_GRU) {
             if (lane == 0) {
-                const float pz = v[0] + a.bias_z[gr], u = v[1] + a.bias_x[gr];
-                const float z = 1.0f / (1.0f + expf(-pz)), keep = 1.0f / (1.0f + expf(pz));
-                const float cand = u >= 0.f ? u + 0.5f : 1.0f / (1.0f + expf(-u));
+                const MinGruGate g = min_gru_gate(v[0] + a.bias_z[gr], v[1] + a.bias_x[gr]);
                 float *st = a.state + (size_t)a.seq[0] * p_width + gr;
-                const float s = (a.pos[0] == 0 ? 0.f : keep * *st) + z * cand;
+                const float s = a.pos[0] == 0 ? g.in : fmaf(g.keep, *st, g.in);
                 *st = s;
-                a.out[gr] = s * (v[2] / (1.0f + expf(-v[2])));
+                a.out[gr] = s * act_silu(v[2]);
             }
         } else {
 #pragma unroll
@@ -121,7 +156,7 @@ __global__ __launch_bounds__(STEP_THREADS) void linear_step_kernel(const uint16_
                 float o = v[r];
                 if constexpr (OUT == STEP_OUT_SIDE) {
                     const float e = bf16_bits_to_f32(a.side[(size_t)a.tok[0] * a.side_stride + a.side_offset + m]);
-                    o = 0.5f * o * (1.0f + tanhf(0.7978845608028654f * (o + 0.044715f * o * o * o))) * e;
+                    o = act_gelu_tanh(o) * e;
                 }
                 if (lane == 0) a.out[m] = o;
                 const float q = o * o;

@@ -7,18 +7,12 @@
 //
 // A sequence's starting state is read in the first launch where the sequence goes on into later windows: those may write
 // its final state while this window still runs.
+#include "act_math.hpp"
 #include "rowops.hpp"
 
 namespace mesh {
 
 constexpr int GRU_WINDOW = 32, GRU_THREADS = 256;
-
-struct GruGate { float z, keep, cand; };
-__device__ __forceinline__ float gru_sigmoid(float v) { return 1.0f / (1.0f + expf(-v)); }
-__device__ __forceinline__ GruGate gru_gate(float pz, float u) {
-    // 1 - z as the sigmoid of the negated argument: no cancellation where the gate is nearly open
-    return {gru_sigmoid(pz), gru_sigmoid(-pz), u >= 0.f ? u + 0.5f : gru_sigmoid(u)};
-}
 
 __global__ __launch_bounds__(GRU_THREADS) void min_gru_compose_kernel(const MinGruArgs a, int T) {
     const int ch = blockIdx.x * GRU_THREADS + threadIdx.x, w = blockIdx.y, W = a.width;
@@ -26,16 +20,16 @@ __global__ __launch_bounds__(GRU_THREADS) void min_gru_compose_kernel(const MinG
     const int t0 = w * GRU_WINDOW, t1 = t0 + GRU_WINDOW < T ? t0 + GRU_WINDOW : T;
     const float bz = a.bias_z[ch], bx = a.bias_x[ch];
     float A = 1.f, B = 0.f, init = 0.f;
-#pragma unroll 4
+#pragma unroll 8
     for (int t = t0; t < t1; ++t) {
         if (t == 0 || a.seq[t] != a.seq[t - 1]) {
             A = 0.f;
             B = init = a.pos[t] == 0 ? 0.f : a.state[(size_t)a.seq[t] * W + ch];
         }
         const float *p = a.zxg + (size_t)t * 3 * W + ch;
-        const GruGate g = gru_gate(p[0] + bz, p[W] + bx);
+        const MinGruGate g = min_gru_gate(p[0] + bz, p[W] + bx);
         A *= g.keep;
-        B = g.keep * B + g.z * g.cand;
+        B = fmaf(g.keep, B, g.in);
     }
     float *ws = a.ws + (size_t)w * 3 * W + ch;
     ws[0] = A; ws[W] = B; ws[2 * W] = init;
@@ -55,13 +49,13 @@ __global__ __launch_bounds__(GRU_THREADS) void min_gru_kernel(const MinGruArgs a
         return;
     }
     float S = 0.f;
-#pragma unroll 4
+#pragma unroll 8
     for (int v = 0; v < w; ++v) S = a.ws[(size_t)v * 3 * W + ch] * S + a.ws[((size_t)v * 3 + 1) * W + ch];
     int last_start = -1;                // the sequence that may go on past this window begins here
     for (int t = t0; t < t1; ++t)
         if (t == 0 || a.seq[t] != a.seq[t - 1]) last_start = t;
     const float bz = a.bias_z[ch], bx = a.bias_x[ch];
-#pragma unroll 4
+#pragma unroll 8
     for (int t = t0; t < t1; ++t) {
         const int seq = a.seq[t];
         if (t == 0 || seq != a.seq[t - 1]) {
@@ -69,10 +63,9 @@ __global__ __launch_bounds__(GRU_THREADS) void min_gru_kernel(const MinGruArgs a
             else S = gridDim.y > 1 && t == last_start ? a.ws[((size_t)w * 3 + 2) * W + ch] : a.state[(size_t)seq * W + ch];
         }
         const float *p = a.zxg + (size_t)t * 3 * W + ch;
-        const GruGate g = gru_gate(p[0] + bz, p[W] + bx);
-        S = g.keep * S + g.z * g.cand;
-        const float o = p[2 * W];
-        put(t, S * (o * gru_sigmoid(o)));
+        const MinGruGate g = min_gru_gate(p[0] + bz, p[W] + bx);
+        S = fmaf(g.keep, S, g.in);
+        put(t, S * act_silu(p[2 * W]));
         if (t + 1 == T || a.seq[t + 1] != seq) a.state[(size_t)seq * W + ch] = S;
     }
 }

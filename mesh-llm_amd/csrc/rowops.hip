@@ -1,6 +1,8 @@
 // See rowops.hpp.  One workgroup per token row; sums of squares in f32.
 #include "rowops.hpp"
 
+#include "act_math.hpp"
+
 #include "kv_cache.hpp"
 
 namespace mesh {
@@ -10,6 +12,27 @@ constexpr int ROW_THREADS = 256, ROW_WAVES = ROW_THREADS / 64;
 template <ActType ACT> __device__ __forceinline__ void act_store(void *out, size_t i, float v) {
     if constexpr (ACT == ACT_BF16) static_cast<uint16_t *>(out)[i] = f32_to_bf16_bits(v);
     else static_cast<float *>(out)[i] = v;
+}
+
+// Rows are walked four elements at a time when their length is a multiple of four (every row then starts on 16 bytes), else
+// one at a time: V elements from i on, and their counterpart on the way out.
+template <int V> struct RowVec { float v[V]; };
+template <int V> __device__ __forceinline__ RowVec<V> row_load(const float *p) {
+    RowVec<V> r;
+    if constexpr (V == 4) { const float4 q = *reinterpret_cast<const float4 *>(p); r.v[0] = q.x; r.v[1] = q.y; r.v[2] = q.z; r.v[3] = q.w; }
+    else r.v[0] = p[0];
+    return r;
+}
+template <int V> __device__ __forceinline__ void row_store(float *p, const RowVec<V> &r) {
+    if constexpr (V == 4) *reinterpret_cast<float4 *>(p) = make_float4(r.v[0], r.v[1], r.v[2], r.v[3]);
+    else p[0] = r.v[0];
+}
+template <ActType ACT, int V> __device__ __forceinline__ void act_store_row(void *out, size_t i, const RowVec<V> &r) {
+    if constexpr (ACT == ACT_F32) row_store<V>(static_cast<float *>(out) + i, r);
+    else if constexpr (V == 4)
+        *reinterpret_cast<uint2 *>(static_cast<uint16_t *>(out) + i) = make_uint2((uint32_t)f32_to_bf16_bits(r.v[0]) | ((uint32_t)f32_to_bf16_bits(r.v[1]) << 16),
+                                                                                  (uint32_t)f32_to_bf16_bits(r.v[2]) | ((uint32_t)f32_to_bf16_bits(r.v[3]) << 16));
+    else act_store<ACT>(out, i, r.v[0]);
 }
 
 __device__ __forceinline__ float row_sum(float v, float *scratch) {
@@ -32,26 +55,34 @@ __global__ __launch_bounds__(ROW_THREADS) void embed_rows_kernel(const uint16_t 
     }
 }
 
-template <ActType ACT>
+template <ActType ACT, int V>
 __global__ __launch_bounds__(ROW_THREADS) void residual_norm_kernel(float *x, const float *y, const float *gain, float eps, int n, void *out, int ld) {
     __shared__ float scratch[ROW_WAVES];
     const size_t at = (size_t)blockIdx.x * n, to = (size_t)blockIdx.x * ld;
     float rinv = 0.f;
     if (y) {
         float ss = 0.f;
-        for (int i = threadIdx.x; i < n; i += ROW_THREADS) ss = fmaf(y[at + i], y[at + i], ss);
+#pragma unroll 4
+        for (int i = threadIdx.x * V; i < n; i += ROW_THREADS * V) {
+            const RowVec<V> r = row_load<V>(y + at + i);
+#pragma unroll
+            for (int j = 0; j < V; ++j) ss = fmaf(r.v[j], r.v[j], ss);
+        }
         rinv = 1.0f / sqrtf(row_sum(ss, scratch) / (float)n + eps);
     }
-    for (int i = threadIdx.x; i < ld; i += ROW_THREADS) {
-        float v = 0.f;
+#pragma unroll 4
+    for (int i = threadIdx.x * V; i < ld; i += ROW_THREADS * V) {
+        RowVec<V> v = {};
         if (i < n) {
-            v = x[at + i];
+            v = row_load<V>(x + at + i);
             if (y) {
-                v = v + y[at + i] * rinv * gain[i];
-                x[at + i] = v;
+                const RowVec<V> r = row_load<V>(y + at + i), g = row_load<V>(gain + i);
+#pragma unroll
+                for (int j = 0; j < V; ++j) v.v[j] = v.v[j] + r.v[j] * rinv * g.v[j];
+                row_store<V>(x + at + i, v);
             }
         }
-        act_store<ACT>(out, to + i, v);
+        act_store_row<ACT, V>(out, to + i, v);
     }
 }
 
@@ -65,41 +96,54 @@ __global__ __launch_bounds__(ROW_THREADS) void scalar_norm_kernel(const float *x
     for (int i = threadIdx.x; i < ld; i += ROW_THREADS) act_store<ACT>(out, to + i, i < n ? x[at + i] * z : 0.f);
 }
 
-template <ActType ACT>
+template <ActType ACT, int V>
 __global__ __launch_bounds__(ROW_THREADS) void poly_norm_kernel(const float *u, const float *coef, float eps, int n, void *out, int ld) {
     __shared__ float scratch[ROW_WAVES];
     const size_t at = (size_t)blockIdx.x * n, to = (size_t)blockIdx.x * ld;
     float p2 = 0.f, p4 = 0.f, p6 = 0.f;
-    for (int i = threadIdx.x; i < n; i += ROW_THREADS) {
-        const float q = u[at + i] * u[at + i];
-        p2 += q; p4 += q * q; p6 += q * q * q;
+#pragma unroll 4
+    for (int i = threadIdx.x * V; i < n; i += ROW_THREADS * V) {
+        const RowVec<V> r = row_load<V>(u + at + i);
+#pragma unroll
+        for (int j = 0; j < V; ++j) {
+            const float q = r.v[j] * r.v[j];
+            p2 += q; p4 += q * q; p6 += q * q * q;
+        }
     }
     p2 = row_sum(p2, scratch); p4 = row_sum(p4, scratch); p6 = row_sum(p6, scratch);
     const float c1 = coef[0] / sqrtf(p2 / (float)n + eps), c2 = coef[1] / sqrtf(p4 / (float)n + eps), c3 = coef[2] / sqrtf(p6 / (float)n + eps), c0 = coef[3];
-    for (int i = threadIdx.x; i < ld; i += ROW_THREADS) {
-        const float v = i < n ? u[at + i] : 0.f;
-        act_store<ACT>(out, to + i, i < n ? ((c3 * v + c2) * v + c1) * v + c0 : 0.f);
+#pragma unroll 4
+    for (int i = threadIdx.x * V; i < ld; i += ROW_THREADS * V) {
+        RowVec<V> v = {};
+        if (i < n) {
+            v = row_load<V>(u + at + i);
+#pragma unroll
+            for (int j = 0; j < V; ++j) v.v[j] = ((c3 * v.v[j] + c2) * v.v[j] + c1) * v.v[j] + c0;
+        }
+        act_store_row<ACT, V>(out, to + i, v);
     }
 }
 
 template <ActType ACT>
-__global__ __launch_bounds__(64) void side_gate_kernel(const float *g, const uint16_t *side, const int32_t *tok, int stride, int offset, int n, void *out, int ld) {
+__global__ __launch_bounds__(64) void side_gate_kernel(const float *g, int slices, size_t slice_stride, const uint16_t *side, const int32_t *tok, int stride, int offset, int n, void *out, int ld) {
     const int t = blockIdx.x;
     const uint16_t *e = side + (size_t)tok[t] * stride + offset;
     for (int i = threadIdx.x; i < ld; i += 64) {
         float v = 0.f;
         if (i < n) {
-            const float z = g[(size_t)t * n + i];
-            v = 0.5f * z * (1.0f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z))) * bf16_bits_to_f32(e[i]);
+            float z = 0.f;
+            for (int s = 0; s < slices; ++s) z += g[s * slice_stride + (size_t)t * n + i];
+            v = act_gelu_tanh(z) * bf16_bits_to_f32(e[i]);
         }
         act_store<ACT>(out, (size_t)t * ld + i, v);
     }
 }
 
-__device__ __forceinline__ void append_value(uint8_t *cache, int type, size_t at, float v, unsigned *sat) {
-    if (type == MESH_F32) { reinterpret_cast<float *>(cache)[at] = v; return; }
-    note_f16_clamp(sat, v, 0.f);
-    reinterpret_cast<uint16_t *>(cache)[at] = f32_to_f16_bits(fminf(fmaxf(v, -65504.f), 65504.f));
+__device__ __forceinline__ void append4(uint8_t *cache, int type, size_t at, const float4 &v, unsigned *sat) {
+    if (type == MESH_F32) { *reinterpret_cast<float4 *>(reinterpret_cast<float *>(cache) + at) = v; return; }
+    note_f16_clamp(sat, v.x, v.y, v.z, v.w);
+    auto h = [](float f) { return (uint32_t)f32_to_f16_bits(fminf(fmaxf(f, -65504.f), 65504.f)); };
+    *reinterpret_cast<uint2 *>(reinterpret_cast<uint16_t *>(cache) + at) = make_uint2(h(v.x) | (h(v.y) << 16), h(v.z) | (h(v.w) << 16));
 }
 
 // grid (slices of the heads, T); every workgroup sums the whole row itself, so that slices need not meet
@@ -107,20 +151,29 @@ __global__ __launch_bounds__(ROW_THREADS) void qk_norm_append_kernel(const QkApp
     __shared__ float scratch[ROW_WAVES];
     const int t = blockIdx.y, nq = a.n_head * a.hd, nk = a.n_kv * a.hd;
     const float *row = a.qk + (size_t)t * (nq + nk);
-    float sq = 0.f, sk = 0.f;
-    for (int i = threadIdx.x; i < nq; i += ROW_THREADS) sq = fmaf(row[i], row[i], sq);
-    for (int i = threadIdx.x; i < nk; i += ROW_THREADS) sk = fmaf(row[nq + i], row[nq + i], sk);
+    float sq = 0.f, sk = 0.f;           // (head rows are a multiple of 64 long: four at a time)
+#pragma unroll 4
+    for (int i = threadIdx.x * 4; i < nq + nk; i += ROW_THREADS * 4) {
+        const float4 v = *reinterpret_cast<const float4 *>(row + i);
+        const float s = v.x * v.x + v.y * v.y + v.z * v.z + v.w * v.w;
+        if (i < nq) sq += s; else sk += s;
+    }
     const float rq = 1.0f / sqrtf(row_sum(sq, scratch) / (float)(a.n_head * a.dim) + a.eps);
     const float rk = 1.0f / sqrtf(row_sum(sk, scratch) / (float)(a.n_kv * a.dim) + a.eps);
     const int pos = a.pos[t], seq = a.seq[t];
-    const int stride = gridDim.x * ROW_THREADS, first = blockIdx.x * ROW_THREADS + threadIdx.x;
-    for (int i = first; i < nq; i += stride) a.q[(size_t)t * nq + i] = row[i] * rq * a.q_norm[i];
-    for (int i = first; i < nk; i += stride) {
-        const int head = i / a.hd, d = i - head * a.hd;
-        const size_t at = (((size_t)seq * a.n_kv + head) * a.n_ctx + pos) * a.hd + d;
-        const float v = row[nq + i];
-        append_value(a.kcache, a.kv_type, at, v * rk * a.k_norm[i], a.sat);
-        append_value(a.vcache, a.kv_type, at, v, a.sat);
+    const int stride = gridDim.x * ROW_THREADS * 4;
+    for (int i = (blockIdx.x * ROW_THREADS + threadIdx.x) * 4; i < nq + nk; i += stride) {
+        const float4 v = *reinterpret_cast<const float4 *>(row + i);
+        if (i < nq) {
+            const float4 g = *reinterpret_cast<const float4 *>(a.q_norm + i);
+            *reinterpret_cast<float4 *>(a.q + (size_t)t * nq + i) = make_float4(v.x * rq * g.x, v.y * rq * g.y, v.z * rq * g.z, v.w * rq * g.w);
+            continue;
+        }
+        const int kk = i - nq, head = kk / a.hd;
+        const float4 g = *reinterpret_cast<const float4 *>(a.k_norm + kk);
+        const size_t at = (((size_t)seq * a.n_kv + head) * a.n_ctx + pos) * a.hd + (kk - head * a.hd);
+        append4(a.kcache, a.kv_type, at, make_float4(v.x * rk * g.x, v.y * rk * g.y, v.z * rk * g.z, v.w * rk * g.w), a.sat);
+        append4(a.vcache, a.kv_type, at, v, a.sat);
     }
 }
 
@@ -128,6 +181,15 @@ __global__ __launch_bounds__(ROW_THREADS) void qk_norm_append_kernel(const QkApp
     do {                                                                                                   \
         if (act == ACT_BF16) MESH_LAUNCH((kernel<ACT_BF16>), grid, block, 0, stream, __VA_ARGS__);         \
         else MESH_LAUNCH((kernel<ACT_F32>), grid, block, 0, stream, __VA_ARGS__);                          \
+        MESH_LAUNCH_CHECK();                                                                               \
+    } while (0)
+
+#define MESH_ROW_LAUNCH(kernel, act, vec, grid, block, ...)                                                \
+    do {                                                                                                   \
+        if (act == ACT_BF16 && (vec)) MESH_LAUNCH((kernel<ACT_BF16, 4>), grid, block, 0, stream, __VA_ARGS__); \
+        else if (act == ACT_BF16) MESH_LAUNCH((kernel<ACT_BF16, 1>), grid, block, 0, stream, __VA_ARGS__);  \
+        else if (vec) MESH_LAUNCH((kernel<ACT_F32, 4>), grid, block, 0, stream, __VA_ARGS__);               \
+        else MESH_LAUNCH((kernel<ACT_F32, 1>), grid, block, 0, stream, __VA_ARGS__);                        \
         MESH_LAUNCH_CHECK();                                                                               \
     } while (0)
 
@@ -141,7 +203,7 @@ int embed_rows(const uint16_t *table, const int32_t *tok, const int32_t *pos, co
 int residual_norm_rows(float *x, const float *y, const float *gain, float eps, int T, int n, void *out, ActType act, int ld, hipStream_t stream) {
     if (T <= 0) return MESH_OK;
     if (ld < n || (y && !gain)) return fail(MESH_ERR_INVALID, "residual_norm_rows: bad operands");
-    MESH_ACT_LAUNCH(residual_norm_kernel, act, dim3((unsigned)T), dim3(ROW_THREADS), x, y, gain, eps, n, out, ld);
+    MESH_ROW_LAUNCH(residual_norm_kernel, act, n % 4 == 0, dim3((unsigned)T), dim3(ROW_THREADS), x, y, gain, eps, n, out, ld);
     return MESH_OK;
 }
 
@@ -155,14 +217,14 @@ int scalar_norm_rows(const float *x, const int32_t *row, const float *gain, floa
 int poly_norm_rows(const float *u, const float *coef, float eps, int T, int n, void *out, ActType act, int ld, hipStream_t stream) {
     if (T <= 0) return MESH_OK;
     if (ld < n) return fail(MESH_ERR_INVALID, "poly_norm_rows: bad operands");
-    MESH_ACT_LAUNCH(poly_norm_kernel, act, dim3((unsigned)T), dim3(ROW_THREADS), u, coef, eps, n, out, ld);
+    MESH_ROW_LAUNCH(poly_norm_kernel, act, n % 4 == 0, dim3((unsigned)T), dim3(ROW_THREADS), u, coef, eps, n, out, ld);
     return MESH_OK;
 }
 
-int side_gate_rows(const float *g, const uint16_t *side, const int32_t *tok, int stride, int offset, int T, int n, void *out, ActType act, int ld, hipStream_t stream) {
+int side_gate_rows(const float *g, int slices, size_t slice_stride, const uint16_t *side, const int32_t *tok, int stride, int offset, int T, int n, void *out, ActType act, int ld, hipStream_t stream) {
     if (T <= 0) return MESH_OK;
     if (ld < n || offset + n > stride) return fail(MESH_ERR_INVALID, "side_gate_rows: bad operands");
-    MESH_ACT_LAUNCH(side_gate_kernel, act, dim3((unsigned)T), dim3(64), g, side, tok, stride, offset, n, out, ld);
+    MESH_ACT_LAUNCH(side_gate_kernel, act, dim3((unsigned)T), dim3(64), g, slices, slice_stride, side, tok, stride, offset, n, out, ld);
     return MESH_OK;
 }
 

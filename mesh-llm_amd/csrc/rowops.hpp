@@ -19,8 +19,8 @@ int scalar_norm_rows(const float *x, const int32_t *row, const float *gain, floa
 // act[t] = c0 N(u) + c1 N(u^2) + c2 N(u^3) + c3 with u = u[t][0..n), powers element by element, N(v) = v / rms(v)
 int poly_norm_rows(const float *u, const float *coef, float eps, int T, int n, void *out, ActType act, int ld, hipStream_t stream);
 
-// act[t][i] = gelu_tanh(g[t][i]) * side[tok[t]][offset + i]
-int side_gate_rows(const float *g, const uint16_t *side, const int32_t *tok, int stride, int offset, int T, int n, void *out, ActType act, int ld, hipStream_t stream);
+// act[t][i] = gelu_tanh(g[t][i]) * side[tok[t]][offset + i]; g as the sum of `slices` partial products (linear_sliced)
+int side_gate_rows(const float *g, int slices, size_t slice_stride, const uint16_t *side, const int32_t *tok, int stride, int offset, int T, int n, void *out, ActType act, int ld, hipStream_t stream);
 
 // Norm over a whole q / k projection and KV append for attention whose values are the un-normalised keys.  qk: [T][(n_head +
 // n_kv) * hd], q first; each head's entries from dim on are zero.  q[t] = q / rms(q over all heads) * q_norm; the cache

@@ -139,6 +139,21 @@ def test_long_prompt_takes_every_kernel(tmp_path, prec):
 
 
 @BOTH
+def test_layers_wide_enough_for_several_tiles_and_slices(tmp_path, prec):
+    """Products whose K spans several batches of a wave, whose rows take more than one per turn, and a side gate cut along K;
+    lengths are no multiple of anything."""
+    cfg = N.config(4500, 1032, 40, [N.attention(8, 2, 128, 50, ff=4200), N.mingru(1100)], scale=0.6)
+    cfg, w, folder, orc = made(tmp_path, cfg)
+    st = open_stage(folder, prec, n_ctx=512, batch=512)
+    t = N.prompt(cfg, 303, 8)
+    want = orc.forward(t)[-20:]
+    for portions in ([303], [150, 150, 1, 1, 1], [290] + [1] * 13):
+        e = N.error(run(st, t, portions, last=20), want)
+        assert e < LIMIT[prec], (portions, prec, e)
+    st.close()
+
+
+@BOTH
 def test_far_token_reaches_through_the_state(tmp_path, prec):
     """A recurrence that hardly forgets: changing one token 300 back changes the last logits as the oracle says."""
     def slow(w, cfg):
