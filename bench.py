@@ -685,6 +685,17 @@ def bench_nadosun(args):
             ses.decode_dev(xs.data_ptr(), [at[0]], out.data_ptr(), T * E * 4, token_ids=ids[:1])
             at[0] += 1
 
+        def portion(n):
+            def run(i):
+                if at[0] + n > NADOSUN_CTX:
+                    at[0] = 0
+                ses.decode_dev(xs.data_ptr(), np.arange(at[0], at[0] + n), out.data_ptr(), T * E * 4, token_ids=ids[:n])
+                at[0] += n
+            return run
+
+        def lportion(n):
+            return lambda i: lses.decode_dev(xs.data_ptr(), np.arange(sp["window"], sp["window"] + n), out.data_ptr(), T * E * 4)
+
         def lprefill(i):
             lses.decode_dev(xs.data_ptr(), np.arange(T), out.data_ptr(), T * E * 4)
 
@@ -709,6 +720,11 @@ def bench_nadosun(args):
                 r[k] = round(min(r[k]), 4)
             pms, _ = kernel_ms(ses_, pf, 1)
             dms, dl = kernel_ms(ses_, sf, 5)
+            for n in (16, 64):                  # short portions of a prompt
+                fn = portion(n) if side == "nadosun" else lportion(n)
+                ms = time_on_stream(torch, s1 if side == "nadosun" else s2, fn, 50, 5)[0]
+                pk, _ = kernel_ms(ses_, fn, 5)
+                r["portion_%d" % n] = {"ms": round(ms, 4), "kernel_ms": pk, "products_frac_hbm": round(by / pk["gemv"] / 1e6 / HBM_PEAK_GBS, 4)}
             r.update({"prefill_tok_s": round(T * 1e3 / r["prefill_ms"], 1), "decode_tok_s": round(1e3 / r["decode_ms"], 1), "weight_GB": round(by / 1e9, 3),
                       "prefill_kernel_ms": pms, "decode_kernel_ms": dms, "decode_launches": dl,
                       "products_prefill_TFLOPs": round(2.0 * mc * T / pms["gemv"] / 1e9, 1),
