@@ -7,6 +7,8 @@
 // are processed together, so each K/V byte is read once per token.
 
 #include "attn.hpp"
+
+#include "act_math.hpp"
 #include "q16.hpp"
 
 namespace mesh {
@@ -268,7 +270,8 @@ __global__ __launch_bounds__(ATTN_THREADS) void attn_kernel(AttnArgs a) {
 // sees them with broadcast reads and the partial rows are fetched with independent loads.
 // (leading scalar arguments: preloaded into SGPRs, see gemv.hip)
 __global__ __launch_bounds__(256) void attn_combine_kernel(const float *p_part, const float *p_ml, float *p_out, _Float16 *p_out16_k8,
-                                                           uint8_t *p_out_q16, uint16_t *p_out_bf16, int p_n_splits, int p_n_head, int p_head_dim) {
+                                                           uint8_t *p_out_q16, uint16_t *p_out_bf16, int p_n_splits, int p_n_head, int p_head_dim,
+                                                           const float *p_gate, int p_gate_ld) {
     __shared__ float s_m[ATTN_SPLITS_CAP], s_l[ATTN_SPLITS_CAP];
     const int h = blockIdx.x, t = blockIdx.y, dd = threadIdx.x;
     const size_t row = (size_t)t * p_n_head + h;
@@ -300,7 +303,8 @@ __global__ __launch_bounds__(256) void attn_combine_kernel(const float *p_part, 
         const size_t kk = (size_t)h * p_head_dim + dd, KK = (size_t)p_n_head * p_head_dim;
         p_out16_k8[(size_t)(t / 16) * 16 * KK + ((kk >> 3) * 16 + (t % 16)) * 8 + (kk & 7)] = (_Float16)(num / den);
     } else if (p_out_bf16) {
-        p_out_bf16[row * p_head_dim + dd] = f32_to_bf16_bits(num / den);
+        const float gate = p_gate ? act_sigmoid(p_gate[(size_t)t * p_gate_ld + h]) : 1.f;
+        p_out_bf16[row * p_head_dim + dd] = f32_to_bf16_bits(num / den * gate);
     } else {
         p_out[row * p_head_dim + dd] = num / den;
     }
@@ -356,7 +360,9 @@ int attention(const AttnArgs &a, int T, hipStream_t stream) {
 }
 
 int attention_combine(const AttnArgs &a, int T, hipStream_t stream) {
-    MESH_LAUNCH(attn_combine_kernel, dim3((unsigned)a.n_head, (unsigned)T), dim3((unsigned)a.head_dim), 0, stream, a.part, a.ml, a.out, a.out16_k8, a.out_q16, a.out_bf16, a.n_splits, a.n_head, a.head_dim);
+    const int dim = a.v_dim ? a.v_dim : a.head_dim;
+    MESH_LAUNCH(attn_combine_kernel, dim3((unsigned)a.n_head, (unsigned)T), dim3((unsigned)dim), 0, stream, a.part, a.ml, a.out, a.out16_k8, a.out_q16, a.out_bf16, a.n_splits, a.n_head, dim,
+                a.head_gate, a.gate_ld);
     MESH_LAUNCH_CHECK();
     return MESH_OK;
 }

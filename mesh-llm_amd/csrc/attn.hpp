@@ -48,6 +48,11 @@ struct AttnArgs {
     int window = 0;                // token t sees the positions (pos[t] - window, pos[t]]; 0: all of [0, pos[t]]
     float scale = 1.f;
     int n_head = 0, n_kv = 0, group = 1, head_dim = 0, n_ctx = 0, n_splits = 1;
+    // attention_chunk only: entries of a value row and of an output head (0: head_dim), and a gate per head, [T][gate_ld], whose
+    // sigmoid multiplies the output (bf16 rows)
+    int v_dim = 0;
+    const float *head_gate = nullptr;
+    int gate_ld = 0;
 };
 // token t attends to cache positions [0, pos[t]] of sequence seq[t], or to the last `window` of them
 int attention(const AttnArgs &a, int T, hipStream_t stream);
@@ -58,7 +63,7 @@ int attention_combine(const AttnArgs &a, int T, hipStream_t stream);
 bool attention_mma_supported(const AttnArgs &a);
 int attention_mma(const AttnArgs &a, int T, hipStream_t stream);
 // The same for a chunk of T consecutive positions pos0 .. pos0 + T - 1 of one sequence, on the matrix cores
-// (attn_prefill.hip; head_dim 64 or 128).  a.pos / a.seq / a.part / a.ml are not used.
+// (attn_prefill.hip; head_dim 64 or 128; with f16 rows and a group of 1 also 128 with values of 64, 192 with values of 128).  a.pos / a.seq / a.part / a.ml are not used.
 int attention_chunk(const AttnArgs &a, int T, int pos0, int seq, hipStream_t stream);
 bool kv_pair_supported(int k_type, int v_type);
 

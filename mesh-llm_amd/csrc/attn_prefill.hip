@@ -22,6 +22,7 @@
 
 #include <algorithm>
 
+#include "act_math.hpp"
 #include "attn.hpp"
 
 namespace mesh {
@@ -61,19 +62,19 @@ __device__ __forceinline__ uint4 pf_row_piece(const uint8_t *row, int piece) {
     }
 }
 
-// NT: tiles of 32 keys per step (1 or 2; two give the wave two independent score chains and half the barriers per key, at
+// HD, VD: entries of a key and of a value row.  NT: tiles of 32 keys per step (1 or 2; two give the wave two independent score chains and half the barriers per key, at
 // ~50 more registers).  NP: (key, 8-dim piece) pairs of a step one thread carries in registers, at least 4 HD NT /
 // (threads of the workgroup); 0 for small workgroups, which load each step's rows where they write them.
-template <int HD, int KT, int VT, int NP, int NT>
+template <int HD, int VD, int KT, int VT, int NP, int NT>
 __global__ __launch_bounds__(512) void attn_chunk_kernel(const AttnArgs a, int T, int pos0, int seq, int hpw, int fwd_from, int qtiles, int n_ksplit) {
-    constexpr int KRB = kv_row_bytes(KT, HD), VRB = kv_row_bytes(VT, HD);
-    constexpr int PIECES = HD / 8;                  // 8-dim pieces of a row
-    constexpr int NKC = HD / 16, NDB = HD / 32;     // steps of the score product along the dims, 32-dim blocks of the output
+    constexpr int KRB = kv_row_bytes(KT, HD), VRB = kv_row_bytes(VT, VD);
+    constexpr int PIECES = HD / 8, VPIECES = VD / 8;      // 8-dim pieces of a row
+    constexpr int NKC = HD / 16, NDB = VD / 32;     // steps of the score product along the dims, 32-dim blocks of the output
     constexpr int PF_KPITCH = HD + 8;               // halfs per key row of the K tile in LDS (bank-conflict padding)
     constexpr int PF_KEYS = 32 * NT;                // keys per step
     constexpr int PF_VPITCH = PF_KEYS / 2 + 2;      // dwords (key pairs) per dim row of the transposed V tile
     __shared__ __align__(16) _Float16 sK[PF_KEYS * PF_KPITCH];
-    __shared__ __align__(16) uint32_t sVt[HD * PF_VPITCH];
+    __shared__ __align__(16) uint32_t sVt[VD * PF_VPITCH];
     const int tid = threadIdx.x, lane = tid & 63, nthreads = blockDim.x;
     // wave -> (head of the workgroup, one of its `qtiles` consecutive query tiles): groups of fewer than four heads fill the
     // workgroup with several query tiles of the same heads, which share the K / V tiles like heads do
@@ -136,13 +137,13 @@ __global__ __launch_bounds__(512) void attn_chunk_kernel(const AttnArgs a, int T
         return pf_row_piece<KT, HD>(a.kcache + (base + kr) * KRB, p % PIECES);
     };
     auto v_row = [&](int k0, int p, int second) {
-        int kr = k0 + 2 * (p / PIECES) + second;
+        int kr = k0 + 2 * (p / VPIECES) + second;
         kr = kr < a.n_ctx ? kr : a.n_ctx - 1;
-        return pf_row_piece<VT, HD>(a.vcache + (base + kr) * VRB, p % PIECES);
+        return pf_row_piece<VT, VD>(a.vcache + (base + kr) * VRB, p % VPIECES);
     };
     auto k_put = [&](int p, const uint4 &r) { *reinterpret_cast<uint4 *>(sK + (p / PIECES) * PF_KPITCH + (p % PIECES) * 8) = r; };
     auto v_put = [&](int p, const uint4 &r0, const uint4 &r1) {
-        const int kp = p / PIECES, piece = p % PIECES;
+        const int kp = p / VPIECES, piece = p % VPIECES;
         const uint32_t w0[4] = {r0.x, r0.y, r0.z, r0.w}, w1[4] = {r1.x, r1.y, r1.z, r1.w};
         uint32_t *dst = sVt + piece * 8 * PF_VPITCH + pf_vcol(piece * 8, kp);
 #pragma unroll
@@ -164,7 +165,7 @@ __global__ __launch_bounds__(512) void attn_chunk_kernel(const AttnArgs a, int T
 #pragma unroll
         for (int i = 0; i < NPV; ++i) {
             const int p = tid + i * nthreads;
-            if (p < PF_KEYS * PIECES / 2) { rv[i][0] = v_row(k0, p, 0); rv[i][1] = v_row(k0, p, 1); }
+            if (p < PF_KEYS * VPIECES / 2) { rv[i][0] = v_row(k0, p, 0); rv[i][1] = v_row(k0, p, 1); }
         }
     };
     if constexpr (NP > 0) fetch_step(k_lo);
@@ -178,11 +179,11 @@ __global__ __launch_bounds__(512) void attn_chunk_kernel(const AttnArgs a, int T
 #pragma unroll
             for (int i = 0; i < NPV; ++i) {
                 const int p = tid + i * nthreads;
-                if (p < PF_KEYS * PIECES / 2) v_put(p, rv[i][0], rv[i][1]);
+                if (p < PF_KEYS * VPIECES / 2) v_put(p, rv[i][0], rv[i][1]);
             }
         } else {
             for (int p = tid; p < PF_KEYS * PIECES; p += nthreads) k_put(p, k_row(k0, p));
-            for (int p = tid; p < PF_KEYS * PIECES / 2; p += nthreads) v_put(p, v_row(k0, p, 0), v_row(k0, p, 1));
+            for (int p = tid; p < PF_KEYS * VPIECES / 2; p += nthreads) v_put(p, v_row(k0, p, 0), v_row(k0, p, 1));
         }
         __syncthreads();
         if constexpr (NP > 0) {
@@ -293,7 +294,7 @@ __global__ __launch_bounds__(512) void attn_chunk_kernel(const AttnArgs a, int T
         // un-normalised partial and (maximum, sum) of this key split, in the layout of the split-KV decode kernels
         if (q_live) {
             const size_t prow = ((size_t)tq * a.n_head + h) * n_ksplit + ks;
-            float *pp = a.part + prow * HD;
+            float *pp = a.part + prow * VD;
 #pragma unroll
             for (int db = 0; db < NDB; ++db)
 #pragma unroll
@@ -310,21 +311,21 @@ __global__ __launch_bounds__(512) void attn_chunk_kernel(const AttnArgs a, int T
         const int t_pad = (T + 15) & ~15;
         if (tq < t_pad) {
             const float inv = q_live ? 1.0f / l : 0.f;
-            const size_t KK = (size_t)a.n_head * HD;
+            const size_t KK = (size_t)a.n_head * VD;
             _Float16 *ob = a.out16_k8 + (size_t)(tq >> 4) * 16 * KK + (size_t)(tq & 15) * 8;
 #pragma unroll
             for (int db = 0; db < NDB; ++db)
 #pragma unroll
                 for (int i4 = 0; i4 < 4; ++i4) {
-                    const size_t kk = (size_t)h * HD + db * 32 + 8 * i4 + 4 * half;
+                    const size_t kk = (size_t)h * VD + db * 32 + 8 * i4 + 4 * half;
                     *reinterpret_cast<uint2 *>(ob + (kk >> 3) * 128 + (kk & 7)) =
                         make_uint2(pf_pack(o[db][4 * i4] * inv, o[db][4 * i4 + 1] * inv), pf_pack(o[db][4 * i4 + 2] * inv, o[db][4 * i4 + 3] * inv));
                 }
         }
     } else if (a.out_bf16) {
         if (q_live) {
-            const float inv = 1.0f / l;
-            uint16_t *op = a.out_bf16 + ((size_t)tq * a.n_head + h) * HD;
+            const float inv = (a.head_gate ? act_sigmoid(a.head_gate[(size_t)tq * a.gate_ld + h]) : 1.0f) / l;
+            uint16_t *op = a.out_bf16 + ((size_t)tq * a.n_head + h) * VD;
             auto two16 = [&](float lo, float hi) { return (uint32_t)f32_to_bf16_bits(lo * inv) | ((uint32_t)f32_to_bf16_bits(hi * inv) << 16); };
 #pragma unroll
             for (int db = 0; db < NDB; ++db)
@@ -335,7 +336,7 @@ __global__ __launch_bounds__(512) void attn_chunk_kernel(const AttnArgs a, int T
         }
     } else if (q_live) {
         const float inv = 1.0f / l;
-        float *op = a.out + ((size_t)tq * a.n_head + h) * HD;
+        float *op = a.out + ((size_t)tq * a.n_head + h) * VD;
 #pragma unroll
         for (int db = 0; db < NDB; ++db)
 #pragma unroll
@@ -375,8 +376,12 @@ static int pf_n_cu() {
 int attention_chunk(const AttnArgs &a_in, int T, int pos0, int seq, hipStream_t stream) {
     if (T <= 0) return MESH_OK;
     AttnArgs a = a_in;
-    if (a.head_dim != 128 && (a.head_dim != 64 || a.k_type != MESH_F16))
-        return fail(MESH_ERR_UNSUPPORTED, "attention_chunk: head_dim %d, cache type %d (128, and 64 with f16 rows)", a.head_dim, a.k_type);
+    const int v_dim = a.v_dim ? a.v_dim : a.head_dim;
+    const bool apart = v_dim != a.head_dim;         // keys and values of different lengths
+    if (apart ? a.group != 1 || a.k_type != MESH_F16 || a.v_type != MESH_F16 || !((a.head_dim == 128 && v_dim == 64) || (a.head_dim == 192 && v_dim == 128))
+              : a.head_dim != 128 && (a.head_dim != 64 || a.k_type != MESH_F16))
+        return fail(MESH_ERR_UNSUPPORTED, "attention_chunk: head_dim %d, values of %d, cache type %d (128, and 64 with f16 rows; 128 with 64 and 192 with 128)", a.head_dim, v_dim, a.k_type);
+    if (a.head_gate && !a.out_bf16) return fail(MESH_ERR_INVALID, "attention_chunk: gated output is bf16");
     if (a.group < 1 || a.n_head != a.group * a.n_kv || pos0 < 0 || pos0 + T > a.n_ctx || seq < 0)
         return fail(MESH_ERR_INVALID, "attention_chunk: bad head layout or chunk [%d, %d) outside the context of %d", pos0, pos0 + T, a.n_ctx);
     if (a.k_type != MESH_F16 && a.chunk_kv16 && T >= PF_EXPAND_MIN_T) {
@@ -427,11 +432,14 @@ int attention_chunk(const AttnArgs &a_in, int T, int pos0, int seq, hipStream_t 
     // NP by the threads of the workgroup: 1024 / threads pairs each, rounded up
 #define MESH_CHUNK_LAUNCH(HD, KT, VT)                                                                                     \
     do {                                                                                                                  \
-        if (waves == 8) MESH_LAUNCH((attn_chunk_kernel<HD, KT, VT, 2, 2>), grid, block, 0, stream, a, T, pos0, seq, hpw, fwd_from, qtiles, n_ksplit);      \
-        else if (waves == 6) MESH_LAUNCH((attn_chunk_kernel<HD, KT, VT, 3, 2>), grid, block, 0, stream, a, T, pos0, seq, hpw, fwd_from, qtiles, n_ksplit); \
-        else MESH_LAUNCH((attn_chunk_kernel<HD, KT, VT, 4, 2>), grid, block, 0, stream, a, T, pos0, seq, hpw, fwd_from, qtiles, n_ksplit);                  \
+        if (waves == 8) MESH_LAUNCH((attn_chunk_kernel<HD, HD, KT, VT, 2, 2>), grid, block, 0, stream, a, T, pos0, seq, hpw, fwd_from, qtiles, n_ksplit);      \
+        else if (waves == 6) MESH_LAUNCH((attn_chunk_kernel<HD, HD, KT, VT, 3, 2>), grid, block, 0, stream, a, T, pos0, seq, hpw, fwd_from, qtiles, n_ksplit); \
+        else MESH_LAUNCH((attn_chunk_kernel<HD, HD, KT, VT, 4, 2>), grid, block, 0, stream, a, T, pos0, seq, hpw, fwd_from, qtiles, n_ksplit);                  \
     } while (0)
-    if (a.head_dim == 64) MESH_CHUNK_LAUNCH(64, MESH_F16, MESH_F16);
+    // (a group of one: four waves)
+    if (apart && a.head_dim == 192) MESH_LAUNCH((attn_chunk_kernel<192, 128, MESH_F16, MESH_F16, 6, 2>), grid, block, 0, stream, a, T, pos0, seq, hpw, fwd_from, qtiles, n_ksplit);
+    else if (apart) MESH_LAUNCH((attn_chunk_kernel<128, 64, MESH_F16, MESH_F16, 4, 2>), grid, block, 0, stream, a, T, pos0, seq, hpw, fwd_from, qtiles, n_ksplit);
+    else if (a.head_dim == 64) MESH_CHUNK_LAUNCH(64, MESH_F16, MESH_F16);
     else if (a.k_type == MESH_F16 && a.v_type == MESH_F16) MESH_CHUNK_LAUNCH(128, MESH_F16, MESH_F16);
     else if (a.k_type == MESH_Q8_0 && a.v_type == MESH_Q4_0) MESH_CHUNK_LAUNCH(128, MESH_Q8_0, MESH_Q4_0);
     else if (a.k_type == MESH_Q4_0 && a.v_type == MESH_Q4_0) MESH_CHUNK_LAUNCH(128, MESH_Q4_0, MESH_Q4_0);

@@ -2,224 +2,11 @@
 #include "hybrid.hpp"
 
 #include <algorithm>
-#include <cmath>
-#include <cstring>
 
 #include "attn.hpp"
-#include "registry.hpp"
-#include "safetensors.hpp"
 #include "stage.hpp"
 
 namespace mesh {
-
-// ------------------------------------------------------------------------------------------------ loading
-namespace {
-
-typedef std::vector<uint64_t> Shape;
-
-struct FolderLoader {
-    const SafetensorsFile &f;
-    mesh_stage &st;
-
-    int dev_alloc(void **p, size_t bytes) {
-        hipError_t e = hipMalloc(p, bytes ? bytes : 16);
-        if (e != hipSuccess) return fail(e == hipErrorOutOfMemory ? MESH_ERR_NOMEM : MESH_ERR_DEVICE, "hipMalloc(%zu) failed: %s", bytes, hipGetErrorString(e));
-        st.allocations.push_back(*p);
-        return MESH_OK;
-    }
-    // bf16 tensor of exactly this shape
-    int get(const std::string &name, const Shape &shape, const uint16_t *&data) {
-        const SafeTensor *t = f.find(name);
-        if (!t) return fail(MESH_ERR_FORMAT, "model.safetensors: tensor '%s' not found", name.c_str());
-        if (t->dtype != "BF16") return fail(MESH_ERR_UNSUPPORTED, "model.safetensors: tensor '%s' is %s (BF16 expected)", name.c_str(), t->dtype.c_str());
-        if (t->shape != shape) {
-            std::string have, want;
-            for (uint64_t d : t->shape) have += std::to_string(d) + " ";
-            for (uint64_t d : shape) want += std::to_string(d) + " ";
-            return fail(MESH_ERR_FORMAT, "model.safetensors: tensor '%s' has shape [ %s], expected [ %s]", name.c_str(), have.c_str(), want.c_str());
-        }
-        data = reinterpret_cast<const uint16_t *>(f.data(*t));       // (read with memcpy only: the file does not promise alignment)
-        st.weight_bytes += t->nbytes;
-        return MESH_OK;
-    }
-    // the tensor as f32 on the host
-    int floats(const std::string &name, const Shape &shape, std::vector<float> &out) {
-        const uint16_t *d = nullptr;
-        int rc = get(name, shape, d);
-        if (rc != MESH_OK) return rc;
-        size_t n = 1;
-        for (uint64_t v : shape) n *= v;
-        out.resize(n);
-        for (size_t i = 0; i < n; ++i) {
-            uint16_t b;
-            memcpy(&b, reinterpret_cast<const uint8_t *>(d) + 2 * i, 2);
-            const uint32_t u = (uint32_t)b << 16;
-            memcpy(&out[i], &u, 4);
-        }
-        return MESH_OK;
-    }
-    int upload(const std::vector<float> &v, float **out) {
-        void *p = nullptr;
-        int rc = dev_alloc(&p, v.size() * sizeof(float));
-        if (rc != MESH_OK) return rc;
-        MESH_HIP_TRY(hipMemcpy(p, v.data(), v.size() * sizeof(float), hipMemcpyHostToDevice));
-        *out = static_cast<float *>(p);
-        return MESH_OK;
-    }
-    int raw(const std::string &name, const Shape &shape, uint16_t **out) {
-        const uint16_t *d = nullptr;
-        int rc = get(name, shape, d);
-        if (rc != MESH_OK) return rc;
-        size_t n = 2;
-        for (uint64_t v : shape) n *= v;
-        void *p = nullptr;
-        if ((rc = dev_alloc(&p, n)) != MESH_OK) return rc;
-        MESH_HIP_TRY(hipMemcpy(p, d, n, hipMemcpyHostToDevice));
-        *out = static_cast<uint16_t *>(p);
-        return MESH_OK;
-    }
-    int matrix_alloc(LinearWeight &W, int M, int K) {
-        W.M = M; W.K = K; W.Mp = linear_rows_padded(M); W.Kp = linear_k_padded(K);
-        void *p = nullptr;
-        int rc = dev_alloc(&p, (size_t)W.Mp * W.Kp * 2);
-        if (rc != MESH_OK) return rc;
-        MESH_HIP_TRY(hipMemset(p, 0, (size_t)W.Mp * W.Kp * 2));
-        W.w = static_cast<const uint16_t *>(p);
-        return MESH_OK;
-    }
-    static int copy(uint16_t *dst, size_t dpitch, const uint8_t *src, size_t spitch, size_t width, size_t rows) {
-        if (dpitch == spitch && width == spitch) MESH_HIP_TRY(hipMemcpy(dst, src, width * rows, hipMemcpyHostToDevice));
-        else MESH_HIP_TRY(hipMemcpy2D(dst, dpitch, src, spitch, width, rows, hipMemcpyHostToDevice));
-        return MESH_OK;
-    }
-    // [rows][cols] into W from row `row0` on; blocks of rb rows are placed rp rows apart, blocks of cb columns cp columns apart
-    int place(LinearWeight &W, const std::string &name, int rows, int cols, int row0, int rb, int rp, int cb, int cp) {
-        const uint16_t *d = nullptr;
-        int rc = get(name, {(uint64_t)rows, (uint64_t)cols}, d);
-        if (rc != MESH_OK) return rc;
-        if (rb == rp) { rb = rp = rows; }
-        if (cb == cp) { cb = cp = cols; }
-        uint16_t *w = const_cast<uint16_t *>(W.w);
-        for (int r = 0, br = 0; r < rows; r += rb, ++br)
-            for (int c = 0, bc = 0; c < cols; c += cb, ++bc) {
-                rc = copy(w + (size_t)(row0 + br * rp) * W.Kp + (size_t)bc * cp, (size_t)W.Kp * 2, reinterpret_cast<const uint8_t *>(d) + ((size_t)r * cols + c) * 2, (size_t)cols * 2,
-                          (size_t)cb * 2, (size_t)rb);
-                if (rc != MESH_OK) return rc;
-            }
-        return MESH_OK;
-    }
-    int matrix(LinearWeight &W, const std::string &name, int M, int K) {
-        int rc = matrix_alloc(W, M, K);
-        return rc != MESH_OK ? rc : place(W, name, M, K, 0, M, M, K, K);
-    }
-    // output norm (one number) times the layer scale
-    int gain(const std::string &norm, const std::string &scale, int n, float **out) {
-        std::vector<float> g, s;
-        int rc;
-        if ((rc = floats(norm, {}, g)) || (rc = floats(scale, {(uint64_t)n}, s))) return rc;
-        for (float &v : s) v *= g[0];
-        return upload(s, out);
-    }
-    int head_norm(const std::string &name, int heads, int dim, int pad, float **out) {
-        std::vector<float> g, p((size_t)heads * pad, 0.f);
-        int rc = floats(name, {(uint64_t)heads * dim}, g);
-        if (rc != MESH_OK) return rc;
-        for (int h = 0; h < heads; ++h)
-            for (int i = 0; i < dim; ++i) p[(size_t)h * pad + i] = g[(size_t)h * dim + i];
-        return upload(p, out);
-    }
-    int layer(HybridLayer &L, const ModelSpec &s, int index) {
-        const std::string p = "l" + std::to_string(index) + ".", mx = p + "mix.";
-        const MixerSpec &m = L.spec.mixer;
-        const int E = s.width;
-        int rc;
-        if (m.kind == MIXER_ATTENTION) {
-            L.head_pad = m.dim <= 64 ? 64 : m.dim <= 128 ? 128 : 256;
-            if (m.dim > 256) return fail(MESH_ERR_UNSUPPORTED, "layer %d: attention heads of %d entries have no kernel (256 at most)", index, m.dim);
-            const int HP = m.heads * L.head_pad, GP = m.kv_heads * L.head_pad;
-            if ((rc = matrix_alloc(L.in, HP + GP, E)) || (rc = place(L.in, mx + "q", m.heads * m.dim, E, 0, m.dim, L.head_pad, E, E)) ||
-                (rc = place(L.in, mx + "k", m.kv_heads * m.dim, E, HP, m.dim, L.head_pad, E, E)) ||
-                (rc = head_norm(mx + "q.norm", m.heads, m.dim, L.head_pad, &L.q_norm)) || (rc = head_norm(mx + "k.norm", m.kv_heads, m.dim, L.head_pad, &L.k_norm)) ||
-                (rc = matrix_alloc(L.out, E, HP)) || (rc = place(L.out, mx + "o", E, m.heads * m.dim, 0, E, E, m.dim, L.head_pad)))
-                return rc;
-        } else {
-            const int W = m.width;
-            std::vector<float> bz, bx;
-            if ((rc = matrix_alloc(L.in, 3 * W, E)) || (rc = place(L.in, mx + "z", W, E, 0, W, W, E, E)) || (rc = place(L.in, mx + "x", W, E, W, W, W, E, E)) ||
-                (rc = place(L.in, mx + "g", W, E, 2 * W, W, W, E, E)) || (rc = floats(mx + "z.b", {(uint64_t)W}, bz)) || (rc = floats(mx + "x.b", {(uint64_t)W}, bx)) ||
-                (rc = upload(bz, &L.bias_z)) || (rc = upload(bx, &L.bias_x)) || (rc = matrix(L.out, mx + "o", E, W)))
-                return rc;
-        }
-        if ((rc = gain(p + "norm1", p + "ls1", E, &L.gain1)) != MESH_OK) return rc;
-        if (L.spec.ff) {
-            std::vector<float> c;
-            if ((rc = matrix(L.up, p + "mlp.up", L.spec.ff, E)) || (rc = matrix(L.down, p + "mlp.down", E, L.spec.ff)) || (rc = floats(p + "mlp.act", {4}, c)) ||
-                (rc = upload(c, &L.coef)) || (rc = gain(p + "norm2", p + "ls2", E, &L.gain2)))
-                return rc;
-        }
-        std::vector<float> g;
-        if ((rc = matrix(L.side_gate, p + "side.gate", s.side_dim, E)) || (rc = matrix(L.side_proj, p + "side.proj", E, s.side_dim)) ||
-            (rc = floats(p + "side.norm", {(uint64_t)E}, g)) || (rc = upload(g, &L.gain_side)))
-            return rc;
-        return MESH_OK;
-    }
-};
-
-}  // namespace
-
-int hybrid_open(const char *folder, int layer_begin, int layer_end, const mesh_stage_opts *opts, mesh_stage *st) {
-    st->hybrid.reset(new HybridModel());
-    HybridModel &hm = *st->hybrid;
-    ModelSpec &s = hm.spec;
-    int rc = model_spec_from_folder(folder, s);
-    if (rc != MESH_OK) return rc;
-    hparams_from_spec(s, st->hp);
-    const int n_layer = (int)s.layers.size();
-    if (layer_end < 0) layer_end = n_layer;
-    if (layer_begin < 0 || layer_begin >= layer_end || layer_end > n_layer)
-        return fail(MESH_ERR_INVALID, "mesh_stage_open: layer range [%d,%d) does not fit a %d-layer model", layer_begin, layer_end, n_layer);
-    st->layer_begin = layer_begin;
-    st->layer_end = layer_end;
-    if (opts && (opts->kv_type || opts->kv_type_v))
-        return fail(MESH_ERR_UNSUPPORTED, "mesh_stage_open: the cache rows of architecture '%s' follow its precision (no kv_type)", s.arch.c_str());
-    hm.act = opts && opts->precision == MESH_PRECISION_F32 ? ACT_F32 : ACT_BF16;
-    st->k_type = st->v_type = hm.act == ACT_F32 ? MESH_F32 : MESH_F16;
-    SafetensorsFile f;
-    if ((rc = f.open((std::string(folder) + "/model.safetensors").c_str())) != MESH_OK) return rc;
-    if ((rc = stage_select_device(opts, st)) != MESH_OK) return rc;
-
-    FolderLoader ld{f, *st};
-    const int E = s.width;
-    hm.width_pad = linear_k_padded(E);
-    hm.layers.resize((size_t)(layer_end - layer_begin));
-    for (int i = layer_begin; i < layer_end; ++i) {
-        HybridLayer &L = hm.layers[(size_t)(i - layer_begin)];
-        L.spec = s.layers[(size_t)i];
-        if ((rc = ld.layer(L, s, i)) != MESH_OK) return rc;
-        hm.in_max = std::max({hm.in_max, L.in.M, L.up.M, L.side_gate.M * LINEAR_SLICES_MAX});
-        hm.act_max = std::max({hm.act_max, L.out.Kp, L.down.Kp, L.side_proj.Kp});
-        if (L.spec.mixer.kind == MIXER_ATTENTION) hm.q_max = std::max(hm.q_max, L.spec.mixer.heads * L.head_pad);
-        else { hm.has_state = true; hm.state_max = std::max(hm.state_max, L.spec.mixer.width); }
-        for (const LinearWeight *w : {&L.in, &L.out, &L.up, &L.down, &L.side_gate, &L.side_proj})
-            if (w->present() && !linear_step_supported(*w)) hm.step_ok = false;
-    }
-    if ((rc = ld.raw("side.embed", {(uint64_t)s.vocab, (uint64_t)n_layer * s.side_dim}, &hm.side)) != MESH_OK) return rc;
-    if (layer_begin == 0) {
-        if ((rc = ld.raw("embed", {(uint64_t)s.vocab, (uint64_t)E}, &hm.embed)) != MESH_OK) return rc;
-        std::vector<float> fr((size_t)(E + 1) / 2);
-        for (size_t i = 0; i < fr.size(); ++i) fr[i] = (float)pow(10000.0, -2.0 * (double)i / E);
-        if ((rc = ld.upload(fr, &hm.freq)) != MESH_OK) return rc;
-        st->tok_embd.data = hm.embed; st->tok_embd.K = E; st->tok_embd.M = s.vocab;
-    }
-    if (layer_end == n_layer) {
-        std::vector<float> g;
-        if ((rc = ld.floats("final.norm", {}, g)) || (rc = ld.upload(g, &hm.final_gain)) || (rc = ld.matrix(hm.head, "head", s.vocab, E))) return rc;
-        if (!linear_step_supported(hm.head)) hm.step_ok = false;
-        st->output.data = const_cast<uint16_t *>(hm.head.w); st->output.K = E; st->output.M = s.vocab;
-    }
-    MESH_HIP_TRY(hipDeviceSynchronize());
-    return MESH_OK;
-}
 
 // ------------------------------------------------------------------------------------------------ session
 int hybrid_session_alloc(mesh_session *s) {
@@ -247,26 +34,36 @@ int hybrid_session_alloc(mesh_session *s) {
     h.part = fbuf(2 * 3 * STEP_PARTS_MAX);
     h.ws = fbuf(hm.state_max ? min_gru_workspace((int)B, hm.state_max) : 0);
     s->attn_part_rows = std::max<size_t>(B, 512);
-    if (hm.q_max) {
+    if (hm.part_max) {
         int heads = 0;
         for (const HybridLayer &L : hm.layers) heads = std::max(heads, L.spec.mixer.heads);
-        s->attn_part = fbuf(s->attn_part_rows * (size_t)hm.q_max);
+        s->attn_part = fbuf(s->attn_part_rows * hm.part_max);
         s->attn_ml = fbuf(s->attn_part_rows * (size_t)heads * 2);
     }
+    h.qx = buf(B * hm.qx_max);
+    h.kvx = fbuf(B * hm.kvx_max);
+    h.kv16 = static_cast<uint16_t *>(buf((size_t)st->n_ctx * hm.kv16_max * 2));
+    h.chunk_cap = (int)B / STATE_CHUNK + std::min((int)B, st->n_seq_max) + 1;        // (a sequence's tokens leave one chunk that is not whole)
+    h.gated_ws = fbuf((size_t)(hm.has_chunks ? h.chunk_cap : 0) * hm.gated_ws_max);
     void *sat = buf(256);
     s->f16_sat = static_cast<unsigned *>(sat);
     for (const HybridLayer &L : hm.layers) {
         const MixerSpec &m = L.spec.mixer;
         uint8_t *k = nullptr, *v = nullptr;
-        float *state = nullptr;
+        float *state = nullptr, *tail = nullptr;
         if (m.kind == MIXER_ATTENTION) {
             const size_t bytes = (size_t)st->n_seq_max * m.kv_heads * (size_t)st->n_ctx * (size_t)kv_row_bytes(st->k_type, L.head_pad);
             k = static_cast<uint8_t *>(buf(bytes));
             v = static_cast<uint8_t *>(buf(bytes));
+        } else if (m.kind == MIXER_LATENT) {
+            if (m.kv_from < 0) k = static_cast<uint8_t *>(buf((size_t)st->n_seq_max * (size_t)st->n_ctx * L.latent.row() * (hm.act == ACT_F32 ? 4 : 2)));
+        } else if (m.has_matrix_state()) {
+            state = fbuf((size_t)st->n_seq_max * m.heads * m.dim * m.vdim);
+            if (L.gated.delta) tail = fbuf((size_t)st->n_seq_max * m.taps * gated_state_channels(L.gated));
         } else {
             state = fbuf((size_t)st->n_seq_max * m.width);
         }
-        h.k.push_back(k); h.v.push_back(v); h.state.push_back(state);
+        h.k.push_back(k); h.v.push_back(v); h.state.push_back(state); h.tail.push_back(tail);
     }
     h.seq_len.assign((size_t)st->n_seq_max, 0);
     return rc;
@@ -296,6 +93,26 @@ void hybrid_note_batch(mesh_session *s, const mesh_batch *b, bool ok) {
     for (int i = 0; i < b->n_tokens; ++i) s->hybrid->seq_len[(size_t)(b->seq_id ? b->seq_id[i] : 0)] = ok ? b->pos[i] + 1 : -1;
 }
 
+bool hybrid_needs_ids(const mesh_stage *st) { return st->hybrid->side(); }
+
+size_t hybrid_chunk_table(mesh_session *s, const mesh_batch *b, int32_t *table, const int32_t *d_table) {
+    HybridSession &h = *s->hybrid;
+    if (!s->stage->hybrid->has_chunks) return 0;
+    const size_t B = (size_t)s->stage->n_batch_max;
+    int32_t *chunk = table, *first = chunk + B + 1, *run = first + B;
+    int nc = 0, nr = 0, start = 0;
+    for (int i = 0; i < b->n_tokens; ++i) {
+        const bool opens = i == 0 || (b->seq_id && b->seq_id[i] != b->seq_id[i - 1]);
+        if (opens) { start = i; run[nr++] = nc; }
+        if (opens || (i - start) % STATE_CHUNK == 0) { chunk[nc] = i; first[nc++] = start; }
+    }
+    chunk[nc] = b->n_tokens;
+    run[nr] = nc;
+    h.chunks.chunk = d_table; h.chunks.first = d_table + B + 1; h.chunks.run = h.chunks.first + B;
+    h.chunks.n_chunks = nc; h.chunks.n_runs = nr;
+    return nr == b->n_tokens ? 0 : 2 * B + 1 + (size_t)nr + 1;
+}
+
 // ------------------------------------------------------------------------------------------------ layers
 bool hybrid_single_step(const mesh_session *s, int T) { return T == 1 && s->tune.step_fused && s->stage->hybrid->step_ok; }
 
@@ -305,17 +122,23 @@ static int layer_splits(const mesh_session *s, const MixerSpec &m, int T, int ma
     return T < 64 ? attn_splits_for(s->tune, T, m.kv_heads, keys_seen(m, max_keys), false) : 1;
 }
 
+static int latent_splits(const mesh_session *s, const LatentShape &ls, int T, int max_keys) { return attn_splits_for(s->tune, T, latent_head_tiles(ls), max_keys, false); }
+
 uint64_t hybrid_graph_key(const mesh_session *s, int T, int max_keys) {
     uint64_t key = 1469598103934665603ull ^ (uint64_t)T;
-    for (const HybridLayer &L : s->stage->hybrid->layers)
-        if (L.spec.mixer.kind == MIXER_ATTENTION) key = (key ^ (uint64_t)layer_splits(s, L.spec.mixer, T, max_keys)) * 1099511628211ull;
+    auto mix = [&](uint64_t v) { key = (key ^ v) * 1099511628211ull; };
+    for (const HybridLayer &L : s->stage->hybrid->layers) {
+        if (L.spec.mixer.kind == MIXER_ATTENTION) mix((uint64_t)layer_splits(s, L.spec.mixer, T, max_keys));
+        if (L.spec.mixer.kind == MIXER_LATENT) mix((uint64_t)latent_splits(s, L.latent, T, max_keys));
+    }
+    if (s->stage->hybrid->has_chunks) mix(((uint64_t)s->hybrid->chunks.n_chunks << 32) | (uint64_t)s->hybrid->chunks.n_runs);
     return key;
 }
 
 int hybrid_embed(mesh_session *s, int T) {
     const HybridModel &hm = *s->stage->hybrid;
     ProfScope ps(s, MESH_PROF_CODEC);
-    return embed_rows(hm.embed, s->d_tok, s->d_pos, hm.freq, hm.spec.embed_scale, T, hm.spec.width, s->x, s->stream);
+    return embed_rows(hm.embed, hm.embed_ld, s->d_tok, s->d_pos, hm.freq, hm.spec.embed_scale, T, hm.spec.width, s->x, s->stream);
 }
 
 // q, k of the call in h.big -> attention output in h.acta: f32 rows for the single-token step, else the product's activations
@@ -353,6 +176,107 @@ static int run_attention(mesh_session *s, size_t il, int T, int max_keys, bool f
     return attention(aa, T, s->stream);
 }
 
+// What the layer's recurrence needs beside its weights.
+static GatedStateArgs gated_args(mesh_session *s, size_t il, void *out, ActType act) {
+    HybridSession &h = *s->hybrid;
+    GatedStateArgs a = s->stage->hybrid->layers[il].gated;
+    a.in = h.big; a.state = h.state[il]; a.tail = h.tail[il]; a.pos = s->d_pos; a.seq = s->d_seq;
+    a.chunks = h.chunks; a.ws = h.gated_ws; a.o = h.q; a.out = out; a.act = act;
+    return a;
+}
+
+static LatentCache latent_cache(mesh_session *s, size_t il) {
+    const HybridModel &hm = *s->stage->hybrid;
+    HybridSession &h = *s->hybrid;
+    const HybridLayer &L = hm.layers[il];
+    LatentCache c;
+    c.rows = h.k[(size_t)L.cache_layer]; c.n_ctx = s->stage->n_ctx;
+    if (L.own_cache((int)il)) { c.in = h.big + L.spec.mixer.q_rank; c.ld = L.in.M; c.gain = L.c_norm; }
+    c.rot = L.rot; c.pos = s->d_pos; c.seq = s->d_seq; c.sat = s->f16_sat; c.eps = hm.spec.eps;
+    return c;
+}
+
+// queries in h.q, this call's rows in the cache unless `append` -> attention output in h.acta (f32 rows for the single-token
+// step, else the product's activations)
+static int run_latent_rows(mesh_session *s, size_t il, int T, int max_keys, bool append, bool f32_out) {
+    mesh_stage *st = s->stage;
+    const HybridModel &hm = *st->hybrid;
+    HybridSession &h = *s->hybrid;
+    const HybridLayer &L = hm.layers[il];
+    const MixerSpec &m = L.spec.mixer;
+    const LatentCache c = latent_cache(s, il);
+    int rc;
+    {
+        ProfScope ps(s, MESH_PROF_ROPE);
+        if ((rc = latent_query(L.latent, c, hm.act, h.q, L.w_uk_t, m.scale, append && c.in, h.qx, T, s->stream)) != MESH_OK) return rc;
+    }
+    LatentAttnArgs a;
+    a.qa = h.qx; a.rows = c.rows; a.pos = s->d_pos; a.seq = s->d_seq; a.part = s->attn_part; a.ml = s->attn_ml; a.n_ctx = st->n_ctx;
+    a.n_splits = latent_splits(s, L.latent, T, max_keys);
+    a.w_uv = L.w_uv; a.gate = h.big + L.in.M - m.heads; a.gate_ld = L.in.M;
+    if (f32_out || hm.act == ACT_F32) a.out = static_cast<float *>(h.acta);
+    else a.out_bf16 = static_cast<uint16_t *>(h.acta);
+    ProfScope ps(s, MESH_PROF_ATTN);
+    if ((rc = latent_attention(L.latent, a, hm.act, T, s->stream)) != MESH_OK) return rc;
+    return latent_out(L.latent, a, T, s->stream);
+}
+
+// the same for a long chunk of one sequence: keys and values of all its positions are projected, then attended to
+static int run_latent_chunk(mesh_session *s, size_t il, int T) {
+    mesh_stage *st = s->stage;
+    const HybridModel &hm = *st->hybrid;
+    HybridSession &h = *s->hybrid;
+    const HybridLayer &L = hm.layers[il];
+    const LatentShape &ls = L.latent;
+    const void *rows = h.k[(size_t)L.cache_layer];
+    uint16_t *k16 = h.kv16, *v16 = k16 + (size_t)ls.heads * st->n_ctx * ls.chunk_k;
+    int rc;
+    {
+        ProfScope ps(s, MESH_PROF_ROPE);
+        if ((rc = latent_chunk_query(ls, L.rot, h.q, s->d_pos, static_cast<float *>(h.qx), T, s->stream)) != MESH_OK) return rc;
+    }
+    const int n_keys = s->chunk_pos0 + T;
+    for (int k0 = 0; k0 < n_keys; k0 += st->n_batch_max) {
+        const int n = std::min(st->n_batch_max, n_keys - k0);
+        {
+            ProfScope ps(s, MESH_PROF_PREP);
+            if ((rc = latent_chunk_rows(ls, rows, st->n_ctx, s->chunk_seq, k0, n, static_cast<uint16_t *>(h.acta), L.ukv.Kp, s->stream)) != MESH_OK) return rc;
+        }
+        {
+            ProfScope ps(s, MESH_PROF_GEMV);
+            if ((rc = linear(L.ukv, h.acta, ACT_BF16, n, h.kvx, L.ukv.M, s->tune.linear_tile_min_tokens, s->stream)) != MESH_OK) return rc;
+        }
+        ProfScope ps(s, MESH_PROF_PREP);
+        if ((rc = latent_chunk_pack(ls, rows, st->n_ctx, s->chunk_seq, k0, n, h.kvx, k16, v16, s->f16_sat, s->stream)) != MESH_OK) return rc;
+    }
+    AttnArgs a;
+    a.q = static_cast<const float *>(h.qx); a.kcache = reinterpret_cast<const uint8_t *>(k16); a.vcache = reinterpret_cast<const uint8_t *>(v16);
+    a.part = s->attn_part; a.ml = s->attn_ml; a.part_rows = s->tune.attn_chunk_ksplit ? s->attn_part_rows : 0;
+    a.out_bf16 = static_cast<uint16_t *>(h.acta);
+    a.scale = L.spec.mixer.scale;
+    a.n_head = a.n_kv = ls.heads; a.head_dim = ls.chunk_k; a.v_dim = ls.chunk_v; a.n_ctx = st->n_ctx;
+    a.head_gate = h.big + L.in.M - ls.heads; a.gate_ld = L.in.M;
+    ProfScope ps(s, MESH_PROF_ATTN);
+    return attention_chunk(a, T, s->chunk_pos0, 0, s->stream);
+}
+
+static int run_latent(mesh_session *s, size_t il, int T, int max_keys) {
+    const HybridModel &hm = *s->stage->hybrid;
+    HybridSession &h = *s->hybrid;
+    const HybridLayer &L = hm.layers[il];
+    int rc;
+    {
+        ProfScope ps(s, MESH_PROF_PREP);
+        if ((rc = latent_rows(L.latent, latent_cache(s, il), hm.act, h.big, L.in.M, L.cq_norm, L.spec.mixer.q_rank, h.acta, L.uq.Kp, T, s->stream)) != MESH_OK) return rc;
+    }
+    {
+        ProfScope ps(s, MESH_PROF_GEMV);
+        if ((rc = linear(L.uq, h.acta, hm.act, T, h.q, L.uq.M, s->tune.linear_tile_min_tokens, s->stream)) != MESH_OK) return rc;
+    }
+    if (L.ukv.present() && s->chunk_pos0 >= 0 && T >= s->tune.latent_chunk_min_tokens) return run_latent_chunk(s, il, T);
+    return run_latent_rows(s, il, T, max_keys, false, false);
+}
+
 // One token: every product derives its input from what the launch before it left (linear.hpp).
 static int run_step(mesh_session *s, int max_keys) {
     mesh_stage *st = s->stage;
@@ -363,67 +287,90 @@ static int run_step(mesh_session *s, int max_keys) {
     HybridPending pend;
     pend.x = s->x;
     int set = 0, rc;
+    const bool ln = hm.spec.out_norm == NORM_LAYER;
     auto base = [&](const LinearWeight &W, float *out, StepOut kind) {
         StepArgs a;
         a.W = W; a.eps = hm.spec.eps; a.out = out; a.out_kind = kind;
         a.pos = s->d_pos; a.seq = s->d_seq; a.tok = s->d_tok;
         return a;
     };
+    auto run = [&](const StepArgs &a) {
+        ProfScope ps(s, MESH_PROF_GEMV);
+        return linear_step(a, stream);
+    };
     // a product that reads the residual stream, completing it first
-    auto from_stream = [&](StepArgs a) {
+    auto from_stream = [&](StepArgs a, const RowNorm &pre) {
         a.in = pend.x;
+        if (pre.kind == NORM_LAYER) { a.in_kind = STEP_IN_LAYER; a.norm_gain = pre.gain; a.norm_bias = pre.bias; }
         if (pend.y) {
-            a.in_kind = STEP_IN_RESIDUAL;
-            a.y = pend.y; a.gain = pend.gain; a.part = pend.part; a.n_part = pend.n_part;
+            if (!ln) a.in_kind = STEP_IN_RESIDUAL;
+            a.y = pend.y; a.gain = pend.post.gain; a.bias = pend.post.bias; a.part = pend.part; a.n_part = pend.n_part;
             a.x_out = pend.x == s->x ? h.x2 : s->x;
         }
-        ProfScope ps(s, MESH_PROF_GEMV);
-        const int r = linear_step(a, stream);
+        const int r = run(a);
         if (pend.y) pend.x = a.x_out;
         pend.y = nullptr;
         return r;
     };
     // a sublayer's last product: its result waits to be normed and added
-    auto to_stream = [&](StepArgs a, const float *gain) {
-        a.out = h.y; a.out_kind = STEP_OUT_SUMSQ;
-        a.out_part = h.part + (size_t)set * 3 * STEP_PARTS_MAX;
-        set ^= 1;
-        pend.y = h.y; pend.gain = gain; pend.part = a.out_part; pend.n_part = linear_step_grid(a);
-        ProfScope ps(s, MESH_PROF_GEMV);
-        return linear_step(a, stream);
+    auto to_stream = [&](StepArgs a, const RowNorm &post) {
+        a.out = h.y;
+        pend.y = h.y; pend.post = post;
+        if (!ln) {
+            a.out_kind = STEP_OUT_SUMSQ;
+            a.out_part = h.part + (size_t)set * 3 * STEP_PARTS_MAX;
+            set ^= 1;
+            pend.part = a.out_part; pend.n_part = linear_step_grid(a);
+        }
+        return run(a);
     };
     for (size_t il = 0; il < hm.layers.size(); ++il) {
         const HybridLayer &L = hm.layers[il];
-        if (L.spec.mixer.kind == MIXER_ATTENTION) {
-            if ((rc = from_stream(base(L.in, h.big, STEP_OUT_PLAIN))) != MESH_OK) return rc;
-            if ((rc = run_attention(s, il, 1, max_keys, true)) != MESH_OK) return rc;
-        } else {
+        const MixerSpec &m = L.spec.mixer;
+        if (m.kind == MIXER_MIN_GRU) {
             StepArgs a = base(L.in, inner, STEP_OUT_MIN_GRU);
-            a.width = L.spec.mixer.width; a.bias_z = L.bias_z; a.bias_x = L.bias_x; a.state = h.state[il];
-            if ((rc = from_stream(a)) != MESH_OK) return rc;
+            a.width = m.width; a.bias_z = L.bias_z; a.bias_x = L.bias_x; a.state = h.state[il];
+            if ((rc = from_stream(a, L.pre1)) != MESH_OK) return rc;
+        } else {
+            if ((rc = from_stream(base(L.in, h.big, STEP_OUT_PLAIN), L.pre1)) != MESH_OK) return rc;
+            if (m.kind == MIXER_ATTENTION) {
+                if ((rc = run_attention(s, il, 1, max_keys, true)) != MESH_OK) return rc;
+            } else if (m.kind == MIXER_LATENT) {
+                StepArgs q = base(L.uq, h.q, STEP_OUT_PLAIN);
+                q.in_kind = STEP_IN_UNIT_RMS; q.in = h.big; q.gain = L.cq_norm;
+                if ((rc = run(q)) != MESH_OK || (rc = run_latent_rows(s, il, 1, max_keys, true, true)) != MESH_OK) return rc;
+            } else {
+                ProfScope ps(s, MESH_PROF_PREP);
+                if ((rc = gated_state_step(gated_args(s, il, inner, ACT_F32), 1, stream)) != MESH_OK) return rc;
+            }
         }
-        StepArgs o = base(L.out, nullptr, STEP_OUT_SUMSQ);
+        StepArgs o = base(L.out, nullptr, STEP_OUT_PLAIN);
         o.in = inner;
-        if ((rc = to_stream(o, L.gain1)) != MESH_OK) return rc;
+        if ((rc = to_stream(o, L.post1)) != MESH_OK) return rc;
         if (L.spec.ff) {
-            StepArgs u = base(L.up, h.big, STEP_OUT_POWERS);
-            u.out_part = h.part + (size_t)set * 3 * STEP_PARTS_MAX;
-            const float *powers = u.out_part;
-            const int n_powers = linear_step_grid(u);
-            set ^= 1;
-            if ((rc = from_stream(u)) != MESH_OK) return rc;
-            StepArgs d = base(L.down, nullptr, STEP_OUT_SUMSQ);
-            d.in_kind = STEP_IN_POLY; d.in = h.big; d.part = powers; d.n_part = n_powers; d.coef = L.coef;
-            if ((rc = to_stream(d, L.gain2)) != MESH_OK) return rc;
+            StepArgs u = base(L.up, h.big, STEP_OUT_PLAIN), d = base(L.down, nullptr, STEP_OUT_PLAIN);
+            d.in = h.big;
+            if (hm.spec.ff == FF_POLY_NORM) {
+                u.out_kind = STEP_OUT_POWERS;
+                u.out_part = h.part + (size_t)set * 3 * STEP_PARTS_MAX;
+                set ^= 1;
+                d.in_kind = STEP_IN_POLY; d.part = u.out_part; d.n_part = linear_step_grid(u); d.coef = L.coef;
+            } else {
+                u.out = inner;
+                d.in_kind = STEP_IN_RELU2; d.in = inner;
+            }
+            if ((rc = from_stream(u, L.pre2)) != MESH_OK || (rc = to_stream(d, L.post2)) != MESH_OK) return rc;
         }
-        StepArgs g = base(L.side_gate, inner, STEP_OUT_SIDE);
-        g.side = hm.side; g.side_stride = (int)hm.spec.layers.size() * hm.spec.side_dim; g.side_offset = (st->layer_begin + (int)il) * hm.spec.side_dim;
-        if ((rc = from_stream(g)) != MESH_OK) return rc;
-        StepArgs p = base(L.side_proj, nullptr, STEP_OUT_SUMSQ);
-        p.in = inner;
-        if ((rc = to_stream(p, L.gain_side)) != MESH_OK) return rc;
+        if (hm.side()) {
+            StepArgs g = base(L.side_gate, inner, STEP_OUT_SIDE);
+            g.side = hm.side_embed; g.side_stride = (int)hm.spec.layers.size() * hm.spec.side_dim; g.side_offset = (st->layer_begin + (int)il) * hm.spec.side_dim;
+            if ((rc = from_stream(g, RowNorm{})) != MESH_OK) return rc;
+            StepArgs p = base(L.side_proj, nullptr, STEP_OUT_PLAIN);
+            p.in = inner;
+            if ((rc = to_stream(p, L.post_side)) != MESH_OK) return rc;
+        }
     }
-    h.tail = pend;
+    h.tail_step = pend;
     return MESH_OK;
 }
 
@@ -441,20 +388,25 @@ int hybrid_run_layers(mesh_session *s, int T, int max_keys) {
         ProfScope ps(s, MESH_PROF_GEMV);
         return linear(W, x, act, T, y, ldy, s->tune.linear_tile_min_tokens, stream);
     };
-    auto add = [&](const float *gain) {
+    // the residual stream after a sublayer, and the next one's input
+    auto add = [&](const float *y, const RowNorm &post, const RowNorm &pre) {
         ProfScope ps(s, MESH_PROF_PREP);
-        return residual_norm_rows(s->x, h.y, gain, eps, T, E, h.xa, act, hm.width_pad, stream);
+        return residual_norm_rows(s->x, y, post, pre, eps, T, E, h.xa, act, hm.width_pad, stream);
     };
-    {
-        ProfScope ps(s, MESH_PROF_PREP);
-        if ((rc = residual_norm_rows(s->x, nullptr, nullptr, eps, T, E, h.xa, act, hm.width_pad, stream)) != MESH_OK) return rc;
-    }
+    if ((rc = add(nullptr, RowNorm{}, hm.layers[0].pre1)) != MESH_OK) return rc;
     for (size_t il = 0; il < hm.layers.size(); ++il) {
         const HybridLayer &L = hm.layers[il];
         const MixerSpec &m = L.spec.mixer;
+        const RowNorm after = hm.side() || il + 1 == hm.layers.size() ? RowNorm{} : hm.layers[il + 1].pre1;
         if ((rc = product(L.in, h.xa, h.big, L.in.M)) != MESH_OK) return rc;
         if (m.kind == MIXER_ATTENTION) {
             if ((rc = run_attention(s, il, T, max_keys, false)) != MESH_OK) return rc;
+        } else if (m.kind == MIXER_LATENT) {
+            if ((rc = run_latent(s, il, T, max_keys)) != MESH_OK) return rc;
+        } else if (m.has_matrix_state()) {
+            const GatedStateArgs a = gated_args(s, il, h.acta, act);
+            ProfScope ps(s, MESH_PROF_PREP);
+            if ((rc = h.chunks.n_runs == T ? gated_state_step(a, T, stream) : gated_state_chunks(a, T, stream)) != MESH_OK) return rc;
         } else {
             MinGruArgs a;
             a.zxg = h.big; a.bias_z = L.bias_z; a.bias_x = L.bias_x; a.state = h.state[il]; a.pos = s->d_pos; a.seq = s->d_seq; a.ws = h.ws;
@@ -462,15 +414,19 @@ int hybrid_run_layers(mesh_session *s, int T, int max_keys) {
             ProfScope ps(s, MESH_PROF_PREP);
             if ((rc = min_gru(a, T, stream)) != MESH_OK) return rc;
         }
-        if ((rc = product(L.out, h.acta, h.y, E)) != MESH_OK || (rc = add(L.gain1)) != MESH_OK) return rc;
+        if ((rc = product(L.out, h.acta, h.y, E)) != MESH_OK || (rc = add(h.y, L.post1, L.spec.ff ? L.pre2 : after)) != MESH_OK) return rc;
         if (L.spec.ff) {
-            if ((rc = product(L.up, h.xa, h.big, L.spec.ff)) != MESH_OK) return rc;
-            {
+            if (hm.spec.ff == FF_POLY_NORM) {
+                if ((rc = product(L.up, h.xa, h.big, L.spec.ff)) != MESH_OK) return rc;
                 ProfScope ps(s, MESH_PROF_PREP);
                 if ((rc = poly_norm_rows(h.big, L.coef, eps, T, L.spec.ff, h.acta, act, L.down.Kp, stream)) != MESH_OK) return rc;
+            } else {
+                ProfScope ps(s, MESH_PROF_GEMV);
+                if ((rc = linear_relu2(L.up, h.xa, act, T, h.acta, L.down.Kp, s->tune.linear_tile_min_tokens, stream)) != MESH_OK) return rc;
             }
-            if ((rc = product(L.down, h.acta, h.y, E)) != MESH_OK || (rc = add(L.gain2)) != MESH_OK) return rc;
+            if ((rc = product(L.down, h.acta, h.y, E)) != MESH_OK || (rc = add(h.y, L.post2, after)) != MESH_OK) return rc;
         }
+        if (!hm.side()) continue;
         int slices;
         const size_t slice = (size_t)T * hm.spec.side_dim;
         {
@@ -479,11 +435,11 @@ int hybrid_run_layers(mesh_session *s, int T, int max_keys) {
         }
         {
             ProfScope ps(s, MESH_PROF_PREP);
-            if ((rc = side_gate_rows(h.big, slices, slice, hm.side, s->d_tok, (int)hm.spec.layers.size() * hm.spec.side_dim, (st->layer_begin + (int)il) * hm.spec.side_dim, T,
+            if ((rc = side_gate_rows(h.big, slices, slice, hm.side_embed, s->d_tok, (int)hm.spec.layers.size() * hm.spec.side_dim, (st->layer_begin + (int)il) * hm.spec.side_dim, T,
                                      hm.spec.side_dim, h.acta, act, L.side_proj.Kp, stream)) != MESH_OK)
                 return rc;
         }
-        if ((rc = product(L.side_proj, h.acta, h.y, E)) != MESH_OK || (rc = add(L.gain_side)) != MESH_OK) return rc;
+        if ((rc = product(L.side_proj, h.acta, h.y, E)) != MESH_OK || (rc = add(h.y, L.post_side, RowNorm{})) != MESH_OK) return rc;
     }
     return MESH_OK;
 }
@@ -493,9 +449,9 @@ int hybrid_finish(mesh_session *s, int T, float **x) {
     HybridSession &h = *s->hybrid;
     *x = s->x;
     if (!hybrid_single_step(s, T)) return MESH_OK;
-    *x = h.tail.x;
+    *x = h.tail_step.x;
     ProfScope ps(s, MESH_PROF_PREP);
-    return residual_norm_rows(h.tail.x, h.tail.y, h.tail.gain, hm.spec.eps, 1, hm.spec.width, h.xa, hm.act, hm.width_pad, s->stream);
+    return residual_norm_rows(h.tail_step.x, h.tail_step.y, h.tail_step.post, RowNorm{}, hm.spec.eps, 1, hm.spec.width, h.xa, hm.act, hm.width_pad, s->stream);
 }
 
 int hybrid_logits(mesh_session *s, int T, const int32_t *d_rows, int n_rows, float *d_out) {
@@ -505,15 +461,19 @@ int hybrid_logits(mesh_session *s, int T, const int32_t *d_rows, int n_rows, flo
     if (hybrid_single_step(s, T)) {
         StepArgs a;
         a.W = hm.head; a.in_kind = STEP_IN_RESIDUAL_NORM; a.out_kind = STEP_OUT_PLAIN;
-        a.in = h.tail.x; a.y = h.tail.y; a.gain = h.tail.gain; a.part = h.tail.part; a.n_part = h.tail.n_part;
-        a.x_out = h.tail.x == s->x ? h.x2 : s->x;
-        a.norm_gain = hm.final_gain; a.eps = hm.spec.eps; a.out = d_out;
+        a.in = h.tail_step.x; a.y = h.tail_step.y; a.gain = h.tail_step.post.gain; a.bias = h.tail_step.post.bias; a.part = h.tail_step.part; a.n_part = h.tail_step.n_part;
+        a.x_out = h.tail_step.x == s->x ? h.x2 : s->x;
+        if (hm.final_norm.kind == NORM_LAYER) { a.in_kind = STEP_IN_LAYER; a.norm_gain = hm.final_norm.gain; a.norm_bias = hm.final_norm.bias; }
+        else a.norm_gain = hm.final_gain;
+        a.eps = hm.spec.eps; a.out = d_out;
         ProfScope ps(s, MESH_PROF_GEMV);
         return linear_step(a, s->stream);
     }
     {
         ProfScope ps(s, MESH_PROF_PREP);
-        if ((rc = scalar_norm_rows(s->x, d_rows, hm.final_gain, hm.spec.eps, n_rows, hm.spec.width, h.xa, hm.act, hm.width_pad, s->stream)) != MESH_OK) return rc;
+        rc = hm.final_norm.kind == NORM_LAYER ? layer_norm_rows(s->x, d_rows, hm.final_norm, hm.spec.eps, n_rows, hm.spec.width, h.xa, hm.act, hm.width_pad, s->stream)
+                                              : scalar_norm_rows(s->x, d_rows, hm.final_gain, hm.spec.eps, n_rows, hm.spec.width, h.xa, hm.act, hm.width_pad, s->stream);
+        if (rc != MESH_OK) return rc;
     }
     ProfScope ps(s, MESH_PROF_GEMV);
     return linear(hm.head, h.xa, hm.act, n_rows, d_out, hm.head.M, s->tune.linear_tile_min_tokens, s->stream);

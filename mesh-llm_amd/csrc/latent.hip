@@ -1,0 +1,510 @@
+// See latent.hpp.
+//
+// latent_attn_kernel: a workgroup takes one (key split, 16 heads, token).  A step stages 32 cache rows in LDS, once as they
+// are and (f16) once with the latents transposed, pairs of keys as dwords, since the second product contracts over keys:
+//   S^T (32 keys x 16 heads)   = rows . Q^T        v_mfma_f32_16x16x32_f16 per 32 elements of a row
+//   O^T (rank x 16 heads)     += latents^T . P^T   the result registers of S^T are the P^T operand as they are
+// Every wave computes the scores (they are few), so that no softmax state crosses waves, and owns a quarter of the rank's
+// rows of O^T.  With f32 rows the same fragments feed v_mfma_f32_16x16x4_f32, eight per 32 elements.
+#include "latent.hpp"
+
+#include <algorithm>
+
+#include "act_math.hpp"
+#include "attn.hpp"
+
+namespace mesh {
+
+typedef _Float16 lt_h8 __attribute__((ext_vector_type(8)));
+typedef _Float16 lt_h2 __attribute__((ext_vector_type(2)));
+typedef float lt_f4 __attribute__((ext_vector_type(4)));
+typedef uint32_t lt_u4 __attribute__((ext_vector_type(4)));
+
+constexpr int LT_THREADS = 256, LT_WAVES = LT_THREADS / 64;
+constexpr int LT_KEYS = 32, LT_VPITCH = LT_KEYS / 2 + 2;      // keys per step; dwords per latent row of the transposed tile
+constexpr int LT_QUERY_TOKENS = 4;                            // tokens that share a workgroup's weight rows in latent_query
+constexpr size_t LT_LDS_MAX = 160 * 1024 - 1024;
+
+__device__ __forceinline__ float lt_exp2(float x) { return __builtin_amdgcn_exp2f(x); }
+__device__ __forceinline__ uint32_t lt_pack(float a, float b) {
+    const lt_h2 h = {(_Float16)a, (_Float16)b};
+    return __builtin_bit_cast(uint32_t, h);
+}
+__device__ __forceinline__ float lt_block_sum(float v, float *scratch) {
+#pragma unroll
+    for (int o = 32; o > 0; o >>= 1) v += __shfl_xor(v, o);
+    __syncthreads();
+    if ((threadIdx.x & 63) == 0) scratch[threadIdx.x >> 6] = v;
+    __syncthreads();
+    return scratch[0] + scratch[1] + scratch[2] + scratch[3];
+}
+// cosine and sine of position times frequency: the product and its whole turns in 64 bits, so that the angle is as exact at
+// the end of a long context as at its start
+__device__ __forceinline__ float2 lt_turn(int pos, double freq, float gain) {
+    const double turns = (double)pos * freq * 0.15915494309189535;
+    const float a = (float)((turns - rint(turns)) * 6.283185307179586);
+    return make_float2(cosf(a) * gain, sinf(a) * gain);
+}
+
+template <ActType ACT> struct LtElem;
+template <> struct LtElem<ACT_BF16> { typedef uint16_t type; };       // f16 bits
+template <> struct LtElem<ACT_F32> { typedef float type; };
+template <ActType ACT> __device__ __forceinline__ void lt_put(void *p, size_t at, float v, unsigned *sat) {
+    if constexpr (ACT == ACT_F32) static_cast<float *>(p)[at] = v;
+    else {
+        note_f16_clamp(sat, v, 0.f);
+        static_cast<uint16_t *>(p)[at] = f32_to_f16_bits(fminf(fmaxf(v, -65504.f), 65504.f));
+    }
+}
+
+// one workgroup: the cache row of token t
+template <ActType ACT>
+__device__ __forceinline__ void lt_append(const LatentShape &s, const LatentCache &c, int t, float *scratch) {
+    const float *p = c.in + (size_t)t * c.ld;
+    const int pos = c.pos[t];
+    const size_t at = ((size_t)c.seq[t] * c.n_ctx + pos) * s.row();
+    float ss = 0.f;
+    for (int i = threadIdx.x; i < s.rank; i += LT_THREADS) ss = fmaf(p[i], p[i], ss);
+    const float r = 1.0f / sqrtf(lt_block_sum(ss, scratch) / (float)s.rank + c.eps);
+    for (int i = threadIdx.x; i < s.rank_pad; i += LT_THREADS) lt_put<ACT>(c.rows, at + i, i < s.rank ? p[i] * r * c.gain[i] : 0.f, c.sat);
+    for (int i = threadIdx.x; i < s.rot_pad / 2; i += LT_THREADS) {
+        float u = 0.f, v = 0.f;
+        if (2 * i < s.rot_dim) {
+            const float2 w = lt_turn(pos, c.rot.freq[i], c.rot.gain);
+            const float x = p[s.rank + 2 * i], y = p[s.rank + 2 * i + 1];
+            u = x * w.x - y * w.y;
+            v = y * w.x + x * w.y;
+        }
+        lt_put<ACT>(c.rows, at + s.rank_pad + 2 * i, u, c.sat);
+        lt_put<ACT>(c.rows, at + s.rank_pad + 2 * i + 1, v, c.sat);
+    }
+}
+
+template <ActType ACT>
+__global__ __launch_bounds__(LT_THREADS) void latent_rows_kernel(const LatentShape s, const LatentCache c, const float *in, int ld, const float *gain, int n, void *out, int ld_out) {
+    __shared__ float scratch[LT_WAVES];
+    const int t = blockIdx.x;
+    const float *p = in + (size_t)t * ld;
+    float ss = 0.f;
+    for (int i = threadIdx.x; i < n; i += LT_THREADS) ss = fmaf(p[i], p[i], ss);
+    const float r = 1.0f / sqrtf(lt_block_sum(ss, scratch) / (float)n + c.eps);
+    for (int i = threadIdx.x; i < ld_out; i += LT_THREADS) {
+        const float v = i < n ? p[i] * r * gain[i] : 0.f;
+        if constexpr (ACT == ACT_BF16) static_cast<uint16_t *>(out)[(size_t)t * ld_out + i] = f32_to_bf16_bits(v);
+        else static_cast<float *>(out)[(size_t)t * ld_out + i] = v;
+    }
+    if (c.in) lt_append<ACT>(s, c, t, scratch);
+}
+
+// eight bf16 weights times eight floats of LDS
+__device__ __forceinline__ float lt_dot8(const uint4 &w, const float *x, float acc) {
+    const uint32_t u[4] = {w.x, w.y, w.z, w.w};
+    const float4 xa = *reinterpret_cast<const float4 *>(x), xb = *reinterpret_cast<const float4 *>(x + 4);
+    const float xf[8] = {xa.x, xa.y, xa.z, xa.w, xb.x, xb.y, xb.z, xb.w};
+#pragma unroll
+    for (int j = 0; j < 8; ++j) acc = fmaf(__uint_as_float((j & 1) ? (u[j >> 1] & 0xFFFF0000u) : (u[j >> 1] << 16)), xf[j], acc);
+    return acc;
+}
+
+// grid (heads, or one more that appends; slices of the rank; groups of TB tokens).  Eight lanes per weight row.
+template <ActType ACT, int TB>
+__global__ __launch_bounds__(LT_THREADS) void latent_query_kernel(const LatentShape s, const LatentCache c, const float *q, const uint16_t *w, float scale, void *qa, int T) {
+    extern __shared__ __align__(16) uint8_t smem[];
+    __shared__ float scratch[LT_WAVES];
+    const int h = blockIdx.x, t0 = blockIdx.z * TB, tid = threadIdx.x;
+    if (h == s.heads) {
+        if (blockIdx.y == 0)
+            for (int t = t0; t < t0 + TB && t < T; ++t) lt_append<ACT>(s, c, t, scratch);
+        return;
+    }
+    float *xs = reinterpret_cast<float *>(smem);          // [TB][dim_pad]
+    const int D = s.dim, P = s.rot_dim, row_q = s.heads * (D + P);
+    const float qs = scale * 1.44269504088896341f;
+    for (int i = tid; i < TB * s.dim_pad; i += LT_THREADS) {
+        const int b = i / s.dim_pad, d = i % s.dim_pad;
+        xs[i] = d < D && t0 + b < T ? q[(size_t)(t0 + b) * row_q + h * (D + P) + d] * qs : 0.f;
+    }
+    if (blockIdx.y == 0) {
+        for (int i = tid; i < TB * (s.rot_pad / 2); i += LT_THREADS) {
+            const int b = i / (s.rot_pad / 2), pr = i % (s.rot_pad / 2), t = t0 + b;
+            if (t >= T) break;
+            float u = 0.f, v = 0.f;
+            if (2 * pr < P) {
+                const float2 cs = lt_turn(c.pos[t], c.rot.freq[pr], c.rot.gain);
+                const float *p = q + (size_t)t * row_q + h * (D + P) + D + 2 * pr;
+                u = (p[0] * cs.x - p[1] * cs.y) * qs;
+                v = (p[1] * cs.x + p[0] * cs.y) * qs;
+            }
+            const size_t at = ((size_t)t * s.heads + h) * s.row() + s.rank_pad + 2 * pr;
+            lt_put<ACT>(qa, at, u, c.sat);
+            lt_put<ACT>(qa, at + 1, v, c.sat);
+        }
+    }
+    __syncthreads();
+    const int per = (s.rank_pad + gridDim.y - 1) / gridDim.y, r1 = min((int)(blockIdx.y + 1) * per, s.rank_pad);
+    const int piece = tid & 7, pieces = s.dim_pad / 8;
+    for (int r0 = blockIdx.y * per; r0 < r1; r0 += LT_THREADS / 8) {
+        const int r = r0 + (tid >> 3), rr = r < r1 ? r : r1 - 1;
+        float acc[TB];
+#pragma unroll
+        for (int b = 0; b < TB; ++b) acc[b] = 0.f;
+        for (int p = piece; p < pieces; p += 8) {
+            const uint4 wv = *reinterpret_cast<const uint4 *>(w + ((size_t)h * s.rank_pad + rr) * s.dim_pad + p * 8);
+#pragma unroll
+            for (int b = 0; b < TB; ++b) acc[b] = lt_dot8(wv, xs + b * s.dim_pad + p * 8, acc[b]);
+        }
+#pragma unroll
+        for (int b = 0; b < TB; ++b) {
+            float v = acc[b];
+            v += __shfl_xor(v, 1); v += __shfl_xor(v, 2); v += __shfl_xor(v, 4);
+            if (piece == 0 && r < r1 && t0 + b < T) lt_put<ACT>(qa, ((size_t)(t0 + b) * s.heads + h) * s.row() + r, v, c.sat);
+        }
+    }
+}
+
+// ---- attention over cache rows
+template <ActType ACT> struct LtFrag;
+template <> struct LtFrag<ACT_BF16> {
+    lt_h8 v;
+    __device__ __forceinline__ void load(const uint16_t *p) { v = __builtin_bit_cast(lt_h8, *reinterpret_cast<const uint4 *>(p)); }
+};
+template <> struct LtFrag<ACT_F32> {
+    float4 a, b;
+    __device__ __forceinline__ void load(const float *p) { a = *reinterpret_cast<const float4 *>(p); b = *reinterpret_cast<const float4 *>(p + 4); }
+};
+__device__ __forceinline__ lt_f4 lt_mma(const LtFrag<ACT_BF16> &a, const LtFrag<ACT_BF16> &b, lt_f4 acc) { return __builtin_amdgcn_mfma_f32_16x16x32_f16(a.v, b.v, acc, 0, 0, 0); }
+__device__ __forceinline__ lt_f4 lt_mma(const LtFrag<ACT_F32> &x, const LtFrag<ACT_F32> &y, lt_f4 acc) {
+    const float xf[8] = {x.a.x, x.a.y, x.a.z, x.a.w, x.b.x, x.b.y, x.b.z, x.b.w}, yf[8] = {y.a.x, y.a.y, y.a.z, y.a.w, y.b.x, y.b.y, y.b.z, y.b.w};
+#pragma unroll
+    for (int j = 0; j < 8; ++j) acc = __builtin_amdgcn_mfma_f32_16x16x4f32(xf[j], yf[j], acc, 0, 0, 0);
+    return acc;
+}
+
+__host__ __device__ constexpr int lt_pitch(ActType act, int row) { return row + (act == ACT_F32 ? 4 : 8); }
+// keys per split: whole steps
+__host__ __device__ constexpr int lt_split_keys(int n_keys, int n_splits) { return ((n_keys + n_splits - 1) / n_splits + LT_KEYS - 1) / LT_KEYS * LT_KEYS; }
+
+// NR: 16-row blocks of the rank per wave (rank_pad = 64 NR)
+template <ActType ACT, int NR>
+__global__ __launch_bounds__(LT_THREADS) void latent_attn_kernel(const LatentAttnArgs a, int heads, int rot_pad) {
+    typedef typename LtElem<ACT>::type E;
+    constexpr int RANK = 64 * NR;
+    extern __shared__ __align__(16) uint8_t smem[];
+    const int row = RANK + rot_pad, pitch = lt_pitch(ACT, row);
+    E *sK = reinterpret_cast<E *>(smem);                                                  // [LT_KEYS][pitch]
+    uint32_t *sV = reinterpret_cast<uint32_t *>(smem + (size_t)LT_KEYS * pitch * sizeof(E));  // f16: [RANK][LT_VPITCH]
+    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, c = lane & 15, g = lane >> 4;
+    const int split = blockIdx.x, t = blockIdx.z, h = blockIdx.y * LATENT_HEADS_TILE + c;
+    const int n_keys = a.pos[t] + 1, per = lt_split_keys(n_keys, a.n_splits);
+    const int j0 = split * per, j1 = min(j0 + per, n_keys);
+    const size_t prow = ((size_t)t * heads + h) * a.n_splits + split;
+    if (j0 >= j1) {
+        if (tid < 16 && h < heads) { a.ml[prow * 2] = -INFINITY; a.ml[prow * 2 + 1] = 0.f; }
+        return;
+    }
+    const E *qp = static_cast<const E *>(a.qa) + ((size_t)t * heads + (h < heads ? h : heads - 1)) * row + 8 * g;
+    const E *rows = static_cast<const E *>(a.rows) + (size_t)a.seq[t] * a.n_ctx * row;
+    lt_f4 o[NR];
+#pragma unroll
+    for (int n = 0; n < NR; ++n) o[n] = lt_f4{0.f, 0.f, 0.f, 0.f};
+    float m = -INFINITY, l = 0.f;
+    for (int k0 = j0; k0 < j1; k0 += LT_KEYS) {
+        // rows past the split are zeros (their scores are masked below)
+        if constexpr (ACT == ACT_BF16) {
+            const int items = 16 * (row / 8);
+            for (int i = tid; i < items; i += LT_THREADS) {
+                const int kp = i & 15, d = (i >> 4) * 8, key = k0 + 2 * kp;
+                uint4 r0 = make_uint4(0, 0, 0, 0), r1 = r0;
+                if (key < j1) r0 = *reinterpret_cast<const uint4 *>(rows + (size_t)key * row + d);
+                if (key + 1 < j1) r1 = *reinterpret_cast<const uint4 *>(rows + (size_t)(key + 1) * row + d);
+                *reinterpret_cast<uint4 *>(sK + (2 * kp) * pitch + d) = r0;
+                *reinterpret_cast<uint4 *>(sK + (2 * kp + 1) * pitch + d) = r1;
+                if (d < RANK) {
+                    const uint32_t w0[4] = {r0.x, r0.y, r0.z, r0.w}, w1[4] = {r1.x, r1.y, r1.z, r1.w};
+                    uint32_t *dst = sV + d * LT_VPITCH + kp;
+#pragma unroll
+                    for (int e = 0; e < 4; ++e) {
+                        dst[(2 * e) * LT_VPITCH] = (w0[e] & 0xffffu) | (w1[e] << 16);
+                        dst[(2 * e + 1) * LT_VPITCH] = (w0[e] >> 16) | (w1[e] & 0xffff0000u);
+                    }
+                }
+            }
+        } else {
+            const int pieces = row / 4;
+            for (int i = tid; i < LT_KEYS * pieces; i += LT_THREADS) {
+                const int kk = i / pieces, d = (i % pieces) * 4;
+                float4 v = make_float4(0.f, 0.f, 0.f, 0.f);
+                if (k0 + kk < j1) v = *reinterpret_cast<const float4 *>(rows + (size_t)(k0 + kk) * row + d);
+                *reinterpret_cast<float4 *>(sK + kk * pitch + d) = v;
+            }
+        }
+        __syncthreads();
+        lt_f4 s[2] = {lt_f4{0.f, 0.f, 0.f, 0.f}, lt_f4{0.f, 0.f, 0.f, 0.f}};
+        auto score = [&](int kc) {
+            LtFrag<ACT> qf, kf[2];
+            qf.load(qp + kc);
+#pragma unroll
+            for (int b = 0; b < 2; ++b) {
+                kf[b].load(sK + (16 * b + c) * pitch + kc + 8 * g);
+                s[b] = lt_mma(kf[b], qf, s[b]);
+            }
+        };
+#pragma unroll
+        for (int kc = 0; kc < RANK; kc += 32) score(kc);
+        for (int kc = RANK; kc < row; kc += 32) score(kc);
+        // register i of tile b: key k0 + 16 b + 4 g + i for head column c; at least key k0 is in range
+        float mx = m;
+#pragma unroll
+        for (int b = 0; b < 2; ++b)
+#pragma unroll
+            for (int i = 0; i < 4; ++i) {
+                if (k0 + 16 * b + 4 * g + i >= j1) s[b][i] = -INFINITY;
+                mx = fmaxf(mx, s[b][i]);
+            }
+        mx = fmaxf(mx, __shfl_xor(mx, 16));
+        mx = fmaxf(mx, __shfl_xor(mx, 32));
+        const float corr = lt_exp2(m - mx);           // exp2(-inf) = 0 the first time
+        m = mx;
+        float p[2][4], ps = 0.f;
+#pragma unroll
+        for (int b = 0; b < 2; ++b)
+#pragma unroll
+            for (int i = 0; i < 4; ++i) { p[b][i] = lt_exp2(s[b][i] - mx); ps += p[b][i]; }
+        l = l * corr + ps;                            // (this lane's keys only)
+#pragma unroll
+        for (int n = 0; n < NR; ++n) o[n] *= corr;
+        if constexpr (ACT == ACT_BF16) {
+            // key slots of lane group g: keys 4g .. 4g + 3 of either tile, which is how P^T lies in the registers
+            const lt_u4 pu = {lt_pack(p[0][0], p[0][1]), lt_pack(p[0][2], p[0][3]), lt_pack(p[1][0], p[1][1]), lt_pack(p[1][2], p[1][3])};
+            const lt_h8 pf = __builtin_bit_cast(lt_h8, pu);
+#pragma unroll
+            for (int n = 0; n < NR; ++n) {
+                const uint32_t *v = sV + (16 * (wave * NR + n) + c) * LT_VPITCH + 2 * g;
+                const uint2 a0 = *reinterpret_cast<const uint2 *>(v), a1 = *reinterpret_cast<const uint2 *>(v + 8);
+                const lt_u4 vu = {a0.x, a0.y, a1.x, a1.y};
+                o[n] = __builtin_amdgcn_mfma_f32_16x16x32_f16(__builtin_bit_cast(lt_h8, vu), pf, o[n], 0, 0, 0);
+            }
+        } else {
+#pragma unroll
+            for (int n = 0; n < NR; ++n)
+#pragma unroll
+                for (int b = 0; b < 2; ++b)
+#pragma unroll
+                    for (int i = 0; i < 4; ++i)
+                        o[n] = __builtin_amdgcn_mfma_f32_16x16x4f32(sK[(16 * b + 4 * g + i) * pitch + 16 * (wave * NR + n) + c], p[b][i], o[n], 0, 0, 0);
+        }
+        __syncthreads();
+    }
+    l += __shfl_xor(l, 16);
+    l += __shfl_xor(l, 32);
+    if (h >= heads) return;
+    if (wave == 0 && g == 0) { a.ml[prow * 2] = m; a.ml[prow * 2 + 1] = l; }
+#pragma unroll
+    for (int n = 0; n < NR; ++n) *reinterpret_cast<float4 *>(a.part + prow * RANK + 16 * (wave * NR + n) + 4 * g) = make_float4(o[n][0], o[n][1], o[n][2], o[n][3]);
+}
+
+// grid (heads, slices of the value rows, T).  Sixteen lanes per weight row.
+__global__ __launch_bounds__(LT_THREADS) void latent_out_kernel(const LatentShape s, const LatentAttnArgs a) {
+    extern __shared__ __align__(16) uint8_t smem[];
+    __shared__ float s_w[ATTN_SPLITS_CAP];
+    __shared__ float s_inv;
+    float *xs = reinterpret_cast<float *>(smem);              // [rank_pad]
+    const int h = blockIdx.x, t = blockIdx.z, tid = threadIdx.x, S = a.n_splits;
+    const int n_keys = a.pos[t] + 1, per = lt_split_keys(n_keys, S), live = (n_keys + per - 1) / per;      // splits that saw a key
+    const size_t row = (size_t)t * s.heads + h;
+    if (tid < 64) {
+        const float m = tid < live ? a.ml[(row * S + tid) * 2] : -INFINITY, l = tid < live ? a.ml[(row * S + tid) * 2 + 1] : 0.f;
+        float mh = m;
+#pragma unroll
+        for (int o = 32; o > 0; o >>= 1) mh = fmaxf(mh, __shfl_xor(mh, o));
+        const float w = tid < live ? lt_exp2(m - mh) : 0.f;
+        float den = l * w;
+#pragma unroll
+        for (int o = 32; o > 0; o >>= 1) den += __shfl_xor(den, o);
+        s_w[tid] = w;
+        if (tid == 0) s_inv = 1.0f / den;
+    }
+    __syncthreads();
+    for (int r = tid; r < s.rank_pad; r += LT_THREADS) {
+        float v = 0.f;
+        const float *p = a.part + row * S * s.rank_pad + r;
+#pragma unroll 8
+        for (int k = 0; k < live; ++k) v = fmaf(p[(size_t)k * s.rank_pad], s_w[k], v);
+        xs[r] = v * s_inv;
+    }
+    __syncthreads();
+    const float gate = act_sigmoid(a.gate[(size_t)t * a.gate_ld + h]);
+    const int slice = (s.v_pad + gridDim.y - 1) / gridDim.y, v1 = min((int)(blockIdx.y + 1) * slice, s.v_pad);
+    const int piece = tid & 15, pieces = s.rank_pad / 8;
+    for (int v0 = blockIdx.y * slice; v0 < v1; v0 += LT_THREADS / 16) {
+        const int v = v0 + (tid >> 4);
+        float acc = 0.f;
+        if (v < s.vdim)
+            for (int p = piece; p < pieces; p += 16) acc = lt_dot8(*reinterpret_cast<const uint4 *>(a.w_uv + ((size_t)h * s.vdim + v) * s.rank_pad + p * 8), xs + p * 8, acc);
+        acc += __shfl_xor(acc, 1); acc += __shfl_xor(acc, 2); acc += __shfl_xor(acc, 4); acc += __shfl_xor(acc, 8);
+        if (piece == 0 && v < v1) {
+            const size_t at = row * s.v_pad + v;
+            if (a.out_bf16) a.out_bf16[at] = f32_to_bf16_bits(acc * gate);
+            else a.out[at] = acc * gate;
+        }
+    }
+}
+
+// ---- many tokens of one sequence
+// grid (heads, T), 64 threads
+__global__ __launch_bounds__(64) void latent_chunk_query_kernel(const LatentShape s, const LatentRotary rot, const float *q, const int32_t *pos, float *out) {
+    const int h = blockIdx.x, t = blockIdx.y;
+    const float *p = q + ((size_t)t * s.heads + h) * (s.dim + s.rot_dim);
+    float *o = out + ((size_t)t * s.heads + h) * s.chunk_k;
+    for (int i = threadIdx.x; i < s.dim; i += 64) o[i] = p[i];
+    for (int i = threadIdx.x; i < s.rot_dim / 2; i += 64) {
+        const float2 w = lt_turn(pos[t], rot.freq[i], rot.gain);
+        const float x = p[s.dim + 2 * i], y = p[s.dim + 2 * i + 1];
+        o[s.dim + 2 * i] = x * w.x - y * w.y;
+        o[s.dim + 2 * i + 1] = y * w.x + x * w.y;
+    }
+    for (int i = s.dim + s.rot_dim + threadIdx.x; i < s.chunk_k; i += 64) o[i] = 0.f;
+}
+
+// one workgroup per position
+__global__ __launch_bounds__(LT_THREADS) void latent_chunk_rows_kernel(const uint16_t *rows, int row, int rank, uint16_t *out, int ld) {
+    const uint16_t *p = rows + (size_t)blockIdx.x * row;
+    for (int i = threadIdx.x; i < ld; i += LT_THREADS) out[(size_t)blockIdx.x * ld + i] = i < rank ? f32_to_bf16_bits(f16_bits_to_f32(p[i])) : 0;
+}
+
+// grid (position, groups of heads); pairs of neighbouring elements
+__global__ __launch_bounds__(LT_THREADS) void latent_chunk_pack_kernel(const LatentShape s, const uint16_t *rows, int n_ctx, int k0, const float *kv, uint16_t *k16, uint16_t *v16, unsigned *sat) {
+    const int key = k0 + blockIdx.x, per = s.chunk_k + s.chunk_v, H = s.heads;
+    const float *y = kv + (size_t)blockIdx.x * H * (s.dim + s.vdim);
+    const uint16_t *r = rows + (size_t)blockIdx.x * s.row() + s.rank_pad;
+    auto f16 = [&](float v) {
+        note_f16_clamp(sat, v, 0.f);
+        return f32_to_f16_bits(fminf(fmaxf(v, -65504.f), 65504.f));
+    };
+    for (int i = (blockIdx.y * LT_THREADS + threadIdx.x) * 2; i < H * per; i += gridDim.y * LT_THREADS * 2) {
+        const int h = i / per, e0 = i % per;
+        uint16_t o[2];
+#pragma unroll
+        for (int j = 0; j < 2; ++j) {
+            const int e = e0 + j;
+            if (e0 < s.chunk_k) o[j] = e < s.dim ? f16(y[h * s.dim + e]) : e < s.dim + s.rot_dim ? r[e - s.dim] : 0;
+            else o[j] = e - s.chunk_k < s.vdim ? f16(y[H * s.dim + h * s.vdim + e - s.chunk_k]) : 0;
+        }
+        uint16_t *dst = e0 < s.chunk_k ? k16 + ((size_t)h * n_ctx + key) * s.chunk_k + e0 : v16 + ((size_t)h * n_ctx + key) * s.chunk_v + e0 - s.chunk_k;
+        *reinterpret_cast<uint32_t *>(dst) = (uint32_t)o[0] | ((uint32_t)o[1] << 16);
+    }
+}
+
+// ------------------------------------------------------------------------------------------------ host
+static size_t attn_lds(ActType act, const LatentShape &s) {
+    const size_t k = (size_t)LT_KEYS * lt_pitch(act, s.row()) * (act == ACT_F32 ? 4 : 2);
+    return act == ACT_F32 ? k : k + (size_t)s.rank_pad * LT_VPITCH * 4;
+}
+
+bool latent_shape(LatentShape &s) {
+    if (s.heads < 1 || s.dim < 1 || s.vdim < 1 || s.rank < 1 || s.rot_dim < 2 || s.rot_dim % 2) return false;
+    s.rank_pad = 64;
+    while (s.rank_pad < s.rank) s.rank_pad *= 2;
+    s.rot_pad = (s.rot_dim + 31) / 32 * 32;
+    s.dim_pad = (s.dim + 7) / 8 * 8;
+    const int k = s.dim + s.rot_dim;
+    s.chunk_k = s.chunk_v = 0;
+    if (s.vdim <= 128 && k <= 192) {
+        s.chunk_k = k <= 64 && s.vdim <= 64 ? 64 : k <= 128 ? 128 : 192;
+        s.chunk_v = s.vdim <= 64 && s.chunk_k < 192 ? 64 : 128;
+    }
+    s.v_pad = s.chunk_v ? s.chunk_v : (s.vdim + 63) / 64 * 64;
+    return s.rank_pad <= 1024 && s.dim_pad <= 4096 && attn_lds(ACT_BF16, s) <= LT_LDS_MAX && attn_lds(ACT_F32, s) <= LT_LDS_MAX;
+}
+
+int latent_rows(const LatentShape &s, const LatentCache &cache, ActType act, const float *in, int ld, const float *gain, int n, void *out, int ld_out, int T, hipStream_t stream) {
+    if (T <= 0) return MESH_OK;
+    if (!in || !gain || !out || ld < n || ld_out < n || (cache.in && (!cache.rows || !cache.gain || !cache.rot.freq))) return fail(MESH_ERR_INVALID, "latent_rows: bad operands");
+    if (act == ACT_BF16) MESH_LAUNCH((latent_rows_kernel<ACT_BF16>), dim3((unsigned)T), dim3(LT_THREADS), 0, stream, s, cache, in, ld, gain, n, out, ld_out);
+    else MESH_LAUNCH((latent_rows_kernel<ACT_F32>), dim3((unsigned)T), dim3(LT_THREADS), 0, stream, s, cache, in, ld, gain, n, out, ld_out);
+    MESH_LAUNCH_CHECK();
+    return MESH_OK;
+}
+
+int latent_query(const LatentShape &s, const LatentCache &cache, ActType act, const float *q, const uint16_t *w_uk_t, float scale, bool append, void *qa, int T, hipStream_t stream) {
+    if (T <= 0) return MESH_OK;
+    if (!q || !w_uk_t || !qa || !cache.rot.freq || (append && (!cache.in || !cache.rows || !cache.gain))) return fail(MESH_ERR_INVALID, "latent_query: bad operands");
+    const int tb = T == 1 ? 1 : LT_QUERY_TOKENS, groups = (T + tb - 1) / tb;
+    // enough workgroups to fill the chip, at least one pass of rows each
+    const int slices = std::max(1, std::min(s.rank_pad / (LT_THREADS / 8), 512 / std::max(1, s.heads * groups)));
+    const dim3 grid((unsigned)(s.heads + (append ? 1 : 0)), (unsigned)slices, (unsigned)groups), block(LT_THREADS);
+    const size_t lds = (size_t)tb * s.dim_pad * sizeof(float);
+    if (act == ACT_BF16 && tb == 1) MESH_LAUNCH((latent_query_kernel<ACT_BF16, 1>), grid, block, lds, stream, s, cache, q, w_uk_t, scale, qa, T);
+    else if (act == ACT_BF16) MESH_LAUNCH((latent_query_kernel<ACT_BF16, LT_QUERY_TOKENS>), grid, block, lds, stream, s, cache, q, w_uk_t, scale, qa, T);
+    else if (tb == 1) MESH_LAUNCH((latent_query_kernel<ACT_F32, 1>), grid, block, lds, stream, s, cache, q, w_uk_t, scale, qa, T);
+    else MESH_LAUNCH((latent_query_kernel<ACT_F32, LT_QUERY_TOKENS>), grid, block, lds, stream, s, cache, q, w_uk_t, scale, qa, T);
+    MESH_LAUNCH_CHECK();
+    return MESH_OK;
+}
+
+template <ActType ACT, int NR>
+static int launch_attn(const LatentShape &s, const LatentAttnArgs &a, int T, hipStream_t stream) {
+    static bool ready = false;        // (hosts are single-threaded per session; a second thread sets the same attribute)
+    if (!ready) {
+        MESH_HIP_TRY(hipFuncSetAttribute(reinterpret_cast<const void *>(latent_attn_kernel<ACT, NR>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)LT_LDS_MAX));
+        ready = true;
+    }
+    MESH_LAUNCH((latent_attn_kernel<ACT, NR>), dim3((unsigned)a.n_splits, (unsigned)latent_head_tiles(s), (unsigned)T), dim3(LT_THREADS), attn_lds(ACT, s), stream, a, s.heads, s.rot_pad);
+    MESH_LAUNCH_CHECK();
+    return MESH_OK;
+}
+template <ActType ACT>
+static int launch_attn_rank(const LatentShape &s, const LatentAttnArgs &a, int T, hipStream_t stream) {
+    switch (s.rank_pad) {
+        case 64: return launch_attn<ACT, 1>(s, a, T, stream);
+        case 128: return launch_attn<ACT, 2>(s, a, T, stream);
+        case 256: return launch_attn<ACT, 4>(s, a, T, stream);
+        case 512: return launch_attn<ACT, 8>(s, a, T, stream);
+        case 1024: return launch_attn<ACT, 16>(s, a, T, stream);
+        default: return fail(MESH_ERR_UNSUPPORTED, "latent_attention: no kernel for a rank of %d", s.rank);
+    }
+}
+
+int latent_attention(const LatentShape &s, const LatentAttnArgs &a, ActType act, int T, hipStream_t stream) {
+    if (T <= 0) return MESH_OK;
+    if (!a.qa || !a.rows || !a.part || !a.ml || a.n_splits < 1 || a.n_splits > ATTN_SPLITS_CAP || T > 65535) return fail(MESH_ERR_INVALID, "latent_attention: bad operands");
+    return act == ACT_BF16 ? launch_attn_rank<ACT_BF16>(s, a, T, stream) : launch_attn_rank<ACT_F32>(s, a, T, stream);
+}
+
+int latent_out(const LatentShape &s, const LatentAttnArgs &a, int T, hipStream_t stream) {
+    if (T <= 0) return MESH_OK;
+    if (!a.w_uv || !a.gate || (!a.out && !a.out_bf16) || a.n_splits > ATTN_SPLITS_CAP || T > 65535) return fail(MESH_ERR_INVALID, "latent_out: bad operands");
+    const int slices = std::max(1, std::min(s.v_pad / (LT_THREADS / 16), 256 / std::max(1, s.heads * T)));
+    MESH_LAUNCH(latent_out_kernel, dim3((unsigned)s.heads, (unsigned)slices, (unsigned)T), dim3(LT_THREADS), (size_t)s.rank_pad * sizeof(float), stream, s, a);
+    MESH_LAUNCH_CHECK();
+    return MESH_OK;
+}
+
+int latent_chunk_query(const LatentShape &s, const LatentRotary &rot, const float *q, const int32_t *pos, float *out, int T, hipStream_t stream) {
+    if (T <= 0) return MESH_OK;
+    if (!s.chunk_k || T > 65535) return fail(MESH_ERR_INVALID, "latent_chunk_query: bad operands");
+    MESH_LAUNCH(latent_chunk_query_kernel, dim3((unsigned)s.heads, (unsigned)T), dim3(64), 0, stream, s, rot, q, pos, out);
+    MESH_LAUNCH_CHECK();
+    return MESH_OK;
+}
+
+int latent_chunk_rows(const LatentShape &s, const void *rows, int n_ctx, int seq, int k0, int n, uint16_t *out, int ld, hipStream_t stream) {
+    if (n <= 0) return MESH_OK;
+    if (k0 < 0 || k0 + n > n_ctx || ld < s.rank) return fail(MESH_ERR_INVALID, "latent_chunk_rows: bad operands");
+    const uint16_t *p = static_cast<const uint16_t *>(rows) + ((size_t)seq * n_ctx + k0) * s.row();
+    MESH_LAUNCH(latent_chunk_rows_kernel, dim3((unsigned)n), dim3(LT_THREADS), 0, stream, p, s.row(), s.rank, out, ld);
+    MESH_LAUNCH_CHECK();
+    return MESH_OK;
+}
+
+int latent_chunk_pack(const LatentShape &s, const void *rows, int n_ctx, int seq, int k0, int n, const float *kv, uint16_t *k16, uint16_t *v16, unsigned *sat, hipStream_t stream) {
+    if (n <= 0) return MESH_OK;
+    if (!s.chunk_k || k0 < 0 || k0 + n > n_ctx) return fail(MESH_ERR_INVALID, "latent_chunk_pack: bad operands");
+    const uint16_t *p = static_cast<const uint16_t *>(rows) + ((size_t)seq * n_ctx + k0) * s.row();
+    const int cols = s.heads * (s.chunk_k + s.chunk_v) / 2;
+    MESH_LAUNCH(latent_chunk_pack_kernel, dim3((unsigned)n, (unsigned)std::max(1, std::min(4, cols / LT_THREADS))), dim3(LT_THREADS), 0, stream, s, p, n_ctx, k0, kv, k16, v16, sat);
+    MESH_LAUNCH_CHECK();
+    return MESH_OK;
+}
+
+}  // namespace mesh

@@ -50,9 +50,20 @@ __device__ __forceinline__ ln_f4 rows_mma(const uint4 &w, const RowsFrag<ACT_F32
     return acc;
 }
 
+// what becomes of a result: stored as it is, or as an activation of the product that follows
+enum LinearOut { LINEAR_OUT_F32 = 0, LINEAR_OUT_RELU2 = 1 };
+template <ActType ACT, LinearOut OUT> __device__ __forceinline__ void linear_store(void *y, size_t at, float v) {
+    if constexpr (OUT == LINEAR_OUT_RELU2) {
+        v = fmaxf(v, 0.f);
+        v *= v;
+    }
+    if constexpr (OUT == LINEAR_OUT_F32 || ACT == ACT_F32) static_cast<float *>(y)[at] = v;
+    else static_cast<uint16_t *>(y)[at] = f32_to_bf16_bits(v);
+}
+
 // grid (row blocks of 16, token blocks of 16 * NT)
-template <ActType ACT, int NT>
-__global__ __launch_bounds__(64 * ROWS_WAVES) void linear_rows_kernel(const uint16_t *w, const void *x, float *y, int K, int M, int T, int ldy) {
+template <ActType ACT, int NT, LinearOut OUT>
+__global__ __launch_bounds__(64 * ROWS_WAVES) void linear_rows_kernel(const uint16_t *w, const void *x, void *y, int K, int M, int T, int ldy) {
     __shared__ float red[ROWS_WAVES][NT][16][17];
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, c = lane & 15, g = lane >> 4;
     const int m0 = blockIdx.x * 16, t0 = blockIdx.y * 16 * NT;
@@ -97,7 +108,7 @@ __global__ __launch_bounds__(64 * ROWS_WAVES) void linear_rows_kernel(const uint
 #pragma unroll
         for (int v = 1; v < ROWS_WAVES; ++v) s += red[v][n][tk][r];
         const int m = m0 + r, t = t0 + 16 * n + tk;
-        if (m < M && t < T) y[(size_t)t * ldy + m] = s;
+        if (m < M && t < T) linear_store<ACT, OUT>(y, (size_t)t * ldy + m, s);
     }
 }
 
@@ -113,11 +124,12 @@ __device__ __forceinline__ void tile_copy16(const uint16_t *src, uint16_t *lds_b
 
 // 1-D grid of (row blocks x token blocks); the workgroups a die is dealt (every eighth) take a contiguous run of tiles with
 // the token block running fastest, so that the weight rows of a run stay in that die's cache
-__global__ __launch_bounds__(TILE_THREADS) void linear_tile_kernel(const uint16_t *w, const uint16_t *x, float *y, int K, int M, int T, int ldy,
+template <LinearOut OUT>
+__global__ __launch_bounds__(TILE_THREADS) void linear_tile_kernel(const uint16_t *w, const uint16_t *x, void *y, int K, int M, int T, int ldy,
                                                                    int n_tblocks, int n_tiles, int k_slice, size_t y_slice) {
     // blockIdx.y: slice of K and the partial result it writes
     const int k_begin = blockIdx.y * k_slice, k_end = k_begin + k_slice < K ? k_begin + k_slice : K;
-    y += blockIdx.y * y_slice;
+    y = static_cast<float *>(y) + blockIdx.y * y_slice;          // (slices are f32 results)
     __shared__ __align__(16) uint16_t sW0[TILE_M * TILE_K], sW1[TILE_M * TILE_K], sX0[TILE_T * TILE_K], sX1[TILE_T * TILE_K];
     const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
     int tile = blockIdx.x;
@@ -195,32 +207,34 @@ __global__ __launch_bounds__(TILE_THREADS) void linear_tile_kernel(const uint16_
 #pragma unroll
             for (int i = 0; i < 16; ++i) {
                 const int t = tb * TILE_T + wt + 32 * a + 8 * (i >> 2) + 4 * half + (i & 3);
-                if (t < T) y[(size_t)t * ldy + m] = acc[a][b][i];
+                if (t < T) linear_store<ACT_BF16, OUT>(y, (size_t)t * ldy + m, acc[a][b][i]);
             }
     }
 }
 
-template <ActType ACT>
-static int launch_rows(const LinearWeight &W, const void *x, int T, float *y, int ldy, hipStream_t stream) {
-    const unsigned mb = (unsigned)((W.M + 15) / 16);
+// M: columns of y to write, at least W.M (the rows of W behind it are zeros)
+template <ActType ACT, LinearOut OUT>
+static int launch_rows(const LinearWeight &W, const void *x, int T, void *y, int ldy, int M, hipStream_t stream) {
+    const unsigned mb = (unsigned)((M + 15) / 16);
     const dim3 block(64 * ROWS_WAVES);
-    if (T <= 16) MESH_LAUNCH((linear_rows_kernel<ACT, 1>), dim3(mb, 1), block, 0, stream, W.w, x, y, W.Kp, W.M, T, ldy);
-    else if (T <= 32) MESH_LAUNCH((linear_rows_kernel<ACT, 2>), dim3(mb, 1), block, 0, stream, W.w, x, y, W.Kp, W.M, T, ldy);
-    else MESH_LAUNCH((linear_rows_kernel<ACT, 4>), dim3(mb, (unsigned)((T + 63) / 64)), block, 0, stream, W.w, x, y, W.Kp, W.M, T, ldy);
+    if (T <= 16) MESH_LAUNCH((linear_rows_kernel<ACT, 1, OUT>), dim3(mb, 1), block, 0, stream, W.w, x, y, W.Kp, M, T, ldy);
+    else if (T <= 32) MESH_LAUNCH((linear_rows_kernel<ACT, 2, OUT>), dim3(mb, 1), block, 0, stream, W.w, x, y, W.Kp, M, T, ldy);
+    else MESH_LAUNCH((linear_rows_kernel<ACT, 4, OUT>), dim3(mb, (unsigned)((T + 63) / 64)), block, 0, stream, W.w, x, y, W.Kp, M, T, ldy);
     MESH_LAUNCH_CHECK();
     return MESH_OK;
 }
 
-static int launch_tile(const LinearWeight &W, const void *x, int T, float *y, int ldy, int slices, size_t stride, hipStream_t stream) {
-    const int mblocks = (W.M + TILE_M - 1) / TILE_M, tblocks = (T + TILE_T - 1) / TILE_T;
+template <LinearOut OUT>
+static int launch_tile(const LinearWeight &W, const void *x, int T, void *y, int ldy, int M, int slices, size_t stride, hipStream_t stream) {
+    const int mblocks = (M + TILE_M - 1) / TILE_M, tblocks = (T + TILE_T - 1) / TILE_T;
     const int steps = W.Kp / TILE_K, k_slice = (steps + slices - 1) / slices * TILE_K;
-    MESH_LAUNCH(linear_tile_kernel, dim3((unsigned)(mblocks * tblocks), (unsigned)slices), dim3(TILE_THREADS), 0, stream, W.w, static_cast<const uint16_t *>(x), y, W.Kp, W.M,
+    MESH_LAUNCH((linear_tile_kernel<OUT>), dim3((unsigned)(mblocks * tblocks), (unsigned)slices), dim3(TILE_THREADS), 0, stream, W.w, static_cast<const uint16_t *>(x), y, W.Kp, M,
                 T, ldy, tblocks, mblocks * tblocks, k_slice, stride);
     MESH_LAUNCH_CHECK();
     return MESH_OK;
 }
 
-static bool linear_ok(const LinearWeight &W, const void *x, int T, const float *y, int ldy) {
+static bool linear_ok(const LinearWeight &W, const void *x, int T, const void *y, int ldy) {
     return W.w && x && y && W.M >= 1 && W.Kp % LINEAR_K_PAD == 0 && W.Mp % LINEAR_ROW_PAD == 0 && W.Mp >= W.M && W.Kp >= W.K && ldy >= W.M && (T + 63) / 64 <= 65535;
 }
 
@@ -235,16 +249,24 @@ int linear_sliced(const LinearWeight &W, const void *x, ActType act, int T, floa
         return rc == MESH_OK ? 1 : rc;
     }
     if (!linear_ok(W, x, T, y, W.M)) return fail(MESH_ERR_INVALID, "linear_sliced: bad operands (%d x %d, %d tokens)", W.M, W.K, T);
-    const int rc = launch_tile(W, x, T, y, W.M, slices, stride, stream);
+    const int rc = launch_tile<LINEAR_OUT_F32>(W, x, T, y, W.M, W.M, slices, stride, stream);
     return rc == MESH_OK ? slices : rc;
 }
 
 int linear(const LinearWeight &W, const void *x, ActType act, int T, float *y, int ldy, int big_from, hipStream_t stream) {
     if (T <= 0) return MESH_OK;
     if (!linear_ok(W, x, T, y, ldy)) return fail(MESH_ERR_INVALID, "linear: bad operands (%d x %d, %d tokens)", W.M, W.K, T);
-    if (act == ACT_F32) return launch_rows<ACT_F32>(W, x, T, y, ldy, stream);
-    if (T < big_from || W.M < TILE_M) return launch_rows<ACT_BF16>(W, x, T, y, ldy, stream);
-    return launch_tile(W, x, T, y, ldy, 1, 0, stream);
+    if (act == ACT_F32) return launch_rows<ACT_F32, LINEAR_OUT_F32>(W, x, T, y, ldy, W.M, stream);
+    if (T < big_from || W.M < TILE_M) return launch_rows<ACT_BF16, LINEAR_OUT_F32>(W, x, T, y, ldy, W.M, stream);
+    return launch_tile<LINEAR_OUT_F32>(W, x, T, y, ldy, W.M, 1, 0, stream);
+}
+
+int linear_relu2(const LinearWeight &W, const void *x, ActType act, int T, void *out, int ld, int big_from, hipStream_t stream) {
+    if (T <= 0) return MESH_OK;
+    if (!linear_ok(W, x, T, out, ld) || ld > W.Mp) return fail(MESH_ERR_INVALID, "linear_relu2: bad operands (%d x %d, %d tokens)", W.M, W.K, T);
+    if (act == ACT_F32) return launch_rows<ACT_F32, LINEAR_OUT_RELU2>(W, x, T, out, ld, ld, stream);
+    if (T < big_from || W.M < TILE_M) return launch_rows<ACT_BF16, LINEAR_OUT_RELU2>(W, x, T, out, ld, ld, stream);
+    return launch_tile<LINEAR_OUT_RELU2>(W, x, T, out, ld, ld, 1, 0, stream);
 }
 
 }  // namespace mesh

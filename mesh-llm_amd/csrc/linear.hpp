@@ -24,6 +24,9 @@ inline int linear_k_padded(int K) { return (K + LINEAR_K_PAD - 1) / LINEAR_K_PAD
 // y[t][m] = sum_k W[m][k] x[t][k] for t < T.  x: rows of W.Kp elements of `act` (columns from K on hold zeros), 16-byte
 // aligned; y: f32 rows of ldy.  big_from: bf16 calls of at least this many tokens take the large-tile kernel.
 int linear(const LinearWeight &W, const void *x, ActType act, int T, float *y, int ldy, int big_from, hipStream_t stream);
+// The same, leaving max(y, 0)^2 as rows of ld elements of `act` (W.M <= ld <= W.Mp; columns from W.M on are zeros) for the
+// product that follows.
+int linear_relu2(const LinearWeight &W, const void *x, ActType act, int T, void *out, int ld, int big_from, hipStream_t stream);
 
 // The same for a matrix of few rows (hundreds), which leaves the large tile with few workgroups: K is cut into slices, each of
 // which writes its own partial y, `stride` floats apart; the reader adds them in order.  Returns the slice count (1: y is
@@ -38,7 +41,10 @@ enum StepIn {
     STEP_IN_VEC = 0,          // x = in
     STEP_IN_RESIDUAL = 1,     // x = in + y / rms(y) * gain, rms from the partial sums its producer left; also written to x_out
     STEP_IN_RESIDUAL_NORM = 2,// the same, then x / rms(x) * norm_gain
-    STEP_IN_POLY = 3          // x = c0 N(u) + c1 N(u^2) + c2 N(u^3) + c3, u = in, N(v) = v / rms(v)
+    STEP_IN_POLY = 3,         // x = c0 N(u) + c1 N(u^2) + c2 N(u^3) + c3, u = in, N(v) = v / rms(v)
+    STEP_IN_LAYER = 4,        // v = in + LN(y) gain + bias (y null: v = in), also written to x_out; x = LN(v) norm_gain + norm_bias, LN(v) = (v - mean) / deviation
+    STEP_IN_UNIT_RMS = 5,     // x = in / rms(in) * gain
+    STEP_IN_RELU2 = 6         // x = max(in, 0)^2
 };
 enum StepOut {
     STEP_OUT_PLAIN = 0,       // out = W x
@@ -53,12 +59,14 @@ struct StepArgs {
     StepIn in_kind = STEP_IN_VEC;
     StepOut out_kind = STEP_OUT_PLAIN;
     const float *in = nullptr;            // [K]
-    const float *y = nullptr;             // RESIDUAL: [K]
-    const float *gain = nullptr;          // RESIDUAL: [K]
+    const float *y = nullptr;             // RESIDUAL, LAYER: [K]
+    const float *gain = nullptr;          // RESIDUAL, LAYER with y, UNIT_RMS: [K]
+    const float *bias = nullptr;          // LAYER with y: [K]
     const float *part = nullptr;          // RESIDUAL: [n_part]; POLY: [3][n_part]
     int n_part = 0;
-    float *x_out = nullptr;               // RESIDUAL: [K], not `in`
-    const float *norm_gain = nullptr;     // RESIDUAL_NORM: one number
+    float *x_out = nullptr;               // RESIDUAL, LAYER with y: [K], not `in`
+    const float *norm_gain = nullptr;     // RESIDUAL_NORM: one number; LAYER: [K]
+    const float *norm_bias = nullptr;     // LAYER: [K]
     const float *coef = nullptr;          // POLY: four numbers
     float eps = 0.f;
     float *out = nullptr;                 // [M] (MIN_GRU: [width])

@@ -53,6 +53,44 @@ __device__ __forceinline__ void step_vec(int K, int Kp, int tid, Load load, Map 
     }
 }
 
+// Mean and sum of squared deviations of `n` values, and of two groups together (Chan, Golub, LeVeque: updating formulae for
+// sample variances): one pass, without the cancellation of sums of squares.
+struct StepMoments {
+    float n = 0.f, mean = 0.f, m2 = 0.f;
+    __device__ __forceinline__ void add(const float *v, int count) {           // count values at once (zero to four)
+        float s = 0.f, d2 = 0.f;
+        for (int j = 0; j < 4; ++j) s += j < count ? v[j] : 0.f;
+        const float m = count ? s / (float)count : 0.f;
+        for (int j = 0; j < 4; ++j) { const float d = j < count ? v[j] - m : 0.f; d2 = fmaf(d, d, d2); }
+        join({(float)count, m, d2});
+    }
+    __device__ __forceinline__ void join(const StepMoments &o) {
+        const float t = n + o.n, f = t > 0.f ? o.n / t : 0.f, d = o.mean - mean;
+        m2 += o.m2 + d * d * n * f;
+        mean = fmaf(d, f, mean);
+        n = t;
+    }
+};
+// over the workgroup in a fixed order, the same in every thread
+__device__ __forceinline__ StepMoments step_block_moments(StepMoments m, float (*scratch)[4], int lane, int wave) {
+#pragma unroll
+    for (int o = 32; o > 0; o >>= 1) {
+        // (the lower lane's group comes first in both, so that the two agree to the bit)
+        StepMoments a = m, b;
+        b.n = __shfl_xor(m.n, o); b.mean = __shfl_xor(m.mean, o); b.m2 = __shfl_xor(m.m2, o);
+        const bool low = !(lane & o);
+        m = low ? a : b;
+        m.join(low ? b : a);
+    }
+    __syncthreads();
+    if (lane == 0) { scratch[wave][0] = m.n; scratch[wave][1] = m.mean; scratch[wave][2] = m.m2; }
+    __syncthreads();
+    StepMoments r = {scratch[0][0], scratch[0][1], scratch[0][2]};
+#pragma unroll
+    for (int w = 1; w < STEP_WAVES; ++w) r.join({scratch[w][0], scratch[w][1], scratch[w][2]});
+    return r;
+}
+
 template <int R, int U, StepIn IN, StepOut OUT>
 __global__ __launch_bounds__(STEP_THREADS) void linear_step_kernel(const uint16_t *p_w, int p_Kp, int p_groups, int p_width, int p_K, const StepArgs a) {
     extern __shared__ __align__(16) uint8_t smem[];
@@ -95,6 +133,71 @@ __global__ __launch_bounds__(STEP_THREADS) void linear_step_kernel(const uint16_
                  [&](int k, const float4 &u) {
                      return make_float4(k < K ? poly(u.x) : 0.f, k + 1 < K ? poly(u.y) : 0.f, k + 2 < K ? poly(u.z) : 0.f, k + 3 < K ? poly(u.w) : 0.f);
                  }, xs);
+    } else if constexpr (IN == STEP_IN_RELU2) {
+        auto sq = [](float v) { const float p = fmaxf(v, 0.f); return p * p; };
+        step_vec(K, Kp, tid, [&](int k) { return ln_load4(a.in, k, K); }, [&](int k, const float4 &v) { return make_float4(sq(v.x), sq(v.y), sq(v.z), sq(v.w)); }, xs);
+    } else if constexpr (IN == STEP_IN_UNIT_RMS) {
+        float ss = 0.f;
+        step_vec(K, Kp, tid, [&](int k) { return ln_load4(a.in, k, K); },
+                 [&](int k, const float4 &v) { ss += v.x * v.x + v.y * v.y + v.z * v.z + v.w * v.w; return v; }, xs);
+        const float rinv = 1.0f / sqrtf(step_block_sum(ss, &scratch[0][0], lane, wave) / (float)K + a.eps);
+        for (int k = tid; k < K; k += STEP_THREADS) xs[k] *= rinv * a.gain[k];
+    } else if constexpr (IN == STEP_IN_LAYER) {
+        constexpr int AHEAD = 2;                // groups of four a thread requests before the first moments are known
+        constexpr int STRIDE = STEP_THREADS * 4;
+        float4 x4[AHEAD], y4[AHEAD];
+        const int k0 = tid * 4;
+#pragma unroll
+        for (int i = 0; i < AHEAD; ++i) {
+            x4[i] = ln_load4(a.in, k0 + i * STRIDE, K);
+            y4[i] = a.y ? ln_load4(a.y, k0 + i * STRIDE, K) : make_float4(0.f, 0.f, 0.f, 0.f);
+        }
+        auto live = [&](int k) { return K - k < 0 ? 0 : K - k < 4 ? K - k : 4; };
+        StepMoments mx;
+        // v of group i -> LDS, x_out and the moments of v
+        auto put = [&](int i, const float4 &v) {
+            const int k = k0 + i * STRIDE;
+            if (k >= Kp) return;
+            *reinterpret_cast<float4 *>(xs + k) = v;
+            const float o[4] = {v.x, v.y, v.z, v.w};
+            const int c = live(k);
+            mx.add(o, c);
+            if (blockIdx.x == 0 && a.y)
+                for (int j = 0; j < c; ++j) a.x_out[k + j] = o[j];
+        };
+        if (a.y) {
+            StepMoments my;
+            auto take = [&](int i, const float4 &v) {
+                const float o[4] = {v.x, v.y, v.z, v.w};
+                my.add(o, live(k0 + i * STRIDE));
+            };
+#pragma unroll
+            for (int i = 0; i < AHEAD; ++i) take(i, y4[i]);
+            for (int i = AHEAD; k0 + i * STRIDE < K; ++i) take(i, ln_load4(a.y, k0 + i * STRIDE, K));
+            my = step_block_moments(my, scratch, lane, wave);
+            const float rs = 1.0f / sqrtf(my.m2 / (float)K + a.eps);
+            auto update = [&](int i, const float4 &x, const float4 &y) {
+                const int k = k0 + i * STRIDE;
+                if (k >= Kp) return;
+                const float4 g = ln_load4(a.gain, k, K), b = ln_load4(a.bias, k, K);
+                put(i, make_float4(x.x + ((y.x - my.mean) * rs * g.x + b.x), x.y + ((y.y - my.mean) * rs * g.y + b.y), x.z + ((y.z - my.mean) * rs * g.z + b.z),
+                                   x.w + ((y.w - my.mean) * rs * g.w + b.w)));
+            };
+#pragma unroll
+            for (int i = 0; i < AHEAD; ++i) update(i, x4[i], y4[i]);
+            for (int i = AHEAD; k0 + i * STRIDE < Kp; ++i) update(i, ln_load4(a.in, k0 + i * STRIDE, K), ln_load4(a.y, k0 + i * STRIDE, K));
+        } else {
+#pragma unroll
+            for (int i = 0; i < AHEAD; ++i) put(i, x4[i]);
+            for (int i = AHEAD; k0 + i * STRIDE < Kp; ++i) put(i, ln_load4(a.in, k0 + i * STRIDE, K));
+        }
+        mx = step_block_moments(mx, scratch, lane, wave);
+        const float rs = 1.0f / sqrtf(mx.m2 / (float)K + a.eps);
+        for (int k = k0; k < Kp; k += STRIDE) {          // (every thread its own groups)
+            const float4 v = *reinterpret_cast<const float4 *>(xs + k), g = ln_load4(a.norm_gain, k, K), b = ln_load4(a.norm_bias, k, K);
+            *reinterpret_cast<float4 *>(xs + k) =
+                make_float4((v.x - mx.mean) * rs * g.x + b.x, (v.y - mx.mean) * rs * g.y + b.y, (v.z - mx.mean) * rs * g.z + b.z, (v.w - mx.mean) * rs * g.w + b.w);
+        }
     } else {
         float ss = 0.f;
         for (int i = tid; i < a.n_part; i += STEP_THREADS) ss += a.part[i];
@@ -244,6 +347,8 @@ int linear_step(const StepArgs &a, hipStream_t stream) {
     if ((resid && (!a.y || !a.gain || !a.part || !a.x_out || a.x_out == a.in || a.n_part < 1 || a.n_part > STEP_PARTS_MAX)) ||
         (a.in_kind == STEP_IN_RESIDUAL_NORM && !a.norm_gain) || (a.in_kind == STEP_IN_POLY && (!a.part || !a.coef || a.n_part < 1 || a.n_part > STEP_PARTS_MAX)))
         return fail(MESH_ERR_INVALID, "linear_step: input description incomplete");
+    if ((a.in_kind == STEP_IN_LAYER && (!a.norm_gain || !a.norm_bias || (a.y && (!a.gain || !a.bias || !a.x_out || a.x_out == a.in)))) || (a.in_kind == STEP_IN_UNIT_RMS && !a.gain))
+        return fail(MESH_ERR_INVALID, "linear_step: input description incomplete");
     if (((a.out_kind == STEP_OUT_SUMSQ || a.out_kind == STEP_OUT_POWERS) && !a.out_part) ||
         (a.out_kind == STEP_OUT_MIN_GRU && (!a.state || !a.pos || !a.seq || !a.bias_z || !a.bias_x || a.width < 1 || W.M != 3 * a.width)) ||
         (a.out_kind == STEP_OUT_SIDE && (!a.side || !a.tok)))
@@ -253,6 +358,9 @@ int linear_step(const StepArgs &a, hipStream_t stream) {
     MESH_STEP_CASE(STEP_IN_VEC, STEP_OUT_PLAIN)
     MESH_STEP_CASE(STEP_IN_RESIDUAL, STEP_OUT_PLAIN)
     MESH_STEP_CASE(STEP_IN_RESIDUAL_NORM, STEP_OUT_PLAIN)
+    MESH_STEP_CASE(STEP_IN_LAYER, STEP_OUT_PLAIN)
+    MESH_STEP_CASE(STEP_IN_UNIT_RMS, STEP_OUT_PLAIN)
+    MESH_STEP_CASE(STEP_IN_RELU2, STEP_OUT_PLAIN)
     MESH_STEP_CASE(STEP_IN_VEC, STEP_OUT_SUMSQ)
     MESH_STEP_CASE(STEP_IN_POLY, STEP_OUT_SUMSQ)
     MESH_STEP_CASE(STEP_IN_RESIDUAL, STEP_OUT_POWERS)

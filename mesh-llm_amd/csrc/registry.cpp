@@ -8,6 +8,7 @@ static const ModelArch ARCHS[] = {
     {"qwen3", CONTAINER_GGUF, FAMILY_KQUANT},
     {"qwen3moe", CONTAINER_GGUF, FAMILY_KQUANT},
     {"Nadosun", CONTAINER_FOLDER, FAMILY_HYBRID},
+    {"Nutavik", CONTAINER_FOLDER, FAMILY_HYBRID},
 };
 
 const ModelArch *find_arch(const std::string &name, ModelContainer container) {

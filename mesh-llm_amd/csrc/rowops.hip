@@ -44,14 +44,18 @@ __device__ __forceinline__ float row_sum(float v, float *scratch) {
     return scratch[0] + scratch[1] + scratch[2] + scratch[3];
 }
 
-__global__ __launch_bounds__(ROW_THREADS) void embed_rows_kernel(const uint16_t *table, const int32_t *tok, const int32_t *pos, const float *freq, float scale,
+__global__ __launch_bounds__(ROW_THREADS) void embed_rows_kernel(const uint16_t *table, int ldt, const int32_t *tok, const int32_t *pos, const float *freq, float scale,
                                                                  int n, float *x) {
     const int t = blockIdx.x;
-    const uint16_t *e = table + (size_t)tok[t] * n;
+    const uint16_t *e = table + (size_t)tok[t] * ldt;
     const float p = (float)pos[t];
     for (int i = threadIdx.x; i < n; i += ROW_THREADS) {
-        const float angle = p * freq[i >> 1];
-        x[(size_t)t * n + i] = bf16_bits_to_f32(e[i]) * scale + ((i & 1) ? cosf(angle) : sinf(angle));
+        float v = bf16_bits_to_f32(e[i]) * scale;
+        if (freq) {
+            const float angle = p * freq[i >> 1];
+            v += (i & 1) ? cosf(angle) : sinf(angle);
+        }
+        x[(size_t)t * n + i] = v;
     }
 }
 
@@ -84,6 +88,89 @@ __global__ __launch_bounds__(ROW_THREADS) void residual_norm_kernel(float *x, co
         }
         act_store_row<ACT, V>(out, to + i, v);
     }
+}
+
+// The same with layer norms on both sides: x += post(y), act = pre(x).  A thread keeps its NV groups of V elements of the row
+// in registers (NV 0: rows of any length, read again for every pass).  Means first, then squared deviations.
+template <ActType ACT, int V, int NV>
+__global__ __launch_bounds__(ROW_THREADS) void layer_norm_kernel(const float *src, const int32_t *row, float *x, const float *y, const RowNorm post, const RowNorm pre,
+                                                                 float eps, int n, void *out, int ld) {
+    __shared__ float scratch[ROW_WAVES];
+    constexpr int NR = NV ? NV : 1;
+    const size_t at = (size_t)(row ? row[blockIdx.x] : (int)blockIdx.x) * n, to = (size_t)blockIdx.x * ld;
+    const float inv_n = 1.0f / (float)n;
+    RowVec<V> r[NR];
+    auto each = [&](auto fn) {         // fn(first element, register group)
+        if constexpr (NV > 0) {
+#pragma unroll
+            for (int k = 0; k < NV; ++k) {
+                const int i = (k * ROW_THREADS + (int)threadIdx.x) * V;
+                if (i < n) fn(i, r[k]);
+            }
+        } else {
+            for (int i = threadIdx.x * V; i < n; i += ROW_THREADS * V) fn(i, r[0]);
+        }
+    };
+    auto moments = [&](const float *p, float &mean, float &rstd) {
+        float s = 0.f;
+        each([&](int i, RowVec<V> &v) {
+            if (NV == 0) v = row_load<V>(p + i);
+#pragma unroll
+            for (int j = 0; j < V; ++j) s += v.v[j];
+        });
+        mean = row_sum(s, scratch) * inv_n;
+        float d2 = 0.f;
+        each([&](int i, RowVec<V> &v) {
+            if (NV == 0) v = row_load<V>(p + i);
+#pragma unroll
+            for (int j = 0; j < V; ++j) { const float d = v.v[j] - mean; d2 = fmaf(d, d, d2); }
+        });
+        rstd = 1.0f / sqrtf(row_sum(d2, scratch) * inv_n + eps);
+    };
+    float mean, rstd;
+    if (y) {
+        if (NV > 0) each([&](int i, RowVec<V> &v) { v = row_load<V>(y + at + i); });
+        moments(y + at, mean, rstd);
+        each([&](int i, RowVec<V> &v) {
+            if (NV == 0) v = row_load<V>(y + at + i);
+            const RowVec<V> g = row_load<V>(post.gain + i), b = row_load<V>(post.bias + i), xv = row_load<V>(src + at + i);
+#pragma unroll
+            for (int j = 0; j < V; ++j) v.v[j] = xv.v[j] + ((v.v[j] - mean) * rstd * g.v[j] + b.v[j]);
+            row_store<V>(x + at + i, v);
+        });
+        src = x;
+    } else if (NV > 0) {
+        each([&](int i, RowVec<V> &v) { v = row_load<V>(src + at + i); });
+    }
+    if (!out) return;
+    mean = 0.f; rstd = 1.f;
+    if (pre.kind == NORM_LAYER) moments(src + at, mean, rstd);
+    each([&](int i, RowVec<V> &v) {
+        if (NV == 0) v = row_load<V>(src + at + i);
+        RowVec<V> o = v;
+        if (pre.kind == NORM_LAYER) {
+            const RowVec<V> g = row_load<V>(pre.gain + i), b = row_load<V>(pre.bias + i);
+#pragma unroll
+            for (int j = 0; j < V; ++j) o.v[j] = (v.v[j] - mean) * rstd * g.v[j] + b.v[j];
+        }
+        act_store_row<ACT, V>(out, to + i, o);
+    });
+    for (int i = n + threadIdx.x; i < ld; i += ROW_THREADS) act_store<ACT>(out, to + i, 0.f);
+}
+
+template <ActType ACT>
+static int launch_layer_norm(const float *src, const int32_t *row, float *x, const float *y, const RowNorm &post, const RowNorm &pre, float eps, int rows, int n, void *out, int ld,
+                             hipStream_t stream) {
+    const dim3 grid((unsigned)rows), block(ROW_THREADS);
+    const int groups = n % 4 == 0 ? (n + 4 * ROW_THREADS - 1) / (4 * ROW_THREADS) : 0;
+    if (groups == 1) MESH_LAUNCH((layer_norm_kernel<ACT, 4, 1>), grid, block, 0, stream, src, row, x, y, post, pre, eps, n, out, ld);
+    else if (groups == 2) MESH_LAUNCH((layer_norm_kernel<ACT, 4, 2>), grid, block, 0, stream, src, row, x, y, post, pre, eps, n, out, ld);
+    else if (groups >= 3 && groups <= 4) MESH_LAUNCH((layer_norm_kernel<ACT, 4, 4>), grid, block, 0, stream, src, row, x, y, post, pre, eps, n, out, ld);
+    else if (groups >= 5 && groups <= 8) MESH_LAUNCH((layer_norm_kernel<ACT, 4, 8>), grid, block, 0, stream, src, row, x, y, post, pre, eps, n, out, ld);
+    else if (groups) MESH_LAUNCH((layer_norm_kernel<ACT, 4, 0>), grid, block, 0, stream, src, row, x, y, post, pre, eps, n, out, ld);
+    else MESH_LAUNCH((layer_norm_kernel<ACT, 1, 0>), grid, block, 0, stream, src, row, x, y, post, pre, eps, n, out, ld);
+    MESH_LAUNCH_CHECK();
+    return MESH_OK;
 }
 
 template <ActType ACT>
@@ -193,18 +280,32 @@ __global__ __launch_bounds__(ROW_THREADS) void qk_norm_append_kernel(const QkApp
         MESH_LAUNCH_CHECK();                                                                               \
     } while (0)
 
-int embed_rows(const uint16_t *table, const int32_t *tok, const int32_t *pos, const float *freq, float scale, int T, int n, float *x, hipStream_t stream) {
+int embed_rows(const uint16_t *table, int ldt, const int32_t *tok, const int32_t *pos, const float *freq, float scale, int T, int n, float *x, hipStream_t stream) {
     if (T <= 0) return MESH_OK;
-    MESH_LAUNCH(embed_rows_kernel, dim3((unsigned)T), dim3(ROW_THREADS), 0, stream, table, tok, pos, freq, scale, n, x);
+    MESH_LAUNCH(embed_rows_kernel, dim3((unsigned)T), dim3(ROW_THREADS), 0, stream, table, ldt, tok, pos, freq, scale, n, x);
     MESH_LAUNCH_CHECK();
     return MESH_OK;
 }
 
-int residual_norm_rows(float *x, const float *y, const float *gain, float eps, int T, int n, void *out, ActType act, int ld, hipStream_t stream) {
+static bool norm_ok(const RowNorm &nm) { return nm.kind == NORM_NONE || (nm.gain && (nm.kind == NORM_RMS || nm.bias)); }
+
+int residual_norm_rows(float *x, const float *y, const RowNorm &post, const RowNorm &pre, float eps, int T, int n, void *out, ActType act, int ld, hipStream_t stream) {
     if (T <= 0) return MESH_OK;
-    if (ld < n || (y && !gain)) return fail(MESH_ERR_INVALID, "residual_norm_rows: bad operands");
-    MESH_ROW_LAUNCH(residual_norm_kernel, act, n % 4 == 0, dim3((unsigned)T), dim3(ROW_THREADS), x, y, gain, eps, n, out, ld);
+    if (ld < n || !norm_ok(post) || !norm_ok(pre) || (y && post.kind == NORM_NONE) || pre.kind == NORM_RMS) return fail(MESH_ERR_INVALID, "residual_norm_rows: bad operands");
+    if (post.kind == NORM_LAYER || pre.kind == NORM_LAYER) {
+        if (y && post.kind != NORM_LAYER) return fail(MESH_ERR_UNSUPPORTED, "residual_norm_rows: no kernel for norm %d before norm %d", (int)post.kind, (int)pre.kind);
+        return act == ACT_BF16 ? launch_layer_norm<ACT_BF16>(x, nullptr, x, y, post, pre, eps, T, n, out, ld, stream)
+                               : launch_layer_norm<ACT_F32>(x, nullptr, x, y, post, pre, eps, T, n, out, ld, stream);
+    }
+    MESH_ROW_LAUNCH(residual_norm_kernel, act, n % 4 == 0, dim3((unsigned)T), dim3(ROW_THREADS), x, y, post.gain, eps, n, out, ld);
     return MESH_OK;
+}
+
+int layer_norm_rows(const float *x, const int32_t *row, const RowNorm &norm, float eps, int n_rows, int n, void *out, ActType act, int ld, hipStream_t stream) {
+    if (n_rows <= 0) return MESH_OK;
+    if (ld < n || norm.kind != NORM_LAYER || !norm_ok(norm)) return fail(MESH_ERR_INVALID, "layer_norm_rows: bad operands");
+    return act == ACT_BF16 ? launch_layer_norm<ACT_BF16>(x, row, nullptr, nullptr, RowNorm{}, norm, eps, n_rows, n, out, ld, stream)
+                           : launch_layer_norm<ACT_F32>(x, row, nullptr, nullptr, RowNorm{}, norm, eps, n_rows, n, out, ld, stream);
 }
 
 int scalar_norm_rows(const float *x, const int32_t *row, const float *gain, float eps, int n_rows, int n, void *out, ActType act, int ld, hipStream_t stream) {

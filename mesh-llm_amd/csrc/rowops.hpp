@@ -4,14 +4,25 @@
 #pragma once
 
 #include "linear.hpp"
+#include "model_config.hpp"
 
 namespace mesh {
 
-// x[t] = table[tok[t]] * scale + position vector of pos[t]: entries 2i and 2i + 1 are sin and cos of pos * freq[i]
-int embed_rows(const uint16_t *table, const int32_t *tok, const int32_t *pos, const float *freq, float scale, int T, int n, float *x, hipStream_t stream);
+// A norm over a row, with what is folded into it: RMS takes gain, LAYER gain and bias.
+struct RowNorm {
+    NormKind kind = NORM_NONE;
+    const float *gain = nullptr, *bias = nullptr;
+};
 
-// x[t] += y[t] / rms(y[t]) * gain (y null: x as it is), and act[t] = x[t]
-int residual_norm_rows(float *x, const float *y, const float *gain, float eps, int T, int n, void *out, ActType act, int ld, hipStream_t stream);
+// x[t] = table[tok[t]] * scale, table rows of ldt, plus (freq set) the position vector of pos[t]: entries 2i and 2i + 1 are
+// sin and cos of pos * freq[i]
+int embed_rows(const uint16_t *table, int ldt, const int32_t *tok, const int32_t *pos, const float *freq, float scale, int T, int n, float *x, hipStream_t stream);
+
+// x[t] += post(y[t]) (y null: x as it is), and act[t] = pre(x[t]): post RMS with pre NONE, or both LAYER
+int residual_norm_rows(float *x, const float *y, const RowNorm &post, const RowNorm &pre, float eps, int T, int n, void *out, ActType act, int ld, hipStream_t stream);
+
+// act[i] = layer norm of x[row[i]] for i < n_rows (row null: i)
+int layer_norm_rows(const float *x, const int32_t *row, const RowNorm &norm, float eps, int n_rows, int n, void *out, ActType act, int ld, hipStream_t stream);
 
 // act[i] = x[row[i]] / rms * gain[0] for i < n_rows (row null: i)
 int scalar_norm_rows(const float *x, const int32_t *row, const float *gain, float eps, int n_rows, int n, void *out, ActType act, int ld, hipStream_t stream);

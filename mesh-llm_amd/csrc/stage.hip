@@ -85,6 +85,10 @@ void hparams_from_spec(const ModelSpec &s, HParams &hp) {
         hp.n_head_kv = std::max(hp.n_head_kv, (uint32_t)l.mixer.kv_heads);
         hp.head_dim = std::max(hp.head_dim, (uint32_t)l.mixer.dim);
         hp.n_ff = std::max(hp.n_ff, (uint32_t)l.ff);
+        if (l.mixer.kind == MIXER_LATENT) {
+            hp.rope_freq_base = (float)l.mixer.rot.base;
+            hp.n_rot = std::max(hp.n_rot, (uint32_t)l.mixer.rot_dim);
+        }
     }
 }
 
@@ -373,6 +377,8 @@ int sess_alloc(mesh_session *s, void **p, size_t bytes) {
 constexpr int ATTN_SPLITS_MAX = ATTN_SPLITS_CAP;
 constexpr int ATTN_PART_ROWS_MIN = 512;     // rows of (token, split) the partial buffers always hold
 constexpr int META_SLOTS = 8;
+// positions, sequence ids, token ids, wanted rows; chunk tables (hybrid_chunk_table)
+static constexpr size_t META_INTS(size_t B) { return 7 * B + 2; }
 constexpr int LOGITS_TOKENS_MAX = MESH_LOGITS_TOKENS_MAX;        // logits rows the host-pointer entry point stages per call
 // Mixture of experts: calls with at least moe_gemm_min_pairs (token, slot) pairs per expert on average run the expert
 // products as tiles of the large-tile GEMM (measured against the other kernels on a 64-expert shard with top-8 routing,
@@ -515,14 +521,14 @@ int session_new(mesh_stage *st, mesh_session **out) {
     int rc = st->hybrid ? hybrid_session_alloc(s.get()) : kquant_session_alloc(s.get());
     if (rc != MESH_OK) return rc;
     void *p = nullptr;
-    if ((rc = sess_alloc(s.get(), &p, 4 * B * sizeof(int32_t))) != MESH_OK) return rc;
+    if ((rc = sess_alloc(s.get(), &p, META_INTS(B) * sizeof(int32_t))) != MESH_OK) return rc;
     s->d_pos = static_cast<int32_t *>(p);
     s->d_seq = s->d_pos + B;
     s->d_tok = s->d_seq + B;
     s->d_rows = s->d_tok + B;
-    MESH_HIP_TRY(hipMemsetAsync(p, 0, 4 * B * sizeof(int32_t), s->stream));
-    MESH_HIP_TRY(hipHostMalloc(reinterpret_cast<void **>(&s->h_meta), META_SLOTS * 4 * B * sizeof(int32_t), hipHostMallocDefault));
-    memset(s->h_meta, 0, META_SLOTS * 4 * B * sizeof(int32_t));
+    MESH_HIP_TRY(hipMemsetAsync(p, 0, META_INTS(B) * sizeof(int32_t), s->stream));
+    MESH_HIP_TRY(hipHostMalloc(reinterpret_cast<void **>(&s->h_meta), META_SLOTS * META_INTS(B) * sizeof(int32_t), hipHostMallocDefault));
+    memset(s->h_meta, 0, META_SLOTS * META_INTS(B) * sizeof(int32_t));
     // staging for packed in/out of the host-pointer entry point: f32 rows of n_embd in; the same or logits rows out
     // (logits of at most LOGITS_TOKENS_MAX tokens per call: a row of a 152k vocabulary is 0.6 MB)
     s->io_stage_bytes = B * (size_t)hp.n_embd * sizeof(float);
@@ -1278,8 +1284,8 @@ static int decode_core(mesh_session *s, const mesh_batch *b, const int32_t *ids,
         for (int i = 0; i < T; ++i) n_rows += b->want[i] != 0;
     }
     if (st->hybrid) {
-        if (!ids) return fail(MESH_ERR_INVALID, "mesh_stage_decode: the layers of architecture '%s' read the token ids (batch.token_id)", hp.arch.c_str());
-        for (int i = 0; i < T; ++i)
+        if (!ids && (tokens_in || hybrid_needs_ids(st))) return fail(MESH_ERR_INVALID, "mesh_stage_decode: the layers of architecture '%s' read the token ids (batch.token_id)", hp.arch.c_str());
+        for (int i = 0; ids && i < T; ++i)
             if (ids[i] < 0 || ids[i] >= (int)hp.n_vocab) return fail(MESH_ERR_INVALID, "mesh_stage_decode: token id %d outside the vocabulary of %u", ids[i], hp.n_vocab);
         if ((rc = hybrid_check_batch(s, b)) != MESH_OK) return rc;
     }
@@ -1298,17 +1304,23 @@ static int decode_core(mesh_session *s, const mesh_batch *b, const int32_t *ids,
     // positions / sequence ids -> device, through a ring of pinned slots so calls may be queued back to back
     const size_t B = (size_t)st->n_batch_max;
     if (s->meta_counter && s->meta_counter % META_SLOTS == 0) MESH_HIP_TRY(hipStreamSynchronize(stream));   // ring wraps: older copies are done
-    int32_t *slot = s->h_meta + (size_t)(s->meta_counter++ % META_SLOTS) * 4 * B;
+    int32_t *slot = s->h_meta + (size_t)(s->meta_counter++ % META_SLOTS) * META_INTS(B);
     for (int i = 0; i < T; ++i) { slot[i] = b->pos[i]; slot[B + i] = b->seq_id ? b->seq_id[i] : 0; }
     size_t meta_ints = B + (size_t)T;
     if (st->hybrid) {
-        for (int i = 0; i < T; ++i) slot[2 * B + i] = ids[i];
-        meta_ints = 2 * B + (size_t)T;
+        if (ids) {
+            for (int i = 0; i < T; ++i) slot[2 * B + i] = ids[i];
+            meta_ints = 2 * B + (size_t)T;
+        }
     }
     if (picked && n_rows < T && n_rows > 0) {
         for (int i = 0, r = 0; i < T; ++i)
             if (b->want[i]) slot[3 * B + (size_t)r++] = i;
         meta_ints = 3 * B + (size_t)n_rows;
+    }
+    if (st->hybrid) {
+        const size_t n = hybrid_chunk_table(s, b, slot + 4 * B, s->d_pos + 4 * B);
+        if (n) meta_ints = 4 * B + n;
     }
     // (one copy for all: the slot and the device buffer have the same layout, positions at 0, sequence ids at B, token ids and
     // wanted rows behind them; a copy is a launch of its own on the stream, and the entries past each list are never read)

@@ -37,6 +37,7 @@ const TuningField *tuning_fields() {
         {"moe_gemm_min_pairs", &Tuning::moe_gemm_min_pairs, 1, 1 << 20, TUNE_SESSION},
         {"grouped_oversub", &Tuning::grouped_oversub, 1, 64, TUNE_SESSION},
         {"linear_tile_min_tokens", &Tuning::linear_tile_min_tokens, 1, 1 << 20, TUNE_SESSION},
+        {"latent_chunk_min_tokens", &Tuning::latent_chunk_min_tokens, 1, 1 << 20, TUNE_SESSION},
         {"step_fused", &Tuning::step_fused, 0, 1, TUNE_SESSION},
         {"graphs", &Tuning::graphs, 0, 1, TUNE_SESSION},
         {nullptr, nullptr, 0, 0, TUNE_STAGE},

@@ -41,6 +41,7 @@ struct Tuning {
     int moe_gemm_min_pairs = 4;    // ... from this many pairs per expert on average
     int grouped_oversub = 8;       // grouped expert mat-vec: workgroups per compute unit and item
     int linear_tile_min_tokens = 128;   // bf16 products of at least this many tokens on the large tile (below: the weight-streaming kernel)
+    int latent_chunk_min_tokens = 128;  // latent attention: a chunk of at least this many tokens projects its sequence's keys and values (below: queries meet the cached latents)
     int step_fused = 1;            // bf16 models, one token: products derive their input from what the launch before left (0: the many-token launches)
     int graphs = 0;                // decode steps of up to 32 tokens replayed from captured HIP graphs
 
