@@ -299,6 +299,7 @@ int mesh_session_f16_saturations(mesh_session *session, uint64_t *count);
  *     moe_gemm=1, moe_gemm_min_pairs=4   prefill-sized expert products on the large-tile GEMM
  *     grouped_oversub=8    grouped expert mat-vec: workgroups per compute unit and item
  *     linear_tile_min_tokens=128  bf16 products of at least this many tokens on the large matrix-core tile
+ *     latent_chunk_min_tokens=128  latent attention: chunks of at least this many tokens project their sequence's keys and values
  *     step_fused=1         bf16 models, one token: norms, activations and residual updates ride in the products
  *     graphs=0             decode steps of up to 32 tokens replayed from captured HIP graphs
  *

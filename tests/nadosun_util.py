@@ -1,9 +1,8 @@
 """Small random Nadosun models for the tests: configurations, weights (as the bf16 values a file can hold) and the folder
 with config.json and model.safetensors, written byte by byte."""
-import json
-import os
-
 import numpy as np
+
+from folder_util import bf16, error, prompt, safetensors_bytes, write_folder  # noqa: F401
 
 
 def attention(heads, kv_heads, dim, window, scale=None, ff=None):
@@ -28,12 +27,6 @@ CONFIGS = {
     "recurrent-only": config(64, 64, 8, [mingru(64), mingru(128, ff=64)]),
     "attention-only": config(64, 128, 16, [attention(2, 2, 64, 16, ff=128), attention(4, 2, 32, 300)]),
 }
-
-
-def bf16(a):
-    """Rounded to bfloat16 (nearest, ties to even), as float32."""
-    u = np.ascontiguousarray(a, np.float32).view(np.uint32)
-    return ((u + 0x7FFF + ((u >> 16) & 1)) & np.uint32(0xFFFF0000)).view(np.float32)
 
 
 def random_weights(cfg, seed):
@@ -74,27 +67,6 @@ def random_weights(cfg, seed):
     return {k: bf16(v).reshape(np.shape(v)) for k, v in w.items()}
 
 
-def safetensors_bytes(tensors):
-    """Weights as BF16 entries."""
-    head, blobs, at = {}, [], 0
-    for name, a in tensors.items():
-        b = (np.ascontiguousarray(a, np.float32).view(np.uint32) >> 16).astype("<u2").tobytes()
-        head[name] = {"dtype": "BF16", "shape": list(np.shape(a)), "data_offsets": [at, at + len(b)]}
-        blobs.append(b)
-        at += len(b)
-    h = json.dumps(head).encode()
-    return len(h).to_bytes(8, "little") + h + b"".join(blobs)
-
-
-def write_folder(path, cfg, tensors):
-    os.makedirs(path, exist_ok=True)
-    with open(os.path.join(path, "config.json"), "w") as f:
-        json.dump(cfg, f)
-    with open(os.path.join(path, "model.safetensors"), "wb") as f:
-        f.write(safetensors_bytes(tensors))
-    return path
-
-
 def only(w, cfg, keep):
     """The weights with every addition to the residual stream but `keep` ("mixer", "ff", "side" or "") scaled to nothing."""
     w = dict(w)
@@ -132,18 +104,3 @@ def needle_weights(cfg, seed, needle, asker, strength):
         w[p + "k.norm"] = np.ones_like(w[p + "k.norm"])
         w["l%d.norm1" % i] = np.float32(8.0)         # what attention finds outweighs the embeddings' own size
     return w
-
-
-def prompt(cfg, n, seed, avoid=()):
-    t = np.random.Generator(np.random.PCG64(seed)).integers(0, cfg["vocab"], n).astype(np.int32)
-    while np.isin(t, avoid).any():
-        t = np.where(np.isin(t, avoid), (t + 1) % cfg["vocab"], t).astype(np.int32)
-    return t
-
-
-def error(got, want):
-    """Largest over the rows: rms of the difference (its mean taken off) over the rms of all of `want`."""
-    got, want = np.asarray(got, np.float64), np.asarray(want, np.float64)
-    d = got - want
-    d -= d.mean(axis=-1, keepdims=True)
-    return float(np.sqrt((d ** 2).mean(axis=-1)).max() / np.sqrt((want ** 2).mean()))

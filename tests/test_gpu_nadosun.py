@@ -12,6 +12,7 @@ import pytest
 
 sys.path.insert(0, os.path.dirname(os.path.abspath(__file__)))
 import nadosun_util as N
+from folder_util import Seq, check_greedy, open_stage, run
 from oracle.nadosun import NadosunOracle
 from util import ROOT, mesh
 
@@ -29,40 +30,6 @@ def made(tmp, name, seed=11, change=None, key=None):
     if change:
         w = change(w, cfg)
     return cfg, w, N.write_folder(str(tmp / "model"), cfg, w), NadosunOracle(cfg, w)
-
-
-def open_stage(folder, prec, begin=0, end=-1, n_ctx=512, n_seq=4, batch=256, **kw):
-    m = mesh()
-    return m.Stage(folder, begin, end, n_ctx=n_ctx, n_seq_max=n_seq, n_batch_max=batch, precision=m.PRECISION_F32 if prec == "f32" else m.PRECISION_DEFAULT, **kw)
-
-
-class Seq:
-    """One sequence of a session, fed in portions."""
-
-    def __init__(self, stage, session, seq=0):
-        self.st, self.ses, self.seq, self.n = stage, session, seq, 0
-
-    def feed(self, tokens, out=None, want=None):
-        m = mesh()
-        pos = np.arange(self.n, self.n + len(tokens), dtype=np.int32)
-        raw = self.ses.decode(np.asarray(tokens, np.int32), pos, seq=np.full(len(tokens), self.seq, np.int32), in_fmt=m.TOKENS,
-                              out_fmt=m.LOGITS if out is None else out, want=want)
-        self.n += len(tokens)
-        return raw.view(np.float32).reshape(-1, self.st.info.n_vocab if out is None else self.st.info.n_embd)
-
-
-def run(stage, tokens, portions, seq=0, session=None, last=10 ** 9, **options):
-    """Logits of the last `last` tokens, fed in portions to a sequence that starts with them."""
-    ses = session or stage.session(**options)
-    s = Seq(stage, ses, seq)
-    rows, at = [], 0
-    for p in portions:
-        rows.append(s.feed(tokens[at:at + p], want=np.arange(at, at + p) >= len(tokens) - last))
-        at += p
-    assert at == len(tokens)
-    if session is None:
-        ses.close()
-    return np.concatenate(rows)
 
 
 # ------------------------------------------------------------------------------------------------ mechanisms
@@ -342,26 +309,6 @@ def test_long_decoding(tmp_path, prec):
 
 
 # ------------------------------------------------------------------------------------------------ generation
-def oracle_greedy(orc, prompt, n, forced=None):
-    orc.reset()
-    lg = orc.forward(prompt)[-1]
-    toks, margins = [], []
-    for i in range(n):
-        top = np.sort(lg)[-2:]
-        toks.append(int(lg.argmax()))
-        margins.append(float(top[1] - top[0]))
-        lg = orc.forward([toks[-1] if forced is None else forced[i]])[-1]
-    return toks, margins
-
-
-def check_greedy(orc, prompt, got, tol):
-    """Every generated token is the oracle's argmax, or one the precision cannot tell from it."""
-    toks, margins = oracle_greedy(orc, prompt, len(got), forced=got)
-    for a, b, mg in zip(got, toks, margins):
-        assert a == b or mg < tol, (a, b, mg)
-    assert sum(a == b for a, b in zip(got, toks)) >= 0.9 * len(got)
-
-
 @BOTH
 def test_greedy_generation_through_the_session(tmp_path, prec):
     m = mesh()
