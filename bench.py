@@ -1,7 +1,7 @@
 #!/usr/bin/env python3
 """Benchmark of the pipeline-stage hot path on one MI355X.  Prints ONE JSON line.
 
-  python bench.py [--gpus 1] [--steps K] [--warmup W] [--workload stage|codec|c4|c5|nadosun] [--batches 1,4,16]
+  python bench.py [--gpus 1] [--steps K] [--warmup W] [--workload stage|codec|c4|c5|nadosun|nutavik] [--batches 1,4,16]
 
 Workloads
   stage   (default) Llama-3-8B-shaped stage, layers 0-15 of 32 (hidden 4096, 32/8 heads, head_dim 128, FFN 14336,
@@ -17,6 +17,8 @@ Workloads
   nadosun Nadosun layers of two sizes (hidden 2048 and 4096: half windowed attention with a feed-forward, half minGRU),
           bf16 random weights, decode of one token behind 2048 and prefill of 2048; beside it a llama stage of the same
           width, heads and feed-forward (Q4_K_M), the closest K-quant model.  value = decode tokens/s at hidden 4096.
+  nutavik Nutavik layers of two sizes (hidden 2048 and 4096: latent attention, gated delta rule, gated linear attention in
+          turn), as above; beside it a Nadosun stage of the same width, depth and feed-forward.  value likewise.
 
 Timing uses HIP events recorded on the stream the kernels run on (the session's own stream for the stage).
 The cpu_baseline leg times the CPU oracle (a restatement of ggml's reference routines, NOT llama.cpp) on the
@@ -580,9 +582,7 @@ def nadosun_config(sp):
             "token_side": {"dim": sp["side"]}, "layers": [att if i % 4 in (0, 3) else gru for i in range(sp["layers"])]}
 
 
-def write_nadosun(folder, cfg):
-    """Random bf16 weights of sigma 1 / sqrt(row length), cut from one random block; norms and layer scales near 1."""
-    os.makedirs(folder, exist_ok=True)
+def nadosun_shapes(cfg):
     E, S, n = cfg["width"], cfg["token_side"]["dim"], len(cfg["layers"])
     shapes = {"embed": (cfg["vocab"], E), "side.embed": (cfg["vocab"], n * S), "final.norm": (), "head": (cfg["vocab"], E)}
     for i, l in enumerate(cfg["layers"]):
@@ -597,6 +597,12 @@ def write_nadosun(folder, cfg):
         shapes.update({p + "norm1": (), p + "ls1": (E,), p + "side.gate": (S, E), p + "side.proj": (E, S), p + "side.norm": (E,)})
         if l["mlp"]:
             shapes.update({p + "mlp.up": (l["mlp"]["ff"], E), p + "mlp.down": (E, l["mlp"]["ff"]), p + "mlp.act": (4,), p + "norm2": (), p + "ls2": (E,)})
+    return shapes
+
+
+def write_model_folder(folder, cfg, shapes, fill=lambda name: 0.8):
+    """Random bf16 weights of sigma 1 / sqrt(row length), cut from one random block; vectors hold the number `fill` gives."""
+    os.makedirs(folder, exist_ok=True)
     rng = np.random.Generator(np.random.PCG64(42))
     base = rng.standard_normal(1 << 24).astype(np.float32)
 
@@ -619,7 +625,7 @@ def write_nadosun(folder, cfg):
         for k, (name, sh) in enumerate(shapes.items()):
             count = int(np.prod(sh, dtype=np.int64))
             if len(sh) < 2:
-                f.write(bits(np.full(count, 0.8)).tobytes())
+                f.write(bits(np.full(count, fill(name))).tobytes())
                 continue
             if sh[1] not in scaled:
                 scaled[sh[1]] = bits(base if "embed" in name else base / np.sqrt(sh[1]))
@@ -659,7 +665,7 @@ def bench_nadosun(args):
     for name, sp in NADOSUN_SIZES.items():
         T, L = NADOSUN_T, sp["layers"]
         folder = os.path.join(models.tmp_dir(), "mesh_bench_nadosun")
-        write_nadosun(folder, nadosun_config(sp))
+        write_model_folder(folder, nadosun_config(sp), nadosun_shapes(nadosun_config(sp)))
         st = m.Stage(folder, 0, L, n_ctx=NADOSUN_CTX, n_batch_max=T)
         shutil.rmtree(folder)
         path = os.path.join(models.tmp_dir(), "mesh_bench_nadosun_llama.gguf")
@@ -741,12 +747,151 @@ def bench_nadosun(args):
             "sizes": sizes}
 
 
+# ------------------------------------------------------------------------------------------------ Nutavik
+NUTAVIK_SIZES = {
+    # width, heads (latent attention; delta, over half as many q / k heads; GLA), feed-forward, layers (latent, delta, GLA, latent over
+    # the first one's cache, delta, GLA, ...); heads of 128 + 64 key and 128 value entries, ranks 512 and 1536, states of 128 x 128
+    "2048": dict(E=2048, H=16, FF=8192, layers=12),
+    "4096": dict(E=4096, H=32, FF=14336, layers=6),
+}
+
+
+def nutavik_config(sp):
+    H, layers = sp["H"], []
+    ff = {"kind": "dense", "ff": sp["FF"]}
+    for i in range(sp["layers"]):
+        if i % 3 == 0:
+            m = {"heads": H, "dim": 128, "rot_dim": 64, "vdim": 128, "kv_rank": 512, "q_rank": 1536, "scale": 192 ** -0.5,
+                 "rot": {"dims": 64, "base": 10000.0, "scaling": {"factor": 4.0, "original": 4096, "fast": 32.0, "slow": 1.0}}}
+            if i % 6 == 3:
+                m["kv_from"] = i - 3
+            layers.append({"type": "latent_attention", "mixer": m, "mlp": ff})
+        elif i % 3 == 1:
+            layers.append({"type": "delta", "mixer": {"heads": H, "kv_heads": H // 2, "dim": 128, "vdim": 128, "conv": 4}, "mlp": ff})
+        else:
+            layers.append({"type": "gla", "mixer": {"heads": H, "dim": 128, "vdim": 128, "tau": 16.0}, "mlp": ff})
+    return {"architecture": "Nutavik", "vocab": NADOSUN_VOCAB, "width": sp["E"], "norm": {"eps": 1e-5}, "residual_mult": 0.7, "logit_scale": 1.0, "layers": layers}
+
+
+def nutavik_shapes(cfg):
+    E = cfg["width"]
+    shapes = {"embed": (cfg["vocab"], E), "final.norm": (E,), "final.norm.b": (E,)}
+    for i, l in enumerate(cfg["layers"]):
+        p, m = "l%d." % i, l["mixer"]
+        x, H, v = p + "mix.", m["heads"], m["heads"] * m["vdim"]
+        if l["type"] == "latent_attention":
+            shapes.update({x + "dq": (m["q_rank"], E), x + "dq.norm": (m["q_rank"],), x + "uq": (H * (m["dim"] + m["rot_dim"]), m["q_rank"]),
+                           x + "uk": (H * m["dim"], m["kv_rank"]), x + "uv": (v, m["kv_rank"]), x + "g": (H, E)})
+            if "kv_from" not in m:
+                shapes.update({x + "dkv": (m["kv_rank"] + m["rot_dim"], E), x + "dkv.norm": (m["kv_rank"],)})
+        else:
+            qk = m.get("kv_heads", H) * m["dim"]
+            shapes.update({x + "q": (qk, E), x + "k": (qk, E), x + "v": (v, E), x + "g": (v, E), x + "norm": (m["vdim"],)})
+            if l["type"] == "delta":
+                shapes.update({x + "q.conv": (qk, m["conv"]), x + "k.conv": (qk, m["conv"]), x + "v.conv": (v, m["conv"]), x + "b": (H, E), x + "a": (H, E),
+                               x + "A_log": (H,), x + "dt_bias": (H,)})
+            else:
+                shapes.update({x + "a1": (16, E), x + "a2": (qk, 16), x + "a2.b": (qk,)})
+        shapes[x + "o"] = (E, v)
+        for n in ("norm1", "norm1b", "norm2", "norm2b"):
+            shapes.update({p + n: (E,), p + n + ".b": (E,)})
+        shapes.update({p + "mlp.up": (l["mlp"]["ff"], E), p + "mlp.down": (E, l["mlp"]["ff"])})
+    return shapes
+
+
+def folder_macs(shapes):
+    """Multiply-adds of one token in the matrices of the layers (every one is read once per step)."""
+    return sum(int(np.prod(sh, dtype=np.int64)) for n, sh in shapes.items() if len(sh) == 2 and "embed" not in n and n != "head" and ".conv" not in n and not n.endswith(".a2"))
+
+
+def bench_nutavik(args):
+    """Nutavik beside Nadosun of the same width, depth and feed-forward (half its layers attention over every earlier token), in turn."""
+    import shutil
+    import torch
+    import __graft_entry__ as graft
+    import models
+    m = graft.load_package()
+    m.lib()
+    sizes = {}
+    T = NADOSUN_T
+    for name, sp in NUTAVIK_SIZES.items():
+        E = sp["E"]
+        nad = nadosun_config(dict(E=E, H=sp["H"], G=sp["H"] // 4, FF=sp["FF"], window=NADOSUN_CTX, side=E // 16, layers=sp["layers"]))
+        for l in nad["layers"]:
+            l["mlp"] = {"kind": "dense", "ff": sp["FF"]}
+        nut = nutavik_config(sp)
+        sides = {}
+        for side, cfg, shapes in (("nutavik", nut, nutavik_shapes(nut)), ("nadosun", nad, nadosun_shapes(nad))):
+            folder = os.path.join(models.tmp_dir(), "mesh_bench_" + side)
+            write_model_folder(folder, cfg, shapes, lambda n: 0.8 if "norm" in n and not n.endswith(".b") or "ls" in n or "act" in n else 0.05)
+            st = m.Stage(folder, 0, sp["layers"], n_ctx=NADOSUN_CTX, n_batch_max=T)
+            shutil.rmtree(folder)
+            sides[side] = dict(st=st, ses=st.session(), macs=folder_macs(shapes), res={"prefill_ms": [], "decode_ms": []})
+        print("[bench] nutavik %s: stages open" % name, file=sys.stderr, flush=True)
+        rng = np.random.Generator(np.random.PCG64(1))
+        xs = torch.from_numpy(rng.standard_normal((T, E)).astype(np.float32)).cuda()
+        out = torch.empty(T * E, dtype=torch.float32, device="cuda")
+        ids = rng.integers(0, NADOSUN_VOCAB, T).astype(np.int32)
+
+        def calls(ses):
+            at = [0]
+
+            def feed(n):
+                def run(i):
+                    if at[0] + n > NADOSUN_CTX:
+                        at[0] = 0
+                    ses.decode_dev(xs.data_ptr(), np.arange(at[0], at[0] + n), out.data_ptr(), T * E * 4, token_ids=ids[:n])
+                    at[0] += n
+                return run
+
+            def prefill(i):
+                at[0] = 0
+                feed(T)(i)
+            return prefill, feed
+
+        for s in sides.values():
+            s["stream"] = torch.cuda.ExternalStream(s["ses"].stream)
+            s["prefill"], s["feed"] = calls(s["ses"])
+        for _ in range(args.burn_in):           # untimed; see bench_stage
+            sides["nadosun"]["feed"](1)(0)
+        torch.cuda.synchronize()
+        steps = min(args.steps, 500)
+        for _ in range(3):
+            for s in sides.values():
+                s["res"]["prefill_ms"].append(time_on_stream(torch, s["stream"], s["prefill"], 3, 1)[0])
+                s["res"]["decode_ms"].append(time_on_stream(torch, s["stream"], s["feed"](1), steps, args.warmup)[0])
+        for side, s in sides.items():
+            r, by, mc = s["res"], 2 * s["macs"], s["macs"]
+            for k in ("prefill_ms", "decode_ms"):
+                r[k] = round(min(r[k]), 4)
+            pms, pl = kernel_ms(s["ses"], s["prefill"], 1)
+            dms, dl = kernel_ms(s["ses"], s["feed"](1), 5)
+            for n in (16, 64):
+                s["prefill"](0)
+                fn = s["feed"](n)
+                ms = time_on_stream(torch, s["stream"], fn, 50, 5)[0]
+                pk, _ = kernel_ms(s["ses"], fn, 5)
+                r["portion_%d" % n] = {"ms": round(ms, 4), "kernel_ms": pk}
+            r.update({"prefill_tok_s": round(T * 1e3 / r["prefill_ms"], 1), "decode_tok_s": round(1e3 / r["decode_ms"], 1), "weight_GB": round(by / 1e9, 3),
+                      "prefill_kernel_ms": pms, "prefill_launches": pl, "decode_kernel_ms": dms, "decode_launches": dl,
+                      "products_prefill_TFLOPs": round(2.0 * mc * T / pms["gemv"] / 1e9, 1), "products_decode_GBps": round(by / dms["gemv"] / 1e6, 1),
+                      "step_frac_hbm": round(by / r["decode_ms"] / 1e6 / HBM_PEAK_GBS, 4)})
+            s["ses"].close(), s["st"].close()
+        sizes[name] = dict(shape=dict(sp, tokens=T), **{k: s["res"] for k, s in sides.items()})
+    head = sizes["4096"]["nutavik"]
+    return {"metric": "Nutavik decode tok/s, hidden 4096, 6 layers", "value": head["decode_tok_s"], "unit": "tok/s", "n_gpus": 1, "steps": args.steps, "warmup": args.warmup,
+            "ms_per_step": head["decode_ms"], "higher_is_better": True, "scaling": "weak", "vs_baseline": None, "dtype": "bf16", "data": "synthetic",
+            "config": {"workload": "Nutavik layers of two sizes, random bf16 weights, single-token decode behind %d tokens and %d-token prefill, beside Nadosun stages of the "
+                                   "same width, depth and feed-forward" % (T, T)},
+            "sizes": sizes}
+
+
 def main():
     ap = argparse.ArgumentParser()
     ap.add_argument("--gpus", type=int, default=1)
     ap.add_argument("--steps", type=int, default=100)
     ap.add_argument("--warmup", type=int, default=10)
-    ap.add_argument("--workload", default="stage", choices=["stage", "codec", "c4", "c5", "nadosun"])
+    ap.add_argument("--workload", default="stage", choices=["stage", "codec", "c4", "c5", "nadosun", "nutavik"])
     ap.add_argument("--batches", default=None, help="decode batch sizes; the first is the headline value (default 1,4,16 for the stage workload, the shape's own list for c4 / c5)")
     ap.add_argument("--kv", default="f16", choices=["f16", "q8_0/q4_0", "q4_0/q4_0"],
                     help="KV cache row types K/V (default f16: the tier the reference picks for an 8B Q4_K_M model)")
@@ -760,7 +905,7 @@ def main():
         sys.exit(2)
     args.kv_given = any(a == "--kv" or a.startswith("--kv=") for a in sys.argv[1:])
     out = bench_stage(args) if args.workload == "stage" else bench_codec(args) if args.workload == "codec" else \
-        bench_nadosun(args) if args.workload == "nadosun" else bench_shape(args)
+        bench_nadosun(args) if args.workload == "nadosun" else bench_nutavik(args) if args.workload == "nutavik" else bench_shape(args)
     print(json.dumps(out))
 
 

@@ -31,13 +31,6 @@ __device__ __forceinline__ gs_f4 gs_mma(const float4 &a, const gs_f4 &b, gs_f4 a
 }
 __device__ __forceinline__ gs_f4 gs_mma(const float4 &a, const float4 &b, gs_f4 acc) { return gs_mma(a, gs_f4{b.x, b.y, b.z, b.w}, acc); }
 
-// logarithm of the decay of key channel `ch` (head * dim + d) of token t: log sigmoid(z) / tau
-__device__ __forceinline__ float gla_log_decay(const GatedStateArgs &a, int t, int ch) {
-    const float *x = a.in + (size_t)t * a.ld + a.at_a, *w = a.a2 + (size_t)ch * a.rank;
-    float z = a.a2_bias[ch];
-    for (int r = 0; r < a.rank; ++r) z = fmaf(w[r], x[r], z);
-    return -gs_softplus(-z) * a.inv_tau;
-}
 __device__ __forceinline__ float delta_log_decay(const GatedStateArgs &a, int t, int h) { return -a.A[h] * gs_softplus(a.in[(size_t)t * a.ld + a.at_a + h] + a.dt_bias[h]); }
 __device__ __forceinline__ float delta_beta(const GatedStateArgs &a, int t, int h) { return act_sigmoid(a.in[(size_t)t * a.ld + a.at_b + h]); }
 
@@ -54,6 +47,34 @@ __device__ __forceinline__ float delta_conv(const GatedStateArgs &a, const float
         v = fmaf(w[j], x, v);
     }
     return act_silu(v);
+}
+
+// The same for tokens t0 .. t0 + 15 (the first `live` of them; zeros behind), up to CONV_WINDOW taps: every input is read once.
+constexpr int CONV_WINDOW = 4, CONV_RUN = 16;
+__device__ __forceinline__ void delta_conv_run(const GatedStateArgs &a, const float *w, int t0, int live, int t_first, int pos0, const float *tail, int at, int channels, float (&y)[CONV_RUN]) {
+    float x[CONV_RUN + CONV_WINDOW - 1], wt[CONV_WINDOW];
+#pragma unroll
+    for (int j = 0; j < CONV_WINDOW; ++j) {
+        const int tap = a.taps - CONV_WINDOW + j;
+        wt[j] = tap >= 0 ? w[tap] : 0.f;
+    }
+#pragma unroll
+    for (int i = 0; i < CONV_RUN + CONV_WINDOW - 1; ++i) {
+        const int k = i - (CONV_WINDOW - 1);              // token t0 + k at position pos0 + k
+        x[i] = 0.f;
+        if (k < 0) {
+            if (-k < a.taps && pos0 + k >= 0) x[i] = t0 + k >= t_first ? a.in[(size_t)(t0 + k) * a.ld + at] : tail[(size_t)((unsigned)(pos0 + k) % (unsigned)a.taps) * channels];
+        } else if (k < live) {
+            x[i] = a.in[(size_t)(t0 + k) * a.ld + at];
+        }
+    }
+#pragma unroll
+    for (int k = 0; k < CONV_RUN; ++k) {
+        float v = 0.f;
+#pragma unroll
+        for (int j = 0; j < CONV_WINDOW; ++j) v = fmaf(wt[j], x[k + j], v);
+        y[k] = k < live ? act_silu(v) : 0.f;
+    }
 }
 
 // ---- one token per sequence
@@ -76,16 +97,24 @@ __global__ __launch_bounds__(THREADS) void gated_step_kernel(const GatedStateArg
     const float *x = a.in + (size_t)t * a.ld;
     float decay = 1.f, beta = 1.f;
     if (a.delta) {
-        const int kvh = h / (a.heads / a.kv_heads), channels = 2 * a.kv_heads * D + a.heads * V;
-        float *slot = a.tail + ((size_t)seq * a.taps + pos % a.taps) * channels;
+        const int kvh = h / (a.heads / a.kv_heads), channels = 2 * a.kv_heads * D + a.heads * V, taps = a.taps, now = pos % taps;
+        float *tail = a.tail + (size_t)seq * taps * channels;
         const bool own = h % (a.heads / a.kv_heads) == 0;           // one head of a group keeps the shared channels' inputs
         for (int i = tid; i < 2 * D + V; i += THREADS) {
             const int part = i < D ? 0 : i < 2 * D ? 1 : 2, e = part == 0 ? i : part == 1 ? i - D : i - 2 * D;
             const int c = part == 2 ? h * V + e : kvh * D + e;
             const int at = (part == 0 ? a.at_q : part == 1 ? a.at_k : a.at_v) + c, ch = (part == 0 ? 0 : part == 1 ? a.kv_heads * D : 2 * a.kv_heads * D) + c;
-            const float y = delta_conv(a, (part == 0 ? a.conv_q : part == 1 ? a.conv_k : a.conv_v) + (size_t)c * a.taps, t, t, at, ch, channels);
-            (part == 0 ? sq : part == 1 ? sk : sv)[e] = y;
-            if (own || part == 2) slot[ch] = x[at];                  // (no slot that is read in this call: those are of taps - 1 other positions)
+            const float *w = (part == 0 ? a.conv_q : part == 1 ? a.conv_k : a.conv_v) + (size_t)c * taps;
+            const float xi = x[at];
+            float y = w[taps - 1] * xi;
+#pragma unroll 4
+            for (int back = 1; back < taps; ++back) {
+                const int slot = now - back < 0 ? now - back + taps : now - back;
+                const float p = pos >= back ? tail[(size_t)slot * channels + ch] : 0.f;
+                y = fmaf(w[taps - 1 - back], p, y);
+            }
+            (part == 0 ? sq : part == 1 ? sk : sv)[e] = act_silu(y);
+            if (own || part == 2) tail[(size_t)now * channels + ch] = xi;       // (not a slot that is read in this call: those are of taps - 1 other positions)
         }
         decay = expf(delta_log_decay(a, t, h));
         beta = delta_beta(a, t, h);
@@ -101,7 +130,19 @@ __global__ __launch_bounds__(THREADS) void gated_step_kernel(const GatedStateArg
         for (int d = tid; d < D; d += THREADS) {
             sq[d] = x[a.at_q + h * D + d] * qs;
             sk[d] = x[a.at_k + h * D + d];
-            sd[d] = expf(gla_log_decay(a, t, h * D + d));
+        }
+        // four lanes per channel
+        for (int d0 = 0; d0 < D; d0 += THREADS / 4) {
+            const int d = d0 + (tid >> 2);
+            float z = 0.f;
+            if (d < D) {
+                const float *w = a.a2 + (size_t)(h * D + d) * a.rank;
+#pragma unroll 4
+                for (int r = tid & 3; r < a.rank; r += 4) z = fmaf(w[r], x[a.at_a + r], z);
+            }
+            z += __shfl_xor(z, 1);
+            z += __shfl_xor(z, 2);
+            if (d < D && (tid & 3) == 0) sd[d] = expf(-gs_softplus(-(z + a.a2_bias[h * D + d])) * a.inv_tau);
         }
         for (int v = tid; v < V; v += THREADS) sv[v] = x[a.at_v + h * V + v];
     }
@@ -116,8 +157,7 @@ __global__ __launch_bounds__(THREADS) void gated_step_kernel(const GatedStateArg
     float dk = 0.f, dq = 0.f;
 #pragma unroll
     for (int i = 0; i < RPT; ++i) {
-        const int d = grp + i * groups;
-        if (d >= D) break;
+        const int d = grp + i * groups < D ? grp + i * groups : D - 1;          // (rows past the state are zeros)
         S[i] *= a.delta ? decay : sd[d];
         dk = fmaf(S[i], sk[d], dk);
         dq = fmaf(S[i], sq[d], dq);
@@ -183,28 +223,39 @@ __global__ __launch_bounds__(PREP_THREADS) void delta_prepare_kernel(const Gated
     const int D = a.dim, V = a.vdim, Dp = gs_pad64(D), Vp = gs_pad16(V), dp = Dp + 4, vp = Vp + 4;
     constexpr int LP = C + 4;
     float *sQ = sm, *sK = sQ + C * dp, *sV = sK + C * dp, *sL = sV + C * vp, *sA = sL + C * LP, *sT = sA + C * LP;
-    float *s_cum = sT + C * LP, *s_beta = s_cum + C;
+    float *s_cum = sT + C * LP, *s_beta = s_cum + C, *s_since = s_beta + C, *s_until = s_since + C;       // decays since the chunk's start, until its end
     const int t0 = a.chunks.chunk[ci], n = a.chunks.chunk[ci + 1] - t0, first = a.chunks.first[ci];
     const int kvh = h / (a.heads / a.kv_heads), channels = 2 * a.kv_heads * D + a.heads * V;
-    for (int i = tid; i < C * Dp; i += PREP_THREADS) {
-        const int r = i / Dp, d = i % Dp, ch = kvh * D + d;
-        float q = 0.f, k = 0.f;
-        if (r < n && d < D) {
-            q = delta_conv(a, a.conv_q + (size_t)ch * a.taps, t0 + r, first, a.at_q + ch, ch, channels);
-            k = delta_conv(a, a.conv_k + (size_t)ch * a.taps, t0 + r, first, a.at_k + ch, a.kv_heads * D + ch, channels);
+    // a channel's half chunk per thread: columns of q, of k, of v
+    const int pos0 = a.pos[t0];
+    const float *tail = a.tail + (size_t)a.seq[t0] * a.taps * channels;
+    for (int i = tid; i < 2 * (2 * Dp + Vp); i += PREP_THREADS) {
+        const int half = i >= 2 * Dp + Vp, e = half ? i - (2 * Dp + Vp) : i, part = e < Dp ? 0 : e < 2 * Dp ? 1 : 2, d = e - part * Dp;
+        const int c0 = part == 2 ? h * V + d : kvh * D + d, r0 = half * CONV_RUN;
+        const int at = (part == 0 ? a.at_q : part == 1 ? a.at_k : a.at_v) + c0, ch = part * a.kv_heads * D + c0;
+        const float *w = (part == 0 ? a.conv_q : part == 1 ? a.conv_k : a.conv_v) + (size_t)c0 * a.taps;
+        float y[CONV_RUN];
+        const int live = d < (part == 2 ? V : D) ? n - r0 : 0;
+        if (live <= 0) {
+#pragma unroll
+            for (int k = 0; k < CONV_RUN; ++k) y[k] = 0.f;
+        } else if (a.taps <= CONV_WINDOW) {
+            delta_conv_run(a, w, t0 + r0, live, first, pos0 + r0, tail + ch, at, channels, y);
+        } else {
+#pragma unroll
+            for (int k = 0; k < CONV_RUN; ++k) y[k] = k < live ? delta_conv(a, w, t0 + r0 + k, first, at, ch, channels) : 0.f;
         }
-        sQ[r * dp + d] = q;
-        sK[r * dp + d] = k;
-    }
-    for (int i = tid; i < C * Vp; i += PREP_THREADS) {
-        const int r = i / Vp, v = i % Vp, ch = h * V + v;
-        sV[r * vp + v] = r < n && v < V ? delta_conv(a, a.conv_v + (size_t)ch * a.taps, t0 + r, first, a.at_v + ch, 2 * a.kv_heads * D + ch, channels) : 0.f;
+        float *dst = (part == 0 ? sQ : part == 1 ? sK : sV) + d;
+        const int pitch = part == 2 ? vp : dp;
+#pragma unroll
+        for (int k = 0; k < CONV_RUN; ++k) dst[(r0 + k) * pitch] = y[k];
     }
     if (wave == 0) {          // logarithms of the decays, summed from the chunk's start
         float s = lane < n ? delta_log_decay(a, t0 + lane, h) : 0.f;
 #pragma unroll
         for (int o = 1; o < C; o <<= 1) { const float p = __shfl_up(s, o); if (lane >= o) s += p; }
-        if (lane < C) { s_cum[lane] = s; s_beta[lane] = lane < n ? delta_beta(a, t0 + lane, h) : 0.f; }
+        const float end = __shfl(s, C - 1);
+        if (lane < C) { s_cum[lane] = s; s_beta[lane] = lane < n ? delta_beta(a, t0 + lane, h) : 0.f; s_since[lane] = expf(s); s_until[lane] = expf(end - s); }
     }
     __syncthreads();
     const float qs = 1.0f / sqrtf((float)D);
@@ -240,28 +291,32 @@ __global__ __launch_bounds__(PREP_THREADS) void delta_prepare_kernel(const Gated
         float x[C];
 #pragma unroll
         for (int r = 0; r < C; ++r) {
-            float v = r == j ? 1.f : 0.f;
+            float v[4] = {r == j ? 1.f : 0.f, 0.f, 0.f, 0.f};          // (four sums: the chain through x is long enough)
 #pragma unroll
-            for (int k = 0; k < r; ++k) v = fmaf(-sL[r * LP + k], x[k], v);
-            x[r] = v;
+            for (int k = 0; k < r; ++k) v[k & 3] = fmaf(-sL[r * LP + k], x[k], v[k & 3]);
+            x[r] = (v[0] + v[1]) + (v[2] + v[3]);
         }
         if (lane < C) {
 #pragma unroll
             for (int r = 0; r < C; ++r) sT[r * LP + j] = x[r];
         }
     } else {
-        const float end = s_cum[C - 1];
         const int id = tid - 64, step = PREP_THREADS - 64;
-        for (int i = id; i < C * Dp; i += step) {
-            const int r = i / Dp, d = i % Dp;
-            m.Q[i] = sQ[r * dp + d] * expf(s_cum[r]);
+        for (int r = wave - 1; r < C; r += 3) {
+            const float f = s_since[r];
+            for (int d = lane * 4; d < Dp; d += 256) {
+                float4 q = *reinterpret_cast<const float4 *>(sQ + r * dp + d);
+                q.x *= f; q.y *= f; q.z *= f; q.w *= f;
+                *reinterpret_cast<float4 *>(m.Q + (size_t)r * Dp + d) = q;
+            }
         }
-        for (int i = id; i < C * Dp; i += step) {
-            const int d = i / C, r = i % C;
-            m.KT[i] = sK[r * dp + d] * expf(end - s_cum[r]);
+        for (int i = id; i < Dp * (C / 4); i += step) {
+            const int d = i / (C / 4), r = i % (C / 4) * 4;
+            *reinterpret_cast<float4 *>(m.KT + (size_t)d * C + r) =
+                make_float4(sK[r * dp + d] * s_until[r], sK[(r + 1) * dp + d] * s_until[r + 1], sK[(r + 2) * dp + d] * s_until[r + 2], sK[(r + 3) * dp + d] * s_until[r + 3]);
         }
-        for (int i = id; i < C * C; i += step) m.A[i] = sA[(i / C) * LP + i % C];
-        for (int i = id; i < Dp; i += step) m.G[i] = expf(end);
+        for (int i = id; i < C * C / 4; i += step) *reinterpret_cast<float4 *>(m.A + 4 * i) = *reinterpret_cast<const float4 *>(sA + (i / (C / 4)) * LP + i % (C / 4) * 4);
+        for (int i = id; i < Dp; i += step) m.G[i] = s_since[C - 1];
     }
     __syncthreads();
     // W = T (beta decay K), U = T (beta V): column tiles dealt to the waves, both row tiles of each
@@ -277,7 +332,7 @@ __global__ __launch_bounds__(PREP_THREADS) void delta_prepare_kernel(const Gated
 #pragma unroll
             for (int j = 0; j < 4; ++j) {
                 const int k = 16 * s + 4 * g + j;
-                b[j] = X[k * xp + c] * s_beta[k] * (w ? expf(s_cum[k]) : 1.f);
+                b[j] = X[k * xp + c] * s_beta[k] * (w ? s_since[k] : 1.f);
             }
 #pragma unroll
             for (int rt = s; rt < 2; ++rt) acc[rt] = gs_mma(*reinterpret_cast<const float4 *>(sT + (16 * rt + c) * LP + 16 * s + 4 * g), b, acc[rt]);
@@ -293,7 +348,7 @@ __global__ __launch_bounds__(PREP_THREADS) void delta_prepare_kernel(const Gated
     }
 }
 static size_t delta_prepare_lds(int dim, int vdim) {
-    return ((size_t)C * (2 * (gs_pad64(dim) + 4) + gs_pad16(vdim) + 4 + 3 * (C + 4)) + 2 * C) * sizeof(float);
+    return ((size_t)C * (2 * (gs_pad64(dim) + 4) + gs_pad16(vdim) + 4 + 3 * (C + 4)) + 4 * C) * sizeof(float);
 }
 
 // grid (chunks, heads)
@@ -303,30 +358,59 @@ __global__ __launch_bounds__(PREP_THREADS) void gla_prepare_kernel(const GatedSt
     const int D = a.dim, Dp = gs_pad64(D), dp = Dp + 4;
     float *sQ = sm, *sK = sQ + C * dp, *sG = sK + C * dp;         // queries, keys, logarithms of the decays summed from the chunk's start
     const int t0 = a.chunks.chunk[ci], n = a.chunks.chunk[ci + 1] - t0;
+    float *sX = sG + C * dp, *sS = sX + C * a.rank;               // a1 rows; sums over the first half chunk
     const float qs = 1.0f / sqrtf((float)D);
-    for (int i = tid; i < C * Dp; i += PREP_THREADS) {
-        const int r = i / Dp, d = i % Dp;
-        const bool live = r < n && d < D;
-        const float *x = a.in + (size_t)(t0 + (live ? r : 0)) * a.ld + h * D + (live ? d : 0);
-        sQ[r * dp + d] = live ? x[a.at_q] * qs : 0.f;
-        sK[r * dp + d] = live ? x[a.at_k] : 0.f;
-        sG[r * dp + d] = live ? gla_log_decay(a, t0 + r, h * D + d) : 0.f;
+    for (int r = wave; r < C; r += 4) {
+        const float *x = a.in + (size_t)(t0 + (r < n ? r : 0)) * a.ld;
+        for (int d = lane; d < Dp; d += 64) {
+            const bool live = r < n && d < D;
+            sQ[r * dp + d] = live ? x[a.at_q + h * D + d] * qs : 0.f;
+            sK[r * dp + d] = live ? x[a.at_k + h * D + d] : 0.f;
+        }
+        for (int k = lane; k < a.rank; k += 64) sX[r * a.rank + k] = r < n ? x[a.at_a + k] : 0.f;
     }
     __syncthreads();
-    for (int d = tid; d < Dp; d += PREP_THREADS) {
-        float s = 0.f;
+    // a channel's half chunk per thread: its pre-activations, then the running sums of their logarithms
+    constexpr int HALF = C / 2;
+    for (int i0 = 0; i0 < 2 * Dp; i0 += PREP_THREADS) {
+        const int i = i0 + tid, half = i >= Dp, d = half ? i - Dp : i, r0 = half * HALF;
+        float z[HALF];
+        if (i < 2 * Dp) {
+            const float *w = a.a2 + (size_t)(h * D + (d < D ? d : 0)) * a.rank;
+            const float bias = d < D ? a.a2_bias[h * D + d] : 0.f;
 #pragma unroll
-        for (int r = 0; r < C; ++r) { s += sG[r * dp + d]; sG[r * dp + d] = s; }
+            for (int k = 0; k < HALF; ++k) z[k] = bias;
+            for (int j = 0; j < a.rank; ++j) {
+                const float wj = w[j];
+#pragma unroll
+                for (int k = 0; k < HALF; ++k) z[k] = fmaf(wj, sX[(r0 + k) * a.rank + j], z[k]);
+            }
+            float sum = 0.f;
+#pragma unroll
+            for (int k = 0; k < HALF; ++k) {
+                sum += d < D && r0 + k < n ? -gs_softplus(-z[k]) * a.inv_tau : 0.f;
+                z[k] = sum;
+            }
+            if (!half) sS[d] = sum;
+        }
+        __syncthreads();            // (first halves are behind when their second halves add them: Dp <= PREP_THREADS)
+        if (i < 2 * Dp) {
+            const float before = half ? sS[d] : 0.f;
+#pragma unroll
+            for (int k = 0; k < HALF; ++k) sG[(r0 + k) * dp + d] = z[k] + before;
+        }
     }
     __syncthreads();
     const GsMats m(a.ws, (size_t)ci * a.heads + h, Dp, 0, false);
-    for (int i = tid; i < C * Dp; i += PREP_THREADS) {
-        const int r = i / Dp, d = i % Dp;
-        m.Q[i] = sQ[r * dp + d] * expf(sG[r * dp + d]);
-    }
-    for (int i = tid; i < C * Dp; i += PREP_THREADS) {
-        const int d = i / C, r = i % C;
-        m.KT[i] = sK[r * dp + d] * expf(sG[(C - 1) * dp + d] - sG[r * dp + d]);
+    for (int r = wave; r < C; r += 4)
+        for (int d = lane; d < Dp; d += 64) m.Q[(size_t)r * Dp + d] = sQ[r * dp + d] * expf(sG[r * dp + d]);
+    for (int i = tid; i < Dp * (C / 4); i += PREP_THREADS) {
+        const int d = i / (C / 4), r = i % (C / 4) * 4;
+        const float end = sG[(C - 1) * dp + d];
+        float k[4];
+#pragma unroll
+        for (int j = 0; j < 4; ++j) k[j] = sK[(r + j) * dp + d] * expf(end - sG[(r + j) * dp + d]);
+        *reinterpret_cast<float4 *>(m.KT + (size_t)d * C + r) = make_float4(k[0], k[1], k[2], k[3]);
     }
     for (int d = tid; d < Dp; d += PREP_THREADS) m.G[d] = expf(sG[(C - 1) * dp + d]);
     // A: a decay per channel does not leave the sum over channels.  Within a 16 x 16 diagonal block each pair takes its own
@@ -369,7 +453,7 @@ __global__ __launch_bounds__(PREP_THREADS) void gla_prepare_kernel(const GatedSt
         }
     }
 }
-static size_t gla_prepare_lds(int dim) { return (size_t)C * 3 * (gs_pad64(dim) + 4) * sizeof(float); }
+static size_t gla_prepare_lds(int dim, int rank) { return ((size_t)C * (3 * (gs_pad64(dim) + 4) + rank) + gs_pad64(dim)) * sizeof(float); }
 
 // grid (heads, 16-column slices of the values, sequences of the call).  Wave w owns rows [16 NT w, 16 NT (w + 1)) of the state.
 template <bool DELTA, int NT>
@@ -395,6 +479,8 @@ __global__ __launch_bounds__(256) void state_scan_kernel(const GatedStateArgs a)
     struct Frag {
         float4 w[DELTA ? 2 : 1][NT], q[2][NT], k[NT][2];
         gs_f4 gd[NT], u[2];
+        float4 a[2];                    // the rows of A of this wave's output tile (waves 0 and 1)
+        int t0, n;
     };
     auto load = [&](int ci, Frag &f) {
         const GsMats m(a.ws, (size_t)ci * a.heads + h, Dp, Vp, DELTA);
@@ -411,6 +497,10 @@ __global__ __launch_bounds__(256) void state_scan_kernel(const GatedStateArgs a)
             f.gd[k] = gs_f4{gv.x, gv.y, gv.z, gv.w};
         }
         const int t0 = a.chunks.chunk[ci], n = a.chunks.chunk[ci + 1] - t0;
+        f.t0 = t0; f.n = n;
+#pragma unroll
+        for (int r = 0; r < 2; ++r)
+            if (r <= wave && wave < 2) f.a[r] = *reinterpret_cast<const float4 *>(m.A + (16 * wave + c) * C + 16 * r + 4 * g);
 #pragma unroll
         for (int r = 0; r < 2; ++r)
 #pragma unroll
@@ -448,18 +538,16 @@ __global__ __launch_bounds__(256) void state_scan_kernel(const GatedStateArgs a)
                 for (int w = 0; w < 4; ++w) u[r] -= *reinterpret_cast<const gs_f4 *>(rd[w][2 + r][lane]);
         }
         if (wave < 2) {                 // the outputs of row tile `wave`
-            const GsMats m(a.ws, (size_t)ci * a.heads + h, Dp, Vp, DELTA);
             gs_f4 o = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
             for (int w = 0; w < 4; ++w) o += *reinterpret_cast<const gs_f4 *>(rd[w][wave][lane]);
 #pragma unroll
             for (int s = 0; s < 2; ++s)
-                if (s <= wave) o = gs_mma(*reinterpret_cast<const float4 *>(m.A + (16 * wave + c) * C + 16 * s + 4 * g), u[s], o);
-            const int t0 = a.chunks.chunk[ci], n = a.chunks.chunk[ci + 1] - t0;
+                if (s <= wave) o = gs_mma(cur.a[s], u[s], o);
 #pragma unroll
             for (int i = 0; i < 4; ++i) {
                 const int tk = 16 * wave + 4 * g + i;
-                if (tk < n && col < V) a.o[(size_t)(t0 + tk) * a.heads * V + h * V + col] = o[i];
+                if (tk < cur.n && col < V) a.o[(size_t)(cur.t0 + tk) * a.heads * V + h * V + col] = o[i];
             }
         }
 #pragma unroll
@@ -516,7 +604,7 @@ __global__ __launch_bounds__(256) void gated_norm_kernel(const GatedStateArgs a,
 static bool args_ok(const GatedStateArgs &a) {
     return a.heads >= 1 && a.kv_heads >= 1 && a.heads % a.kv_heads == 0 && a.dim >= 1 && a.vdim >= 1 && gated_state_supported(a.dim, a.vdim) && a.in && a.norm && a.state && a.pos &&
            a.seq && a.out && a.ld_out >= a.heads * a.vdim &&
-           (a.delta ? a.taps >= 1 && a.tail && a.conv_q && a.conv_k && a.conv_v && a.A && a.dt_bias : a.kv_heads == a.heads && a.rank >= 1 && a.a2 && a.a2_bias);
+           (a.delta ? a.taps >= 1 && a.tail && a.conv_q && a.conv_k && a.conv_v && a.A && a.dt_bias : a.kv_heads == a.heads && a.rank >= 1 && a.rank <= STATE_RANK_MAX && a.a2 && a.a2_bias);
 }
 
 int gated_state_step(const GatedStateArgs &a, int T, hipStream_t stream) {
@@ -554,11 +642,11 @@ int gated_state_chunks(const GatedStateArgs &a, int T, hipStream_t stream) {
     if (!args_ok(a) || !a.ws || !a.o || !ch.chunk || !ch.first || !ch.run || ch.n_chunks < 1 || ch.n_runs < 1 || ch.n_runs > 65535 || a.heads > 65535)
         return fail(MESH_ERR_INVALID, "gated_state_chunks: bad operands");
     const dim3 grid((unsigned)ch.n_chunks, (unsigned)a.heads), block(PREP_THREADS);
-    const size_t lds = a.delta ? delta_prepare_lds(a.dim, a.vdim) : gla_prepare_lds(a.dim);
+    const size_t lds = a.delta ? delta_prepare_lds(a.dim, a.vdim) : gla_prepare_lds(a.dim, a.rank);
     static bool ready = false;        // (hosts are single-threaded per session; a second thread sets the same attributes)
     if (!ready) {
         MESH_HIP_TRY(hipFuncSetAttribute(reinterpret_cast<const void *>(delta_prepare_kernel), hipFuncAttributeMaxDynamicSharedMemorySize, (int)delta_prepare_lds(STATE_DIM_MAX, STATE_DIM_MAX)));
-        MESH_HIP_TRY(hipFuncSetAttribute(reinterpret_cast<const void *>(gla_prepare_kernel), hipFuncAttributeMaxDynamicSharedMemorySize, (int)gla_prepare_lds(STATE_DIM_MAX)));
+        MESH_HIP_TRY(hipFuncSetAttribute(reinterpret_cast<const void *>(gla_prepare_kernel), hipFuncAttributeMaxDynamicSharedMemorySize, (int)gla_prepare_lds(STATE_DIM_MAX, STATE_RANK_MAX)));
         ready = true;
     }
     if (a.delta) MESH_LAUNCH(delta_prepare_kernel, grid, block, lds, stream, a);

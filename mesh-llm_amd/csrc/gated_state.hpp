@@ -19,6 +19,7 @@ namespace mesh {
 
 constexpr int STATE_CHUNK = 32;
 constexpr int STATE_DIM_MAX = 256;          // of dim and of vdim
+constexpr int STATE_RANK_MAX = 256;         // of GLA's decay projection
 
 // The calls' tokens by sequence: chunk i is tokens [chunk[i], chunk[i + 1]), all of one sequence, whose run of tokens begins
 // at first[i]; sequence j of the call has chunks [run[j], run[j + 1]).  Device arrays.

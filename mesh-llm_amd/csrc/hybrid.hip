@@ -33,7 +33,7 @@ int hybrid_session_alloc(mesh_session *s) {
     h.q = fbuf(B * (size_t)hm.q_max);
     h.part = fbuf(2 * 3 * STEP_PARTS_MAX);
     h.ws = fbuf(hm.state_max ? min_gru_workspace((int)B, hm.state_max) : 0);
-    s->attn_part_rows = std::max<size_t>(B, 512);
+    s->attn_part_rows = std::max<size_t>(B, 256 * LATENT_GROUP);
     if (hm.part_max) {
         int heads = 0;
         for (const HybridLayer &L : hm.layers) heads = std::max(heads, L.spec.mixer.heads);
@@ -122,14 +122,17 @@ static int layer_splits(const mesh_session *s, const MixerSpec &m, int T, int ma
     return T < 64 ? attn_splits_for(s->tune, T, m.kv_heads, keys_seen(m, max_keys), false) : 1;
 }
 
-static int latent_splits(const mesh_session *s, const LatentShape &ls, int T, int max_keys) { return attn_splits_for(s->tune, T, latent_head_tiles(ls), max_keys, false); }
+// (the partial sums have room for 1024 (token, split) rows at least)
+static int latent_layer_splits(const mesh_session *s, const LatentShape &ls, int T, int max_keys) {
+    return latent_splits(ls, T, latent_group(ls, T, s->chunk_pos0 >= 0), max_keys, std::min(s->tune.attn_split_target, 256));
+}
 
 uint64_t hybrid_graph_key(const mesh_session *s, int T, int max_keys) {
     uint64_t key = 1469598103934665603ull ^ (uint64_t)T;
     auto mix = [&](uint64_t v) { key = (key ^ v) * 1099511628211ull; };
     for (const HybridLayer &L : s->stage->hybrid->layers) {
         if (L.spec.mixer.kind == MIXER_ATTENTION) mix((uint64_t)layer_splits(s, L.spec.mixer, T, max_keys));
-        if (L.spec.mixer.kind == MIXER_LATENT) mix((uint64_t)latent_splits(s, L.latent, T, max_keys));
+        if (L.spec.mixer.kind == MIXER_LATENT) mix((uint64_t)latent_layer_splits(s, L.latent, T, max_keys) << 1 | (s->chunk_pos0 >= 0 ? 1 : 0));
     }
     if (s->stage->hybrid->has_chunks) mix(((uint64_t)s->hybrid->chunks.n_chunks << 32) | (uint64_t)s->hybrid->chunks.n_runs);
     return key;
@@ -212,7 +215,8 @@ static int run_latent_rows(mesh_session *s, size_t il, int T, int max_keys, bool
     }
     LatentAttnArgs a;
     a.qa = h.qx; a.rows = c.rows; a.pos = s->d_pos; a.seq = s->d_seq; a.part = s->attn_part; a.ml = s->attn_ml; a.n_ctx = st->n_ctx;
-    a.n_splits = latent_splits(s, L.latent, T, max_keys);
+    a.group = latent_group(L.latent, T, s->chunk_pos0 >= 0);
+    a.n_splits = latent_layer_splits(s, L.latent, T, max_keys);
     a.w_uv = L.w_uv; a.gate = h.big + L.in.M - m.heads; a.gate_ld = L.in.M;
     if (f32_out || hm.act == ACT_F32) a.out = static_cast<float *>(h.acta);
     else a.out_bf16 = static_cast<uint16_t *>(h.acta);

@@ -231,6 +231,7 @@ struct FolderLoader {
             const SafeTensor *a1 = f.find(mx + "a1");
             if (!a1 || a1->shape.size() != 2 || a1->shape[0] < 1 || a1->shape[0] > 4096) return fail(MESH_ERR_FORMAT, "model.safetensors: tensor '%sa1' not found or not a matrix", mx.c_str());
             g.rank = (int)a1->shape[0];
+            if (g.rank > STATE_RANK_MAX) return fail(MESH_ERR_UNSUPPORTED, "layer %d: a decay projection of rank %d has no kernel (%d at most)", index, g.rank, STATE_RANK_MAX);
             g.at_a = g.at_g + v;
             g.inv_tau = 1.0f / m.tau;
             in.push_back({mx + "a1", g.rank});

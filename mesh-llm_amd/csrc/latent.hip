@@ -1,11 +1,11 @@
 // See latent.hpp.
 //
-// latent_attn_kernel: a workgroup takes one (key split, 16 heads, token).  A step stages 32 cache rows in LDS, once as they
+// latent_attn_kernel: a workgroup takes one (key split, 16 heads, token or four consecutive tokens of a sequence).  A step stages 32 cache rows in LDS, once as they
 // are and (f16) once with the latents transposed, pairs of keys as dwords, since the second product contracts over keys:
 //   S^T (32 keys x 16 heads)   = rows . Q^T        v_mfma_f32_16x16x32_f16 per 32 elements of a row
 //   O^T (rank x 16 heads)     += latents^T . P^T   the result registers of S^T are the P^T operand as they are
-// Every wave computes the scores (they are few), so that no softmax state crosses waves, and owns a quarter of the rank's
-// rows of O^T.  With f32 rows the same fragments feed v_mfma_f32_16x16x4_f32, eight per 32 elements.
+// With one token every wave computes the scores (they are few), so that no softmax state crosses waves, and owns a quarter of
+// the rank's rows of O^T; with four each wave has a token.  With f32 rows the same fragments feed v_mfma_f32_16x16x4_f32, eight per 32 elements.
 #include "latent.hpp"
 
 #include <algorithm>
@@ -184,50 +184,82 @@ __host__ __device__ constexpr int lt_pitch(ActType act, int row) { return row + 
 // keys per split: whole steps
 __host__ __device__ constexpr int lt_split_keys(int n_keys, int n_splits) { return ((n_keys + n_splits - 1) / n_splits + LT_KEYS - 1) / LT_KEYS * LT_KEYS; }
 
-// NR: 16-row blocks of the rank per wave (rank_pad = 64 NR)
-template <ActType ACT, int NR>
-__global__ __launch_bounds__(LT_THREADS) void latent_attn_kernel(const LatentAttnArgs a, int heads, int rot_pad) {
+// key range of a group of tokens: positions ascend by one within it
+__device__ __forceinline__ int lt_group_keys(const int32_t *pos, int t0, int tokens, int T) { return pos[min(t0 + tokens, T) - 1] + 1; }
+
+// NR: rank_pad / 64.  TOK 1: a workgroup has one token, and each wave owns NR 16-row blocks of O^T.  TOK 4: it has four
+// consecutive tokens of one sequence, a wave each, which share the staged rows.
+template <ActType ACT, int NR, int TOK>
+__global__ __launch_bounds__(LT_THREADS) void latent_attn_kernel(const LatentAttnArgs a, int heads, int rot_pad, int T) {
     typedef typename LtElem<ACT>::type E;
-    constexpr int RANK = 64 * NR;
+    constexpr int RANK = 64 * NR, NO = TOK == 1 ? NR : 4 * NR;
     extern __shared__ __align__(16) uint8_t smem[];
     const int row = RANK + rot_pad, pitch = lt_pitch(ACT, row);
     E *sK = reinterpret_cast<E *>(smem);                                                  // [LT_KEYS][pitch]
     uint32_t *sV = reinterpret_cast<uint32_t *>(smem + (size_t)LT_KEYS * pitch * sizeof(E));  // f16: [RANK][LT_VPITCH]
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, c = lane & 15, g = lane >> 4;
-    const int split = blockIdx.x, t = blockIdx.z, h = blockIdx.y * LATENT_HEADS_TILE + c;
-    const int n_keys = a.pos[t] + 1, per = lt_split_keys(n_keys, a.n_splits);
-    const int j0 = split * per, j1 = min(j0 + per, n_keys);
+    const int split = blockIdx.x, t0 = blockIdx.z * TOK, h = blockIdx.y * LATENT_HEADS_TILE + c;
+    const bool live = TOK == 1 || t0 + wave < T;
+    const int t = TOK == 1 ? t0 : live ? t0 + wave : T - 1;
+    const int ob = TOK == 1 ? wave * NR : 0;                  // first 16-row block of this wave
+    const int n_keys = lt_group_keys(a.pos, t0, TOK, T), mine = a.pos[t] + 1, per = lt_split_keys(n_keys, a.n_splits);
+    const int j0 = split * per, j1 = min(j0 + per, n_keys), jm = min(j1, mine);
     const size_t prow = ((size_t)t * heads + h) * a.n_splits + split;
     if (j0 >= j1) {
-        if (tid < 16 && h < heads) { a.ml[prow * 2] = -INFINITY; a.ml[prow * 2 + 1] = 0.f; }
+        if ((TOK > 1 ? live && lane < 16 : tid < 16) && h < heads) { a.ml[prow * 2] = -INFINITY; a.ml[prow * 2 + 1] = 0.f; }
         return;
     }
-    const E *qp = static_cast<const E *>(a.qa) + ((size_t)t * heads + (h < heads ? h : heads - 1)) * row + 8 * g;
     const E *rows = static_cast<const E *>(a.rows) + (size_t)a.seq[t] * a.n_ctx * row;
-    lt_f4 o[NR];
+    // rows on their way to LDS (f16): 8 elements of two neighbouring keys per item; a thread fetches its items of a step while
+    // the step before it is multiplied.  Rows past the split are zeros (their scores are masked below).
+    constexpr int ITEMS = ACT == ACT_BF16 ? (2 * (RANK + 64) + LT_THREADS - 1) / LT_THREADS : 1;
+    uint4 r0[ITEMS], r1[ITEMS];
+    auto fetch_item = [&](int k0, int i, uint4 &x, uint4 &y) {
+        const int key = k0 + 2 * (i & 15), d = (i >> 4) * 8;
+        x = y = make_uint4(0, 0, 0, 0);
+        if (key < j1) x = *reinterpret_cast<const uint4 *>(rows + (size_t)key * row + d);
+        if (key + 1 < j1) y = *reinterpret_cast<const uint4 *>(rows + (size_t)(key + 1) * row + d);
+    };
+    auto put_item = [&](int i, const uint4 &x, const uint4 &y) {
+        const int kp = i & 15, d = (i >> 4) * 8;
+        *reinterpret_cast<uint4 *>(sK + (2 * kp) * pitch + d) = x;
+        *reinterpret_cast<uint4 *>(sK + (2 * kp + 1) * pitch + d) = y;
+        if (d >= RANK) return;
+        const uint32_t w0[4] = {x.x, x.y, x.z, x.w}, w1[4] = {y.x, y.y, y.z, y.w};
+        uint32_t *dst = sV + d * LT_VPITCH + kp;
 #pragma unroll
-    for (int n = 0; n < NR; ++n) o[n] = lt_f4{0.f, 0.f, 0.f, 0.f};
+        for (int e = 0; e < 4; ++e) {
+            dst[(2 * e) * LT_VPITCH] = (w0[e] & 0xffffu) | (w1[e] << 16);
+            dst[(2 * e + 1) * LT_VPITCH] = (w0[e] >> 16) | (w1[e] & 0xffff0000u);
+        }
+    };
+    const int items = 2 * row;
+    auto fetch = [&](int k0) {
+#pragma unroll
+        for (int n = 0; n < ITEMS; ++n)
+            if (tid + n * LT_THREADS < items) fetch_item(k0, tid + n * LT_THREADS, r0[n], r1[n]);
+    };
+    if constexpr (ACT == ACT_BF16) fetch(j0);
+    const E *qp = static_cast<const E *>(a.qa) + ((size_t)t * heads + (h < heads ? h : heads - 1)) * row + 8 * g;
+    constexpr int NQ = ACT == ACT_BF16 ? 2 * NR : 1;
+    LtFrag<ACT> qf[NQ];
+    if constexpr (ACT == ACT_BF16) {
+#pragma unroll
+        for (int n = 0; n < NQ; ++n) qf[n].load(qp + 32 * n);
+    }
+    lt_f4 o[NO];
+#pragma unroll
+    for (int n = 0; n < NO; ++n) o[n] = lt_f4{0.f, 0.f, 0.f, 0.f};
     float m = -INFINITY, l = 0.f;
     for (int k0 = j0; k0 < j1; k0 += LT_KEYS) {
-        // rows past the split are zeros (their scores are masked below)
         if constexpr (ACT == ACT_BF16) {
-            const int items = 16 * (row / 8);
-            for (int i = tid; i < items; i += LT_THREADS) {
-                const int kp = i & 15, d = (i >> 4) * 8, key = k0 + 2 * kp;
-                uint4 r0 = make_uint4(0, 0, 0, 0), r1 = r0;
-                if (key < j1) r0 = *reinterpret_cast<const uint4 *>(rows + (size_t)key * row + d);
-                if (key + 1 < j1) r1 = *reinterpret_cast<const uint4 *>(rows + (size_t)(key + 1) * row + d);
-                *reinterpret_cast<uint4 *>(sK + (2 * kp) * pitch + d) = r0;
-                *reinterpret_cast<uint4 *>(sK + (2 * kp + 1) * pitch + d) = r1;
-                if (d < RANK) {
-                    const uint32_t w0[4] = {r0.x, r0.y, r0.z, r0.w}, w1[4] = {r1.x, r1.y, r1.z, r1.w};
-                    uint32_t *dst = sV + d * LT_VPITCH + kp;
 #pragma unroll
-                    for (int e = 0; e < 4; ++e) {
-                        dst[(2 * e) * LT_VPITCH] = (w0[e] & 0xffffu) | (w1[e] << 16);
-                        dst[(2 * e + 1) * LT_VPITCH] = (w0[e] >> 16) | (w1[e] & 0xffff0000u);
-                    }
-                }
+            for (int n = 0; n < ITEMS; ++n)
+                if (tid + n * LT_THREADS < items) put_item(tid + n * LT_THREADS, r0[n], r1[n]);
+            for (int i = tid + ITEMS * LT_THREADS; i < items; i += LT_THREADS) {           // (rotated parts of more than 64)
+                uint4 x, y;
+                fetch_item(k0, i, x, y);
+                put_item(i, x, y);
             }
         } else {
             const int pieces = row / 4;
@@ -239,113 +271,144 @@ __global__ __launch_bounds__(LT_THREADS) void latent_attn_kernel(const LatentAtt
             }
         }
         __syncthreads();
+        if constexpr (ACT == ACT_BF16) {
+            if (k0 + LT_KEYS < j1) fetch(k0 + LT_KEYS);
+        }
         lt_f4 s[2] = {lt_f4{0.f, 0.f, 0.f, 0.f}, lt_f4{0.f, 0.f, 0.f, 0.f}};
-        auto score = [&](int kc) {
-            LtFrag<ACT> qf, kf[2];
-            qf.load(qp + kc);
+        auto score = [&](int kc, const LtFrag<ACT> &q) {
+            LtFrag<ACT> kf;
 #pragma unroll
             for (int b = 0; b < 2; ++b) {
-                kf[b].load(sK + (16 * b + c) * pitch + kc + 8 * g);
-                s[b] = lt_mma(kf[b], qf, s[b]);
+                kf.load(sK + (16 * b + c) * pitch + kc + 8 * g);
+                s[b] = lt_mma(kf, q, s[b]);
             }
         };
+        auto score_at = [&](int kc) {
+            LtFrag<ACT> q;
+            q.load(qp + kc);
+            score(kc, q);
+        };
+        if constexpr (ACT == ACT_BF16) {
 #pragma unroll
-        for (int kc = 0; kc < RANK; kc += 32) score(kc);
-        for (int kc = RANK; kc < row; kc += 32) score(kc);
-        // register i of tile b: key k0 + 16 b + 4 g + i for head column c; at least key k0 is in range
+            for (int n = 0; n < NQ; ++n) score(32 * n, qf[n]);
+        } else {
+            for (int kc = 0; kc < RANK; kc += 32) score_at(kc);
+        }
+        for (int kc = RANK; kc < row; kc += 32) score_at(kc);
+        // register i of tile b: key k0 + 16 b + 4 g + i for head column c
         float mx = m;
 #pragma unroll
         for (int b = 0; b < 2; ++b)
 #pragma unroll
             for (int i = 0; i < 4; ++i) {
-                if (k0 + 16 * b + 4 * g + i >= j1) s[b][i] = -INFINITY;
+                if (k0 + 16 * b + 4 * g + i >= jm) s[b][i] = -INFINITY;
                 mx = fmaxf(mx, s[b][i]);
             }
         mx = fmaxf(mx, __shfl_xor(mx, 16));
         mx = fmaxf(mx, __shfl_xor(mx, 32));
-        const float corr = lt_exp2(m - mx);           // exp2(-inf) = 0 the first time
+        // (a token before the group's last may see no key of the split: all is -inf then, and the reference 0 gives zeros)
+        const float ref = mx == -INFINITY ? 0.f : mx;
+        const float corr = lt_exp2(m - ref);          // exp2(-inf) = 0 the first time
         m = mx;
         float p[2][4], ps = 0.f;
 #pragma unroll
         for (int b = 0; b < 2; ++b)
 #pragma unroll
-            for (int i = 0; i < 4; ++i) { p[b][i] = lt_exp2(s[b][i] - mx); ps += p[b][i]; }
+            for (int i = 0; i < 4; ++i) { p[b][i] = lt_exp2(s[b][i] - ref); ps += p[b][i]; }
         l = l * corr + ps;                            // (this lane's keys only)
+        if (__builtin_amdgcn_ballot_w64(corr != 1.0f) != 0ull) {
 #pragma unroll
-        for (int n = 0; n < NR; ++n) o[n] *= corr;
+            for (int n = 0; n < NO; ++n) o[n] *= corr;
+        }
         if constexpr (ACT == ACT_BF16) {
             // key slots of lane group g: keys 4g .. 4g + 3 of either tile, which is how P^T lies in the registers
             const lt_u4 pu = {lt_pack(p[0][0], p[0][1]), lt_pack(p[0][2], p[0][3]), lt_pack(p[1][0], p[1][1]), lt_pack(p[1][2], p[1][3])};
             const lt_h8 pf = __builtin_bit_cast(lt_h8, pu);
 #pragma unroll
-            for (int n = 0; n < NR; ++n) {
-                const uint32_t *v = sV + (16 * (wave * NR + n) + c) * LT_VPITCH + 2 * g;
+            for (int n = 0; n < NO; ++n) {
+                const uint32_t *v = sV + (16 * (ob + n) + c) * LT_VPITCH + 2 * g;
                 const uint2 a0 = *reinterpret_cast<const uint2 *>(v), a1 = *reinterpret_cast<const uint2 *>(v + 8);
                 const lt_u4 vu = {a0.x, a0.y, a1.x, a1.y};
                 o[n] = __builtin_amdgcn_mfma_f32_16x16x32_f16(__builtin_bit_cast(lt_h8, vu), pf, o[n], 0, 0, 0);
             }
         } else {
 #pragma unroll
-            for (int n = 0; n < NR; ++n)
+            for (int n = 0; n < NO; ++n)
 #pragma unroll
                 for (int b = 0; b < 2; ++b)
 #pragma unroll
                     for (int i = 0; i < 4; ++i)
-                        o[n] = __builtin_amdgcn_mfma_f32_16x16x4f32(sK[(16 * b + 4 * g + i) * pitch + 16 * (wave * NR + n) + c], p[b][i], o[n], 0, 0, 0);
+                        o[n] = __builtin_amdgcn_mfma_f32_16x16x4f32(sK[(16 * b + 4 * g + i) * pitch + 16 * (ob + n) + c], p[b][i], o[n], 0, 0, 0);
         }
         __syncthreads();
     }
     l += __shfl_xor(l, 16);
     l += __shfl_xor(l, 32);
-    if (h >= heads) return;
-    if (wave == 0 && g == 0) { a.ml[prow * 2] = m; a.ml[prow * 2 + 1] = l; }
+    if (h >= heads || !live) return;
+    if ((TOK > 1 || wave == 0) && g == 0) { a.ml[prow * 2] = m; a.ml[prow * 2 + 1] = l; }
 #pragma unroll
-    for (int n = 0; n < NR; ++n) *reinterpret_cast<float4 *>(a.part + prow * RANK + 16 * (wave * NR + n) + 4 * g) = make_float4(o[n][0], o[n][1], o[n][2], o[n][3]);
+    for (int n = 0; n < NO; ++n) *reinterpret_cast<float4 *>(a.part + prow * RANK + 16 * (ob + n) + 4 * g) = make_float4(o[n][0], o[n][1], o[n][2], o[n][3]);
 }
 
-// grid (heads, slices of the value rows, T).  Sixteen lanes per weight row.
-__global__ __launch_bounds__(LT_THREADS) void latent_out_kernel(const LatentShape s, const LatentAttnArgs a) {
+// grid (heads, slices of the value rows, groups of TB tokens).  Sixteen lanes per weight row.
+template <int TB>
+__global__ __launch_bounds__(LT_THREADS) void latent_out_kernel(const LatentShape s, const LatentAttnArgs a, int T) {
     extern __shared__ __align__(16) uint8_t smem[];
-    __shared__ float s_w[ATTN_SPLITS_CAP];
-    __shared__ float s_inv;
-    float *xs = reinterpret_cast<float *>(smem);              // [rank_pad]
-    const int h = blockIdx.x, t = blockIdx.z, tid = threadIdx.x, S = a.n_splits;
-    const int n_keys = a.pos[t] + 1, per = lt_split_keys(n_keys, S), live = (n_keys + per - 1) / per;      // splits that saw a key
-    const size_t row = (size_t)t * s.heads + h;
-    if (tid < 64) {
-        const float m = tid < live ? a.ml[(row * S + tid) * 2] : -INFINITY, l = tid < live ? a.ml[(row * S + tid) * 2 + 1] : 0.f;
+    __shared__ float s_w[TB][ATTN_SPLITS_CAP];
+    float *xs = reinterpret_cast<float *>(smem);              // [TB][rank_pad]
+    const int h = blockIdx.x, t0 = blockIdx.z * TB, tid = threadIdx.x, lane = tid & 63, S = a.n_splits;
+    for (int b = tid >> 6; b < TB; b += LT_WAVES) {
+        const int t = min(t0 + b, T - 1), tg = t / a.group * a.group;          // the attention launch's group of this token
+        const int n_keys = lt_group_keys(a.pos, tg, a.group, T), per = lt_split_keys(n_keys, S), live = (n_keys + per - 1) / per;      // splits that had keys
+        const size_t row = (size_t)t * s.heads + h;
+        const float m = lane < live ? a.ml[(row * S + lane) * 2] : -INFINITY, l = lane < live ? a.ml[(row * S + lane) * 2 + 1] : 0.f;
         float mh = m;
 #pragma unroll
         for (int o = 32; o > 0; o >>= 1) mh = fmaxf(mh, __shfl_xor(mh, o));
-        const float w = tid < live ? lt_exp2(m - mh) : 0.f;
+        const float w = lane < live ? lt_exp2(m - mh) : 0.f;
         float den = l * w;
 #pragma unroll
         for (int o = 32; o > 0; o >>= 1) den += __shfl_xor(den, o);
-        s_w[tid] = w;
-        if (tid == 0) s_inv = 1.0f / den;
+        s_w[b][lane] = w / den;
     }
     __syncthreads();
-    for (int r = tid; r < s.rank_pad; r += LT_THREADS) {
-        float v = 0.f;
-        const float *p = a.part + row * S * s.rank_pad + r;
+#pragma unroll
+    for (int b = 0; b < TB; ++b) {
+        const int t = min(t0 + b, T - 1), tg = t / a.group * a.group, n_keys = lt_group_keys(a.pos, tg, a.group, T), per = lt_split_keys(n_keys, S), live = (n_keys + per - 1) / per;
+        for (int r = tid; r < s.rank_pad; r += LT_THREADS) {
+            float v = 0.f;
+            const float *p = a.part + ((size_t)t * s.heads + h) * S * s.rank_pad + r;
 #pragma unroll 8
-        for (int k = 0; k < live; ++k) v = fmaf(p[(size_t)k * s.rank_pad], s_w[k], v);
-        xs[r] = v * s_inv;
+            for (int k = 0; k < live; ++k) v = fmaf(p[(size_t)k * s.rank_pad], s_w[b][k], v);
+            xs[b * s.rank_pad + r] = v;
+        }
     }
     __syncthreads();
-    const float gate = act_sigmoid(a.gate[(size_t)t * a.gate_ld + h]);
     const int slice = (s.v_pad + gridDim.y - 1) / gridDim.y, v1 = min((int)(blockIdx.y + 1) * slice, s.v_pad);
     const int piece = tid & 15, pieces = s.rank_pad / 8;
+    float gate[TB];
+#pragma unroll
+    for (int b = 0; b < TB; ++b) gate[b] = act_sigmoid(a.gate[(size_t)min(t0 + b, T - 1) * a.gate_ld + h]);
     for (int v0 = blockIdx.y * slice; v0 < v1; v0 += LT_THREADS / 16) {
         const int v = v0 + (tid >> 4);
-        float acc = 0.f;
+        float acc[TB];
+#pragma unroll
+        for (int b = 0; b < TB; ++b) acc[b] = 0.f;
         if (v < s.vdim)
-            for (int p = piece; p < pieces; p += 16) acc = lt_dot8(*reinterpret_cast<const uint4 *>(a.w_uv + ((size_t)h * s.vdim + v) * s.rank_pad + p * 8), xs + p * 8, acc);
-        acc += __shfl_xor(acc, 1); acc += __shfl_xor(acc, 2); acc += __shfl_xor(acc, 4); acc += __shfl_xor(acc, 8);
-        if (piece == 0 && v < v1) {
-            const size_t at = row * s.v_pad + v;
-            if (a.out_bf16) a.out_bf16[at] = f32_to_bf16_bits(acc * gate);
-            else a.out[at] = acc * gate;
+            for (int p = piece; p < pieces; p += 16) {
+                const uint4 wv = *reinterpret_cast<const uint4 *>(a.w_uv + ((size_t)h * s.vdim + v) * s.rank_pad + p * 8);
+#pragma unroll
+                for (int b = 0; b < TB; ++b) acc[b] = lt_dot8(wv, xs + b * s.rank_pad + p * 8, acc[b]);
+            }
+#pragma unroll
+        for (int b = 0; b < TB; ++b) {
+            float y = acc[b];
+            y += __shfl_xor(y, 1); y += __shfl_xor(y, 2); y += __shfl_xor(y, 4); y += __shfl_xor(y, 8);
+            if (piece == 0 && v < v1 && t0 + b < T) {
+                const size_t at = ((size_t)(t0 + b) * s.heads + h) * s.v_pad + v;
+                if (a.out_bf16) a.out_bf16[at] = f32_to_bf16_bits(y * gate[b]);
+                else a.out[at] = y * gate[b];
+            }
         }
     }
 }
@@ -442,40 +505,60 @@ int latent_query(const LatentShape &s, const LatentCache &cache, ActType act, co
     return MESH_OK;
 }
 
-template <ActType ACT, int NR>
+int latent_group(const LatentShape &s, int T, bool one_run) { return one_run && T > 1 && s.rank_pad <= 512 ? LATENT_GROUP : 1; }
+
+int latent_splits(const LatentShape &s, int T, int group, int max_keys, int target) {
+    const int wgs = (T + group - 1) / group * latent_head_tiles(s);
+    const int n = std::min((target ? target : 256) / std::max(1, wgs), (max_keys + LT_KEYS - 1) / LT_KEYS);
+    return std::max(1, std::min(n, ATTN_SPLITS_CAP));
+}
+
+template <ActType ACT, int NR, int TOK>
 static int launch_attn(const LatentShape &s, const LatentAttnArgs &a, int T, hipStream_t stream) {
     static bool ready = false;        // (hosts are single-threaded per session; a second thread sets the same attribute)
     if (!ready) {
-        MESH_HIP_TRY(hipFuncSetAttribute(reinterpret_cast<const void *>(latent_attn_kernel<ACT, NR>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)LT_LDS_MAX));
+        MESH_HIP_TRY(hipFuncSetAttribute(reinterpret_cast<const void *>(latent_attn_kernel<ACT, NR, TOK>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)LT_LDS_MAX));
         ready = true;
     }
-    MESH_LAUNCH((latent_attn_kernel<ACT, NR>), dim3((unsigned)a.n_splits, (unsigned)latent_head_tiles(s), (unsigned)T), dim3(LT_THREADS), attn_lds(ACT, s), stream, a, s.heads, s.rot_pad);
+    MESH_LAUNCH((latent_attn_kernel<ACT, NR, TOK>), dim3((unsigned)a.n_splits, (unsigned)latent_head_tiles(s), (unsigned)((T + TOK - 1) / TOK)), dim3(LT_THREADS), attn_lds(ACT, s), stream, a,
+                s.heads, s.rot_pad, T);
     MESH_LAUNCH_CHECK();
     return MESH_OK;
+}
+template <ActType ACT, int NR>
+static int launch_attn_group(const LatentShape &s, const LatentAttnArgs &a, int T, hipStream_t stream) {
+    if (a.group == 1) return launch_attn<ACT, NR, 1>(s, a, T, stream);
+    if constexpr (NR <= 8) return launch_attn<ACT, NR, LATENT_GROUP>(s, a, T, stream);
+    return fail(MESH_ERR_UNSUPPORTED, "latent_attention: no grouped kernel for a rank of %d", s.rank);
 }
 template <ActType ACT>
 static int launch_attn_rank(const LatentShape &s, const LatentAttnArgs &a, int T, hipStream_t stream) {
     switch (s.rank_pad) {
-        case 64: return launch_attn<ACT, 1>(s, a, T, stream);
-        case 128: return launch_attn<ACT, 2>(s, a, T, stream);
-        case 256: return launch_attn<ACT, 4>(s, a, T, stream);
-        case 512: return launch_attn<ACT, 8>(s, a, T, stream);
-        case 1024: return launch_attn<ACT, 16>(s, a, T, stream);
+        case 64: return launch_attn_group<ACT, 1>(s, a, T, stream);
+        case 128: return launch_attn_group<ACT, 2>(s, a, T, stream);
+        case 256: return launch_attn_group<ACT, 4>(s, a, T, stream);
+        case 512: return launch_attn_group<ACT, 8>(s, a, T, stream);
+        case 1024: return launch_attn_group<ACT, 16>(s, a, T, stream);
         default: return fail(MESH_ERR_UNSUPPORTED, "latent_attention: no kernel for a rank of %d", s.rank);
     }
 }
 
 int latent_attention(const LatentShape &s, const LatentAttnArgs &a, ActType act, int T, hipStream_t stream) {
     if (T <= 0) return MESH_OK;
-    if (!a.qa || !a.rows || !a.part || !a.ml || a.n_splits < 1 || a.n_splits > ATTN_SPLITS_CAP || T > 65535) return fail(MESH_ERR_INVALID, "latent_attention: bad operands");
+    if (!a.qa || !a.rows || !a.part || !a.ml || a.n_splits < 1 || a.n_splits > ATTN_SPLITS_CAP || T > 65535 || (a.group != 1 && a.group != LATENT_GROUP))
+        return fail(MESH_ERR_INVALID, "latent_attention: bad operands");
     return act == ACT_BF16 ? launch_attn_rank<ACT_BF16>(s, a, T, stream) : launch_attn_rank<ACT_F32>(s, a, T, stream);
 }
 
 int latent_out(const LatentShape &s, const LatentAttnArgs &a, int T, hipStream_t stream) {
     if (T <= 0) return MESH_OK;
     if (!a.w_uv || !a.gate || (!a.out && !a.out_bf16) || a.n_splits > ATTN_SPLITS_CAP || T > 65535) return fail(MESH_ERR_INVALID, "latent_out: bad operands");
-    const int slices = std::max(1, std::min(s.v_pad / (LT_THREADS / 16), 256 / std::max(1, s.heads * T)));
-    MESH_LAUNCH(latent_out_kernel, dim3((unsigned)s.heads, (unsigned)slices, (unsigned)T), dim3(LT_THREADS), (size_t)s.rank_pad * sizeof(float), stream, s, a);
+    const int tb = T == 1 ? 1 : LT_QUERY_TOKENS, groups = (T + tb - 1) / tb;
+    const int slices = std::max(1, std::min(s.v_pad / (LT_THREADS / 16), 256 / std::max(1, s.heads * groups)));
+    const dim3 grid((unsigned)s.heads, (unsigned)slices, (unsigned)groups), block(LT_THREADS);
+    const size_t lds = (size_t)tb * s.rank_pad * sizeof(float);
+    if (tb == 1) MESH_LAUNCH((latent_out_kernel<1>), grid, block, lds, stream, s, a, T);
+    else MESH_LAUNCH((latent_out_kernel<LT_QUERY_TOKENS>), grid, block, lds, stream, s, a, T);
     MESH_LAUNCH_CHECK();
     return MESH_OK;
 }

@@ -55,6 +55,7 @@ struct LatentAttnArgs {
     float *part = nullptr;             // [T][heads][n_splits][rank_pad]
     float *ml = nullptr;               // [T][heads][n_splits][2]: maximum (log2 units) and sum
     int n_ctx = 0, n_splits = 1;
+    int group = 1;                     // tokens a workgroup takes: 1, or LATENT_GROUP where the call is one run of positions of a sequence
     // latent_out
     const uint16_t *w_uv = nullptr;    // [heads][vdim][rank_pad]
     const float *gate = nullptr;       // [T][gate_ld], one per head, through a sigmoid
@@ -62,6 +63,10 @@ struct LatentAttnArgs {
     float *out = nullptr;              // [T][heads * v_pad], or
     uint16_t *out_bf16 = nullptr;
 };
+constexpr int LATENT_GROUP = 4;
+int latent_group(const LatentShape &s, int T, bool one_run);
+// key splits of a launch that aims at `target` workgroups (0: one per compute unit); splits * T is at most LATENT_GROUP * target or T
+int latent_splits(const LatentShape &s, int T, int group, int max_keys, int target);
 // token t over positions [0, pos[t]] of sequence seq[t]: partial sums of latents per key split
 int latent_attention(const LatentShape &s, const LatentAttnArgs &a, ActType act, int T, hipStream_t stream);
 // splits merged, projected to values, times the head's gate

@@ -15,9 +15,15 @@ namespace mesh {
 constexpr int STEP_THREADS = 512, STEP_WAVES = STEP_THREADS / 64;
 constexpr size_t STEP_LDS_MAX = 160 * 1024 - 1024;
 
+// over the wave, in every lane: data-parallel-primitive moves inside a row of 16 lanes (swap neighbours, swap pairs, mirror the
+// 8, mirror the 16), permutes across rows
 __device__ __forceinline__ float step_wave_sum(float v) {
-#pragma unroll
-    for (int o = 32; o > 0; o >>= 1) v += __shfl_xor(v, o);
+    v += __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), 0xB1, 0xF, 0xF, false));
+    v += __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), 0x4E, 0xF, 0xF, false));
+    v += __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), 0x141, 0xF, 0xF, false));
+    v += __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), 0x140, 0xF, 0xF, false));
+    v += __shfl_xor(v, 16);
+    v += __shfl_xor(v, 32);
     return v;
 }
 // sum over the workgroup in a fixed order, the same in every thread
@@ -51,44 +57,6 @@ __device__ __forceinline__ void step_vec(int K, int Kp, int tid, Load load, Map 
             if (k < Kp) *reinterpret_cast<float4 *>(xs + k) = map(k, v[i]);
         }
     }
-}
-
-// Mean and sum of squared deviations of `n` values, and of two groups together (Chan, Golub, LeVeque: updating formulae for
-// sample variances): one pass, without the cancellation of sums of squares.
-struct StepMoments {
-    float n = 0.f, mean = 0.f, m2 = 0.f;
-    __device__ __forceinline__ void add(const float *v, int count) {           // count values at once (zero to four)
-        float s = 0.f, d2 = 0.f;
-        for (int j = 0; j < 4; ++j) s += j < count ? v[j] : 0.f;
-        const float m = count ? s / (float)count : 0.f;
-        for (int j = 0; j < 4; ++j) { const float d = j < count ? v[j] - m : 0.f; d2 = fmaf(d, d, d2); }
-        join({(float)count, m, d2});
-    }
-    __device__ __forceinline__ void join(const StepMoments &o) {
-        const float t = n + o.n, f = t > 0.f ? o.n / t : 0.f, d = o.mean - mean;
-        m2 += o.m2 + d * d * n * f;
-        mean = fmaf(d, f, mean);
-        n = t;
-    }
-};
-// over the workgroup in a fixed order, the same in every thread
-__device__ __forceinline__ StepMoments step_block_moments(StepMoments m, float (*scratch)[4], int lane, int wave) {
-#pragma unroll
-    for (int o = 32; o > 0; o >>= 1) {
-        // (the lower lane's group comes first in both, so that the two agree to the bit)
-        StepMoments a = m, b;
-        b.n = __shfl_xor(m.n, o); b.mean = __shfl_xor(m.mean, o); b.m2 = __shfl_xor(m.m2, o);
-        const bool low = !(lane & o);
-        m = low ? a : b;
-        m.join(low ? b : a);
-    }
-    __syncthreads();
-    if (lane == 0) { scratch[wave][0] = m.n; scratch[wave][1] = m.mean; scratch[wave][2] = m.m2; }
-    __syncthreads();
-    StepMoments r = {scratch[0][0], scratch[0][1], scratch[0][2]};
-#pragma unroll
-    for (int w = 1; w < STEP_WAVES; ++w) r.join({scratch[w][0], scratch[w][1], scratch[w][2]});
-    return r;
 }
 
 template <int R, int U, StepIn IN, StepOut OUT>
@@ -143,61 +111,73 @@ __global__ __launch_bounds__(STEP_THREADS) void linear_step_kernel(const uint16_
         const float rinv = 1.0f / sqrtf(step_block_sum(ss, &scratch[0][0], lane, wave) / (float)K + a.eps);
         for (int k = tid; k < K; k += STEP_THREADS) xs[k] *= rinv * a.gain[k];
     } else if constexpr (IN == STEP_IN_LAYER) {
-        constexpr int AHEAD = 2;                // groups of four a thread requests before the first moments are known
-        constexpr int STRIDE = STEP_THREADS * 4;
-        float4 x4[AHEAD], y4[AHEAD];
+        // a thread's first AHEAD groups of four, of every vector, are requested before the first sum; means first, then squared
+        // deviations
+        constexpr int AHEAD = 2, STRIDE = STEP_THREADS * 4;
         const int k0 = tid * 4;
+        const float inv_n = 1.0f / (float)K;
+        float4 x4[AHEAD], y4[AHEAD], g4[AHEAD], b4[AHEAD], ng4[AHEAD], nb4[AHEAD];
 #pragma unroll
         for (int i = 0; i < AHEAD; ++i) {
-            x4[i] = ln_load4(a.in, k0 + i * STRIDE, K);
-            y4[i] = a.y ? ln_load4(a.y, k0 + i * STRIDE, K) : make_float4(0.f, 0.f, 0.f, 0.f);
-        }
-        auto live = [&](int k) { return K - k < 0 ? 0 : K - k < 4 ? K - k : 4; };
-        StepMoments mx;
-        // v of group i -> LDS, x_out and the moments of v
-        auto put = [&](int i, const float4 &v) {
             const int k = k0 + i * STRIDE;
-            if (k >= Kp) return;
-            *reinterpret_cast<float4 *>(xs + k) = v;
-            const float o[4] = {v.x, v.y, v.z, v.w};
-            const int c = live(k);
-            mx.add(o, c);
-            if (blockIdx.x == 0 && a.y)
-                for (int j = 0; j < c; ++j) a.x_out[k + j] = o[j];
+            x4[i] = ln_load4(a.in, k, K);
+            if (a.y) { y4[i] = ln_load4(a.y, k, K); g4[i] = ln_load4(a.gain, k, K); b4[i] = ln_load4(a.bias, k, K); }
+            ng4[i] = ln_load4(a.norm_gain, k, K); nb4[i] = ln_load4(a.norm_bias, k, K);
+        }
+        auto sum4 = [](const float4 &v) { return (v.x + v.y) + (v.z + v.w); };
+        auto dev4 = [&](int k, const float4 &v, float mean) {
+            const float d[4] = {v.x - mean, v.y - mean, v.z - mean, v.w - mean};
+            float s = 0.f;
+#pragma unroll
+            for (int j = 0; j < 4; ++j) s = fmaf(k + j < K ? d[j] : 0.f, d[j], s);
+            return s;
         };
         if (a.y) {
-            StepMoments my;
-            auto take = [&](int i, const float4 &v) {
-                const float o[4] = {v.x, v.y, v.z, v.w};
-                my.add(o, live(k0 + i * STRIDE));
+            float s = 0.f;
+#pragma unroll
+            for (int i = 0; i < AHEAD; ++i) s += sum4(y4[i]);
+            for (int k = k0 + AHEAD * STRIDE; k < K; k += STRIDE) s += sum4(ln_load4(a.y, k, K));
+            const float mean = step_block_sum(s, &scratch[0][0], lane, wave) * inv_n;
+            s = 0.f;
+#pragma unroll
+            for (int i = 0; i < AHEAD; ++i) s += dev4(k0 + i * STRIDE, y4[i], mean);
+            for (int k = k0 + AHEAD * STRIDE; k < K; k += STRIDE) s += dev4(k, ln_load4(a.y, k, K), mean);
+            const float rs = 1.0f / sqrtf(step_block_sum(s, &scratch[0][0], lane, wave) * inv_n + a.eps);
+            auto update = [&](int k, const float4 &x, const float4 &y, const float4 &g, const float4 &b) {
+                const float4 v = make_float4(x.x + ((y.x - mean) * rs * g.x + b.x), x.y + ((y.y - mean) * rs * g.y + b.y), x.z + ((y.z - mean) * rs * g.z + b.z),
+                                             x.w + ((y.w - mean) * rs * g.w + b.w));
+                if (blockIdx.x == 0) {
+                    const float o[4] = {v.x, v.y, v.z, v.w};
+#pragma unroll
+                    for (int j = 0; j < 4; ++j)
+                        if (k + j < K) a.x_out[k + j] = o[j];
+                }
+                return v;
             };
 #pragma unroll
-            for (int i = 0; i < AHEAD; ++i) take(i, y4[i]);
-            for (int i = AHEAD; k0 + i * STRIDE < K; ++i) take(i, ln_load4(a.y, k0 + i * STRIDE, K));
-            my = step_block_moments(my, scratch, lane, wave);
-            const float rs = 1.0f / sqrtf(my.m2 / (float)K + a.eps);
-            auto update = [&](int i, const float4 &x, const float4 &y) {
-                const int k = k0 + i * STRIDE;
-                if (k >= Kp) return;
-                const float4 g = ln_load4(a.gain, k, K), b = ln_load4(a.bias, k, K);
-                put(i, make_float4(x.x + ((y.x - my.mean) * rs * g.x + b.x), x.y + ((y.y - my.mean) * rs * g.y + b.y), x.z + ((y.z - my.mean) * rs * g.z + b.z),
-                                   x.w + ((y.w - my.mean) * rs * g.w + b.w)));
-            };
-#pragma unroll
-            for (int i = 0; i < AHEAD; ++i) update(i, x4[i], y4[i]);
-            for (int i = AHEAD; k0 + i * STRIDE < Kp; ++i) update(i, ln_load4(a.in, k0 + i * STRIDE, K), ln_load4(a.y, k0 + i * STRIDE, K));
+            for (int i = 0; i < AHEAD; ++i) x4[i] = update(k0 + i * STRIDE, x4[i], y4[i], g4[i], b4[i]);
+            for (int k = k0 + AHEAD * STRIDE; k < Kp; k += STRIDE)
+                *reinterpret_cast<float4 *>(xs + k) = update(k, ln_load4(a.in, k, K), ln_load4(a.y, k, K), ln_load4(a.gain, k, K), ln_load4(a.bias, k, K));
         } else {
+            for (int k = k0 + AHEAD * STRIDE; k < Kp; k += STRIDE) *reinterpret_cast<float4 *>(xs + k) = ln_load4(a.in, k, K);
+        }
+        // (groups behind the first AHEAD wait in LDS, every thread's its own)
+        float s = 0.f;
 #pragma unroll
-            for (int i = 0; i < AHEAD; ++i) put(i, x4[i]);
-            for (int i = AHEAD; k0 + i * STRIDE < Kp; ++i) put(i, ln_load4(a.in, k0 + i * STRIDE, K));
-        }
-        mx = step_block_moments(mx, scratch, lane, wave);
-        const float rs = 1.0f / sqrtf(mx.m2 / (float)K + a.eps);
-        for (int k = k0; k < Kp; k += STRIDE) {          // (every thread its own groups)
-            const float4 v = *reinterpret_cast<const float4 *>(xs + k), g = ln_load4(a.norm_gain, k, K), b = ln_load4(a.norm_bias, k, K);
-            *reinterpret_cast<float4 *>(xs + k) =
-                make_float4((v.x - mx.mean) * rs * g.x + b.x, (v.y - mx.mean) * rs * g.y + b.y, (v.z - mx.mean) * rs * g.z + b.z, (v.w - mx.mean) * rs * g.w + b.w);
-        }
+        for (int i = 0; i < AHEAD; ++i) s += sum4(x4[i]);
+        for (int k = k0 + AHEAD * STRIDE; k < Kp; k += STRIDE) s += sum4(*reinterpret_cast<const float4 *>(xs + k));
+        const float mean = step_block_sum(s, &scratch[0][0], lane, wave) * inv_n;
+        s = 0.f;
+#pragma unroll
+        for (int i = 0; i < AHEAD; ++i) s += dev4(k0 + i * STRIDE, x4[i], mean);
+        for (int k = k0 + AHEAD * STRIDE; k < Kp; k += STRIDE) s += dev4(k, *reinterpret_cast<const float4 *>(xs + k), mean);
+        const float rs = 1.0f / sqrtf(step_block_sum(s, &scratch[0][0], lane, wave) * inv_n + a.eps);
+        auto put = [&](int k, const float4 &v, const float4 &g, const float4 &b) {
+            if (k < Kp) *reinterpret_cast<float4 *>(xs + k) = make_float4((v.x - mean) * rs * g.x + b.x, (v.y - mean) * rs * g.y + b.y, (v.z - mean) * rs * g.z + b.z, (v.w - mean) * rs * g.w + b.w);
+        };
+#pragma unroll
+        for (int i = 0; i < AHEAD; ++i) put(k0 + i * STRIDE, x4[i], ng4[i], nb4[i]);
+        for (int k = k0 + AHEAD * STRIDE; k < Kp; k += STRIDE) put(k, *reinterpret_cast<const float4 *>(xs + k), ln_load4(a.norm_gain, k, K), ln_load4(a.norm_bias, k, K));
     } else {
         float ss = 0.f;
         for (int i = tid; i < a.n_part; i += STEP_THREADS) ss += a.part[i];

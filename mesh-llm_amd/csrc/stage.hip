@@ -1218,8 +1218,8 @@ static int run_layers_graphed(mesh_session *s, int T, int max_keys) {
     // A prefill chunk (consecutive positions of one sequence, enough tokens for the large-tile GEMM) runs the chunk
     // attention kernel, whose first position and sequence are launch arguments: a replay would carry the captured
     // chunk's.  Such calls are always launched eagerly.
-    if (s->chunk_pos0 >= 0 && T >= PREFILL_MIN_TOKENS) return run_layers(s, T, max_keys);
     const mesh_stage *st = s->stage;
+    if (s->chunk_pos0 >= 0 && (T >= PREFILL_MIN_TOKENS || (st->hybrid && T >= s->tune.latent_chunk_min_tokens))) return run_layers(s, T, max_keys);
     const int n_splits = st->hybrid ? 0 : attn_splits_for(s->tune, T, (int)st->hp.n_head_kv, max_keys, st->k_type != MESH_F16);
     const uint64_t key = st->hybrid ? hybrid_graph_key(s, T, max_keys) : (uint64_t)T | ((uint64_t)n_splits << 8) | ((uint64_t)(s->expert_mask_on ? 1 : 0) << 20);
     auto it = s->graphs.find(key);
