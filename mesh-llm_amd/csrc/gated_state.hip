@@ -96,7 +96,12 @@ __global__ __launch_bounds__(THREADS) void gated_step_kernel(const GatedStateArg
     }
     const float *x = a.in + (size_t)t * a.ld;
     float decay = 1.f, beta = 1.f;
+    // (so are the vectors that the token's output ends with: V <= THREADS)
+    const int vi = tid < V ? tid : V - 1;
+    const float out_norm = a.norm[vi], out_gate = x[a.at_g + h * V + vi];
     if (a.delta) {
+        decay = expf(delta_log_decay(a, t, h));
+        beta = delta_beta(a, t, h);
         const int kvh = h / (a.heads / a.kv_heads), channels = 2 * a.kv_heads * D + a.heads * V, taps = a.taps, now = pos % taps;
         float *tail = a.tail + (size_t)seq * taps * channels;
         const bool own = h % (a.heads / a.kv_heads) == 0;           // one head of a group keeps the shared channels' inputs
@@ -116,8 +121,6 @@ __global__ __launch_bounds__(THREADS) void gated_step_kernel(const GatedStateArg
             (part == 0 ? sq : part == 1 ? sk : sv)[e] = act_silu(y);
             if (own || part == 2) tail[(size_t)now * channels + ch] = xi;       // (not a slot that is read in this call: those are of taps - 1 other positions)
         }
-        decay = expf(delta_log_decay(a, t, h));
-        beta = delta_beta(a, t, h);
         __syncthreads();
         if (wave < 2) {
             float *u = wave == 0 ? sq : sk, ss = 0.f;
@@ -188,7 +191,7 @@ __global__ __launch_bounds__(THREADS) void gated_step_kernel(const GatedStateArg
         if (a.act == ACT_BF16) static_cast<uint16_t *>(a.out)[to + i] = f32_to_bf16_bits(y);
         else static_cast<float *>(a.out)[to + i] = y;
     };
-    for (int i = tid; i < V; i += THREADS) put(h * V + i, so[i] * r * a.norm[i] * act_silu(x[a.at_g + h * V + i]));
+    if (tid < V) put(h * V + tid, so[tid] * r * out_norm * act_silu(out_gate));
     if (h == a.heads - 1)
         for (int i = a.heads * V + tid; i < a.ld_out; i += THREADS) put(i, 0.f);
 }
@@ -259,11 +262,23 @@ __global__ __launch_bounds__(PREP_THREADS) void delta_prepare_kernel(const Gated
     }
     __syncthreads();
     const float qs = 1.0f / sqrtf((float)D);
-    for (int r = wave; r < 2 * C; r += 4) {
+    // sixteen lanes per row (the columns past dim are zeros)
+#pragma unroll
+    for (int r0 = 0; r0 < 2 * C; r0 += PREP_THREADS / 16) {
+        const int r = r0 + (tid >> 4);
         float *u = (r < C ? sQ : sK) + (r & (C - 1)) * dp, ss = 0.f;
-        for (int d = lane; d < D; d += 64) ss = fmaf(u[d], u[d], ss);
-        const float f = (r < C ? qs : 1.0f) / sqrtf(gs_wave_sum(ss) + UNIT_EPS);
-        for (int d = lane; d < D; d += 64) u[d] *= f;
+        for (int d = 4 * c; d < Dp; d += 64) {
+            const float4 v = *reinterpret_cast<const float4 *>(u + d);
+            ss = fmaf(v.x, v.x, fmaf(v.y, v.y, fmaf(v.z, v.z, fmaf(v.w, v.w, ss))));
+        }
+#pragma unroll
+        for (int o = 8; o > 0; o >>= 1) ss += __shfl_xor(ss, o);
+        const float f = (r < C ? qs : 1.0f) / sqrtf(ss + UNIT_EPS);
+        for (int d = 4 * c; d < Dp; d += 64) {
+            float4 v = *reinterpret_cast<const float4 *>(u + d);
+            v.x *= f; v.y *= f; v.z *= f; v.w *= f;
+            *reinterpret_cast<float4 *>(u + d) = v;
+        }
     }
     __syncthreads();
     // products of keys with keys and queries with keys, one 16 x 16 tile a wave
@@ -380,10 +395,17 @@ __global__ __launch_bounds__(PREP_THREADS) void gla_prepare_kernel(const GatedSt
             const float bias = d < D ? a.a2_bias[h * D + d] : 0.f;
 #pragma unroll
             for (int k = 0; k < HALF; ++k) z[k] = bias;
-            for (int j = 0; j < a.rank; ++j) {
-                const float wj = w[j];
+            constexpr int WB = 8;             // weights of a channel on their way at once
+            for (int j0 = 0; j0 < a.rank; j0 += WB) {
+                float wj[WB];
 #pragma unroll
-                for (int k = 0; k < HALF; ++k) z[k] = fmaf(wj, sX[(r0 + k) * a.rank + j], z[k]);
+                for (int j = 0; j < WB; ++j) wj[j] = j0 + j < a.rank ? w[j0 + j] : 0.f;
+#pragma unroll
+                for (int j = 0; j < WB; ++j) {
+                    const int at = j0 + j < a.rank ? j0 + j : 0;
+#pragma unroll
+                    for (int k = 0; k < HALF; ++k) z[k] = fmaf(wj[j], sX[(r0 + k) * a.rank + at], z[k]);
+                }
             }
             float sum = 0.f;
 #pragma unroll
@@ -414,15 +436,27 @@ __global__ __launch_bounds__(PREP_THREADS) void gla_prepare_kernel(const GatedSt
     }
     for (int d = tid; d < Dp; d += PREP_THREADS) m.G[d] = expf(sG[(C - 1) * dp + d]);
     // A: a decay per channel does not leave the sum over channels.  Within a 16 x 16 diagonal block each pair takes its own
-    // exponentials; the block below them is a product of queries decayed since token 15 and keys decayed until it.  No exponent
-    // is ever positive.
-    constexpr int PAIRS = 16 * 17 / 2;
-    for (int i = tid; i < 2 * PAIRS; i += PREP_THREADS) {
-        const int b = i / PAIRS, p = i % PAIRS;
-        int r = (int)((sqrtf(8.f * p + 1.f) - 1.f) * 0.5f);
-        r += (r + 1) * (r + 2) / 2 <= p ? 1 : 0;
-        r -= r * (r + 1) / 2 > p ? 1 : 0;
-        const int j = 16 * b + p - r * (r + 1) / 2;
+    // exponentials (a token with itself has none: eight lanes share its sum); the block below them is a product of queries decayed
+    // since token 15 and keys decayed until it.  No exponent is ever positive.
+    constexpr int PAIRS = 16 * 15 / 2;
+    static_assert(2 * PAIRS <= PREP_THREADS && PREP_THREADS == 8 * C, "one turn per thread");
+    {
+        const int r = tid >> 3;
+        float s = 0.f;
+        for (int d = 4 * (tid & 7); d < Dp; d += 32) {
+            const float4 q = *reinterpret_cast<const float4 *>(sQ + r * dp + d), k = *reinterpret_cast<const float4 *>(sK + r * dp + d);
+            s = fmaf(q.x, k.x, fmaf(q.y, k.y, fmaf(q.z, k.z, fmaf(q.w, k.w, s))));
+        }
+        s += __shfl_xor(s, 1); s += __shfl_xor(s, 2); s += __shfl_xor(s, 4);
+        if ((tid & 7) == 0) m.A[r * C + r] = s;
+    }
+    if (tid < 2 * PAIRS) {
+        // pair p of a block: row r >= 1, column p - r (r - 1) / 2 < r
+        const int b = tid / PAIRS, p = tid % PAIRS;
+        int r = (int)((sqrtf(8.f * p + 1.f) - 1.f) * 0.5f) + 1;
+        r += r * (r + 1) / 2 <= p ? 1 : 0;
+        r -= r * (r - 1) / 2 > p ? 1 : 0;
+        const int j = 16 * b + p - r * (r - 1) / 2;
         r += 16 * b;
         float s = 0.f;
         for (int d = 0; d < Dp; d += 4) {
@@ -434,7 +468,7 @@ __global__ __launch_bounds__(PREP_THREADS) void gla_prepare_kernel(const GatedSt
             s = fmaf(q.w * k.w, act_exp_neg(gj.w - gr.w), s);
         }
         m.A[r * C + j] = s;
-        if (r != j) m.A[j * C + r] = 0.f;
+        m.A[j * C + r] = 0.f;
     }
     if (wave == 3) {
         gs_f4 acc = {0.f, 0.f, 0.f, 0.f};
@@ -480,8 +514,9 @@ __global__ __launch_bounds__(256) void state_scan_kernel(const GatedStateArgs a)
         float4 w[DELTA ? 2 : 1][NT], q[2][NT], k[NT][2];
         gs_f4 gd[NT], u[2];
         float4 a[2];                    // the rows of A of this wave's output tile (waves 0 and 1)
-        int t0, n;
     };
+    // (every chunk of a run but its last is whole)
+    const int t_end = a.chunks.chunk[c1];
     auto load = [&](int ci, Frag &f) {
         const GsMats m(a.ws, (size_t)ci * a.heads + h, Dp, Vp, DELTA);
 #pragma unroll
@@ -496,8 +531,7 @@ __global__ __launch_bounds__(256) void state_scan_kernel(const GatedStateArgs a)
             const float4 gv = *reinterpret_cast<const float4 *>(m.G + d);
             f.gd[k] = gs_f4{gv.x, gv.y, gv.z, gv.w};
         }
-        const int t0 = a.chunks.chunk[ci], n = a.chunks.chunk[ci + 1] - t0;
-        f.t0 = t0; f.n = n;
+        const int t0 = t_first + (ci - c0) * C, n = t_end - t0;
 #pragma unroll
         for (int r = 0; r < 2; ++r)
             if (r <= wave && wave < 2) f.a[r] = *reinterpret_cast<const float4 *>(m.A + (16 * wave + c) * C + 16 * r + 4 * g);
@@ -510,11 +544,10 @@ __global__ __launch_bounds__(256) void state_scan_kernel(const GatedStateArgs a)
                 else f.u[r][i] = tk < n && col < V ? a.in[(size_t)(t0 + tk) * a.ld + a.at_v + h * V + col] : 0.f;
             }
     };
-    Frag cur;
-    load(c0, cur);
-    for (int ci = c0; ci < c1; ++ci) {
-        Frag next;
-        if (ci + 1 < c1) load(ci + 1, next);
+    // the chunk in `cur`, while the one AHEAD behind it is fetched into `ahead` (as many as the registers hold)
+    constexpr int AHEAD = NT < 4 ? 2 : 1;
+    auto step = [&](int ci, const Frag &cur, Frag &ahead) {
+        if (ci + AHEAD < c1) load(ci + AHEAD, ahead);
         float (*rd)[DELTA ? 4 : 2][64][4] = red[(ci - c0) & 1];
         gs_f4 ws[2], qs[2];
 #pragma unroll
@@ -547,7 +580,8 @@ __global__ __launch_bounds__(256) void state_scan_kernel(const GatedStateArgs a)
 #pragma unroll
             for (int i = 0; i < 4; ++i) {
                 const int tk = 16 * wave + 4 * g + i;
-                if (tk < cur.n && col < V) a.o[(size_t)(cur.t0 + tk) * a.heads * V + h * V + col] = o[i];
+                const int t = t_first + (ci - c0) * C + tk;
+                if (t < t_end && col < V) a.o[(size_t)t * a.heads * V + h * V + col] = o[i];
             }
         }
 #pragma unroll
@@ -556,7 +590,22 @@ __global__ __launch_bounds__(256) void state_scan_kernel(const GatedStateArgs a)
             s = gs_mma(cur.k[k][0], u[0], s);
             S[k] = gs_mma(cur.k[k][1], u[1], s);
         }
-        cur = next;
+    };
+    Frag f0, f1;
+    load(c0, f0);
+    if constexpr (AHEAD == 2) {
+        Frag f2;
+        if (c0 + 1 < c1) load(c0 + 1, f1);
+        for (int ci = c0; ci < c1; ci += 3) {
+            step(ci, f0, f2);
+            if (ci + 1 < c1) step(ci + 1, f1, f0);
+            if (ci + 2 < c1) step(ci + 2, f2, f1);
+        }
+    } else {
+        for (int ci = c0; ci < c1; ci += 2) {
+            step(ci, f0, f1);
+            if (ci + 1 < c1) step(ci + 1, f1, f0);
+        }
     }
 #pragma unroll
     for (int k = 0; k < NT; ++k)
@@ -567,7 +616,8 @@ __global__ __launch_bounds__(256) void state_scan_kernel(const GatedStateArgs a)
         }
 }
 
-// grid (T): a wave per head; the convolutions' inputs of a sequence's last tokens go to the tail (read by the launches before)
+// grid (T, groups of heads): a wave per head; the convolutions' inputs of a sequence's last tokens go to the tail (read by the
+// launches before)
 template <ActType ACT>
 __global__ __launch_bounds__(256) void gated_norm_kernel(const GatedStateArgs a, int T) {
     const int t = blockIdx.x, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, V = a.vdim, n = a.heads * V;
@@ -577,26 +627,28 @@ __global__ __launch_bounds__(256) void gated_norm_kernel(const GatedStateArgs a,
         if constexpr (ACT == ACT_BF16) static_cast<uint16_t *>(a.out)[to + i] = f32_to_bf16_bits(y);
         else static_cast<float *>(a.out)[to + i] = y;
     };
-    for (int h = wave; h < a.heads; h += 4) {
-        float ss = 0.f, v[STATE_DIM_MAX / 64];
+    for (int h = blockIdx.y * 4 + wave; h < a.heads; h += 4 * gridDim.y) {
+        float ss = 0.f, v[STATE_DIM_MAX / 64], gate[STATE_DIM_MAX / 64];
 #pragma unroll
         for (int k = 0; k < STATE_DIM_MAX / 64; ++k) {
             const int i = lane + 64 * k;
             v[k] = i < V ? o[h * V + i] : 0.f;
+            gate[k] = i < V ? x[a.at_g + h * V + i] : 0.f;
             ss = fmaf(v[k], v[k], ss);
         }
         const float r = 1.0f / sqrtf(gs_wave_sum(ss) / (float)V + a.eps);
 #pragma unroll
         for (int k = 0; k < STATE_DIM_MAX / 64; ++k) {
             const int i = lane + 64 * k;
-            if (i < V) put(h * V + i, v[k] * r * a.norm[i] * act_silu(x[a.at_g + h * V + i]));
+            if (i < V) put(h * V + i, v[k] * r * a.norm[i] * act_silu(gate[k]));
         }
     }
-    for (int i = n + tid; i < a.ld_out; i += 256) put(i, 0.f);
+    if (blockIdx.y == 0)
+        for (int i = n + tid; i < a.ld_out; i += 256) put(i, 0.f);
     if (a.delta && a.taps > 1 && (t + a.taps - 1 >= T || a.seq[t + a.taps - 1] != a.seq[t])) {
         const int qk = a.kv_heads * a.dim, channels = 2 * qk + n;
         float *slot = a.tail + ((size_t)a.seq[t] * a.taps + a.pos[t] % a.taps) * channels;
-        for (int i = tid; i < channels; i += 256) slot[i] = x[i < qk ? a.at_q + i : i < 2 * qk ? a.at_k + i - qk : a.at_v + i - 2 * qk];
+        for (int i = blockIdx.y * 256 + tid; i < channels; i += 256 * gridDim.y) slot[i] = x[i < qk ? a.at_q + i : i < 2 * qk ? a.at_k + i - qk : a.at_v + i - 2 * qk];
     }
 }
 
@@ -654,8 +706,9 @@ int gated_state_chunks(const GatedStateArgs &a, int T, hipStream_t stream) {
     MESH_LAUNCH_CHECK();
     const int rc = a.delta ? launch_scan<true>(a, stream) : launch_scan<false>(a, stream);
     if (rc != MESH_OK) return rc;
-    if (a.act == ACT_BF16) MESH_LAUNCH((gated_norm_kernel<ACT_BF16>), dim3((unsigned)T), dim3(256), 0, stream, a, T);
-    else MESH_LAUNCH((gated_norm_kernel<ACT_F32>), dim3((unsigned)T), dim3(256), 0, stream, a, T);
+    const dim3 norm_grid((unsigned)T, (unsigned)((a.heads + 7) / 8));          // two heads per wave
+    if (a.act == ACT_BF16) MESH_LAUNCH((gated_norm_kernel<ACT_BF16>), norm_grid, dim3(256), 0, stream, a, T);
+    else MESH_LAUNCH((gated_norm_kernel<ACT_F32>), norm_grid, dim3(256), 0, stream, a, T);
     MESH_LAUNCH_CHECK();
     return MESH_OK;
 }
