@@ -375,14 +375,30 @@ __global__ __launch_bounds__(PREP_THREADS) void gla_prepare_kernel(const GatedSt
     const int t0 = a.chunks.chunk[ci], n = a.chunks.chunk[ci + 1] - t0;
     float *sX = sG + C * dp, *sS = sX + C * a.rank;               // a1 rows; sums over the first half chunk
     const float qs = 1.0f / sqrtf((float)D);
-    for (int r = wave; r < C; r += 4) {
-        const float *x = a.in + (size_t)(t0 + (r < n ? r : 0)) * a.ld;
-        for (int d = lane; d < Dp; d += 64) {
+    // a wave's rows of 64 columns are all on their way before the first is kept
+    constexpr int ROWS = C / 4;
+    const float *xr[ROWS];
+#pragma unroll
+    for (int i = 0; i < ROWS; ++i) xr[i] = a.in + (size_t)(t0 + (wave + 4 * i < n ? wave + 4 * i : 0)) * a.ld;
+    for (int k = lane; k < a.rank; k += 64) {
+        float v[ROWS];
+#pragma unroll
+        for (int i = 0; i < ROWS; ++i) v[i] = xr[i][a.at_a + k];
+#pragma unroll
+        for (int i = 0; i < ROWS; ++i) sX[(wave + 4 * i) * a.rank + k] = wave + 4 * i < n ? v[i] : 0.f;
+    }
+    for (int d = lane; d < Dp; d += 64) {
+        float q[ROWS], k[ROWS];
+        const int from = h * D + (d < D ? d : 0);
+#pragma unroll
+        for (int i = 0; i < ROWS; ++i) { q[i] = xr[i][a.at_q + from]; k[i] = xr[i][a.at_k + from]; }
+#pragma unroll
+        for (int i = 0; i < ROWS; ++i) {
+            const int r = wave + 4 * i;
             const bool live = r < n && d < D;
-            sQ[r * dp + d] = live ? x[a.at_q + h * D + d] * qs : 0.f;
-            sK[r * dp + d] = live ? x[a.at_k + h * D + d] : 0.f;
+            sQ[r * dp + d] = live ? q[i] * qs : 0.f;
+            sK[r * dp + d] = live ? k[i] : 0.f;
         }
-        for (int k = lane; k < a.rank; k += 64) sX[r * a.rank + k] = r < n ? x[a.at_a + k] : 0.f;
     }
     __syncthreads();
     // a channel's half chunk per thread: its pre-activations, then the running sums of their logarithms

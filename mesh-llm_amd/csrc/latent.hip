@@ -143,21 +143,35 @@ __global__ __launch_bounds__(LT_THREADS) void latent_query_kernel(const LatentSh
     __syncthreads();
     const int per = (s.rank_pad + gridDim.y - 1) / gridDim.y, r1 = min((int)(blockIdx.y + 1) * per, s.rank_pad);
     const int piece = tid & 7, pieces = s.dim_pad / 8;
-    for (int r0 = blockIdx.y * per; r0 < r1; r0 += LT_THREADS / 8) {
-        const int r = r0 + (tid >> 3), rr = r < r1 ? r : r1 - 1;
-        float acc[TB];
+    constexpr int ROWS = LT_THREADS / 8, UR = TB == 1 ? 1 : 4;            // rows of a thread on their way at once
+    for (int r0 = blockIdx.y * per; r0 < r1; r0 += UR * ROWS) {
+        float acc[UR][TB];
+        const uint16_t *wr[UR];
 #pragma unroll
-        for (int b = 0; b < TB; ++b) acc[b] = 0.f;
+        for (int u = 0; u < UR; ++u) {
+            wr[u] = w + ((size_t)h * s.rank_pad + min(r0 + u * ROWS + (tid >> 3), r1 - 1)) * s.dim_pad;
+#pragma unroll
+            for (int b = 0; b < TB; ++b) acc[u][b] = 0.f;
+        }
+#pragma unroll 2
         for (int p = piece; p < pieces; p += 8) {
-            const uint4 wv = *reinterpret_cast<const uint4 *>(w + ((size_t)h * s.rank_pad + rr) * s.dim_pad + p * 8);
+            uint4 wv[UR];
 #pragma unroll
-            for (int b = 0; b < TB; ++b) acc[b] = lt_dot8(wv, xs + b * s.dim_pad + p * 8, acc[b]);
+            for (int u = 0; u < UR; ++u) wv[u] = *reinterpret_cast<const uint4 *>(wr[u] + p * 8);
+#pragma unroll
+            for (int u = 0; u < UR; ++u)
+#pragma unroll
+                for (int b = 0; b < TB; ++b) acc[u][b] = lt_dot8(wv[u], xs + b * s.dim_pad + p * 8, acc[u][b]);
         }
 #pragma unroll
-        for (int b = 0; b < TB; ++b) {
-            float v = acc[b];
-            v += __shfl_xor(v, 1); v += __shfl_xor(v, 2); v += __shfl_xor(v, 4);
-            if (piece == 0 && r < r1 && t0 + b < T) lt_put<ACT>(qa, ((size_t)(t0 + b) * s.heads + h) * s.row() + r, v, c.sat);
+        for (int u = 0; u < UR; ++u) {
+            const int r = r0 + u * ROWS + (tid >> 3);
+#pragma unroll
+            for (int b = 0; b < TB; ++b) {
+                float v = acc[u][b];
+                v += __shfl_xor(v, 1); v += __shfl_xor(v, 2); v += __shfl_xor(v, 4);
+                if (piece == 0 && r < r1 && t0 + b < T) lt_put<ACT>(qa, ((size_t)(t0 + b) * s.heads + h) * s.row() + r, v, c.sat);
+            }
         }
     }
 }
@@ -355,6 +369,7 @@ template <int TB>
 __global__ __launch_bounds__(LT_THREADS) void latent_out_kernel(const LatentShape s, const LatentAttnArgs a, int T) {
     extern __shared__ __align__(16) uint8_t smem[];
     __shared__ float s_w[TB][ATTN_SPLITS_CAP];
+    static_assert(ATTN_SPLITS_CAP == 64, "a lane per split");
     float *xs = reinterpret_cast<float *>(smem);              // [TB][rank_pad]
     const int h = blockIdx.x, t0 = blockIdx.z * TB, tid = threadIdx.x, lane = tid & 63, S = a.n_splits;
     for (int b = tid >> 6; b < TB; b += LT_WAVES) {
@@ -372,16 +387,38 @@ __global__ __launch_bounds__(LT_THREADS) void latent_out_kernel(const LatentShap
         s_w[b][lane] = w / den;
     }
     __syncthreads();
+    int live = 0, last[TB];       // splits of the group's longest token (the others' weights end in zeros); every token's last one
 #pragma unroll
     for (int b = 0; b < TB; ++b) {
-        const int t = min(t0 + b, T - 1), tg = t / a.group * a.group, n_keys = lt_group_keys(a.pos, tg, a.group, T), per = lt_split_keys(n_keys, S), live = (n_keys + per - 1) / per;
-        for (int r = tid; r < s.rank_pad; r += LT_THREADS) {
-            float v = 0.f;
-            const float *p = a.part + ((size_t)t * s.heads + h) * S * s.rank_pad + r;
-#pragma unroll 8
-            for (int k = 0; k < live; ++k) v = fmaf(p[(size_t)k * s.rank_pad], s_w[b][k], v);
-            xs[b * s.rank_pad + r] = v;
+        const int tg = min(t0 + b, T - 1) / a.group * a.group, n_keys = lt_group_keys(a.pos, tg, a.group, T), per = lt_split_keys(n_keys, S);
+        last[b] = (n_keys + per - 1) / per - 1;
+        live = max(live, last[b] + 1);
+    }
+    const float *part[TB];
+#pragma unroll
+    for (int b = 0; b < TB; ++b) part[b] = a.part + ((size_t)min(t0 + b, T - 1) * s.heads + h) * S * s.rank_pad;
+    for (int r = tid * 2; r < s.rank_pad; r += LT_THREADS * 2) {
+        float2 v[TB];
+#pragma unroll
+        for (int b = 0; b < TB; ++b) v[b] = make_float2(0.f, 0.f);
+        constexpr int KB = TB == 1 ? 16 : 8;            // splits on their way at once
+        for (int k0 = 0; k0 < live; k0 += KB) {
+            float2 x[KB][TB];
+#pragma unroll
+            for (int k = 0; k < KB; ++k)
+#pragma unroll
+                for (int b = 0; b < TB; ++b) x[k][b] = *reinterpret_cast<const float2 *>(part[b] + (size_t)min(k0 + k, last[b]) * s.rank_pad + r);
+#pragma unroll
+            for (int k = 0; k < KB; ++k)
+#pragma unroll
+                for (int b = 0; b < TB; ++b) {
+                    const float f = k0 + k < live ? s_w[b][k0 + k] : 0.f;
+                    v[b].x = fmaf(x[k][b].x, f, v[b].x);
+                    v[b].y = fmaf(x[k][b].y, f, v[b].y);
+                }
         }
+#pragma unroll
+        for (int b = 0; b < TB; ++b) *reinterpret_cast<float2 *>(xs + b * s.rank_pad + r) = v[b];
     }
     __syncthreads();
     const int slice = (s.v_pad + gridDim.y - 1) / gridDim.y, v1 = min((int)(blockIdx.y + 1) * slice, s.v_pad);
@@ -389,27 +426,40 @@ __global__ __launch_bounds__(LT_THREADS) void latent_out_kernel(const LatentShap
     float gate[TB];
 #pragma unroll
     for (int b = 0; b < TB; ++b) gate[b] = act_sigmoid(a.gate[(size_t)min(t0 + b, T - 1) * a.gate_ld + h]);
-    for (int v0 = blockIdx.y * slice; v0 < v1; v0 += LT_THREADS / 16) {
+    constexpr int ROWS = LT_THREADS / 16, UR = TB == 1 ? 1 : 4;           // rows of a thread on their way at once
+    for (int v0 = blockIdx.y * slice; v0 < v1; v0 += UR * ROWS) {
         const int v = v0 + (tid >> 4);
-        float acc[TB];
+        float acc[UR][TB];
 #pragma unroll
-        for (int b = 0; b < TB; ++b) acc[b] = 0.f;
-        if (v < s.vdim)
-            for (int p = piece; p < pieces; p += 16) {
-                const uint4 wv = *reinterpret_cast<const uint4 *>(a.w_uv + ((size_t)h * s.vdim + v) * s.rank_pad + p * 8);
+        for (int u = 0; u < UR; ++u)
 #pragma unroll
-                for (int b = 0; b < TB; ++b) acc[b] = lt_dot8(wv, xs + b * s.rank_pad + p * 8, acc[b]);
+            for (int b = 0; b < TB; ++b) acc[u][b] = 0.f;
+        const int end = min(v1, s.vdim);          // (rows past the values are zeros)
+#pragma unroll 4
+        for (int p = piece; p < pieces; p += 16) {
+            uint4 wv[UR];
+#pragma unroll
+            for (int u = 0; u < UR; ++u) {
+                wv[u] = make_uint4(0, 0, 0, 0);
+                if (v + u * ROWS < end) wv[u] = *reinterpret_cast<const uint4 *>(a.w_uv + ((size_t)h * s.vdim + v + u * ROWS) * s.rank_pad + p * 8);
             }
 #pragma unroll
-        for (int b = 0; b < TB; ++b) {
-            float y = acc[b];
-            y += __shfl_xor(y, 1); y += __shfl_xor(y, 2); y += __shfl_xor(y, 4); y += __shfl_xor(y, 8);
-            if (piece == 0 && v < v1 && t0 + b < T) {
-                const size_t at = ((size_t)(t0 + b) * s.heads + h) * s.v_pad + v;
-                if (a.out_bf16) a.out_bf16[at] = f32_to_bf16_bits(y * gate[b]);
-                else a.out[at] = y * gate[b];
-            }
+            for (int u = 0; u < UR; ++u)
+#pragma unroll
+                for (int b = 0; b < TB; ++b) acc[u][b] = lt_dot8(wv[u], xs + b * s.rank_pad + p * 8, acc[u][b]);
         }
+#pragma unroll
+        for (int u = 0; u < UR; ++u)
+#pragma unroll
+            for (int b = 0; b < TB; ++b) {
+                float y = acc[u][b];
+                y += __shfl_xor(y, 1); y += __shfl_xor(y, 2); y += __shfl_xor(y, 4); y += __shfl_xor(y, 8);
+                if (piece == 0 && v + u * ROWS < v1 && t0 + b < T) {
+                    const size_t at = ((size_t)(t0 + b) * s.heads + h) * s.v_pad + v + u * ROWS;
+                    if (a.out_bf16) a.out_bf16[at] = f32_to_bf16_bits(y * gate[b]);
+                    else a.out[at] = y * gate[b];
+                }
+            }
     }
 }
 
