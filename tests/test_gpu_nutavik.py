@@ -4,6 +4,7 @@ trace runner."""
 import json
 import os
 import subprocess
+import urllib.request
 
 import numpy as np
 import pytest
@@ -350,6 +351,31 @@ def test_greedy_generation_through_the_session(tmp_path, prec):
         check_greedy(orc, p, o, 1e-3 if prec == "f32" else 1.0)
     ses.close()
     st.close()
+
+
+def test_greedy_generation_through_the_plugin_endpoint(tmp_path):
+    from plugin_host import PB, PluginHost
+    cfg, w, folder, orc = made(tmp_path, "mixed")
+    host = PluginHost(os.path.join(ROOT, "mesh-llm_amd", "mesh-stage-plugin"), ["--model", folder, "--precision", "f32", "-c", "128", "--batch", "64"], tmp_path, name="latent")
+    info = json.loads(host.initialize().initialize_response.server_info_json)
+    assert info["arch"] == "Nutavik" and info["stage_open"] is True
+    env = host.request(initialize_request=PB["InitializeRequest"](host_protocol_version=2, host_version="t", host_info_json="{}", mesh_visibility=1))
+    address = env.initialize_response.manifest.endpoints[0].address
+
+    def post(ids, pos0):
+        req = urllib.request.Request(address + "/stage/decode", data=np.asarray(ids, np.int32).tobytes(), method="POST",
+                                     headers={"X-Mesh-Tokens": str(len(ids)), "X-Mesh-Pos0": str(pos0), "X-Mesh-In-Format": "tokens", "X-Mesh-Out-Format": "logits",
+                                              "X-Mesh-Want": str(len(ids) - 1)})
+        with urllib.request.urlopen(req, timeout=60) as r:
+            return np.frombuffer(r.read(), np.float32)
+
+    p = prompt(cfg, 39, 77)
+    out = [int(post(p, 0).argmax())]
+    for i in range(15):
+        out.append(int(post(out[-1:], len(p) + i).argmax()))
+    check_greedy(orc, p, out, 1e-3)
+    host.request(shutdown_request=PB["ShutdownRequest"](reason="done"))
+    host.close()
 
 
 @BOTH
